@@ -54,13 +54,9 @@ def ensure_gateway_binaries() -> Path:
 
 
 def ensure_kernels() -> None:
-    lib = REPO / "llmlb_amd" / "ops" / "libllmlb_kernels.so"
-    if not lib.exists():
-        srcs = sorted((REPO / "llmlb_amd/ops/csrc").glob("*.hip"))
-        subprocess.run(["/opt/rocm/bin/hipcc", "--offload-arch=gfx950",
-                        "-O3", "-std=c++17", "-shared", "-fPIC",
-                        *[str(s) for s in srcs], "-o", str(lib)],
-                       check=True)
+    from llmlb_amd.ops.build import LIBRARIES, ensure_library
+    for name in LIBRARIES:
+        ensure_library(name)
 
 
 # ---------------------------------------------------------------------

@@ -22,8 +22,13 @@ Optional serving features (all measured in profiles/):
   * chunked prefill for long prompts (prefill_chunk),
   * prompt-lookup speculative decoding (spec_ngram / LLMLB_SPEC_NGRAM),
   * FP8 e4m3 KV cache (kv_dtype="fp8_e4m3"),
-  * HF-safetensors checkpoint loading (weights_path),
+  * safetensors checkpoint loading (weights_path),
   * request cancellation (abort()).
+
+Hybrid models (``ragged`` model classes) take the same requests through
+one packed forward per step: every running sequence's next token beside
+portions of the prompts still being read (``run_batch``), against a
+HybridCache whose state slots are the decode rows.
 """
 from __future__ import annotations
 
@@ -39,8 +44,10 @@ log = logging.getLogger("llmlb.engine")
 import torch
 
 from .. import ops
-from ..models.llama import LlamaConfig, LlamaForCausalLM
-from .kv_cache import BLOCK_SIZE, KVCache, PrefixCache
+from ..models.llama import LlamaConfig
+from ..models.registry import model_class
+from .kv_cache import BLOCK_SIZE, HybridCache, KVCache, PrefixCache
+from .ragged import RaggedBatch
 from .sampler import SamplingParams, sample
 
 
@@ -54,7 +61,7 @@ def os_env_flag(name: str, default: bool) -> bool:
 
 @dataclass
 class EngineConfig:
-    model: LlamaConfig
+    model: LlamaConfig          # or another config of models/registry.py
     device: str = "cuda:0"
     dtype: str = "bfloat16"
     kv_cache_blocks: int | None = None     # None = size from HBM budget
@@ -225,17 +232,67 @@ class _DecodeGraph:
         return self.logits[:n]
 
 
+class _RaggedGraph:
+    """A hipGraph of one decode forward of a ``ragged`` model at a padded
+    batch size.  A step fills one int buffer and replays.  Padded rows
+    use table row ``max_rows``, whose pages are all the sacrificial block
+    0 and whose state slot no sequence owns."""
+
+    BUCKETS = (1, 2, 4) + _DecodeGraph.BUCKETS
+
+    def __init__(self, engine: "Engine", S: int):
+        self.S, self._engine = S, engine
+        self.flat = torch.zeros(RaggedBatch.int_count(S, S),
+                                dtype=torch.int32, device=engine.device)
+        self.batch = None
+
+    def _fill(self, runs) -> None:
+        runs = runs + [(self._engine.max_rows, 0, [0])] \
+            * (self.S - len(runs))
+        self.flat.copy_(torch.tensor(RaggedBatch.pack(runs),
+                                     dtype=torch.int32))
+        if self.batch is None:
+            self.batch = RaggedBatch.over(self.flat, runs,
+                                          self._engine._bt_dev)
+
+    def _forward(self) -> torch.Tensor:
+        model = self._engine.model
+        return model.logits(model.forward(self.batch, self._engine.kv))
+
+    def capture(self) -> None:
+        self._fill([])
+        torch.cuda.synchronize()
+        side = torch.cuda.Stream()
+        side.wait_stream(torch.cuda.current_stream())
+        with torch.cuda.stream(side):
+            for _ in range(2):
+                self._forward()
+        torch.cuda.current_stream().wait_stream(side)
+        torch.cuda.synchronize()
+        self.graph = torch.cuda.CUDAGraph()
+        with torch.cuda.graph(self.graph):
+            self.logits = self._forward()
+
+    def run(self, runs) -> torch.Tensor:
+        self._fill(runs)
+        self.graph.replay()
+        return self.logits[:len(runs)]
+
+
 class Engine:
     def __init__(self, cfg: EngineConfig):
         self.cfg = cfg
         self.device = torch.device(cfg.device)
         dtype = getattr(torch, cfg.dtype)
-        self.model = LlamaForCausalLM(cfg.model, tp=cfg.tp_ctx, dtype=dtype,
-                                      device=cfg.device, seed=cfg.seed,
-                                      init_weights=not cfg.weights_path)
+        cls = model_class(cfg.model)
+        self.ragged = getattr(cls, "ragged", False)
+        self.model = cls(cfg.model, tp=cfg.tp_ctx, dtype=dtype,
+                         device=cfg.device, seed=cfg.seed,
+                         init_weights=not cfg.weights_path)
         if cfg.weights_path:
             self.model.load_safetensors(cfg.weights_path)
-        if ((ops.w8a8_active() or ops._FP8_WEIGHTS)
+        if (not self.ragged
+                and (ops.w8a8_active() or ops._FP8_WEIGHTS)
                 and self.device.type == "cuda"):
             # pre-quantize the fp8 weight copies NOW: lazily they are
             # built inside the first decode's graph capture, which the
@@ -298,23 +355,14 @@ class Engine:
                 except Exception:
                     pass
         m = cfg.model
-        n_kv_local = m.kv_heads // self.model.tp.world_size
-        import os as _os0
-        self.kv_dtype = _os0.environ.get("LLMLB_KV_DTYPE",
-                                         cfg.kv_dtype) or "bfloat16"
-        if (self.kv_dtype == "fp8_e4m3" and self.device.type == "cuda"
-                and (m.head_dim != 128
-                     or m.q_heads // m.kv_heads > 16)):
-            raise ValueError(
-                "fp8_e4m3 KV on GPU requires head_dim=128 and GQA "
-                f"group <= 16 (got D={m.head_dim}, "
-                f"group={m.q_heads // m.kv_heads})")
-        num_blocks = cfg.kv_cache_blocks or self._auto_blocks(n_kv_local)
-        self.kv = KVCache(m.layers, num_blocks, n_kv_local, m.head_dim,
-                          self.device, dtype, kv_dtype=self.kv_dtype)
+        self.max_rows = cfg.max_batch
+        self._init_cache(dtype)
         import os as _os
         self.spec_ngram = int(_os.environ.get("LLMLB_SPEC_NGRAM",
                                               str(cfg.spec_ngram)) or 0)
+        if self.ragged:
+            # a rejected draft cannot be taken out of a recurrent state
+            self.spec_ngram = 0
         # decode piggyback at prefill-chunk boundaries (A/B knob)
         self._piggyback = _os.environ.get(
             "LLMLB_PREFILL_PIGGYBACK", "1").lower() not in (
@@ -322,7 +370,7 @@ class Engine:
         self.spec_proposed = 0
         self.spec_accepted = 0
         self.prefix = (PrefixCache(self.kv)
-                       if cfg.enable_prefix_cache
+                       if cfg.enable_prefix_cache and not self.ragged
                        and os_env_flag("LLMLB_PREFIX_CACHE", True)
                        else None)
         self.running: list[_Sequence] = []
@@ -332,9 +380,6 @@ class Engine:
         self._abort_rids: set[int] = set()
         self._stop = threading.Event()
         self._thread: threading.Thread | None = None
-        self.scale = m.head_dim ** -0.5
-        self.n_q_local = m.q_heads // self.model.tp.world_size
-        self.n_kv_local = n_kv_local
         self.steps_done = 0
         self.tokens_out = 0
         # observability: hipEvent-tagged decode-step GPU time (sampled
@@ -349,11 +394,12 @@ class Engine:
         self._ev_end = None
 
         # persistent decode state (device-resident)
-        self.max_rows = cfg.max_batch
         self.max_blocks_per_seq = min(
-            (m.max_pos + BLOCK_SIZE - 1) // BLOCK_SIZE, num_blocks)
+            (m.max_pos + BLOCK_SIZE - 1) // BLOCK_SIZE, self.kv.num_blocks)
         dev = self.device
-        self._bt_dev = torch.zeros(self.max_rows, self.max_blocks_per_seq,
+        # one row more than sequences: padded rows of captured steps
+        self._bt_dev = torch.zeros(self.max_rows + 1,
+                                   self.max_blocks_per_seq,
                                    dtype=torch.int32, device=dev)
         self._len_dev = torch.zeros(self.max_rows, dtype=torch.int32,
                                     device=dev)
@@ -365,7 +411,7 @@ class Engine:
         # hipGraph-captured decode steps, one per padded batch bucket
         self.use_graphs = (self.device.type == "cuda"
                            and self.model.tp.world_size == 1
-                           and cfg.model.layers > 0
+                           and bool(cfg.model.layers)
                            and os_env_flag("LLMLB_DECODE_GRAPHS", True))
         self._graphs: dict[int, _DecodeGraph] = {}
         self.timing = defaultdict(float) \
@@ -377,17 +423,56 @@ class Engine:
                                    or cfg.max_prefill_tokens))
 
     # -- sizing ----------------------------------------------------------
+    def _init_cache(self, dtype) -> None:
+        import os
+        cfg, m = self.cfg, self.cfg.model
+        if self.ragged:
+            self.kv_dtype = os.environ.get("LLMLB_KV_DTYPE",
+                                           cfg.kv_dtype) or "bfloat16"
+            if self.kv_dtype == "fp8_e4m3":
+                raise ValueError("fp8_e4m3 KV is not available for "
+                                 f"{m.architecture}")
+            specs = self.model.specs
+            per_block = HybridCache.block_bytes(specs, dtype)
+            state = HybridCache.state_bytes(specs, self.max_rows, dtype)
+            blocks = cfg.kv_cache_blocks
+            if blocks is None:
+                blocks = max((self._cache_budget() - state)
+                             // max(per_block, 1), 16)
+                # no more than every row at full length can use
+                blocks = min(blocks, 1 + self.max_rows
+                             * -(-m.max_pos // BLOCK_SIZE))
+            self.kv = self.model.make_cache(blocks, self.max_rows)
+            return
+        n_kv_local = m.kv_heads // self.model.tp.world_size
+        self.kv_dtype = os.environ.get("LLMLB_KV_DTYPE",
+                                         cfg.kv_dtype) or "bfloat16"
+        if (self.kv_dtype == "fp8_e4m3" and self.device.type == "cuda"
+                and (m.head_dim != 128
+                     or m.q_heads // m.kv_heads > 16)):
+            raise ValueError(
+                "fp8_e4m3 KV on GPU requires head_dim=128 and GQA "
+                f"group <= 16 (got D={m.head_dim}, "
+                f"group={m.q_heads // m.kv_heads})")
+        num_blocks = cfg.kv_cache_blocks or self._auto_blocks(n_kv_local)
+        self.kv = KVCache(m.layers, num_blocks, n_kv_local, m.head_dim,
+                          self.device, dtype, kv_dtype=self.kv_dtype)
+        self.scale = m.head_dim ** -0.5
+        self.n_q_local = m.q_heads // self.model.tp.world_size
+        self.n_kv_local = n_kv_local
+
+    def _cache_budget(self) -> int:
+        if self.device.type == "cuda":
+            free, _total = torch.cuda.mem_get_info(self.device)
+            return int(free * self.cfg.hbm_fraction)
+        return 64 * 1024 * 1024  # CPU tests: small
+
     def _auto_blocks(self, n_kv_local: int) -> int:
         m = self.cfg.model
         per_block = KVCache.bytes_per_block(m.layers, n_kv_local,
                                             m.head_dim,
                                             kv_dtype=self.kv_dtype)
-        if self.device.type == "cuda":
-            free, _total = torch.cuda.mem_get_info(self.device)
-            budget = int(free * self.cfg.hbm_fraction)
-        else:
-            budget = 64 * 1024 * 1024  # CPU tests: small
-        return max(budget // per_block, 16)
+        return max(self._cache_budget() // per_block, 16)
 
     # -- public API ------------------------------------------------------
     def submit(self, prompt_ids: list[int],
@@ -559,9 +644,11 @@ class Engine:
         """One scheduler iteration.  Returns True if any work was done."""
         self._apply_aborts()
         prefills = self._admit()
-        if prefills:
+        if self.ragged:
+            self._ragged_step(prefills)
+        elif prefills:
             self._prefill_batch(prefills)
-        if self.running:
+        if self.running and not self.ragged:
             if (self.spec_ngram > 0
                     and all(s.params.temperature < 1e-5
                             and not s.params.needs_slow_path()
@@ -845,6 +932,163 @@ class Engine:
             self.timing["emit"] += time.monotonic() - _t3
             self.timing["steps"] += 1
 
+    # -- packed batches (hybrid models) ----------------------------------
+    def open_sequence(self, params: SamplingParams | None = None
+                      ) -> _Sequence:
+        """A live sequence fed through ``run_batch`` by the caller: it
+        takes a decode row (and with it a state slot), pages as its
+        tokens come.  End it with ``close_sequence``."""
+        if not self.ragged:
+            raise ValueError(f"{self.cfg.model.name} does not run packed "
+                             "batches")
+        if not self._free_rows:
+            raise RuntimeError(f"all {self.max_rows} sequence slots are "
+                               "in use")
+        with self._rid_lock:
+            rid = self._next_rid
+            self._next_rid += 1
+        seq = _Sequence(rid, [], params or SamplingParams(), queue.Queue(),
+                        None)
+        seq.row = self._free_rows.pop()
+        return seq
+
+    def close_sequence(self, seq: _Sequence) -> None:
+        """Give back what the sequence holds."""
+        self._retire(seq)
+
+    def _grow_tables(self, work) -> None:
+        """Pages for every run's tokens, all or nothing."""
+        need = [(seq, -(-(seq.length + len(toks)) // BLOCK_SIZE)
+                 - len(seq.block_table)) for seq, toks, _ in work]
+        total = sum(max(n, 0) for _, n in need)
+        if not total:
+            return
+        if total > self.kv.free_blocks():
+            raise MemoryError(f"KV cache exhausted: want {total} blocks, "
+                              f"{self.kv.free_blocks()} free")
+        self._write_tables([(seq, self.kv.allocate(n))
+                            for seq, n in need if n > 0])
+
+    def _write_tables(self, new) -> None:
+        """Append page lists to sequences and to the device table."""
+        cells = []
+        for seq, blocks in new:
+            at = len(seq.block_table)
+            seq.block_table = seq.block_table + blocks
+            cells += [(seq.row, at + i, blk) for i, blk in enumerate(blocks)]
+        rows, cols, vals = torch.tensor(cells, device=self.device).unbind(1)
+        self._bt_dev[rows, cols] = vals.to(torch.int32)
+
+    @torch.inference_mode()
+    def run_batch(self, work) -> torch.Tensor:
+        """Run the next tokens of several sequences as one batch.
+
+        ``work``: [(sequence, token ids, wanted places among them)].
+        Returns float32 logits [wanted, vocab] in that order.  Only the
+        given tokens are computed; everything before them comes from the
+        cache and the recurrent state."""
+        vocab = self.cfg.model.vocab
+        cap = min(self.cfg.model.max_pos,
+                  self.max_blocks_per_seq * BLOCK_SIZE)
+        for seq, toks, want in work:
+            if not toks or min(toks) < 0 or max(toks) >= vocab:
+                raise ValueError("token ids must be in [0, vocab)")
+            if seq.length + len(toks) > cap:
+                raise ValueError(f"sequence longer than {cap} tokens")
+            if any(not 0 <= i < len(toks) for i in want):
+                raise ValueError("wanted place outside the tokens")
+        if len({id(seq) for seq, _, _ in work}) != len(work):
+            raise ValueError("a sequence may appear once in a batch")
+        if not work:
+            return torch.empty(0, vocab, device=self.device)
+        self._grow_tables(work)
+        order = sorted(range(len(work)), key=lambda i: len(work[i][1]))
+        runs = [(work[i][0].row, work[i][0].length, work[i][1])
+                for i in order]
+        start, at = {}, 0
+        for i in order:
+            start[i] = at
+            at += len(work[i][1])
+        index = [start[i] + j for i, (_, _, want) in enumerate(work)
+                 for j in want]
+        graph = self._graph_for(len(runs)) if at == len(runs) else None
+        if graph is not None:
+            logits = graph.run(runs)
+            if index != list(range(len(runs))):
+                logits = logits[torch.tensor(index, dtype=torch.long,
+                                             device=self.device)]
+        else:
+            x = self.model.forward(RaggedBatch.build(runs, self._bt_dev),
+                                   self.kv)
+            logits = self.model.logits(x, torch.tensor(
+                index, dtype=torch.int32, device=self.device)) \
+                if index else torch.empty(0, vocab, device=self.device)
+        for seq, toks, _ in work:
+            seq.length += len(toks)
+        return logits
+
+    def _reject_reason(self, seq: _Sequence) -> str | None:
+        """Why a request can never run, or None."""
+        m, ids = self.cfg.model, seq.prompt_ids
+        if not ids:
+            return "empty prompt"
+        if min(ids) < 0 or max(ids) >= m.vocab:
+            return "token id outside the vocabulary"
+        if len(ids) + seq.max_new > min(
+                m.max_pos, self.max_blocks_per_seq * BLOCK_SIZE):
+            return "prompt longer than the context window"
+        return None
+
+    def _ragged_step(self, admitted: list[_Sequence]) -> None:
+        """One packed forward: a token of every decoding sequence, and
+        up to ``prefill_chunk`` tokens of prompts still being read."""
+        for seq in admitted:
+            blocks, seq.block_table = seq.block_table, []
+            self._write_tables([(seq, blocks)])
+            self.running.append(seq)
+            reason = self._reject_reason(seq)
+            if reason is not None:
+                seq.out_queue.put((0, "error", {"error": reason}))
+                self._retire(seq)
+        budget = max(self.cfg.prefill_chunk, 1)
+        work = []
+        for seq in self.running:
+            left = len(seq.prompt_ids) - seq.length
+            if left > 0:
+                n = min(left, budget)
+                if not n:
+                    continue
+                budget -= n
+                toks = seq.prompt_ids[seq.length:seq.length + n]
+                work.append((seq, toks, [n - 1] if n == left else []))
+            else:
+                work.append((seq, [seq.out_ids[-1]], [0]))
+        if not work:
+            return
+        timed = self.device.type == "cuda" and self.steps_done % 32 == 0
+        if timed:
+            if self._ev_start is None:
+                self._ev_start = torch.cuda.Event(enable_timing=True)
+                self._ev_end = torch.cuda.Event(enable_timing=True)
+            self._ev_start.record()
+        logits = self.run_batch(work)
+        seqs = [seq for seq, _, want in work if want]
+        toks = sample(logits, [s.params for s in seqs],
+                      [s.generator for s in seqs],
+                      histories=[(s.prompt_ids, s.out_ids) for s in seqs])
+        if timed:
+            self._ev_end.record()
+        toks_cpu = toks.tolist()
+        if timed and toks_cpu:
+            ms = self._ev_start.elapsed_time(self._ev_end)
+            self.gpu_step_ms_ema = (ms if self.gpu_step_ms_ema == 0
+                                    else 0.2 * ms
+                                    + 0.8 * self.gpu_step_ms_ema)
+        extras = self._logprob_extras(logits, toks, seqs)
+        for seq, tok, ex in zip(seqs, toks_cpu, extras):
+            if not self._push_token(seq, tok, ex):
+                self._retire(seq)
+
     # -- prompt-lookup speculative decoding ------------------------------
     def _draft_for(self, seq: _Sequence) -> list[int]:
         """Prompt-lookup draft v2: match the trailing TRIGRAM first
@@ -1042,8 +1286,9 @@ class Engine:
     def _graph_for(self, S: int) -> "_DecodeGraph | None":
         if not self.use_graphs:
             return None
+        kind = _RaggedGraph if self.ragged else _DecodeGraph
         bucket = None
-        for b in _DecodeGraph.BUCKETS:
+        for b in kind.BUCKETS:
             if S <= b <= self.max_rows:
                 bucket = b
                 break
@@ -1051,7 +1296,7 @@ class Engine:
             return None
         g = self._graphs.get(bucket)
         if g is None:
-            g = _DecodeGraph(self, bucket)
+            g = kind(self, bucket)
             try:
                 g.capture()
             except Exception as e:  # graphs are an optimization only

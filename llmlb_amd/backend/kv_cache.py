@@ -16,18 +16,47 @@ reuses those KV pages and prefills only the suffix.  Retired pages
 with no active users park in an LRU pool and are evicted back to the
 free list on demand — with 288 GB of HBM3E the pool is effectively a
 multi-gigabyte prompt cache.
+
+``HybridCache`` serves models that mix latent attention with recurrent
+layers: the same pages hold latents, and each live sequence owns one
+slot of recurrent state.
 """
 from __future__ import annotations
 
 import hashlib
 from collections import OrderedDict
+from dataclasses import dataclass
 
 import torch
 
 BLOCK_SIZE = 16  # tokens per page (matches PA_BLOCK in kernels.hip)
 
 
-class KVCache:
+class PagePool:
+    """Free list of cache pages.  Block 0 is reserved as the sacrificial
+    target of padded rows in hipGraph-captured decode steps
+    (engine._DecodeGraph)."""
+
+    block_size = BLOCK_SIZE
+
+    def __init__(self, num_blocks: int):
+        self.num_blocks = num_blocks
+        self._free: list[int] = list(range(num_blocks - 1, 0, -1))
+
+    def free_blocks(self) -> int:
+        return len(self._free)
+
+    def allocate(self, n: int) -> list[int]:
+        if n > len(self._free):
+            raise MemoryError(f"KV cache exhausted: want {n} blocks, "
+                              f"{len(self._free)} free")
+        return [self._free.pop() for _ in range(n)]
+
+    def release(self, blocks: list[int]) -> None:
+        self._free.extend(blocks)
+
+
+class KVCache(PagePool):
     """``kv_dtype="fp8_e4m3"`` stores K/V as OCP e4m3 bytes (gfx950's
     native FP8) with one fp32 scale per (page, head, token) — half the
     attention bandwidth and double the resident context of bf16."""
@@ -35,8 +64,7 @@ class KVCache:
     def __init__(self, layers: int, num_blocks: int, n_kv: int,
                  head_dim: int, device, dtype=torch.bfloat16,
                  kv_dtype: str = "bfloat16"):
-        self.block_size = BLOCK_SIZE
-        self.num_blocks = num_blocks
+        super().__init__(num_blocks)
         self.fp8 = kv_dtype == "fp8_e4m3"
         store = torch.uint8 if self.fp8 else dtype
         self.k = [torch.zeros(num_blocks, n_kv, BLOCK_SIZE, head_dim,
@@ -57,9 +85,6 @@ class KVCache:
         else:
             self.k_scale = self.v_scale = None
         self.out_dtype = dtype
-        # block 0 is reserved as the sacrificial target of padded rows
-        # in hipGraph-captured decode steps (engine._DecodeGraph)
-        self._free: list[int] = list(range(num_blocks - 1, 0, -1))
 
     def gather(self, li: int, blks: torch.Tensor, offs: torch.Tensor):
         """K/V rows at (block, offset) as compute-dtype tensors
@@ -83,17 +108,71 @@ class KVCache:
         esize = torch.tensor([], dtype=dtype).element_size()
         return 2 * layers * n_kv * BLOCK_SIZE * head_dim * esize
 
-    def free_blocks(self) -> int:
-        return len(self._free)
 
-    def allocate(self, n: int) -> list[int]:
-        if n > len(self._free):
-            raise MemoryError(f"KV cache exhausted: want {n} blocks, "
-                              f"{len(self._free)} free")
-        return [self._free.pop() for _ in range(n)]
+@dataclass(frozen=True)
+class LatentSpec:
+    """A layer that keeps ``width`` numbers per token in the pages."""
+    width: int
 
-    def release(self, blocks: list[int]) -> None:
-        self._free.extend(blocks)
+    def page_bytes(self, esize: int) -> int:
+        return BLOCK_SIZE * self.width * esize
+
+
+@dataclass(frozen=True)
+class DeltaSpec:
+    """A recurrent layer: per sequence a float state of
+    heads x vdim x dim and the last ``taps`` inputs of ``channels``
+    convolved channels."""
+    heads: int
+    vdim: int
+    dim: int
+    channels: int
+    taps: int
+
+    def slot_bytes(self, esize: int) -> int:
+        return (4 * self.heads * self.vdim * self.dim
+                + esize * self.taps * self.channels)
+
+
+class HybridCache(PagePool):
+    """Pages of latents and slots of recurrent state for one model.
+
+    ``specs[i]`` is layer i's LatentSpec, DeltaSpec or None (a layer
+    that reads another's latents).  All latent layers share one block
+    table.  State slots are the engine's decode rows, plus one more for
+    the padded rows of captured decode steps.  Nothing is cleared when a
+    page or slot changes hands: kernels read only positions that the
+    sequence itself has written, and position 0 starts from a zero
+    state."""
+
+    fp8 = False
+
+    def __init__(self, specs, num_blocks: int, slots: int, device, dtype):
+        super().__init__(num_blocks)
+        self.slots = slots
+        self.latent, self.state, self.ring = {}, {}, {}
+        for i, s in enumerate(specs):
+            if isinstance(s, LatentSpec):
+                self.latent[i] = torch.zeros(num_blocks, BLOCK_SIZE, s.width,
+                                             dtype=dtype, device=device)
+            elif isinstance(s, DeltaSpec):
+                self.state[i] = torch.zeros(
+                    slots + 1, s.heads, s.vdim, s.dim,
+                    dtype=torch.float32, device=device)
+                self.ring[i] = torch.zeros(slots + 1, s.taps, s.channels,
+                                           dtype=dtype, device=device)
+
+    @staticmethod
+    def block_bytes(specs, dtype) -> int:
+        esize = torch.tensor([], dtype=dtype).element_size()
+        return sum(s.page_bytes(esize) for s in specs
+                   if isinstance(s, LatentSpec))
+
+    @staticmethod
+    def state_bytes(specs, slots: int, dtype) -> int:
+        esize = torch.tensor([], dtype=dtype).element_size()
+        return (slots + 1) * sum(s.slot_bytes(esize) for s in specs
+                                 if isinstance(s, DeltaSpec))
 
 
 class PrefixCache:

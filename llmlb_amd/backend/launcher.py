@@ -5,7 +5,8 @@ CLI (also used by bench.py and the gateway's node tooling):
   python -m llmlb_amd.backend.launcher --model llama-3-8b \
       --device cuda:0 --port 9200 [--served-name NAME] [--kv-blocks N]
 
-Model configs resolve through LlamaConfig presets; TP replicas use
+Model configs resolve through models/registry.py: a preset, or a folder
+with config.json and *.safetensors.  TP replicas use
 torchrun with --tp N (each rank binds cuda:LOCAL_RANK; rank 0 serves
 HTTP and broadcasts per-step schedules — see parallel/tp.py).
 """
@@ -15,17 +16,8 @@ import argparse
 
 import torch
 
-from ..models.llama import LlamaConfig
+from ..models.registry import PRESETS, resolve  # noqa: F401
 from .engine import Engine, EngineConfig
-
-PRESETS = {
-    "llama-3-8b": LlamaConfig.llama3_8b,
-    "llama-3-70b": LlamaConfig.llama3_70b,
-    "qwen2-7b": LlamaConfig.qwen2_7b,
-    "qwen2-0.5b": LlamaConfig.qwen2_0_5b,
-    "llama-tiny": LlamaConfig.tiny,
-    "llama-small": LlamaConfig.small,
-}
 
 
 def build_engine(model: str, device: str, kv_blocks: int | None = None,
@@ -35,11 +27,8 @@ def build_engine(model: str, device: str, kv_blocks: int | None = None,
                  max_prefill_tokens: int | None = None) -> Engine:
     """tp_ctx=None means 'infer from torch.distributed' — pass
     TPContext.solo() for DP replicas inside a larger world."""
-    cfg_fn = PRESETS.get(model)
-    if cfg_fn is None:
-        raise SystemExit(f"unknown model preset '{model}' "
-                         f"(have: {', '.join(PRESETS)})")
-    mcfg = cfg_fn()
+    mcfg, folder = resolve(model)
+    weights = weights or folder
     dtype = "bfloat16" if device.startswith("cuda") else "float32"
     ecfg = EngineConfig(model=mcfg, device=device, dtype=dtype,
                         kv_cache_blocks=kv_blocks, max_batch=max_batch,
@@ -52,7 +41,8 @@ def build_engine(model: str, device: str, kv_blocks: int | None = None,
 
 def main(argv=None) -> None:
     ap = argparse.ArgumentParser(description="llmlb_amd backend replica")
-    ap.add_argument("--model", default="llama-3-8b")
+    ap.add_argument("--model", default="llama-3-8b",
+                    help="preset, or a folder with config.json and weights")
     ap.add_argument("--served-name", default=None,
                     help="model id to serve (defaults to preset name)")
     ap.add_argument("--device", default=None)
@@ -60,7 +50,7 @@ def main(argv=None) -> None:
     ap.add_argument("--port", type=int, default=9200)
     ap.add_argument("--kv-blocks", type=int, default=None)
     ap.add_argument("--weights", default=None,
-                    help="HF safetensors checkpoint (file or dir)")
+                    help="safetensors checkpoint (file or dir)")
     ap.add_argument("--tokenizer", default=None,
                     help="local tokenizer.json (tokenizers format)")
     ap.add_argument("--max-batch", type=int, default=256)

@@ -1,0 +1,83 @@
+"""One packed forward batch of unequal token runs.
+
+A step of a hybrid model runs portions of prompts beside single decoded
+tokens.  Their tokens lie packed one after another; kernels find a
+token's place through per-token and per-entry arrays that travel to the
+GPU in a single copy.  Entries with few tokens come first, so that each
+attention form finds its tokens in one run.
+"""
+from __future__ import annotations
+
+from dataclasses import dataclass
+
+import torch
+
+# longest entry whose queries attend through the absorbed form (the
+# cache read once for all heads); longer ones expand keys and values
+SHORT_ENTRY = 8
+
+
+@dataclass
+class RaggedBatch:
+    ids: torch.Tensor        # [T] token ids (all int32)
+    pos: torch.Tensor        # [T] place in the sequence, from 0
+    row: torch.Tensor        # [T] block-table row = state slot
+    tstart: torch.Tensor     # [T] packed index of the entry's first token
+    tend: torch.Tensor       # [T] packed index after the entry's last token
+    e_start: torch.Tensor    # [E] per entry: first packed token,
+    e_len: torch.Tensor      # [E] tokens,
+    e_pos: torch.Tensor      # [E] tokens already in the cache,
+    e_row: torch.Tensor      # [E] row
+    block_tables: torch.Tensor   # [rows, max blocks]
+    n_tok: int
+    decode: bool             # every entry is one token
+    # host copies of the entries, for launches sized by them
+    entries: list            # [(start, length, position, row)]
+    n_short: int             # packed tokens in entries <= SHORT_ENTRY
+
+    @staticmethod
+    def int_count(n_tok: int, n_entries: int) -> int:
+        return 5 * n_tok + 4 * n_entries
+
+    @staticmethod
+    def pack(runs) -> list[int]:
+        """``runs``: [(row, position, token ids)], short ones first ->
+        the flat int array ``over`` splits."""
+        ids, pos, row, ts, te = [], [], [], [], []
+        es, el, ep, er = [], [], [], []
+        at = 0
+        for r, p, toks in runs:
+            n = len(toks)
+            ids += toks
+            pos += range(p, p + n)
+            row += [r] * n
+            ts += [at] * n
+            te += [at + n] * n
+            es.append(at)
+            el.append(n)
+            ep.append(p)
+            er.append(r)
+            at += n
+        return ids + pos + row + ts + te + es + el + ep + er
+
+    @classmethod
+    def over(cls, flat: torch.Tensor, runs, block_tables) -> "RaggedBatch":
+        """View a device int32 buffer filled from ``pack(runs)``."""
+        T = sum(len(t) for _, _, t in runs)
+        E = len(runs)
+        parts = torch.split(flat, [T] * 5 + [E] * 4)
+        entries, at, short = [], 0, 0
+        for r, p, toks in runs:
+            n = len(toks)
+            entries.append((at, n, p, r))
+            at += n
+            if n <= SHORT_ENTRY:
+                short = at
+        return cls(*parts, block_tables=block_tables, n_tok=T,
+                   decode=T == E, entries=entries, n_short=short)
+
+    @classmethod
+    def build(cls, runs, block_tables) -> "RaggedBatch":
+        dev = block_tables.device
+        flat = torch.tensor(cls.pack(runs), dtype=torch.int32, device=dev)
+        return cls.over(flat, runs, block_tables)

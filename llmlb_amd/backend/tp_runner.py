@@ -24,9 +24,9 @@ import time
 import torch
 import torch.distributed as dist
 
+from ..models.registry import resolve
 from ..parallel.tp import TPContext
 from .engine import Engine, EngineConfig
-from .launcher import PRESETS
 from .sampler import SamplingParams
 
 
@@ -136,12 +136,12 @@ def main(argv=None):
         torch.cuda.set_device(device)
 
     tp = TPContext()
-    mcfg = PRESETS[args.model]()
+    mcfg, folder = resolve(args.model)
     ecfg = EngineConfig(
         model=mcfg, device=device,
         dtype="bfloat16" if have_gpu else "float32",
         kv_cache_blocks=args.kv_blocks, max_batch=args.max_batch,
-        tp_ctx=tp)
+        tp_ctx=tp, weights_path=folder)
     engine = Engine(ecfg)
     coord = TPEngineCoordinator(engine, group_cpu)
 

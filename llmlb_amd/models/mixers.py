@@ -1,0 +1,192 @@
+"""Token mixers and feed-forwards of the hybrid models.
+
+Each takes its sizes and constants as arguments, reads the layer's input
+[T, width] in the storage type and returns the sublayer's output before
+any norm.  Projections of the same input are one matrix product.
+"""
+from __future__ import annotations
+
+import torch
+import torch.nn as nn
+import torch.nn.functional as F
+
+from ..backend.kv_cache import DeltaSpec, LatentSpec
+from ..ops import hybrid as hy
+from ..ops import linear_decode
+
+FULL_CONTEXT = 2 ** 30     # the window of an unmasked causal layer
+
+
+def _linear(x, w):
+    return linear_decode(x, w) if x.shape[0] <= 128 else F.linear(x, w)
+
+
+def _param(t):
+    return nn.Parameter(t, requires_grad=False)
+
+
+def _stack_rows(parts, align: int = 8):
+    """Concatenate weights along their output rows, each part padded to
+    a multiple of ``align`` so that every section of the product starts
+    on a whole vector.  Returns (weight, offsets)."""
+    rows, offs, at = [], [], 0
+    for w in parts:
+        offs.append(at)
+        rows.append(w)
+        at += w.shape[0]
+        gap = -at % align
+        if gap:
+            rows.append(w.new_zeros(gap, w.shape[1]))
+            at += gap
+    return torch.cat(rows).contiguous(), offs
+
+
+class LatentAttention(nn.Module):
+    """Multi-head attention whose keys and values are linear maps of one
+    cached latent per token, plus a rotated key part shared by the
+    heads.  ``kv_from`` names the layer whose latents this one reads
+    (None: its own)."""
+
+    def __init__(self, *, width, heads, dim, rot_dim, vdim, kv_rank, scale,
+                 window, kv_from, eps, dtype, device):
+        super().__init__()
+        self.heads, self.dim, self.rot, self.vdim = heads, dim, rot_dim, vdim
+        self.rank, self.scale, self.kv_from = kv_rank, scale, kv_from
+        self.window = min(window or FULL_CONTEXT, FULL_CONTEXT)
+        self.eps, self.width = eps, width
+        self.dtype, self.device = dtype, device
+        self.cos_sin = None            # set by the model, [max_pos, rot]
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        H, R = self.heads, self.rank
+        out = {"q": (H * (self.dim + self.rot), self.width),
+               "uk": (H * self.dim, R), "uv": (H * self.vdim, R),
+               "o": (self.width, H * self.vdim)}
+        if self.kv_from is None:
+            out["dkv"] = (R + self.rot, self.width)
+            out["dkv.norm"] = (R,)
+        return out
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        to = dict(dtype=self.dtype, device=self.device)
+        own = self.kv_from is None
+        stacked, offs = _stack_rows(
+            [w["q"], w["dkv"]] if own else [w["q"]])
+        self.w_in = _param(stacked.to(**to))
+        self.c_off = offs[1] if own else 0
+        self.w_uk = _param(w["uk"].reshape(
+            self.heads, self.dim, self.rank).to(**to).contiguous())
+        uv = w["uv"].reshape(self.heads, self.vdim, self.rank).to(**to)
+        self.w_uv = _param(uv.contiguous())
+        self.w_uv_t = _param(uv.transpose(1, 2).contiguous())
+        self.w_o = _param(w["o"].to(**to))
+        self.w_norm = _param(w["dkv.norm"].float().to(self.device)) \
+            if own else None
+
+    def cache_spec(self):
+        return LatentSpec(self.rank + self.rot) \
+            if self.kv_from is None else None
+
+    def forward(self, x, b, cache, index: int):
+        own = self.kv_from is None
+        pages = cache.latent[index if own else self.kv_from]
+        proj = _linear(x, self.w_in)
+        hy.latent_prep(proj, self.heads, self.dim, self.rot, self.rank,
+                       self.c_off, self.w_norm, self.eps, self.cos_sin, b,
+                       pages, own)
+        return _linear(self._absorbed(proj, b, pages, b.n_tok), self.w_o)
+
+    def _absorbed(self, proj, b, pages, n):
+        """The first n tokens of the batch -> [n, heads * vdim]."""
+        H, D = self.heads, self.dim
+        q = proj[:n, :H * (D + self.rot)].unflatten(
+            1, (H, D + self.rot))[..., :D].transpose(0, 1)
+        qa = torch.bmm(q, self.w_uk)
+        lat = hy.latent_rows(qa, proj, D, self.rot, pages, b, self.window,
+                             self.scale)
+        o = torch.bmm(lat, self.w_uv_t)                 # [H, n, vdim]
+        return o.transpose(0, 1).reshape(n, H * self.vdim)
+
+
+class ChannelDelta(nn.Module):
+    """Gated delta rule with a decay per head and key channel, short
+    convolutions on q, k and v, and a gated norm on each head's
+    output."""
+
+    def __init__(self, *, width, heads, kv_heads, dim, vdim, taps,
+                 decay_rank, gate_rank, eps, dtype, device):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.heads, self.kv_heads, self.dim, self.vdim = \
+            heads, kv_heads, dim, vdim
+        self.taps, self.eps, self.width = taps, eps, width
+        self.decay_rank, self.gate_rank = decay_rank, gate_rank
+        self.dtype, self.device = dtype, device
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, qk, v = self.width, self.kv_heads * self.dim, \
+            self.heads * self.vdim
+        n = self.heads * self.dim
+        return {"q": (qk, W), "k": (qk, W), "v": (v, W),
+                "q.conv": (qk, self.taps), "k.conv": (qk, self.taps),
+                "v.conv": (v, self.taps), "b": (self.heads, W),
+                "A_log": (self.heads,), "norm": (self.vdim,),
+                "a1": (self.decay_rank, W), "a2": (n, self.decay_rank),
+                "dt_bias": (n,), "g1": (self.gate_rank, W),
+                "g2": (v, self.gate_rank), "o": (W, v)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        to = dict(dtype=self.dtype, device=self.device)
+        qkv = torch.cat([w["q"], w["k"], w["v"]])
+        stacked, (_, self.a_off, self.g_off, self.b_off) = _stack_rows(
+            [qkv, w["a1"], w["g1"], w["b"]])
+        self.w_in = _param(stacked.to(**to))
+        self.w_a2 = _param(w["a2"].to(**to))
+        self.w_g2 = _param(w["g2"].to(**to))
+        self.w_o = _param(w["o"].to(**to))
+
+        def wide(t):
+            return _param(t.float().to(self.device).contiguous())
+
+        self.w_conv = wide(torch.cat(
+            [w["q.conv"], w["k.conv"], w["v.conv"]]).t())   # [taps, C]
+        self.a_log, self.dt_bias = wide(w["A_log"]), wide(w["dt_bias"])
+        self.w_norm = wide(w["norm"])
+
+    def cache_spec(self):
+        C = 2 * self.kv_heads * self.dim + self.heads * self.vdim
+        return DeltaSpec(self.heads, self.vdim, self.dim, C, self.taps)
+
+    def forward(self, x, b, cache, index: int):
+        proj = _linear(x, self.w_in)
+        dec = _linear(proj[:, self.a_off:self.a_off + self.decay_rank],
+                      self.w_a2)
+        gate = _linear(proj[:, self.g_off:self.g_off + self.gate_rank],
+                       self.w_g2)
+        o = hy.gated_delta(
+            proj, self.b_off, dec, gate, cache.state[index],
+            cache.ring[index], b, self.w_conv, self.a_log, self.dt_bias,
+            self.w_norm, self.kv_heads, self.heads, self.dim, self.vdim,
+            self.taps, self.eps)
+        return _linear(o, self.w_o)
+
+
+class DenseFF(nn.Module):
+    """down(gelu(up x)), the tanh form of gelu."""
+
+    def __init__(self, *, width, ff, dtype, device):
+        super().__init__()
+        self.width, self.ff, self.dtype, self.device = \
+            width, ff, dtype, device
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        return {"up": (self.ff, self.width), "down": (self.width, self.ff)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        to = dict(dtype=self.dtype, device=self.device)
+        self.w_up = _param(w["up"].to(**to))
+        self.w_down = _param(w["down"].to(**to))
+
+    def forward(self, x):
+        return _linear(hy.gelu_tanh_(_linear(x, self.w_up)), self.w_down)

@@ -1,0 +1,174 @@
+// Attention over a cache of latents.
+//
+// A cached token is one row of rank + R numbers: a normed latent c and a
+// rotated key part that all heads share.  Head h's key is (W_uk c, kr)
+// and its value W_uv c, so with qa = W_uk^T q (the "absorbed" query)
+//   score = (qa . c + qr . kr) * scale,   out = W_uv (sum_j p_j c_j):
+// the cache is read as it is, once for all heads.  A query at position i
+// sees the keys j with 0 <= i - j < window.
+//
+// Cache layout: [pages][16 tokens][rank + R].
+#include "common.h"
+
+// Per token of a packed batch: norm the latent, rotate the key part and
+// put both into the cache; rotate every head's query part in place.
+// Column offsets are into a row of ``proj`` (ld columns).  The pair
+// (i, i + R/2) turns; cos_sin row p is cos[R/2] | sin[R/2].
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(
+    T* __restrict__ proj, int ld, int H, int D, int R, int c_off, int rank,
+    const float* __restrict__ w_norm, float eps,
+    const float* __restrict__ cos_sin, const int* __restrict__ pos_,
+    const int* __restrict__ row_, const int* __restrict__ bt, int max_blocks,
+    T* __restrict__ cache, int writes_kv) {
+  __shared__ float red[4];
+  const int t = blockIdx.x;
+  const int pos = pos_[t];
+  T* p = proj + (size_t)t * ld;
+  const int half = R / 2;
+  const float* cs = cos_sin + (size_t)pos * R;
+  for (int i = threadIdx.x; i < H * half; i += 256) {
+    const int h = i / half, j = i % half;
+    T* q = p + (size_t)h * (D + R) + D + j;
+    const float u = to_f(q[0]), v = to_f(q[half]);
+    const float c = cs[j], s = cs[half + j];
+    q[0] = from_f<T>(u * c - v * s);
+    q[half] = from_f<T>(v * c + u * s);
+  }
+  if (!writes_kv) return;
+  T* dst = cache + page_slot(bt, max_blocks, row_[t], pos) * (rank + R);
+  const T* src = p + c_off;
+  float ssq = 0.f;
+  for (int i = threadIdx.x; i < rank; i += 256) {
+    const float f = to_f(src[i]);
+    ssq += f * f;
+  }
+  const float r = 1.f / sqrtf(block_sum_256(ssq, red) / rank + eps);
+  for (int i = threadIdx.x; i < rank; i += 256)
+    dst[i] = from_f<T>(to_f(src[i]) * r * w_norm[i]);
+  for (int j = threadIdx.x; j < half; j += 256) {
+    const float u = to_f(src[rank + j]), v = to_f(src[rank + half + j]);
+    const float c = cs[j], s = cs[half + j];
+    dst[rank + j] = from_f<T>(u * c - v * s);
+    dst[rank + half + j] = from_f<T>(v * c + u * s);
+  }
+}
+
+// Absorbed attention of any sizes, one workgroup per (query, head): the
+// waves take every fourth key each and merge at the end.  The 32-bit
+// path, and 16-bit sizes that the tiled kernels do not cover.
+//   qa  [H][N][rank], proj rows carry the rotated query parts
+//   out [H][N][rank]
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void latent_rows_kernel(
+    T* __restrict__ out, const T* __restrict__ qa, const T* __restrict__ proj,
+    int ld, int D, int R, int rank, const T* __restrict__ cache,
+    const int* __restrict__ pos_, const int* __restrict__ row_,
+    const int* __restrict__ bt, int max_blocks, int window, float scale,
+    int N) {
+  extern __shared__ float lds[];
+  float* lq = lds;               // rank + R query numbers
+  float* lacc = lds + rank + R;  // 4 waves x rank
+  __shared__ float lm[4], ll[4];
+  const int n = blockIdx.x, h = blockIdx.y;
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int pos = pos_[n], row = row_[n];
+  const int first = pos - window + 1 > 0 ? pos - window + 1 : 0;
+  const T* q = qa + ((size_t)h * N + n) * rank;
+  for (int i = threadIdx.x; i < rank; i += 256) lq[i] = to_f(q[i]) * scale;
+  const T* qr = proj + (size_t)n * ld + (size_t)h * (D + R) + D;
+  for (int i = threadIdx.x; i < R; i += 256)
+    lq[rank + i] = to_f(qr[i]) * scale;
+  __syncthreads();
+
+  float m = -INFINITY, l = 0.f, acc[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) acc[i] = 0.f;
+  for (int j = first + wave; j <= pos; j += 4) {
+    const T* key = cache + page_slot(bt, max_blocks, row, j) * (rank + R);
+    float c[NR], s = 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      const int d = lane + i * WAVE;
+      c[i] = d < rank ? to_f(key[d]) : 0.f;
+      s += d < rank ? c[i] * lq[d] : 0.f;
+    }
+    for (int d = lane; d < R; d += WAVE) s += to_f(key[rank + d]) * lq[rank + d];
+    s = wave_sum(s);
+    const float mn = fmaxf(m, s);
+    const float keep = expf(m - mn), w = expf(s - mn);
+    l = l * keep + w;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) acc[i] = acc[i] * keep + w * c[i];
+    m = mn;
+  }
+  if (lane == 0) {
+    lm[wave] = m;
+    ll[wave] = l;
+  }
+#pragma unroll
+  for (int i = 0; i < NR; ++i)
+    if (lane + i * WAVE < rank) lacc[wave * rank + lane + i * WAVE] = acc[i];
+  __syncthreads();
+  const float mx = fmaxf(fmaxf(lm[0], lm[1]), fmaxf(lm[2], lm[3]));
+  float f[4], sum = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) {
+    f[w] = ll[w] > 0.f ? expf(lm[w] - mx) : 0.f;
+    sum += f[w] * ll[w];
+  }
+  const float inv = 1.f / sum;
+  T* o = out + ((size_t)h * N + n) * rank;
+  for (int i = threadIdx.x; i < rank; i += 256) {
+    float v = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) v += f[w] * lacc[w * rank + i];
+    o[i] = from_f<T>(v * inv);
+  }
+}
+
+extern "C" {
+
+int hy_latent_prep(void* proj, int ld, int H, int D, int R, int c_off,
+                   int rank, const void* w_norm, float eps,
+                   const void* cos_sin, const void* pos, const void* row,
+                   const void* bt, int max_blocks, void* cache, int writes_kv,
+                   int n_tok, int dtype, void* stream) {
+  if (R % 2 || rank <= 0) return -2;
+  if (n_tok <= 0) return 0;
+  HY_DTYPE(dtype, hipLaunchKernelGGL(
+      latent_prep_kernel<T>, dim3(n_tok), dim3(256), 0, (hipStream_t)stream,
+      (T*)proj, ld, H, D, R, c_off, rank, (const float*)w_norm, eps,
+      (const float*)cos_sin, (const int*)pos, (const int*)row,
+      (const int*)bt, max_blocks, (T*)cache, writes_kv));
+  HY_CHECK();
+  return 0;
+}
+
+int hy_latent_rows(void* out, const void* qa, const void* proj, int ld, int H,
+                   int D, int R, int rank, const void* cache, const void* pos,
+                   const void* row, const void* bt, int max_blocks,
+                   int window, float scale, int n_rows, int dtype,
+                   void* stream) {
+  if (rank <= 0 || rank > 2048 || R > 2048 || window <= 0 || H > 65535)
+    return -2;
+  if (n_rows <= 0) return 0;
+  const size_t lds = (size_t)(5 * rank + R) * sizeof(float);
+  const dim3 grid(n_rows, H), block(256);
+#define GO(NR)                                                               \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (latent_rows_kernel<T, NR>), grid, block, lds, (hipStream_t)stream,    \
+      (T*)out, (const T*)qa, (const T*)proj, ld, D, R, rank,                 \
+      (const T*)cache, (const int*)pos, (const int*)row, (const int*)bt,     \
+      max_blocks, window, scale, n_rows))
+  if (rank <= 128) GO(2);
+  else if (rank <= 256) GO(4);
+  else if (rank <= 512) GO(8);
+  else if (rank <= 1024) GO(16);
+  else GO(32);
+#undef GO
+  HY_CHECK();
+  return 0;
+}
+
+}  // extern "C"
