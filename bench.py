@@ -216,7 +216,19 @@ def main() -> None:
     ap.add_argument("--model", default=None,
                     help="model preset (default llama-3-8b on GPU, "
                          "llama-tiny on CPU)")
-    args = ap.parse_args()
+    ap.add_argument("--hybrid", action="store_true",
+                    help="instead: prefill and decode throughput of the "
+                         "hybrid family beside Llama at equal size "
+                         "(benchmarks/hybrid_bench.py)")
+    args, rest = ap.parse_known_args()
+    if args.hybrid:
+        ensure_kernels()
+        from benchmarks.hybrid_bench import main as hybrid_main
+        hybrid_main(["--steps", str(args.steps), "--warmup",
+                     str(args.warmup), *rest])
+        return
+    if rest:
+        ap.error(f"unrecognized arguments: {' '.join(rest)}")
 
     rank = int(os.environ.get("RANK", "0"))
     world = int(os.environ.get("WORLD_SIZE", "1"))

@@ -252,8 +252,10 @@ class _RaggedGraph:
         self.flat.copy_(torch.tensor(RaggedBatch.pack(runs),
                                      dtype=torch.int32))
         if self.batch is None:
-            self.batch = RaggedBatch.over(self.flat, runs,
-                                          self._engine._bt_dev)
+            eng = self._engine
+            self.batch = RaggedBatch.over(
+                self.flat, runs, eng._bt_dev,
+                max_keys=eng.max_blocks_per_seq * BLOCK_SIZE)
 
     def _forward(self) -> torch.Tensor:
         model = self._engine.model
@@ -1041,7 +1043,7 @@ class Engine:
 
     def _ragged_step(self, admitted: list[_Sequence]) -> None:
         """One packed forward: a token of every decoding sequence, and
-        up to ``prefill_chunk`` tokens of prompts still being read."""
+        prompts still being read up to the step's token budget."""
         for seq in admitted:
             blocks, seq.block_table = seq.block_table, []
             self._write_tables([(seq, blocks)])
@@ -1050,7 +1052,7 @@ class Engine:
             if reason is not None:
                 seq.out_queue.put((0, "error", {"error": reason}))
                 self._retire(seq)
-        budget = max(self.cfg.prefill_chunk, 1)
+        budget = max(self._step_budget, 1)
         work = []
         for seq in self.running:
             left = len(seq.prompt_ids) - seq.length

@@ -8,7 +8,7 @@ attention form finds its tokens in one run.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, field
 
 import torch
 
@@ -34,6 +34,36 @@ class RaggedBatch:
     # host copies of the entries, for launches sized by them
     entries: list            # [(start, length, position, row)]
     n_short: int             # packed tokens in entries <= SHORT_ENTRY
+    max_keys: int            # longest context any query may see
+    plans: dict = field(default_factory=dict)
+
+    def long_plan(self, window: int):
+        """Work lists of the long entries for attention over the last
+        ``window`` keys: what to copy out of the pages, 64 key rows a
+        block, and tiles of up to 128 queries.
+
+        Returns (blocks, items, block count, item count); blocks are
+        (row, first key position, valid keys), items (packed query,
+        query position, queries, key row, key position)."""
+        plan = self.plans.get(window)
+        if plan is None:
+            blocks, items = [], []
+            for start, n, pos, row in self.entries:
+                if n <= SHORT_ENTRY:
+                    continue
+                first, end = max(0, pos - window + 1), pos + n
+                at = 64 * (len(blocks) // 3)
+                for k in range(first, end, 64):
+                    blocks += (row, k, min(64, end - k))
+                # last queries first: they see the most keys
+                for q in reversed(range(0, n, 128)):
+                    items += (start + q, pos + q, min(128, n - q), at, first)
+            flat = torch.tensor(blocks + items, dtype=torch.int32,
+                                device=self.pos.device)
+            plan = (flat[:len(blocks)], flat[len(blocks):],
+                    len(blocks) // 3, len(items) // 5)
+            self.plans[window] = plan
+        return plan
 
     @staticmethod
     def int_count(n_tok: int, n_entries: int) -> int:
@@ -61,8 +91,11 @@ class RaggedBatch:
         return ids + pos + row + ts + te + es + el + ep + er
 
     @classmethod
-    def over(cls, flat: torch.Tensor, runs, block_tables) -> "RaggedBatch":
-        """View a device int32 buffer filled from ``pack(runs)``."""
+    def over(cls, flat: torch.Tensor, runs, block_tables,
+             max_keys: int | None = None) -> "RaggedBatch":
+        """View a device int32 buffer filled from ``pack(runs)``.
+        ``max_keys``: the bound to plan for when the buffer will be
+        filled again (captured steps)."""
         T = sum(len(t) for _, _, t in runs)
         E = len(runs)
         parts = torch.split(flat, [T] * 5 + [E] * 4)
@@ -74,7 +107,8 @@ class RaggedBatch:
             if n <= SHORT_ENTRY:
                 short = at
         return cls(*parts, block_tables=block_tables, n_tok=T,
-                   decode=T == E, entries=entries, n_short=short)
+                   decode=T == E, entries=entries, n_short=short,
+                   max_keys=max_keys or max(p + n for _, n, p, _ in entries))
 
     @classmethod
     def build(cls, runs, block_tables) -> "RaggedBatch":

@@ -55,6 +55,8 @@ class LatentAttention(nn.Module):
         self.window = min(window or FULL_CONTEXT, FULL_CONTEXT)
         self.eps, self.width = eps, width
         self.dtype, self.device = dtype, device
+        self.tiled = hy.can_decode_tiled(dtype, dim, rot_dim, kv_rank)
+        self.flash = hy.can_flash(dtype, dim, rot_dim, kv_rank, vdim)
         self.cos_sin = None            # set by the model, [max_pos, rot]
 
     def weight_shapes(self) -> dict[str, tuple]:
@@ -94,7 +96,19 @@ class LatentAttention(nn.Module):
         hy.latent_prep(proj, self.heads, self.dim, self.rot, self.rank,
                        self.c_off, self.w_norm, self.eps, self.cos_sin, b,
                        pages, own)
-        return _linear(self._absorbed(proj, b, pages, b.n_tok), self.w_o)
+        T = b.n_tok
+        n = b.n_short if self.flash and x.is_cuda else T
+        if n == T:
+            o = self._absorbed(proj, b, pages, n)
+        else:
+            o = torch.empty(T, self.heads * self.vdim, dtype=x.dtype,
+                            device=x.device)
+            if n:
+                o[:n] = self._absorbed(proj, b, pages, n)
+            hy.latent_flash(o, proj, self.heads, self.dim, self.rot,
+                            self.w_uk, self.w_uv, pages, b, self.window,
+                            self.scale)
+        return _linear(o, self.w_o)
 
     def _absorbed(self, proj, b, pages, n):
         """The first n tokens of the batch -> [n, heads * vdim]."""
@@ -102,8 +116,10 @@ class LatentAttention(nn.Module):
         q = proj[:n, :H * (D + self.rot)].unflatten(
             1, (H, D + self.rot))[..., :D].transpose(0, 1)
         qa = torch.bmm(q, self.w_uk)
-        lat = hy.latent_rows(qa, proj, D, self.rot, pages, b, self.window,
-                             self.scale)
+        attend = hy.latent_decode if self.tiled and proj.is_cuda \
+            else hy.latent_rows
+        lat = attend(qa, proj, D, self.rot, pages, b, self.window,
+                     self.scale)
         o = torch.bmm(lat, self.w_uv_t)                 # [H, n, vdim]
         return o.transpose(0, 1).reshape(n, H * self.vdim)
 

@@ -157,6 +157,70 @@ def latent_rows(qa, proj, dim, rot, cache, b, window, scale):
     return out
 
 
+def can_decode_tiled(dtype, dim, rot, rank) -> bool:
+    """Sizes that ``latent_decode`` takes."""
+    return (dtype == torch.bfloat16 and rank % 8 == 0 and rot % 8 == 0
+            and dim % 8 == 0 and rot <= 64 and rank <= 512)
+
+
+def decode_parts(n: int, heads: int, window: int, max_keys: int) -> int:
+    """How many workgroups share one query's keys: enough to fill the
+    chip twice, with at least two tiles of keys each."""
+    groups = n * ((heads + 31) // 32 if heads > 16 else 1)
+    keys = min(window, max_keys)
+    return max(1, min(512 // groups, keys // 128, 16))
+
+
+def latent_decode(qa, proj, dim, rot, cache, b, window, scale):
+    """``latent_rows`` on the matrix cores (bf16, GPU)."""
+    H, N, rank = qa.shape
+    assert qa.is_contiguous()
+    bt = b.block_tables
+    parts = decode_parts(N, H, window, b.max_keys)
+    out = torch.empty_like(qa)
+    acc = ml = None
+    if parts > 1:
+        acc = torch.empty(N, H, parts, rank, dtype=torch.float32,
+                          device=qa.device)
+        ml = torch.empty(N, H, parts, 2, dtype=torch.float32,
+                         device=qa.device)
+    _check(native().hy_latent_decode(
+        _ptr(out), _p(acc), _p(ml), _ptr(qa), _ptr(proj),
+        _i(proj.stride(0)), _i(H), _i(dim), _i(rot), _i(rank), _ptr(cache),
+        _ptr(b.pos), _ptr(b.row), _ptr(bt), _i(bt.shape[1]), _i(window),
+        _f(scale), _i(N), _i(parts), _stream()), "hy_latent_decode")
+    return out
+
+
+def can_flash(dtype, dim, rot, rank, vdim) -> bool:
+    """Sizes that ``latent_flash`` takes."""
+    return (dtype == torch.bfloat16 and dim % 8 == 0 and rot % 8 == 0
+            and rank % 8 == 0 and dim + rot <= 256 and vdim <= 256)
+
+
+def latent_flash(out, proj, heads, dim, rot, w_uk, w_uv, cache, b, window,
+                 scale) -> None:
+    """Attention of the batch's long entries into ``out`` [T, H * vdim]:
+    their visible latents are copied out of the pages and expanded to
+    keys and (transposed) values.  w_uk [H, dim, rank], w_uv
+    [H, vdim, rank]."""
+    H, V, rank = w_uv.shape
+    blocks, items, n_blocks, n_items = b.long_plan(window)
+    n = 64 * n_blocks
+    lib, bt, st = native(), b.block_tables, _stream()
+    c = torch.empty(n, rank, dtype=proj.dtype, device=proj.device)
+    kr = torch.empty(n, rot, dtype=proj.dtype, device=proj.device)
+    _check(lib.hy_latent_gather(
+        _ptr(c), _ptr(kr), _ptr(cache), _ptr(blocks), _i(n_blocks), _ptr(bt),
+        _i(bt.shape[1]), _i(rank), _i(rot), st), "hy_latent_gather")
+    kx = torch.nn.functional.linear(c, w_uk.view(H * dim, rank))
+    vt = torch.nn.functional.linear(w_uv.view(H * V, rank), c)
+    _check(lib.hy_latent_flash(
+        _ptr(out), _ptr(proj), _i(proj.stride(0)), _ptr(kx), _ptr(kr),
+        _ptr(vt), _i(n), _ptr(items), _i(n_items), _i(H), _i(dim), _i(rot),
+        _i(V), _i(window), _f(scale), st), "hy_latent_flash")
+
+
 # -- gated delta rule ------------------------------------------------------
 
 def gated_delta(proj, b_off, dec, gate, state, ring, b, wconv, a_log,
