@@ -123,6 +123,250 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
   }
 }
 
+// N consecutive elements, as wide as alignment allows; VEC: the address
+// is aligned to the whole run (or to 16 bytes).
+template <int N, bool VEC>
+__device__ __forceinline__ void load_run(const bf16_t* p, float* f) {
+  if (VEC && N % 8 == 0) {
+#pragma unroll
+    for (int i = 0; i < N; i += 8) load8(p + i, f + i);
+  } else if (VEC && N == 4) {
+    const uint2 v = *reinterpret_cast<const uint2*>(p);
+    f[0] = __uint_as_float(v.x << 16);
+    f[1] = __uint_as_float(v.x & 0xffff0000u);
+    f[2] = __uint_as_float(v.y << 16);
+    f[3] = __uint_as_float(v.y & 0xffff0000u);
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) f[i] = to_f(p[i]);
+  }
+}
+template <int N, bool VEC>
+__device__ __forceinline__ void load_run(const float* p, float* f) {
+  if (VEC && N % 4 == 0) {
+#pragma unroll
+    for (int i = 0; i < N; i += 4) {
+      const float4 v = *reinterpret_cast<const float4*>(p + i);
+      f[i] = v.x; f[i + 1] = v.y; f[i + 2] = v.z; f[i + 3] = v.w;
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) f[i] = p[i];
+  }
+}
+template <int N, bool VEC>
+__device__ __forceinline__ void store_run(float* p, const float* f) {
+  if (VEC && N % 4 == 0) {
+#pragma unroll
+    for (int i = 0; i < N; i += 4)
+      *reinterpret_cast<float4*>(p + i) =
+          make_float4(f[i], f[i + 1], f[i + 2], f[i + 3]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) p[i] = f[i];
+  }
+}
+template <int N, bool VEC>
+__device__ __forceinline__ void store_run(bf16_t* p, const float* f) {
+  if (VEC && N % 8 == 0) {
+#pragma unroll
+    for (int i = 0; i < N; i += 8) store8(p + i, f + i);
+  } else if (VEC && N == 4) {
+    *reinterpret_cast<uint2*>(p) =
+        make_uint2(pack2(f[0], f[1]), pack2(f[2], f[3]));
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) p[i] = from_f<bf16_t>(f[i]);
+  }
+}
+// only the first ``valid`` of N elements exist
+template <int N, bool VEC, typename T>
+__device__ __forceinline__ void load_some(const T* p, int valid, float* f) {
+  if (VEC || valid >= N) {
+    load_run<N, VEC>(p, f);
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i) f[i] = i < valid ? to_f(p[i]) : 0.f;
+  }
+}
+template <int N, bool VEC, typename T>
+__device__ __forceinline__ void store_some(T* p, int valid, const float* f) {
+  if (VEC || valid >= N) {
+    store_run<N, VEC>(p, f);
+  } else {
+#pragma unroll
+    for (int i = 0; i < N; ++i)
+      if (i < valid) p[i] = from_f<T>(f[i]);
+  }
+}
+
+// 16-bit results take the hardware's exponential and logarithm
+template <typename T>
+__device__ __forceinline__ float sigmoid_t(float x) {
+  return sizeof(T) == 2 ? 1.f / (1.f + __expf(-x)) : sigmoid_f(x);
+}
+template <typename T>
+__device__ __forceinline__ float decay_t(float z, float rate) {
+  if (sizeof(T) == 2) {
+    const float e = __expf(-fabsf(z));
+    // log(1 + e) by its series where 1 + e would lose e
+    const float lp = e < 1e-3f ? e * (1.f - 0.5f * e) : __logf(1.f + e);
+    return __expf(-rate * (fmaxf(z, 0.f) + lp));
+  }
+  return expf(-rate * softplus_f(z));
+}
+
+// The convolution of N neighbouring channels over consecutive tokens,
+// each input read once: ``hist`` holds the last taps - 1 inputs.
+#define TAPS_MAX 4
+template <typename T, int N, bool VEC>
+struct ConvRun {
+  float w[TAPS_MAX][N], hist[TAPS_MAX - 1][N];
+  const T* proj;
+  const T* ring;
+  int ld, C, taps, c, valid;
+
+  __device__ __forceinline__ ConvRun(const T* proj_, int ld_, const T* ring_,
+                                     const float* wconv, int C_, int taps_,
+                                     int c_, int valid_)
+      : proj(proj_), ring(ring_), ld(ld_), C(C_), taps(taps_), c(c_),
+        valid(valid_) {
+#pragma unroll
+    for (int b = 0; b < TAPS_MAX; ++b)
+      if (b < taps)
+        load_some<N, VEC>(wconv + (size_t)(taps - 1 - b) * C + c, valid,
+                          w[b]);
+  }
+  // inputs before token t, from the batch or the sequence's ring
+  __device__ __forceinline__ void start(int t, int pos, int tstart,
+                                        int slot) {
+#pragma unroll
+    for (int b = 1; b < TAPS_MAX; ++b) {
+#pragma unroll
+      for (int i = 0; i < N; ++i) hist[b - 1][i] = 0.f;
+      if (b < taps && pos - b >= 0)
+        load_some<N, VEC>(
+            t - b >= tstart
+                ? proj + (size_t)(t - b) * ld + c
+                : ring + ((size_t)slot * taps + (pos - b) % taps) * C + c,
+            valid, hist[b - 1]);
+    }
+  }
+  __device__ __forceinline__ void step(int t, float* y) {
+    float x[N];
+    load_some<N, VEC>(proj + (size_t)t * ld + c, valid, x);
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      float acc = x[i] * w[0][i];
+#pragma unroll
+      for (int b = 1; b < TAPS_MAX; ++b)
+        if (b < taps) acc += hist[b - 1][i] * w[b][i];
+#pragma unroll
+      for (int b = TAPS_MAX - 1; b > 1; --b) hist[b - 1][i] = hist[b - 2][i];
+      hist[0][i] = x[i];
+      y[i] = acc * sigmoid_t<T>(acc);
+    }
+  }
+};
+
+// delta_prep for at most TAPS_MAX taps and D <= 256: a workgroup walks
+// PREP_TOK tokens.  blockIdx.y ranges: q/k heads (16 lanes a head, 16
+// heads a workgroup), then value channels, then decays (8 channels a
+// thread).  VEC: all sections start on whole vectors.
+#define PREP_TOK 16
+template <typename T, int RPL, bool VEC>
+__global__ __launch_bounds__(256) void delta_prep_run_kernel(
+    float* __restrict__ ws, const T* __restrict__ proj, int ld, int b_off,
+    const T* __restrict__ dec, const T* __restrict__ ring,
+    const float* __restrict__ wconv, const float* __restrict__ a_log,
+    const float* __restrict__ dt_bias, const int* __restrict__ pos_,
+    const int* __restrict__ row_, const int* __restrict__ tstart_, int n_tok,
+    int KH, int H, int D, int V, int taps, float q_scale, int qk_blocks,
+    int v_blocks) {
+  const int t0 = blockIdx.x * PREP_TOK;
+  const int t1 = t0 + PREP_TOK < n_tok ? t0 + PREP_TOK : n_tok;
+  const int C = 2 * KH * D + H * V;
+  const WsLayout at(KH, H, D, V);
+  int y = blockIdx.y;
+  if (y < qk_blocks) {
+    const int unit = y * 16 + threadIdx.x / 16;
+    if (unit >= KH) return;  // whole groups of 16 lanes
+    const int r0 = (threadIdx.x & 15) * RPL;
+    const int valid = D - r0 < RPL ? (D - r0 > 0 ? D - r0 : 0) : RPL;
+    const int cq = unit * D + (valid ? r0 : 0), ck = KH * D + cq;
+    ConvRun<T, RPL, VEC> q(proj, ld, ring, wconv, C, taps, cq, valid);
+    ConvRun<T, RPL, VEC> k(proj, ld, ring, wconv, C, taps, ck, valid);
+    for (int t = t0; t < t1; ++t) {
+      const int ts = tstart_[t];
+      if (t == t0 || t == ts) {
+        q.start(t, pos_[t], ts, row_[t]);
+        k.start(t, pos_[t], ts, row_[t]);
+      }
+      float a[RPL], b[RPL], qq = 0.f, kk = 0.f, qk = 0.f;
+      q.step(t, a);
+      k.step(t, b);
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) {
+        if (!VEC && i >= valid) a[i] = b[i] = 0.f;
+        qq += a[i] * a[i];
+        kk += b[i] * b[i];
+        qk += a[i] * b[i];
+      }
+      const float qs = q_scale / sqrtf(row16_sum(qq) + 1e-6f);
+      const float ks = 1.f / sqrtf(row16_sum(kk) + 1e-6f);
+      qk = row16_sum(qk) * qs * ks;
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) {
+        a[i] *= qs;
+        b[i] *= ks;
+      }
+      float* w = ws + (size_t)t * at.size;
+      store_some<RPL, VEC>(w + cq, valid, a);
+      store_some<RPL, VEC>(w + ck, valid, b);
+      if ((threadIdx.x & 15) == 0) w[at.qk + unit] = qk;
+    }
+    return;
+  }
+  y -= qk_blocks;
+  if (y < v_blocks) {
+    const int j = (y * 256 + threadIdx.x) * 8;
+    if (j >= H * V) return;
+    const int valid = H * V - j < 8 ? H * V - j : 8;
+    ConvRun<T, 8, VEC> v(proj, ld, ring, wconv, C, taps, 2 * KH * D + j,
+                         valid);
+    for (int t = t0; t < t1; ++t) {
+      const int ts = tstart_[t];
+      if (t == t0 || t == ts) v.start(t, pos_[t], ts, row_[t]);
+      float f[8];
+      v.step(t, f);
+      store_some<8, VEC>(ws + (size_t)t * at.size + at.v + j, valid, f);
+    }
+    return;
+  }
+  y -= v_blocks;
+  const int j = (y * 256 + threadIdx.x) * 8;
+  if (y == 0)
+    for (int i = threadIdx.x; i < (t1 - t0) * H; i += 256) {
+      const int t = t0 + i / H, h = i % H;
+      ws[(size_t)t * at.size + at.beta + h] =
+          sigmoid_t<T>(to_f(proj[(size_t)t * ld + b_off + h]));
+    }
+  if (j >= H * D) return;
+  const int valid = H * D - j < 8 ? H * D - j : 8;
+  float bias[8], rate[8];
+  load_some<8, VEC>(dt_bias + j, valid, bias);
+#pragma unroll
+  for (int i = 0; i < 8; ++i)
+    rate[i] = i < valid ? expf(a_log[(j + i) / D]) : 0.f;
+  for (int t = t0; t < t1; ++t) {
+    float f[8];
+    load_some<8, VEC>(dec + (size_t)t * H * D + j, valid, f);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f[i] = decay_t<T>(f[i] + bias[i], rate[i]);
+    store_some<8, VEC>(ws + (size_t)t * at.size + at.g + j, valid, f);
+  }
+}
+
 template <int RPL, bool EXACT>
 __device__ __forceinline__ void load_rows(const float* __restrict__ p, int r0,
                                           int D, float* f) {
@@ -155,10 +399,12 @@ __device__ __forceinline__ void store_rows(float* __restrict__ p, int r0,
   }
 }
 
-// One wave = 4 value columns of one head of one sequence; 16 lanes a
-// column, RPL key channels a lane.  The operands of the next PF tokens
-// are in flight while a token is worked on.
-template <int RPL, bool EXACT>
+// One wave = 4 CPL value columns of one head of one sequence: 16 lanes a
+// column, RPL key channels and CPL columns a lane.  The operands of the
+// next PF tokens are in flight while a token is worked on; they are the
+// same for every column, so CPL > 1 divides the load on the vector
+// memory path, which is what limits a chip full of waves.
+template <int RPL, bool EXACT, int CPL>
 __global__ __launch_bounds__(64) void delta_scan_kernel(
     float* __restrict__ o, float* __restrict__ state,
     const float* __restrict__ ws, const int* __restrict__ e_start,
@@ -166,7 +412,7 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(
     const int* __restrict__ e_row, int KH, int H, int D, int V) {
   constexpr int PF = RPL <= 8 ? 4 : (RPL == 16 ? 2 : 1);
   const int e = blockIdx.y;
-  const int nb = (V + 3) / 4;
+  const int nb = (V + 4 * CPL - 1) / (4 * CPL);
   int head, cb;
   if (H % 8 == 0) {  // all columns of a head on one XCD: its L2 serves them
     const int x = blockIdx.x & 7, r = blockIdx.x >> 3;
@@ -177,28 +423,35 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(
     cb = blockIdx.x % nb;
   }
   const int lane = threadIdx.x;
-  const int col = cb * 4 + lane / 16;
-  const int colc = col < V ? col : V - 1;
+  const int col = (cb * 4 + lane / 16) * CPL;  // the lane's first column
   const int r0 = (lane & 15) * RPL;
   const int kh = head / (H / KH);
   const WsLayout at(KH, H, D, V);
   const int len = e_len[e];
   const float* base = ws + (size_t)e_start[e] * at.size;
   float* out = o + ((size_t)e_start[e] * H + head) * V;
-  float* sp = state + (((size_t)e_row[e] * H + head) * V + colc) * D;
-
-  float S[RPL];
+  float* sp = state + ((size_t)e_row[e] * H + head) * V * D;
+  int cc[CPL];
 #pragma unroll
-  for (int i = 0; i < RPL; ++i) S[i] = 0.f;
-  if (e_pos[e] > 0) load_rows<RPL, EXACT>(sp, r0, D, S);
+  for (int c = 0; c < CPL; ++c) cc[c] = col + c < V ? col + c : V - 1;
 
-  float q[PF][RPL], k[PF][RPL], g[PF][RPL], v[PF], qk[PF], beta[PF];
+  float S[CPL][RPL];
+  const bool resume = e_pos[e] > 0;
+#pragma unroll
+  for (int c = 0; c < CPL; ++c) {
+#pragma unroll
+    for (int i = 0; i < RPL; ++i) S[c][i] = 0.f;
+    if (resume) load_rows<RPL, EXACT>(sp + (size_t)cc[c] * D, r0, D, S[c]);
+  }
+
+  float q[PF][RPL], k[PF][RPL], g[PF][RPL], v[PF][CPL], qk[PF], beta[PF];
   auto fetch = [&](int s, int t) {
     const float* w = base + (size_t)(t < len ? t : len - 1) * at.size;
     load_rows<RPL, EXACT>(w + (size_t)kh * D, r0, D, q[s]);
     load_rows<RPL, EXACT>(w + (size_t)(KH + kh) * D, r0, D, k[s]);
     load_rows<RPL, EXACT>(w + at.g + (size_t)head * D, r0, D, g[s]);
-    v[s] = w[at.v + head * V + colc];
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) v[s][c] = w[at.v + head * V + cc[c]];
     qk[s] = w[at.qk + kh];
     beta[s] = w[at.beta + head];
   };
@@ -209,25 +462,43 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(
 #pragma unroll
     for (int s = 0; s < PF; ++s) {
       if (t0 + s < len) {
-        float a = 0.f, b = 0.f;
+        float a[CPL], b[CPL];
 #pragma unroll
-        for (int i = 0; i < RPL; ++i) {
-          S[i] *= g[s][i];
-          a += k[s][i] * S[i];
-          b += q[s][i] * S[i];
+        for (int c = 0; c < CPL; ++c) {
+          a[c] = b[c] = 0.f;
+#pragma unroll
+          for (int i = 0; i < RPL; ++i) {
+            S[c][i] *= g[s][i];
+            a[c] += k[s][i] * S[c][i];
+            b[c] += q[s][i] * S[c][i];
+          }
         }
-        a = row16_sum(a);
-        b = row16_sum(b);
-        const float u = beta[s] * (v[s] - a);
 #pragma unroll
-        for (int i = 0; i < RPL; ++i) S[i] += k[s][i] * u;
-        if ((lane & 15) == 0 && col < V)
-          out[(size_t)(t0 + s) * H * V + col] = b + qk[s] * u;
+        for (int c = 0; c < CPL; ++c) {
+          a[c] = row16_sum(a[c]);
+          b[c] = row16_sum(b[c]);
+        }
+#pragma unroll
+        for (int c = 0; c < CPL; ++c) {
+          const float u = beta[s] * (v[s][c] - a[c]);
+#pragma unroll
+          for (int i = 0; i < RPL; ++i) S[c][i] += k[s][i] * u;
+          b[c] += qk[s] * u;
+        }
+        // lane c of a group of 16 writes its column c
+        float mine = b[0];
+#pragma unroll
+        for (int c = 1; c < CPL; ++c) mine = (lane & 15) == c ? b[c] : mine;
+        if ((lane & 15) < CPL && col + (lane & 15) < V)
+          out[(size_t)(t0 + s) * H * V + col + (lane & 15)] = mine;
         fetch(s, t0 + s + PF);
       }
     }
   }
-  if (col < V) store_rows<RPL, EXACT>(sp, r0, D, S);
+#pragma unroll
+  for (int c = 0; c < CPL; ++c)
+    if (col + c < V)
+      store_rows<RPL, EXACT>(sp + (size_t)(col + c) * D, r0, D, S[c]);
 }
 
 // out = o / rms(o) * w * sigmoid(gate) per head; and, once nothing reads
@@ -255,6 +526,38 @@ __global__ __launch_bounds__(256) void delta_out_kernel(
   for (int j = lane; j < V; j += WAVE)
     out[base + j] =
         from_f<T>(o[base + j] * r * w[j] * sigmoid_f(to_f(gate[base + j])));
+}
+
+// The same with 16 lanes a head and RPL value channels a lane (V <= 256);
+// VEC: V = 16 RPL.
+template <typename T, int RPL, bool VEC>
+__global__ __launch_bounds__(256) void delta_out_run_kernel(
+    T* __restrict__ out, const float* __restrict__ o,
+    const T* __restrict__ gate, const float* __restrict__ w, float eps,
+    const T* __restrict__ proj, int ld, T* __restrict__ ring,
+    const int* __restrict__ pos_, const int* __restrict__ row_,
+    const int* __restrict__ tend_, int H, int V, int C, int taps) {
+  const int t = blockIdx.x;
+  const int h = blockIdx.y * 16 + threadIdx.x / 16;
+  if (blockIdx.y == 0 && tend_[t] - t <= taps) {
+    T* dst = ring + ((size_t)row_[t] * taps + pos_[t] % taps) * C;
+    for (int c = threadIdx.x; c < C; c += 256)
+      dst[c] = proj[(size_t)t * ld + c];
+  }
+  if (h >= H) return;  // whole groups of 16 lanes
+  const int r0 = (threadIdx.x & 15) * RPL;
+  const int valid = V - r0 < RPL ? (V - r0 > 0 ? V - r0 : 0) : RPL;
+  const size_t at = ((size_t)t * H + h) * V + (valid ? r0 : 0);
+  float x[RPL], gt[RPL], wn[RPL], ssq = 0.f;
+  load_some<RPL, VEC>(o + at, valid, x);
+  load_some<RPL, VEC>(gate + at, valid, gt);
+  load_some<RPL, VEC>(w + (valid ? r0 : 0), valid, wn);
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) ssq += x[i] * x[i];
+  const float r = 1.f / sqrtf(row16_sum(ssq) / V + eps);
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) x[i] *= r * wn[i] * sigmoid_t<T>(gt[i]);
+  store_some<RPL, VEC>(out + at, valid, x);
 }
 
 // Decode: one token of every sequence, all of the above in one launch.
@@ -431,6 +734,39 @@ int hy_delta_prep(void* ws, const void* proj, int ld, int b_off,
                   void* stream) {
   if (!delta_ok(KH, H, D, V, taps)) return -2;
   if (n_tok <= 0) return 0;
+  if (taps <= TAPS_MAX && D <= 256) {
+    const int qk_blocks = (KH + 15) / 16;
+    const int v_blocks = (H * V + 2047) / 2048;
+    const int g_blocks = (H * D + 2047) / 2048;
+    const dim3 grid((n_tok + PREP_TOK - 1) / PREP_TOK,
+                    qk_blocks + v_blocks + g_blocks);
+    const bool whole = rows_per_lane(D) * 16 == D && D % 8 == 0 &&
+                       V % 8 == 0 && ld % 8 == 0;
+#define RUN(RPL, VEC)                                                        \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (delta_prep_run_kernel<T, RPL, VEC>), grid, dim3(256), 0,              \
+      (hipStream_t)stream, (float*)ws, (const T*)proj, ld, b_off,            \
+      (const T*)dec, (const T*)ring, (const float*)wconv,                    \
+      (const float*)a_log, (const float*)dt_bias, (const int*)pos,           \
+      (const int*)row, (const int*)tstart, n_tok, KH, H, D, V, taps,         \
+      q_scale, qk_blocks, v_blocks))
+#define PICK(RPL)            \
+  do {                       \
+    if (whole) RUN(RPL, true); \
+    else RUN(RPL, false);    \
+  } while (0)
+    switch (rows_per_lane(D)) {
+      case 1: PICK(1); break;
+      case 2: PICK(2); break;
+      case 4: PICK(4); break;
+      case 8: PICK(8); break;
+      default: PICK(16); break;
+    }
+#undef PICK
+#undef RUN
+    HY_CHECK();
+    return 0;
+  }
   const dim3 grid(n_tok, (KH + H + 3) / 4), block(256);
 #define GO(NJ)                                                               \
   HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
@@ -453,11 +789,21 @@ int hy_delta_scan(void* o, void* state, const void* ws, const void* e_start,
                   int n_entries, int KH, int H, int D, int V, void* stream) {
   if (!delta_ok(KH, H, D, V, 1) || n_entries > 65535) return -2;
   if (n_entries <= 0) return 0;
-  const dim3 grid(H * ((V + 3) / 4), n_entries), block(64);
-  HY_RPL(D, hipLaunchKernelGGL(
-      (delta_scan_kernel<RPL, EXACT>), grid, block, 0, (hipStream_t)stream,
-      (float*)o, (float*)state, (const float*)ws, (const int*)e_start,
-      (const int*)e_len, (const int*)e_pos, (const int*)e_row, KH, H, D, V));
+  // wide lanes where they still fill the chip's 1024 SIMDs
+  const long long waves = (long long)n_entries * H * ((V + 3) / 4);
+#define GO(CPL)                                                               \
+  do {                                                                        \
+    const dim3 grid(H * ((V + 4 * CPL - 1) / (4 * CPL)), n_entries);          \
+    HY_RPL(D, hipLaunchKernelGGL(                                             \
+        (delta_scan_kernel<RPL, EXACT, CPL>), grid, dim3(64), 0,              \
+        (hipStream_t)stream, (float*)o, (float*)state, (const float*)ws,      \
+        (const int*)e_start, (const int*)e_len, (const int*)e_pos,            \
+        (const int*)e_row, KH, H, D, V));                                     \
+  } while (0)
+  if (V >= 16 && D <= 128 && waves >= 4096) GO(4);
+  else if (V >= 8 && D <= 256 && waves >= 2048) GO(2);
+  else GO(1);
+#undef GO
   HY_CHECK();
   return 0;
 }
@@ -470,6 +816,32 @@ int hy_delta_out(void* out, const void* o, const void* gate, const void* w,
   if (!delta_ok(KH, H, D, V, taps)) return -2;
   if (n_tok <= 0) return 0;
   const int C = 2 * KH * D + H * V;
+  if (V <= 256) {
+    const dim3 grid(n_tok, (H + 15) / 16);
+    const bool whole = rows_per_lane(V) * 16 == V;
+#define RUN(RPL, VEC)                                                       \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                       \
+      (delta_out_run_kernel<T, RPL, VEC>), grid, dim3(256), 0,              \
+      (hipStream_t)stream, (T*)out, (const float*)o, (const T*)gate,        \
+      (const float*)w, eps, (const T*)proj, ld, (T*)ring, (const int*)pos,  \
+      (const int*)row, (const int*)tend, H, V, C, taps))
+#define PICK(RPL)            \
+  do {                       \
+    if (whole) RUN(RPL, true); \
+    else RUN(RPL, false);    \
+  } while (0)
+    switch (rows_per_lane(V)) {
+      case 1: PICK(1); break;
+      case 2: PICK(2); break;
+      case 4: PICK(4); break;
+      case 8: PICK(8); break;
+      default: PICK(16); break;
+    }
+#undef PICK
+#undef RUN
+    HY_CHECK();
+    return 0;
+  }
   HY_DTYPE(dtype, hipLaunchKernelGGL(
       delta_out_kernel<T>, dim3(n_tok, (H + 3) / 4), dim3(256), 0,
       (hipStream_t)stream, (T*)out, (const float*)o, (const T*)gate,

@@ -58,7 +58,8 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(
 //   q   = proj + h * (D + R), kx [keys][H D], kr [keys][R],
 //   vt [H V][key_ld]  (values transposed), out [tokens][H V]
 template <int DQ, int DV>
-__global__ __launch_bounds__(256, 1) void latent_flash_kernel(
+__global__ __launch_bounds__(256, DQ * 2 + DV <= 512 ? 2 : 1)
+void latent_flash_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ proj, int ld,
     const bf16_t* __restrict__ kx, const bf16_t* __restrict__ kr,
     const bf16_t* __restrict__ vt, int key_ld, const int* __restrict__ items,
@@ -249,7 +250,8 @@ __global__ __launch_bounds__(256, 1) void latent_flash_kernel(
 // the rank for all heads.
 //   qa [H][N][rank]; parts: acc [N][H][parts][rank] and (max, sum)
 template <int NT, int HT>
-__global__ __launch_bounds__(256, 1) void latent_decode_kernel(
+__global__ __launch_bounds__(256, NT == 8 && HT == 1 ? 1 : 2)
+void latent_decode_kernel(
     bf16_t* __restrict__ out, float* __restrict__ ws_acc,
     float* __restrict__ ws_ml, const bf16_t* __restrict__ qa,
     const bf16_t* __restrict__ proj, int ld, int D, int R, int rank, int H,
@@ -273,25 +275,49 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(
 
   const int pos = pos_[q], row = row_[q];
   const int first = pos - window + 1 > 0 ? pos - window + 1 : 0;
-  const int tiles = (pos - first + KEYS) / KEYS;
+  const int base = first & ~(PAGE - 1);  // tiles are whole pages
+  const int tiles = (pos - base + KEYS) / KEYS;
   const int per = (tiles + parts - 1) / parts;
   const int t_lo = part * per;
   const int t_hi = t_lo + per < tiles ? t_lo + per : tiles;
+  const int* pages = bt + (size_t)row * max_blocks;
+  const int last_page = pos / PAGE;
 
+  // the thread's pieces of a tile: place in the row and in LDS
+  int p_row[PL], p_off[PL];
+#pragma unroll
+  for (int i = 0; i < PL; ++i) {
+    const int p = tid + i * 256;
+    p_row[i] = p / pieces;
+    p_off[i] = (p - p_row[i] * pieces) * 8;
+  }
+  // page numbers are wave-uniform and fetched a tile ahead of the rows
+  int pg[KEYS / PAGE];
+  auto fetch_pages = [&](int t) {
+#pragma unroll
+    for (int i = 0; i < KEYS / PAGE; ++i) {
+      const int b = base / PAGE + t * (KEYS / PAGE) + i;
+      pg[i] = pages[b < last_page ? b : last_page];
+    }
+  };
   u32x4 pk[PL];
   auto fetch = [&](int t) {
 #pragma unroll
     for (int i = 0; i < PL; ++i) {
-      const int p = tid + i * 256;
-      const int r = p / pieces;
-      int key = first + t * KEYS + r;
-      key = key < pos ? key : pos;
-      pk[i] = r < KEYS ? *reinterpret_cast<const u32x4*>(
-                             cache + page_slot(bt, max_blocks, row, key) *
-                                         width + (p % pieces) * 8)
-                       : u32x4{0, 0, 0, 0};
+      int page = pg[0];
+#pragma unroll
+      for (int k = 1; k < KEYS / PAGE; ++k)
+        page = p_row[i] / PAGE == k ? pg[k] : page;
+      pk[i] = p_row[i] < KEYS
+                  ? *reinterpret_cast<const u32x4*>(
+                        cache +
+                        ((size_t)page * PAGE + p_row[i] % PAGE) * width +
+                        p_off[i])
+                  : u32x4{0, 0, 0, 0};
     }
+    if (t + 1 < t_hi) fetch_pages(t + 1);
   };
+  if (t_lo < t_hi) fetch_pages(t_lo);
   if (t_lo < t_hi) fetch(t_lo);
 
   u32x4 qf[KD];
@@ -326,25 +352,26 @@ __global__ __launch_bounds__(256, 1) void latent_decode_kernel(
   }
   for (int t = t_lo; t < t_hi; ++t) {
 #pragma unroll
-    for (int i = 0; i < PL; ++i) {
-      const int p = tid + i * 256;
-      const int r = p / pieces;
-      if (r < KEYS)
-        *reinterpret_cast<u32x4*>(&lk[r * PITCH + (p % pieces) * 8]) = pk[i];
-    }
+    for (int i = 0; i < PL; ++i)
+      if (p_row[i] < KEYS)
+        *reinterpret_cast<u32x4*>(&lk[p_row[i] * PITCH + p_off[i]]) = pk[i];
     __syncthreads();
     if (t + 1 < t_hi) fetch(t + 1);
-    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+    f32x4 s = {0.f, 0.f, 0.f, 0.f}, s1 = s;
 #pragma unroll
-    for (int k = 0; k < KD; ++k)
-      s = mfma(*reinterpret_cast<const u32x4*>(
-                   &lk[(kt * 16 + n) * PITCH + k * 32 + g * 8]),
-               qf[k], s);
-    const int j = first + t * KEYS + kt * 16 + g * 4;
+    for (int k = 0; k < KD; k += 2) {
+      const unsigned short* c =
+          &lk[(kt * 16 + n) * PITCH + k * 32 + g * 8];
+      s = mfma(*reinterpret_cast<const u32x4*>(c), qf[k], s);
+      s1 = mfma(*reinterpret_cast<const u32x4*>(c + 32), qf[k + 1], s1);
+    }
+    s += s1;
+    const int j = base + t * KEYS + kt * 16 + g * 4;
     float mx = -INFINITY;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      s[i] = j + i <= pos ? s[i] * scale_log2 : -INFINITY;
+      s[i] = j + i >= first && j + i <= pos ? s[i] * scale_log2
+                                            : -INFINITY;
       mx = fmaxf(mx, s[i]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));

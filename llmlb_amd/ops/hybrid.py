@@ -165,10 +165,10 @@ def can_decode_tiled(dtype, dim, rot, rank) -> bool:
 
 def decode_parts(n: int, heads: int, window: int, max_keys: int) -> int:
     """How many workgroups share one query's keys: enough to fill the
-    chip twice, with at least two tiles of keys each."""
+    chip, with at least two tiles of keys each."""
     groups = n * ((heads + 31) // 32 if heads > 16 else 1)
     keys = min(window, max_keys)
-    return max(1, min(512 // groups, keys // 128, 16))
+    return max(1, min(256 // groups, keys // 64, 16))
 
 
 def latent_decode(qa, proj, dim, rot, cache, b, window, scale):
