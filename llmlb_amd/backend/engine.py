@@ -41,6 +41,7 @@ from dataclasses import dataclass, field
 
 log = logging.getLogger("llmlb.engine")
 
+import numpy as np
 import torch
 
 from .. import ops
@@ -249,8 +250,7 @@ class _RaggedGraph:
     def _fill(self, runs) -> None:
         runs = runs + [(self._engine.max_rows, 0, [0])] \
             * (self.S - len(runs))
-        self.flat.copy_(torch.tensor(RaggedBatch.pack(runs),
-                                     dtype=torch.int32))
+        self.flat.copy_(torch.from_numpy(RaggedBatch.pack(runs)))
         if self.batch is None:
             eng = self._engine
             self.batch = RaggedBatch.over(
@@ -356,6 +356,9 @@ class Engine:
                             self.model.lm_head.data)
                 except Exception:
                     pass
+        if self.ragged and self.device.type == "cuda":
+            ops.tune_decode_shapes(
+                [p for p in self.model.parameters() if p.dim() == 2])
         m = cfg.model
         self.max_rows = cfg.max_batch
         self._init_cache(dtype)
@@ -992,8 +995,10 @@ class Engine:
         vocab = self.cfg.model.vocab
         cap = min(self.cfg.model.max_pos,
                   self.max_blocks_per_seq * BLOCK_SIZE)
+        work = [(seq, np.asarray(toks, dtype=np.int64), want)
+                for seq, toks, want in work]
         for seq, toks, want in work:
-            if not toks or min(toks) < 0 or max(toks) >= vocab:
+            if not len(toks) or toks.min() < 0 or toks.max() >= vocab:
                 raise ValueError("token ids must be in [0, vocab)")
             if seq.length + len(toks) > cap:
                 raise ValueError(f"sequence longer than {cap} tokens")

@@ -10,6 +10,7 @@ from __future__ import annotations
 
 from dataclasses import dataclass, field
 
+import numpy as np
 import torch
 
 # longest entry whose queries attend through the absorbed form (the
@@ -70,25 +71,19 @@ class RaggedBatch:
         return 5 * n_tok + 4 * n_entries
 
     @staticmethod
-    def pack(runs) -> list[int]:
+    def pack(runs) -> np.ndarray:
         """``runs``: [(row, position, token ids)], short ones first ->
-        the flat int array ``over`` splits."""
-        ids, pos, row, ts, te = [], [], [], [], []
-        es, el, ep, er = [], [], [], []
-        at = 0
-        for r, p, toks in runs:
-            n = len(toks)
-            ids += toks
-            pos += range(p, p + n)
-            row += [r] * n
-            ts += [at] * n
-            te += [at + n] * n
-            es.append(at)
-            el.append(n)
-            ep.append(p)
-            er.append(r)
-            at += n
-        return ids + pos + row + ts + te + es + el + ep + er
+        the flat int32 array that ``over`` splits."""
+        n = np.array([len(t) for _, _, t in runs], dtype=np.int32)
+        row = np.array([r for r, _, _ in runs], dtype=np.int32)
+        pos = np.array([p for _, p, _ in runs], dtype=np.int32)
+        end = np.cumsum(n, dtype=np.int32)
+        start = end - n
+        at = np.arange(end[-1], dtype=np.int32)
+        return np.concatenate(
+            [np.asarray(t, dtype=np.int32) for _, _, t in runs]
+            + [at + np.repeat(pos - start, n), np.repeat(row, n),
+               np.repeat(start, n), np.repeat(end, n), start, n, pos, row])
 
     @classmethod
     def over(cls, flat: torch.Tensor, runs, block_tables,
@@ -113,5 +108,5 @@ class RaggedBatch:
     @classmethod
     def build(cls, runs, block_tables) -> "RaggedBatch":
         dev = block_tables.device
-        flat = torch.tensor(cls.pack(runs), dtype=torch.int32, device=dev)
+        flat = torch.from_numpy(cls.pack(runs)).to(dev)
         return cls.over(flat, runs, block_tables)

@@ -678,6 +678,53 @@ def quantize_fp8_weight(w: torch.Tensor):
     return q.view(torch.uint8).contiguous(), scale.squeeze(1).contiguous()
 
 
+# shapes (M, K) whose products with 17..128 rows take the staged decode
+# GEMM because the library's pick was measured far behind it
+_DECODE_CHOICE: dict[tuple[int, int], bool] = {}
+
+
+def tune_decode_shapes(weights) -> int:
+    """Time hipBLASLt against the staged decode GEMM at 64 rows for each
+    [M, K] weight the latter can take, and keep the staged kernel where
+    it is at least a third faster (split-K down-projections of uncommon
+    depth, where the library runs a handful of workgroups).  Called once
+    at engine init; returns the number of shapes switched."""
+    if _lib is None:
+        return 0
+    flush = None
+    for w in weights:
+        M, K = w.shape
+        if ((M, K) in _DECODE_CHOICE or w.dtype != torch.bfloat16
+                or K % 256 or M % 128 or K < 4096):
+            continue
+        x = torch.randn(64, K, dtype=w.dtype, device=w.device)
+        if flush is None:      # weights must come from HBM, not the cache
+            flush = torch.empty(320 << 20, dtype=torch.uint8,
+                                device=w.device)
+
+        def timed(fn):
+            best = float("inf")
+            for i in range(5):
+                flush.fill_(i)
+                a = torch.cuda.Event(enable_timing=True)
+                b = torch.cuda.Event(enable_timing=True)
+                a.record()
+                fn()
+                b.record()
+                torch.cuda.synchronize()
+                best = min(best, a.elapsed_time(b)) if i else best
+            return best
+
+        try:
+            staged = timed(lambda: decode_gemm_v2(x, w))
+        except ValueError:
+            _DECODE_CHOICE[(M, K)] = False
+            continue
+        library = timed(lambda: torch.nn.functional.linear(x, w))
+        _DECODE_CHOICE[(M, K)] = staged < library / 1.5
+    return sum(_DECODE_CHOICE.values())
+
+
 def linear_decode(x: torch.Tensor, weight: torch.Tensor,
                   w8: tuple | None = None) -> torch.Tensor:
     """out = x @ W^T.
@@ -716,7 +763,7 @@ def linear_decode(x: torch.Tensor, weight: torch.Tensor,
         try:
             if N <= 16:
                 return decode_gemm_v2(x, weight, ver="2")
-            if mode != "auto":
+            if mode != "auto" or _DECODE_CHOICE.get((M, K)):
                 return decode_gemm_v2(x, weight)
         except ValueError:
             pass

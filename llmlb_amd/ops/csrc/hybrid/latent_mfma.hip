@@ -23,6 +23,20 @@ __device__ __forceinline__ f32x4 mfma(u32x4 a, u32x4 b, f32x4 c) {
       0);
 }
 
+// An operand whose 8 elements lie in 8 successive LDS rows: 16 lanes
+// address a 4 x 16 block (lane i: row i / 4, columns 4 (i % 4) ..) and
+// each gets one of its columns; the second block is ``down`` further.
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
+__device__ __forceinline__ u32x4 load_columns(const unsigned short* p,
+                                              int down) {
+  const uint2 a = __builtin_bit_cast(
+      uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)p));
+  const uint2 b = __builtin_bit_cast(
+      uint2, __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(p + down)));
+  return u32x4{a.x, a.y, b.x, b.y};
+}
+
 #define LOG2E 1.4426950408889634f
 
 // ---------------------------------------------------------------------------
@@ -97,27 +111,38 @@ void latent_flash_kernel(
   const int lo = (seen_lo > 0 ? seen_lo : 0) & ~63;
   const int hi = q_pos + n_q - k_pos;  // one past the last
 
+  // the thread's pieces of a tile: pointers that move from tile to tile.
+  // Columns past D + R meet a zero of the query, rows past V are dropped.
   u32x4 pk[KL], pv[VL];
-  auto fetch = [&](int j0) {
+  const bf16_t* k_src[KL];
+  int k_step[KL];
+  unsigned v_off[VL];
+#pragma unroll
+  for (int i = 0; i < KL; ++i) {
+    const int p = tid + i * 256;
+    const int d = (p % (DQ / 8)) * 8;
+    const size_t key = (size_t)k_row + lo + p / (DQ / 8);
+    const bool rotated = d >= D && R > 0;
+    k_src[i] = rotated ? kr + key * R + (d < DR ? d - D : 0)
+                       : kx + key * H * D + (size_t)h * D + (d < D ? d : 0);
+    k_step[i] = 64 * (rotated ? R : H * D);
+  }
+#pragma unroll
+  for (int i = 0; i < VL; ++i) {
+    const int p = tid + i * 256;
+    v_off[i] = (unsigned)(p / 8 < V ? p / 8 : V - 1) * key_ld + (p % 8) * 8;
+  }
+  const bf16_t* v_src = vt + (size_t)h * V * key_ld + k_row + lo;
+  auto fetch = [&]() {
 #pragma unroll
     for (int i = 0; i < KL; ++i) {
-      const int p = tid + i * 256;
-      const int r = p / (DQ / 8), d = (p % (DQ / 8)) * 8;
-      const size_t key = (size_t)k_row + j0 + r;
-      pk[i] = d < D ? *reinterpret_cast<const u32x4*>(
-                          kx + key * ((size_t)H * D) + (size_t)h * D + d)
-              : d < DR
-                  ? *reinterpret_cast<const u32x4*>(kr + key * R + (d - D))
-                  : u32x4{0, 0, 0, 0};
+      pk[i] = *reinterpret_cast<const u32x4*>(k_src[i]);
+      k_src[i] += k_step[i];
     }
 #pragma unroll
-    for (int i = 0; i < VL; ++i) {
-      const int p = tid + i * 256;
-      const int r = p / 8, d = (p % 8) * 8;
-      pv[i] = r < V ? *reinterpret_cast<const u32x4*>(
-                          vt + ((size_t)h * V + r) * key_ld + k_row + j0 + d)
-                    : u32x4{0, 0, 0, 0};
-    }
+    for (int i = 0; i < VL; ++i)
+      pv[i] = *reinterpret_cast<const u32x4*>(v_src + v_off[i]);
+    v_src += 64;
   };
 
   f32x4 o[2][VT];
@@ -132,7 +157,7 @@ void latent_flash_kernel(
   const int w_lo = q_pos + wave * 32 - k_pos;  // this wave's queries, as
   const int w_hi = w_lo + 31;                  // places in the key rows
 
-  fetch(lo);
+  fetch();
   for (int j0 = lo; j0 < hi; j0 += 64) {
 #pragma unroll
     for (int i = 0; i < KL; ++i) {
@@ -146,7 +171,7 @@ void latent_flash_kernel(
       *reinterpret_cast<u32x4*>(&lv[(p / 8) * VP + (p % 8) * 8]) = pv[i];
     }
     __syncthreads();
-    if (j0 + 64 < hi) fetch(j0 + 64);
+    if (j0 + 64 < hi) fetch();
     // a tile none of the wave's queries sees costs nothing
     if (j0 <= w_hi && j0 + 63 > w_lo - window) {
       f32x4 s[2][4];
@@ -168,17 +193,21 @@ void latent_flash_kernel(
         const int qi = w_lo + a * 16 + n;
         float mx = m[a];
 #pragma unroll
+        for (int t = 0; t < 4; ++t) s[a][t] *= scale_log2;
+        if (!whole) {
+          const int age = qi - j0 - g * 4;  // of key (t, i): age - 16t - i
+#pragma unroll
+          for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+              s[a][t][i] = (unsigned)(age - t * 16 - i) < (unsigned)window
+                               ? s[a][t][i]
+                               : -INFINITY;
+        }
+#pragma unroll
         for (int t = 0; t < 4; ++t)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            float x = s[a][t][i] * scale_log2;
-            if (!whole) {
-              const int j = j0 + t * 16 + g * 4 + i;
-              if (j > qi || qi - j >= window) x = -INFINITY;
-            }
-            s[a][t][i] = x;
-            mx = fmaxf(mx, x);
-          }
+          for (int i = 0; i < 4; ++i) mx = fmaxf(mx, s[a][t][i]);
         mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
         mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
         const float keep = __builtin_amdgcn_exp2f(m[a] - mx);
@@ -261,7 +290,8 @@ void latent_decode_kernel(
   constexpr int KD = NT * 2 + 2;         // 32-wide steps over rank + R
   constexpr int KEYS = 64 / HT, KT = KEYS / 16;
   constexpr int PITCH = KD * 32 + 8;
-  constexpr int PL = (KEYS * KD * 4 + 255) / 256;
+  constexpr int PAGES = KEYS / PAGE;
+  constexpr int PL = (PAGE * KD * 4 + 255) / 256;  // loads per page
   constexpr int PP = KEYS + 8;
   extern __shared__ unsigned short lk[];  // KEYS x PITCH
   __shared__ unsigned short lp[HT * 16 * PP];
@@ -283,37 +313,34 @@ void latent_decode_kernel(
   const int* pages = bt + (size_t)row * max_blocks;
   const int last_page = pos / PAGE;
 
-  // the thread's pieces of a tile: place in the row and in LDS
-  int p_row[PL], p_off[PL];
+  // the thread's pieces of a page, as offsets into it and into LDS
+  // (threads past the last piece repeat it)
+  int p_from[PL], p_to[PL];
 #pragma unroll
   for (int i = 0; i < PL; ++i) {
-    const int p = tid + i * 256;
-    p_row[i] = p / pieces;
-    p_off[i] = (p - p_row[i] * pieces) * 8;
+    int p = tid + i * 256;
+    p = p < PAGE * pieces ? p : PAGE * pieces - 1;
+    p_from[i] = p * 8;
+    p_to[i] = p / pieces * PITCH + p % pieces * 8;
   }
   // page numbers are wave-uniform and fetched a tile ahead of the rows
-  int pg[KEYS / PAGE];
+  int pg[PAGES];
   auto fetch_pages = [&](int t) {
 #pragma unroll
-    for (int i = 0; i < KEYS / PAGE; ++i) {
-      const int b = base / PAGE + t * (KEYS / PAGE) + i;
+    for (int i = 0; i < PAGES; ++i) {
+      const int b = base / PAGE + t * PAGES + i;
       pg[i] = pages[b < last_page ? b : last_page];
     }
   };
-  u32x4 pk[PL];
+  u32x4 pk[PAGES][PL];
   auto fetch = [&](int t) {
 #pragma unroll
-    for (int i = 0; i < PL; ++i) {
-      int page = pg[0];
+    for (int k = 0; k < PAGES; ++k) {
+      const bf16_t* src =
+          cache + (size_t)__builtin_amdgcn_readfirstlane(pg[k]) * PAGE * width;
 #pragma unroll
-      for (int k = 1; k < KEYS / PAGE; ++k)
-        page = p_row[i] / PAGE == k ? pg[k] : page;
-      pk[i] = p_row[i] < KEYS
-                  ? *reinterpret_cast<const u32x4*>(
-                        cache +
-                        ((size_t)page * PAGE + p_row[i] % PAGE) * width +
-                        p_off[i])
-                  : u32x4{0, 0, 0, 0};
+      for (int i = 0; i < PL; ++i)
+        pk[k][i] = *reinterpret_cast<const u32x4*>(src + p_from[i]);
     }
     if (t + 1 < t_hi) fetch_pages(t + 1);
   };
@@ -352,9 +379,11 @@ void latent_decode_kernel(
   }
   for (int t = t_lo; t < t_hi; ++t) {
 #pragma unroll
-    for (int i = 0; i < PL; ++i)
-      if (p_row[i] < KEYS)
-        *reinterpret_cast<u32x4*>(&lk[p_row[i] * PITCH + p_off[i]]) = pk[i];
+    for (int k = 0; k < PAGES; ++k)
+#pragma unroll
+      for (int i = 0; i < PL; ++i)
+        *reinterpret_cast<u32x4*>(&lk[k * PAGE * PITCH + p_to[i]]) =
+            pk[k][i];
     __syncthreads();
     if (t + 1 < t_hi) fetch(t + 1);
     f32x4 s = {0.f, 0.f, 0.f, 0.f}, s1 = s;
@@ -417,13 +446,10 @@ void latent_decode_kernel(
             &lp[(a * 16 + n) * PP + ks * 32 + g * 8]);
 #pragma unroll
       for (int r = 0; r < NT; ++r) {
-        const unsigned short* c =
-            &lk[(ks * 32 + g * 8) * PITCH + (wave * NT + r) * 16 + n];
-        u32x4 cf;
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-          cf[i] = (unsigned)c[(2 * i) * PITCH] |
-                  ((unsigned)c[(2 * i + 1) * PITCH] << 16);
+        const u32x4 cf = load_columns(
+            &lk[(ks * 32 + g * 8 + (n >> 2)) * PITCH +
+                (wave * NT + r) * 16 + (n & 3) * 4],
+            4 * PITCH);
 #pragma unroll
         for (int a = 0; a < HT; ++a) o[a][r] = mfma(cf, pf[a], o[a][r]);
       }
