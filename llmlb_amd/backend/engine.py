@@ -32,6 +32,8 @@ HybridCache whose state slots are the decode rows.
 """
 from __future__ import annotations
 
+import contextlib
+import gc
 import logging
 import queue
 import threading
@@ -131,6 +133,23 @@ class _Sequence:
         self.max_new = params.max_new_tokens # clamped to max_pos at submit
 
 
+@contextlib.contextmanager
+def _capturing(graph):
+    """Stream capture with the garbage collector held off: an engine and
+    its graphs form a cycle, and a collection inside the capture would
+    destroy a dropped engine's graphs there, which the runtime forbids
+    (the failed destructor aborts the process)."""
+    enabled = gc.isenabled()
+    gc.collect()
+    gc.disable()
+    try:
+        with torch.cuda.graph(graph):
+            yield
+    finally:
+        if enabled:
+            gc.enable()
+
+
 class _DecodeGraph:
     """One hipGraph-captured decode forward at a fixed (padded) batch.
 
@@ -213,7 +232,7 @@ class _DecodeGraph:
         torch.cuda.current_stream().wait_stream(side)
         torch.cuda.synchronize()
         self.graph = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(self.graph):
+        with _capturing(self.graph):
             self.logits = self._forward()
 
     def run(self, ids, lens, bt, slots, seq_lens) -> torch.Tensor:
@@ -272,7 +291,7 @@ class _RaggedGraph:
         torch.cuda.current_stream().wait_stream(side)
         torch.cuda.synchronize()
         self.graph = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(self.graph):
+        with _capturing(self.graph):
             self.logits = self._forward()
 
     def run(self, runs) -> torch.Tensor:

@@ -131,11 +131,7 @@ __device__ __forceinline__ void load_run(const bf16_t* p, float* f) {
 #pragma unroll
     for (int i = 0; i < N; i += 8) load8(p + i, f + i);
   } else if (VEC && N == 4) {
-    const uint2 v = *reinterpret_cast<const uint2*>(p);
-    f[0] = __uint_as_float(v.x << 16);
-    f[1] = __uint_as_float(v.x & 0xffff0000u);
-    f[2] = __uint_as_float(v.y << 16);
-    f[3] = __uint_as_float(v.y & 0xffff0000u);
+    load4(p, f);
   } else {
 #pragma unroll
     for (int i = 0; i < N; ++i) f[i] = to_f(p[i]);
@@ -145,10 +141,7 @@ template <int N, bool VEC>
 __device__ __forceinline__ void load_run(const float* p, float* f) {
   if (VEC && N % 4 == 0) {
 #pragma unroll
-    for (int i = 0; i < N; i += 4) {
-      const float4 v = *reinterpret_cast<const float4*>(p + i);
-      f[i] = v.x; f[i + 1] = v.y; f[i + 2] = v.z; f[i + 3] = v.w;
-    }
+    for (int i = 0; i < N; i += 4) load4(p + i, f + i);
   } else {
 #pragma unroll
     for (int i = 0; i < N; ++i) f[i] = p[i];
@@ -158,9 +151,7 @@ template <int N, bool VEC>
 __device__ __forceinline__ void store_run(float* p, const float* f) {
   if (VEC && N % 4 == 0) {
 #pragma unroll
-    for (int i = 0; i < N; i += 4)
-      *reinterpret_cast<float4*>(p + i) =
-          make_float4(f[i], f[i + 1], f[i + 2], f[i + 3]);
+    for (int i = 0; i < N; i += 4) store4(p + i, f + i);
   } else {
 #pragma unroll
     for (int i = 0; i < N; ++i) p[i] = f[i];
@@ -172,8 +163,7 @@ __device__ __forceinline__ void store_run(bf16_t* p, const float* f) {
 #pragma unroll
     for (int i = 0; i < N; i += 8) store8(p + i, f + i);
   } else if (VEC && N == 4) {
-    *reinterpret_cast<uint2*>(p) =
-        make_uint2(pack2(f[0], f[1]), pack2(f[2], f[3]));
+    store4(p, f);
   } else {
 #pragma unroll
     for (int i = 0; i < N; ++i) p[i] = from_f<bf16_t>(f[i]);

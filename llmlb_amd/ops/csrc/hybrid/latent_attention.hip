@@ -27,13 +27,32 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
   T* p = proj + (size_t)t * ld;
   const int half = R / 2;
   const float* cs = cos_sin + (size_t)pos * R;
-  for (int i = threadIdx.x; i < H * half; i += 256) {
-    const int h = i / half, j = i % half;
-    T* q = p + (size_t)h * (D + R) + D + j;
-    const float u = to_f(q[0]), v = to_f(q[half]);
-    const float c = cs[j], s = cs[half + j];
-    q[0] = from_f<T>(u * c - v * s);
-    q[half] = from_f<T>(v * c + u * s);
+  if (half % 4 == 0 && D % 4 == 0 && ld % 4 == 0) {
+    const int quads = half / 4;
+    for (int i = threadIdx.x; i < H * quads; i += 256) {
+      const int h = i / quads, j = i % quads * 4;
+      T* q = p + (size_t)h * (D + R) + D + j;
+      float u[4], v[4];
+      load4(q, u);
+      load4(q + half, v);
+      const float4 c = *reinterpret_cast<const float4*>(cs + j);
+      const float4 s = *reinterpret_cast<const float4*>(cs + half + j);
+      const float a[4] = {u[0] * c.x - v[0] * s.x, u[1] * c.y - v[1] * s.y,
+                          u[2] * c.z - v[2] * s.z, u[3] * c.w - v[3] * s.w};
+      const float b[4] = {v[0] * c.x + u[0] * s.x, v[1] * c.y + u[1] * s.y,
+                          v[2] * c.z + u[2] * s.z, v[3] * c.w + u[3] * s.w};
+      store4(q, a);
+      store4(q + half, b);
+    }
+  } else {
+    for (int i = threadIdx.x; i < H * half; i += 256) {
+      const int h = i / half, j = i % half;
+      T* q = p + (size_t)h * (D + R) + D + j;
+      const float u = to_f(q[0]), v = to_f(q[half]);
+      const float c = cs[j], s = cs[half + j];
+      q[0] = from_f<T>(u * c - v * s);
+      q[half] = from_f<T>(v * c + u * s);
+    }
   }
   if (!writes_kv) return;
   T* dst = cache + page_slot(bt, max_blocks, row_[t], pos) * (rank + R);

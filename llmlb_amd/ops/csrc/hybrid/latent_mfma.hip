@@ -40,7 +40,7 @@ __device__ __forceinline__ u32x4 load_columns(const unsigned short* p,
 #define LOG2E 1.4426950408889634f
 
 // ---------------------------------------------------------------------------
-// Copy the latents that a portion's queries can see out of the pages, 64
+// Copy the latents that a portion's queries can see out of the pages, 16
 // rows a workgroup: c [rows][rank], kr [rows][R].  ``blocks`` holds
 // (table row, first key position, valid keys) per 64 rows; rows past the
 // valid ones are zeroed.
@@ -48,16 +48,18 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(
     bf16_t* __restrict__ c, bf16_t* __restrict__ kr,
     const bf16_t* __restrict__ cache, const int* __restrict__ blocks,
     const int* __restrict__ bt, int max_blocks, int rank, int R) {
-  const int* blk = blocks + blockIdx.x * 3;
+  const int* blk = blocks + blockIdx.x / 4 * 3;
   const int row = blk[0], first = blk[1], valid = blk[2];
   const int pieces = (rank + R) / 8;
-  for (int i = threadIdx.x; i < 64 * pieces; i += 256) {
-    const int r = i / pieces, d = (i % pieces) * 8;
+  const int r0 = blockIdx.x % 4 * 16;
+#pragma unroll 4
+  for (int i = threadIdx.x; i < 16 * pieces; i += 256) {
+    const int r = r0 + i / pieces, d = (i % pieces) * 8;
     uint4 v = make_uint4(0, 0, 0, 0);
     if (r < valid)
       v = *reinterpret_cast<const uint4*>(
           cache + page_slot(bt, max_blocks, row, first + r) * (rank + R) + d);
-    const size_t to = (size_t)blockIdx.x * 64 + r;
+    const size_t to = (size_t)(blockIdx.x / 4) * 64 + r;
     bf16_t* dst = d < rank ? c + to * rank + d : kr + to * R + (d - rank);
     *reinterpret_cast<uint4*>(dst) = v;
   }
@@ -552,7 +554,7 @@ int hy_latent_gather(void* c, void* kr, const void* cache, const void* blocks,
                      int R, void* stream) {
   if (rank % 8 || R % 8) return -2;
   if (n_blocks <= 0) return 0;
-  hipLaunchKernelGGL(latent_gather_kernel, dim3(n_blocks), dim3(256), 0,
+  hipLaunchKernelGGL(latent_gather_kernel, dim3(n_blocks * 4), dim3(256), 0,
                      (hipStream_t)stream, (bf16_t*)c, (bf16_t*)kr,
                      (const bf16_t*)cache, (const int*)blocks,
                      (const int*)bt, max_blocks, rank, R);

@@ -13,6 +13,15 @@ __global__ __launch_bounds__(256) void embed_rows_kernel(
   const int id = ids[t];
   const bool ok = id >= 0 && id < vocab;
   const T* src = table + (size_t)(ok ? id : 0) * width;
+  if (ok && (width & 7) == 0) {
+    for (int i = threadIdx.x * 8; i < width; i += 2048) {
+      float f[8];
+      load8(src + i, f);
+      store8(x + (size_t)t * width + i, f);
+      if (xb) store8(xb + (size_t)t * width + i, f);
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < width; i += 256) {
     const float v = ok ? to_f(src[i]) : 0.f;
     x[(size_t)t * width + i] = v;

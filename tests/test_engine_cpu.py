@@ -259,3 +259,21 @@ def test_decode_piggyback_between_prefill_chunks():
     # the running stream got a token at each of the 3 interior chunk
     # boundaries plus the step's own decode
     assert q1.qsize() - before >= 4, (before, q1.qsize())
+
+
+def test_capture_holds_off_the_collector(monkeypatch):
+    """No garbage collection inside a graph capture, and the collector
+    is back afterwards, also after a failed capture."""
+    import contextlib
+    import gc
+
+    from llmlb_amd.backend import engine as E
+    monkeypatch.setattr(torch.cuda, "graph",
+                        lambda g: contextlib.nullcontext())
+    with E._capturing(None):
+        assert not gc.isenabled()
+    assert gc.isenabled()
+    with pytest.raises(ValueError):
+        with E._capturing(None):
+            raise ValueError
+    assert gc.isenabled()
