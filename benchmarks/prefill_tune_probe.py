@@ -2,7 +2,7 @@
 tuner timings (cache-evicted) AND a cold-stream style comparison for
 the llama-3-8b prefill GEMM shapes.
 
-  gpurun -- 'LLMLB_FP8_A8=1 python benchmarks/prefill_tune_probe.py'
+  LLMLB_FP8_A8=1 python benchmarks/prefill_tune_probe.py
 """
 import os
 import sys

@@ -4,7 +4,7 @@ path with a bool mask (profiles/r02_fp8_prefill_ab.md).  Try the same
 shapes with (a) bool mask, (b) bf16 additive mask, (c) explicit
 backend restriction, and time each — the round-3 prefill lever.
 
-  gpurun -- 'python benchmarks/sdpa_mask_probe.py'
+  python benchmarks/sdpa_mask_probe.py
 """
 import sys
 import time

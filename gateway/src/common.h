@@ -2,7 +2,7 @@
 // Design: epoll event loops (one per core, SO_REUSEPORT), non-blocking
 // sockets, single-buffer forwarding (scan-in-place SSE tap, no per-chunk
 // copies).  Mirrors the behavior of the reference gateway's hot path
-//  with a zero-copy pump.
+// with a zero-copy pump.
 #pragma once
 
 #include <algorithm>

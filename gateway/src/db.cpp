@@ -98,7 +98,7 @@ int Db::changes() { return sqlite3_changes(db_); }
 
 // ---------------------------------------------------------------------
 // Schema.  One migration set (idempotent CREATE IF NOT EXISTS), covering
-// the reference's table groups (SURVEY.md §2 component 27): endpoints,
+// the reference's table groups: endpoints,
 // endpoint_models, registered models, request_history, daily stats,
 // users, api_keys, invitations, audit_log, settings, health history.
 // ---------------------------------------------------------------------

@@ -1,6 +1,6 @@
 // SQLite persistence for the gateway (endpoints, models, request
 // history, daily stats, users, api keys, audit log) — the L2 layer of
-// SURVEY.md §1, reimplemented natively.
+// reimplemented natively.
 //
 // The build environment ships libsqlite3.so.0 but no sqlite3.h, so we
 // declare the handful of stable public C-API entry points we use

@@ -1,6 +1,6 @@
 // Pull-based health checking, endpoint type detection and model sync —
 // the reference's health/endpoint_checker.rs, detection/ and sync/
-// subsystems (SURVEY.md §3.4), as one background thread with a blocking
+// subsystems, as one background thread with a blocking
 // mini HTTP client (off the hot path).
 #include <poll.h>
 #include <sys/socket.h>

@@ -1,6 +1,6 @@
 // Mock OpenAI-compatible echo backend — BASELINE config 1's backend and
 // the integration-test fake (the reference tests use wiremock servers
-// the same way, SURVEY.md §4).
+// the same way).
 //
 //   llmlb-mock [--port N] [--models a,b] [--delay-ms D] [--workers N]
 //              [--stream-chunks K] [--fail-rate F]

@@ -1,7 +1,7 @@
 // Routing core: endpoint registry + TPS-weighted selection.
 //
 // Reimplements the behavior of the reference's balancer::LoadManager /
-// registry::EndpointRegistry (SURVEY.md §2 components 5-8) natively:
+// registry::EndpointRegistry natively:
 //   * per-(endpoint, model, api_kind) tokens/sec EMA, alpha = 0.2
 //     (balancer/types.rs:109), stale after 120 s (types.rs:20);
 //   * selection sorts candidates by TPS score desc with round-robin

@@ -1,7 +1,7 @@
 // llmlb-test: native unit tests for the gateway internals (TPS math,
 // selection, admission, HTTP parsing, chunked scanner, SSE tap, JSON,
 // crypto).  Mirrors the reference's in-file unit-test tier
-// (SURVEY.md §4).  Exit code 0 = all pass.
+// Exit code 0 = all pass.
 #include <cstdio>
 #include <unistd.h>
 
@@ -355,7 +355,7 @@ static void test_anthropic_stream_encoder_fragmented() {
 }
 
 static void test_permission_matrix() {
-  // exact token matching: no substring grants (ADVICE r1)
+  // exact token matching: no substring grants
   CHECK(!AuthStore::perms_grant("badminton", "admin"));
   CHECK(!AuthStore::perms_grant("inference-disabled", "openai.inference"));
   CHECK(!AuthStore::perms_grant("inferenc", "openai.inference"));

@@ -16,7 +16,7 @@ balancer written in Rust) redesigned for a single 8x MI355X node:
                      replica placement.
   * ``telemetry/`` — amdsmi HBM/busy polling, hipEvent queue depth.
 
-The reference gateway hosts no model kernels (SURVEY.md §0); the GPU
+The reference gateway hosts no model kernels; the GPU
 surface here (backends, kernels, telemetry, placement) is new work
 specified by BASELINE.json.
 """

@@ -6,7 +6,7 @@ drill-downs, auth/users, invitations, audit queries, TPS benchmarks,
 catalog, WS events) to this FastAPI app over loopback
 (LLMLB_CONTROL_PLANE_URL).  Shares the gateway's SQLite database (WAL).
 
-Reference coverage (SURVEY.md §2): components 20 (dashboard API), 21
+Reference coverage: components 20 (dashboard API), 21
 (dashboard WS), 22 (benchmarks), 23 (catalog), 24 (users/api_keys/
 invitations/audit API), 25 (auth: JWT login, password policy).
 bcrypt is not in this image, so passwords use PBKDF2-HMAC-SHA256

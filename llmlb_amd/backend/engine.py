@@ -569,7 +569,7 @@ class Engine:
                 # A step() failure (OOM, kernel error, scheduler bug)
                 # must not kill the daemon thread and hang every
                 # in-flight and queued request: fail them all with an
-                # "error" finish and keep serving (ADVICE r1 #2).
+                # "error" finish and keep serving.
                 log.exception("engine step failed; failing in-flight work")
                 self._fail_all_inflight("engine step error")
                 busy = False
@@ -718,7 +718,7 @@ class Engine:
                 if c1 == L:
                     break
                 c0 = c1
-                # decode piggyback (VERDICT r1 #8): one decode step for
+                # decode piggyback: one decode step for
                 # the running streams between prefill chunks, so a long
                 # prompt no longer stalls everyone's time-between-tokens
                 # for its whole multi-chunk prefill.  Intermediate chunk
@@ -1190,7 +1190,6 @@ class Engine:
             # also bound by what the KV pool can actually grow to right
             # now: pages beyond the current table must be allocatable,
             # else truncate the draft instead of raising mid-step
-            # 
             free_room = (len(s.block_table) * BLOCK_SIZE
                          + self.kv.free_blocks() * BLOCK_SIZE
                          - s.length - 1)

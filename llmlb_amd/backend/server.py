@@ -2,7 +2,7 @@
 
 One server per engine (one engine per GPU; TP replicas run one server
 on rank 0 of the TP group).  Serves the surface the gateway's model
-sync and routing expect (SURVEY.md §3):
+sync and routing expect:
 
   GET  /v1/models            — model listing (sync source)
   POST /v1/chat/completions  — chat, stream + non-stream

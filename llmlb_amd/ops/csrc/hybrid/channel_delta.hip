@@ -448,43 +448,53 @@ __global__ __launch_bounds__(64) void delta_scan_kernel(
 #pragma unroll
   for (int s = 0; s < PF; ++s) fetch(s, s);
 
-  for (int t0 = 0; t0 < len; t0 += PF) {
+  // Every lane stores, the same value from several of them (and columns
+  // past the last one repeat it): no branch between the loads in flight
+  // and their use, so that waiting for one token's operands does not
+  // wait for the next ones'.
+  int oc = cc[0];
 #pragma unroll
-    for (int s = 0; s < PF; ++s) {
-      if (t0 + s < len) {
-        float a[CPL], b[CPL];
+  for (int c = 1; c < CPL; ++c) oc = lane % CPL == c ? cc[c] : oc;
+  auto token = [&](int s, int t) {
+    float a[CPL], b[CPL];
 #pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          a[c] = b[c] = 0.f;
+    for (int c = 0; c < CPL; ++c) {
+      a[c] = b[c] = 0.f;
 #pragma unroll
-          for (int i = 0; i < RPL; ++i) {
-            S[c][i] *= g[s][i];
-            a[c] += k[s][i] * S[c][i];
-            b[c] += q[s][i] * S[c][i];
-          }
-        }
-#pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          a[c] = row16_sum(a[c]);
-          b[c] = row16_sum(b[c]);
-        }
-#pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          const float u = beta[s] * (v[s][c] - a[c]);
-#pragma unroll
-          for (int i = 0; i < RPL; ++i) S[c][i] += k[s][i] * u;
-          b[c] += qk[s] * u;
-        }
-        // lane c of a group of 16 writes its column c
-        float mine = b[0];
-#pragma unroll
-        for (int c = 1; c < CPL; ++c) mine = (lane & 15) == c ? b[c] : mine;
-        if ((lane & 15) < CPL && col + (lane & 15) < V)
-          out[(size_t)(t0 + s) * H * V + col + (lane & 15)] = mine;
-        fetch(s, t0 + s + PF);
+      for (int i = 0; i < RPL; ++i) {
+        S[c][i] *= g[s][i];
+        a[c] += k[s][i] * S[c][i];
+        b[c] += q[s][i] * S[c][i];
       }
     }
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+      a[c] = row16_sum(a[c]);
+      b[c] = row16_sum(b[c]);
+    }
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+      const float u = beta[s] * (v[s][c] - a[c]);
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) S[c][i] += k[s][i] * u;
+      b[c] += qk[s] * u;
+    }
+    float mine = b[0];
+#pragma unroll
+    for (int c = 1; c < CPL; ++c) mine = lane % CPL == c ? b[c] : mine;
+    out[(size_t)t * H * V + oc] = mine;
+  };
+  int t0 = 0;
+  for (; t0 + PF <= len; t0 += PF) {
+#pragma unroll
+    for (int s = 0; s < PF; ++s) {
+      token(s, t0 + s);
+      fetch(s, t0 + s + PF);
+    }
   }
+#pragma unroll
+  for (int s = 0; s < PF; ++s)
+    if (t0 + s < len) token(s, t0 + s);
 #pragma unroll
   for (int c = 0; c < CPL; ++c)
     if (col + c < V)
@@ -779,7 +789,7 @@ int hy_delta_scan(void* o, void* state, const void* ws, const void* e_start,
                   int n_entries, int KH, int H, int D, int V, void* stream) {
   if (!delta_ok(KH, H, D, V, 1) || n_entries > 65535) return -2;
   if (n_entries <= 0) return 0;
-  // wide lanes where they still fill the chip's 1024 SIMDs
+  // wide lanes where they still put waves enough on the 1024 SIMDs
   const long long waves = (long long)n_entries * H * ((V + 3) / 4);
 #define GO(CPL)                                                               \
   do {                                                                        \
@@ -790,7 +800,7 @@ int hy_delta_scan(void* o, void* state, const void* ws, const void* e_start,
         (const int*)e_start, (const int*)e_len, (const int*)e_pos,            \
         (const int*)e_row, KH, H, D, V));                                     \
   } while (0)
-  if (V >= 16 && D <= 128 && waves >= 4096) GO(4);
+  if (V >= 16 && D <= 128 && waves >= 8192) GO(4);
   else if (V >= 8 && D <= 256 && waves >= 2048) GO(2);
   else GO(1);
 #undef GO

@@ -2,7 +2,7 @@
 //
 // These are the inference-backend hot ops for the Llama-3 family served
 // behind the gateway.  The reference gateway
-// (akiojin/llmlb) hosts no model kernels (SURVEY.md §2c); this file is the
+// (akiojin/llmlb) hosts no model kernels; this file is the
 // new MI355X-native backend surface.
 //
 // Design notes (per /opt/skills/guides/cdna_hip_programming.md):

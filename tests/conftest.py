@@ -13,7 +13,7 @@ os.environ.setdefault("OMP_NUM_THREADS", "4")
 
 def pytest_configure(config):
     config.addinivalue_line(
-        "markers", "gpu: needs a real MI355X GPU (run via gpurun)")
+        "markers", "gpu: needs a real MI355X GPU")
 
 
 def pytest_collection_modifyitems(config, items):

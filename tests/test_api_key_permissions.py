@@ -150,7 +150,7 @@ def test_scoped_permission_matrix(gw):
     assert _req("GET", gw + "/api/dashboard/summary",
                 headers=inf)[0] in (401, 403)
 
-    # substring tokens must not grant anything (ADVICE r1)
+    # substring tokens must not grant anything
     bad = mint("badminton")
     assert _req("POST", gw + "/v1/chat/completions", chat,
                 headers=bad)[0] in (401, 403)

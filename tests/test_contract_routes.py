@@ -1,5 +1,5 @@
 """Contract sweep: every data-plane route answers with its documented
-status + JSON shape (reference tests/contract/* tier, SURVEY §4).
+status + JSON shape (reference tests/contract/* tier).
 One shared stack; each case asserts status, content type and key
 fields — shapes, not values."""
 import json

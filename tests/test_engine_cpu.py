@@ -237,7 +237,7 @@ def test_logit_bias(tiny_engine):
 
 def test_decode_piggyback_between_prefill_chunks():
     """A long chunked prefill must not starve running streams: each
-    chunk boundary runs one decode step for them (VERDICT r1 #8)."""
+    chunk boundary runs one decode step for them."""
     from llmlb_amd.backend.engine import Engine, EngineConfig
     from llmlb_amd.backend.launcher import PRESETS
     from llmlb_amd.backend.sampler import SamplingParams

@@ -1,5 +1,5 @@
 """Integration tests: real llmlb-gw + llmlb-mock binaries over loopback
-(the reference tests the same flows with wiremock backends, SURVEY.md §4).
+(the reference tests the same flows with wiremock backends).
 CPU-only; binaries are built by __graft_entry__.build() / make.
 """
 import json
