@@ -284,7 +284,7 @@ def main() -> None:
     kv_gb = float(os.environ.get("LLMLB_BENCH_KV_GB", "0"))
     if kv_gb == 0 and oversubscribed:
         kv_gb = 8.0   # fixed cap: ranks share one GPU in validation
-    if kv_gb > 0 and have_gpu:
+    if kv_gb > 0 and have_gpu and model_name.startswith(("llama", "qwen")):
         from llmlb_amd.backend.kv_cache import KVCache
         from llmlb_amd.backend.launcher import PRESETS
         m = PRESETS[model_name]()

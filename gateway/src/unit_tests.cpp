@@ -1,6 +1,6 @@
 // llmlb-test: native unit tests for the gateway internals (TPS math,
 // selection, admission, HTTP parsing, chunked scanner, SSE tap, JSON,
-// crypto).  Mirrors the reference's in-file unit-test tier
+// crypto).  Mirrors the reference's in-file unit-test tier.
 // Exit code 0 = all pass.
 #include <cstdio>
 #include <unistd.h>

@@ -13,24 +13,54 @@
 // Per token of a packed batch: norm the latent, rotate the key part and
 // put both into the cache; rotate every head's query part in place.
 // Column offsets are into a row of ``proj`` (ld columns).  The pair
-// (i, i + R/2) turns; cos_sin row p is cos[R/2] | sin[R/2].
-template <typename T>
+// (i, i + R/2) turns; cos_sin row p is cos[R/2] | sin[R/2].  One wave a
+// token; VQ and VC: query parts and latents come in whole vectors.
+template <typename T, bool VQ, bool VC>
 __global__ __launch_bounds__(256) void latent_prep_kernel(
     T* __restrict__ proj, int ld, int H, int D, int R, int c_off, int rank,
     const float* __restrict__ w_norm, float eps,
     const float* __restrict__ cos_sin, const int* __restrict__ pos_,
     const int* __restrict__ row_, const int* __restrict__ bt, int max_blocks,
-    T* __restrict__ cache, int writes_kv) {
-  __shared__ float red[4];
-  const int t = blockIdx.x;
+    T* __restrict__ cache, int writes_kv, int n_tok) {
+  const int t = blockIdx.x * 4 + threadIdx.x / WAVE;
+  if (t >= n_tok) return;
+  const int lane = threadIdx.x & (WAVE - 1);
   const int pos = pos_[t];
   T* p = proj + (size_t)t * ld;
   const int half = R / 2;
   const float* cs = cos_sin + (size_t)pos * R;
-  if (half % 4 == 0 && D % 4 == 0 && ld % 4 == 0) {
+  // the latent's loads and the page lookup go first: the longest chains
+  constexpr int KEEP = 2;
+  float keep[KEEP][8], ssq = 0.f;
+  const T* src = p + c_off;
+  T* dst = nullptr;
+  float kr[2] = {0.f, 0.f};
+  if (writes_kv) {
+    dst = cache + page_slot(bt, max_blocks, row_[t], pos) * (rank + R);
+    if (lane < half) {
+      kr[0] = to_f(src[rank + lane]);
+      kr[1] = to_f(src[rank + half + lane]);
+    }
+    if (VC) {
+#pragma unroll
+      for (int n = 0; n < KEEP; ++n) {
+        const int i = (lane + n * WAVE) * 8;
+        if (i < rank) {
+          load8(src + i, keep[n]);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) ssq += keep[n][j] * keep[n][j];
+        }
+      }
+    }
+    for (int i = lane + (VC ? KEEP * WAVE * 8 : 0); i < rank; i += WAVE) {
+      const float f = to_f(src[i]);
+      ssq += f * f;
+    }
+  }
+  if (VQ) {
     const int quads = half / 4;
-    for (int i = threadIdx.x; i < H * quads; i += 256) {
-      const int h = i / quads, j = i % quads * 4;
+    for (int i = lane; i < H * quads; i += WAVE) {
+      const int h = i / quads, j = (i - h * quads) * 4;
       T* q = p + (size_t)h * (D + R) + D + j;
       float u[4], v[4];
       load4(q, u);
@@ -45,7 +75,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
       store4(q + half, b);
     }
   } else {
-    for (int i = threadIdx.x; i < H * half; i += 256) {
+    for (int i = lane; i < H * half; i += WAVE) {
       const int h = i / half, j = i % half;
       T* q = p + (size_t)h * (D + R) + D + j;
       const float u = to_f(q[0]), v = to_f(q[half]);
@@ -55,18 +85,25 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     }
   }
   if (!writes_kv) return;
-  T* dst = cache + page_slot(bt, max_blocks, row_[t], pos) * (rank + R);
-  const T* src = p + c_off;
-  float ssq = 0.f;
-  for (int i = threadIdx.x; i < rank; i += 256) {
-    const float f = to_f(src[i]);
-    ssq += f * f;
+  const float r = 1.f / sqrtf(wave_sum(ssq) / rank + eps);
+  if (VC) {
+#pragma unroll
+    for (int n = 0; n < KEEP; ++n) {
+      const int i = (lane + n * WAVE) * 8;
+      if (i < rank) {
+        float w[8];
+        load8(w_norm + i, w);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) keep[n][j] *= r * w[j];
+        store8(dst + i, keep[n]);
+      }
+    }
   }
-  const float r = 1.f / sqrtf(block_sum_256(ssq, red) / rank + eps);
-  for (int i = threadIdx.x; i < rank; i += 256)
+  for (int i = lane + (VC ? KEEP * WAVE * 8 : 0); i < rank; i += WAVE)
     dst[i] = from_f<T>(to_f(src[i]) * r * w_norm[i]);
-  for (int j = threadIdx.x; j < half; j += 256) {
-    const float u = to_f(src[rank + j]), v = to_f(src[rank + half + j]);
+  for (int j = lane; j < half; j += WAVE) {
+    const float u = j == lane ? kr[0] : to_f(src[rank + j]);
+    const float v = j == lane ? kr[1] : to_f(src[rank + half + j]);
     const float c = cs[j], s = cs[half + j];
     dst[rank + j] = from_f<T>(u * c - v * s);
     dst[rank + half + j] = from_f<T>(v * c + u * s);
@@ -155,11 +192,21 @@ int hy_latent_prep(void* proj, int ld, int H, int D, int R, int c_off,
                    int n_tok, int dtype, void* stream) {
   if (R % 2 || rank <= 0) return -2;
   if (n_tok <= 0) return 0;
-  HY_DTYPE(dtype, hipLaunchKernelGGL(
-      latent_prep_kernel<T>, dim3(n_tok), dim3(256), 0, (hipStream_t)stream,
-      (T*)proj, ld, H, D, R, c_off, rank, (const float*)w_norm, eps,
-      (const float*)cos_sin, (const int*)pos, (const int*)row,
-      (const int*)bt, max_blocks, (T*)cache, writes_kv));
+  const bool vq = R % 8 == 0 && D % 4 == 0 && ld % 4 == 0;
+  const bool vc = rank % 8 == 0 && R % 8 == 0 && ld % 8 == 0 &&
+                  c_off % 8 == 0;
+#define GO(VQ, VC)                                                           \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (latent_prep_kernel<T, VQ, VC>), dim3((n_tok + 3) / 4), dim3(256), 0,  \
+      (hipStream_t)stream, (T*)proj, ld, H, D, R, c_off, rank,               \
+      (const float*)w_norm, eps, (const float*)cos_sin, (const int*)pos,     \
+      (const int*)row, (const int*)bt, max_blocks, (T*)cache, writes_kv,     \
+      n_tok))
+  if (vq && vc) GO(true, true);
+  else if (vq) GO(true, false);
+  else if (vc) GO(false, true);
+  else GO(false, false);
+#undef GO
   HY_CHECK();
   return 0;
 }

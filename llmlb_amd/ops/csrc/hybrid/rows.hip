@@ -103,6 +103,24 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(
   const size_t src = (size_t)(index ? index[blockIdx.x] : blockIdx.x) * width;
   const size_t dst = (size_t)blockIdx.x * width;
   float ssq = 0.f;
+  if ((width & 7) == 0) {
+    for (int i = threadIdx.x * 8; i < width; i += 2048) {
+      float f[8];
+      load8(x + src + i, f);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ssq += f[j] * f[j];
+    }
+    const float r = 1.f / sqrtf(block_sum_256(ssq, red) / width + eps);
+    for (int i = threadIdx.x * 8; i < width; i += 2048) {
+      float f[8], wr[8];
+      load8(x + src + i, f);
+      load8(w + i, wr);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] *= r * (w_offset + wr[j]);
+      store8(out + dst + i, f);
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < width; i += 256)
     ssq += x[src + i] * x[src + i];
   const float r = 1.f / sqrtf(block_sum_256(ssq, red) / width + eps);
@@ -145,8 +163,18 @@ __global__ __launch_bounds__(256) void soft_cap_kernel(
     float* __restrict__ out, const T* __restrict__ in, float cap,
     long long n) {
   const long long step = (long long)gridDim.x * 256;
-  for (long long i = (long long)blockIdx.x * 256 + threadIdx.x; i < n;
-       i += step) {
+  const long long id = (long long)blockIdx.x * 256 + threadIdx.x;
+  const long long nvec = n >> 3;
+  for (long long i = id; i < nvec; i += step) {
+    float f[8];
+    load8(in + i * 8, f);
+    if (cap > 0.f) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] = cap * tanhf(f[j] / cap);
+    }
+    store8(out + i * 8, f);
+  }
+  for (long long i = nvec * 8 + id; i < n; i += step) {
     const float v = to_f(in[i]);
     out[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
   }
@@ -206,7 +234,7 @@ int hy_soft_cap(void* out, const void* in, float cap, long long n, int dtype,
                 void* stream) {
   if (n <= 0) return 0;
   HY_DTYPE(dtype, hipLaunchKernelGGL(
-      soft_cap_kernel<T>, dim3(grid_for(n)), dim3(256), 0,
+      soft_cap_kernel<T>, dim3(grid_for((n + 7) / 8)), dim3(256), 0,
       (hipStream_t)stream, (float*)out, (const T*)in, cap, n));
   HY_CHECK();
   return 0;

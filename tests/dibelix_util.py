@@ -49,11 +49,13 @@ ODD = config([latent(5, 6, 2, 7, 20, 19), delta(3, 1, 10, 5, 2, (7, 9)),
               latent(2, 10, 2, 9, 20, 33, scale=0.4, kv_from=0),
               delta(4, 2, 17, 6, 3, (5, 11))],
              vocab=131, width=52, ff=[70, None, 44, 58], eps=1e-4)
-# sizes of the tiled kernels, more than 16 heads, grouped delta heads
+# sizes of the tiled kernels, more than 16 heads, grouped delta heads, a
+# second rotation
 TILED = config([delta(8, 4, 128, 64, 4, (24, 40)),
                 latent(20, 32, 16, 48, 136, 70, base=5e4),
                 latent(12, 64, 16, 64, 136, 29, base=5e4, kv_from=1),
-                delta(4, 4, 32, 48, 1, (16, 8))],
+                delta(4, 4, 32, 48, 1, (16, 8)),
+                latent(16, 24, 32, 40, 88, 41, base=900.0)],
                vocab=320, width=256, ff=208, eps=1e-6, softcap=20.0)
 # one layer of each kind, for long runs
 PLAIN = config([latent(3, 16, 8, 24, 40, 27), delta(4, 2, 24, 16, 4)],
