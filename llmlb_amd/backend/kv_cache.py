@@ -17,9 +17,10 @@ with no active users park in an LRU pool and are evicted back to the
 free list on demand — with 288 GB of HBM3E the pool is effectively a
 multi-gigabyte prompt cache.
 
-``HybridCache`` serves models that mix latent attention with recurrent
-layers: the same pages hold latents, and each live sequence owns one
-slot of recurrent state.
+``HybridCache`` serves models that mix attention with recurrent layers:
+the same pages hold whatever an attention layer keeps per token (a
+latent, or keys beside values), and each live sequence owns one slot of
+recurrent state.
 """
 from __future__ import annotations
 
@@ -110,7 +111,7 @@ class KVCache(PagePool):
 
 
 @dataclass(frozen=True)
-class LatentSpec:
+class PageSpec:
     """A layer that keeps ``width`` numbers per token in the pages."""
     width: int
 
@@ -119,10 +120,10 @@ class LatentSpec:
 
 
 @dataclass(frozen=True)
-class DeltaSpec:
+class StateSpec:
     """A recurrent layer: per sequence a float state of
     heads x vdim x dim and the last ``taps`` inputs of ``channels``
-    convolved channels."""
+    convolved channels (both 0: no convolution)."""
     heads: int
     vdim: int
     dim: int
@@ -135,11 +136,11 @@ class DeltaSpec:
 
 
 class HybridCache(PagePool):
-    """Pages of latents and slots of recurrent state for one model.
+    """Pages and slots of recurrent state for one model.
 
-    ``specs[i]`` is layer i's LatentSpec, DeltaSpec or None (a layer
-    that reads another's latents).  All latent layers share one block
-    table.  State slots are the engine's decode rows, plus one more for
+    ``specs[i]`` is layer i's PageSpec, StateSpec or None (a layer
+    that reads another's pages).  All layers with pages share one block
+    table; how a layer lays out its part of a page is its own affair.  State slots are the engine's decode rows, plus one more for
     the padded rows of captured decode steps.  Nothing is cleared when a
     page or slot changes hands: kernels read only positions that the
     sequence itself has written, and position 0 starts from a zero
@@ -150,12 +151,12 @@ class HybridCache(PagePool):
     def __init__(self, specs, num_blocks: int, slots: int, device, dtype):
         super().__init__(num_blocks)
         self.slots = slots
-        self.latent, self.state, self.ring = {}, {}, {}
+        self.pages, self.state, self.ring = {}, {}, {}
         for i, s in enumerate(specs):
-            if isinstance(s, LatentSpec):
-                self.latent[i] = torch.zeros(num_blocks, BLOCK_SIZE, s.width,
+            if isinstance(s, PageSpec):
+                self.pages[i] = torch.zeros(num_blocks, BLOCK_SIZE, s.width,
                                              dtype=dtype, device=device)
-            elif isinstance(s, DeltaSpec):
+            elif isinstance(s, StateSpec):
                 self.state[i] = torch.zeros(
                     slots + 1, s.heads, s.vdim, s.dim,
                     dtype=torch.float32, device=device)
@@ -166,13 +167,13 @@ class HybridCache(PagePool):
     def block_bytes(specs, dtype) -> int:
         esize = torch.tensor([], dtype=dtype).element_size()
         return sum(s.page_bytes(esize) for s in specs
-                   if isinstance(s, LatentSpec))
+                   if isinstance(s, PageSpec))
 
     @staticmethod
     def state_bytes(specs, slots: int, dtype) -> int:
         esize = torch.tensor([], dtype=dtype).element_size()
         return (slots + 1) * sum(s.slot_bytes(esize) for s in specs
-                                 if isinstance(s, DeltaSpec))
+                                 if isinstance(s, StateSpec))
 
 
 class PrefixCache:

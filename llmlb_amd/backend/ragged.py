@@ -13,8 +13,9 @@ from dataclasses import dataclass, field
 import numpy as np
 import torch
 
-# longest entry whose queries attend through the absorbed form (the
-# cache read once for all heads); longer ones expand keys and values
+# longest entry whose queries attend one by one, as single tokens do
+# (the cache read once for all heads of a query); longer ones attend in
+# tiles of queries
 SHORT_ENTRY = 8
 
 
@@ -64,6 +65,24 @@ class RaggedBatch:
             plan = (flat[:len(blocks)], flat[len(blocks):],
                     len(blocks) // 3, len(items) // 5)
             self.plans[window] = plan
+        return plan
+
+    def query_tiles(self, size: int):
+        """Work list of the long entries in tiles of up to ``size``
+        queries: (items, item count), an item being (packed query, query
+        position, queries, block-table row), those with the most keys
+        first."""
+        plan = self.plans.get(("tiles", size))
+        if plan is None:
+            items = []
+            for start, n, pos, row in self.entries:
+                if n > SHORT_ENTRY:
+                    items += [(start + q, pos + q, min(size, n - q), row)
+                              for q in range(0, n, size)]
+            items.sort(key=lambda it: -it[1])
+            plan = (torch.tensor(items, dtype=torch.int32,
+                                 device=self.pos.device), len(items))
+            self.plans["tiles", size] = plan
         return plan
 
     @staticmethod

@@ -9,21 +9,19 @@ configuration, low-rank sizes from the weights' shapes.
 """
 from __future__ import annotations
 
-import json
 from dataclasses import dataclass, field
 from pathlib import Path
 
 import torch
 import torch.nn as nn
 
-from ..backend.kv_cache import BLOCK_SIZE, HybridCache
+from ..backend.kv_cache import HybridCache
 from ..backend.ragged import RaggedBatch
 from ..ops import hybrid as hy
 from ..ops.reference import build_cos_sin_table
-from ..parallel.tp import TPContext, get_tp_context
-from .mixers import ChannelDelta, DenseFF, LatentAttention, _linear, _param
-
-NORM_OFFSET = 1.0          # norm weights are stored around zero
+from ..parallel.tp import TPContext
+from .mixers import ChannelDelta, DenseFF, LatentAttention
+from .packed import PackedCausalLM, read_folder
 
 
 @dataclass
@@ -56,15 +54,8 @@ class DibelixConfig:
 
     @classmethod
     def from_dir(cls, path) -> "DibelixConfig":
-        from safetensors import safe_open
-        path = Path(path)
-        shapes = {}
-        for f in sorted(path.glob("*.safetensors")):
-            with safe_open(str(f), framework="pt") as sf:
-                for name in sf.keys():
-                    shapes[name] = sf.get_slice(name).get_shape()
-        return cls.from_json(json.loads((path / "config.json").read_text()),
-                             shapes, name=path.resolve().name)
+        c, shapes = read_folder(path)
+        return cls.from_json(c, shapes, name=Path(path).resolve().name)
 
     @classmethod
     def build(cls, pattern: str, *, vocab, width, ff, heads, dim, rot_dim,
@@ -163,26 +154,16 @@ class DibelixLayer(nn.Module):
             width=cfg.width, ff=mlp["ff"], dtype=dtype, device=device)
 
 
-class DibelixForCausalLM(nn.Module):
-    """Runs packed batches (backend.ragged.RaggedBatch) against a
-    HybridCache; the engine owns both."""
-
-    ragged = True
+class DibelixForCausalLM(PackedCausalLM):
+    norm_offset = 1.0          # norm weights are stored around zero
 
     def __init__(self, cfg: DibelixConfig, tp: TPContext | None = None,
                  dtype: torch.dtype = torch.bfloat16, device="cpu",
                  seed: int = 1234, init_weights: bool = True):
-        super().__init__()
-        self.tp = tp or get_tp_context()
-        if self.tp.world_size != 1:
-            raise ValueError("Dibelix runs on one GPU per replica "
-                             "(tensor parallel size 1)")
-        self.cfg, self.dtype = cfg, dtype
-        self.device = torch.device(device)
+        super().__init__(cfg, tp, dtype, device)
         self.layers_ = nn.ModuleList(
             [DibelixLayer(cfg, i, dtype, self.device)
              for i in range(len(cfg.layers))])
-        self.specs = [ly.mix.cache_spec() for ly in self.layers_]
         tables: dict = {}
         for i, ly in enumerate(self.layers_):
             if isinstance(ly.mix, LatentAttention):
@@ -197,92 +178,29 @@ class DibelixForCausalLM(nn.Module):
 
     # -- weights ----------------------------------------------------------
 
-    def weight_shapes(self) -> dict[str, tuple]:
-        W = self.cfg.width
-        out = {"embed": (self.cfg.vocab, W), "final.norm": (W,),
-               "head": (self.cfg.vocab, W)}
-        for i, ly in enumerate(self.layers_):
-            out[f"l{i}.norm1"] = (W,)
-            for k, s in ly.mix.weight_shapes().items():
-                out[f"l{i}.mix.{k}"] = s
-            if ly.ff is not None:
-                out[f"l{i}.norm2"] = (W,)
-                for k, s in ly.ff.weight_shapes().items():
-                    out[f"l{i}.mlp.{k}"] = s
-        return out
+    def load_layer(self, i: int, take, vec) -> None:
+        ly = self.layers_[i]
+        ly.norm1 = vec("norm1")
+        ly.mix.load({k: take(f"mix.{k}") for k in ly.mix.weight_shapes()})
+        if ly.ff is not None:
+            ly.norm2 = vec("norm2")
+            ly.ff.load({k: take(f"mlp.{k}") for k in ly.ff.weight_shapes()})
 
-    def _assign(self, take) -> None:
-        """``take(name)`` -> tensor.  Matrices keep the storage type;
-        norms, convolutions and decay parameters are kept in 32-bit."""
-        def mat(name):
-            return _param(take(name).to(dtype=self.dtype,
-                                        device=self.device).contiguous())
-
-        def vec(name):
-            return _param(take(name).float().to(self.device).contiguous())
-
-        self.embed, self.head = mat("embed"), mat("head")
-        self.final_norm = vec("final.norm")
-        for i, ly in enumerate(self.layers_):
-            ly.norm1 = vec(f"l{i}.norm1")
-            ly.mix.load({k: take(f"l{i}.mix.{k}")
-                         for k in ly.mix.weight_shapes()})
-            if ly.ff is not None:
-                ly.norm2 = vec(f"l{i}.norm2")
-                ly.ff.load({k: take(f"l{i}.mlp.{k}")
-                            for k in ly.ff.weight_shapes()})
-
-    def load_safetensors(self, path) -> int:
-        """Load a *.safetensors file or a folder of shards.  Returns the
-        number of tensors consumed."""
-        from safetensors import safe_open
-        p = Path(path)
-        files = sorted(p.glob("*.safetensors")) if p.is_dir() else [p]
-        if not files:
-            raise FileNotFoundError(f"no .safetensors under {path}")
-        tensors = {}
-        for f in files:
-            with safe_open(str(f), framework="pt") as sf:
-                for name in sf.keys():
-                    tensors[name] = sf.get_tensor(name)
-        want = self.weight_shapes()
-        for name, shape in want.items():
-            if name not in tensors:
-                raise KeyError(f"{name} is missing from {path}")
-            if tuple(tensors[name].shape) != tuple(shape):
-                raise ValueError(
-                    f"{name}: {tuple(tensors[name].shape)} in the file, "
-                    f"{tuple(shape)} by the configuration")
-        self._assign(lambda name: tensors[name])
-        return len(want)
-
-    def _init_weights(self, seed: int) -> None:
-        shapes = self.weight_shapes()
-        g = torch.Generator(device=self.device).manual_seed(seed)
-
-        def take(name):
-            s = shapes[name]
-            n = torch.randn(s, generator=g, device=self.device)
-            if name.endswith("mix.norm") or name.endswith("dkv.norm"):
-                return torch.ones_like(n)
-            if ".norm" in name:
-                return torch.zeros_like(n)
-            if name.endswith("A_log"):
-                return n.abs().mul_(0.5)
-            if name.endswith("dt_bias"):
-                return n.mul_(0.5).sub_(4.0)
-            if name.endswith(".conv"):
-                return n.mul_(0.5)
-            return n.mul_(0.02 if name in ("embed", "head")
-                          else s[-1] ** -0.5)
-
-        self._assign(take)
+    def random_tensor(self, name: str, noise: torch.Tensor) -> torch.Tensor:
+        if name.endswith("mix.norm") or name.endswith("dkv.norm"):
+            return torch.ones_like(noise)
+        if ".norm" in name:
+            return torch.zeros_like(noise)
+        if name.endswith("A_log"):
+            return noise.abs().mul_(0.5)
+        if name.endswith("dt_bias"):
+            return noise.mul_(0.5).sub_(4.0)
+        if name.endswith(".conv"):
+            return noise.mul_(0.5)
+        return noise.mul_(0.02 if name in ("embed", "head")
+                          else noise.shape[-1] ** -0.5)
 
     # -- forward ----------------------------------------------------------
-
-    def make_cache(self, num_blocks: int, slots: int) -> HybridCache:
-        return HybridCache(self.specs, num_blocks, slots, self.device,
-                           self.dtype)
 
     def forward(self, b: RaggedBatch, cache: HybridCache,
                 on_layer=None) -> torch.Tensor:
@@ -292,31 +210,10 @@ class DibelixForCausalLM(nn.Module):
         x, xb = hy.embed_rows(self.embed, b.ids)
         for i, ly in enumerate(self.layers_):
             hy.post_norm_add(x, xb, ly.mix(xb, b, cache, i), ly.norm1, eps,
-                             NORM_OFFSET)
+                             self.norm_offset)
             if ly.ff is not None:
                 hy.post_norm_add(x, xb, ly.ff(xb), ly.norm2, eps,
-                                 NORM_OFFSET)
+                                 self.norm_offset)
             if on_layer is not None:
                 on_layer(i, x)
         return x
-
-    def logits(self, x: torch.Tensor, index=None) -> torch.Tensor:
-        """float32 logits of the rows ``index`` (int32; None: all)."""
-        h = hy.norm_rows(x, index, self.final_norm, self.cfg.eps, self.dtype,
-                         NORM_OFFSET)
-        return hy.soft_cap(_linear(h, self.head), self.cfg.logit_softcap)
-
-    @torch.inference_mode()
-    def forward_dense(self, input_ids: torch.Tensor) -> torch.Tensor:
-        """Final-norm hidden states [B, L, width] of whole sequences,
-        through a cache of their own (embeddings)."""
-        B, L = input_ids.shape
-        nb = (L + BLOCK_SIZE - 1) // BLOCK_SIZE
-        cache = self.make_cache(1 + B * nb, B)
-        bt = torch.arange(1, 1 + B * nb, dtype=torch.int32,
-                          device=self.device).view(B, nb)
-        batch = RaggedBatch.build(
-            [(i, 0, toks) for i, toks in enumerate(input_ids.tolist())], bt)
-        x = self.forward(batch, cache)
-        return hy.norm_rows(x, None, self.final_norm, self.cfg.eps,
-                            self.dtype, NORM_OFFSET).view(B, L, -1)

@@ -1,8 +1,13 @@
 """Token mixers and feed-forwards of the hybrid models.
 
-Each takes its sizes and constants as arguments, reads the layer's input
-[T, width] in the storage type and returns the sublayer's output before
-any norm.  Projections of the same input are one matrix product.
+Each takes its sizes and constants as arguments and reads the layer's
+input [T, width] in the storage type.  Projections of the same input are
+one matrix product.
+
+``forward`` returns the sublayer's output before any norm.  Modules for
+parallel layers have ``inner`` instead: it writes what the output
+projection reads (``out_width`` columns of a wider row), so that the
+layer applies the projections of mixer and feed-forward as one product.
 """
 from __future__ import annotations
 
@@ -10,7 +15,7 @@ import torch
 import torch.nn as nn
 import torch.nn.functional as F
 
-from ..backend.kv_cache import DeltaSpec, LatentSpec
+from ..backend.kv_cache import StateSpec, PageSpec
 from ..ops import hybrid as hy
 from ..ops import linear_decode
 
@@ -86,12 +91,12 @@ class LatentAttention(nn.Module):
             if own else None
 
     def cache_spec(self):
-        return LatentSpec(self.rank + self.rot) \
+        return PageSpec(self.rank + self.rot) \
             if self.kv_from is None else None
 
     def forward(self, x, b, cache, index: int):
         own = self.kv_from is None
-        pages = cache.latent[index if own else self.kv_from]
+        pages = cache.pages[index if own else self.kv_from]
         proj = _linear(x, self.w_in)
         hy.latent_prep(proj, self.heads, self.dim, self.rot, self.rank,
                        self.c_off, self.w_norm, self.eps, self.cos_sin, b,
@@ -172,7 +177,7 @@ class ChannelDelta(nn.Module):
 
     def cache_spec(self):
         C = 2 * self.kv_heads * self.dim + self.heads * self.vdim
-        return DeltaSpec(self.heads, self.vdim, self.dim, C, self.taps)
+        return StateSpec(self.heads, self.vdim, self.dim, C, self.taps)
 
     def forward(self, x, b, cache, index: int):
         proj = _linear(x, self.w_in)
@@ -206,3 +211,175 @@ class DenseFF(nn.Module):
 
     def forward(self, x):
         return _linear(hy.gelu_tanh_(_linear(x, self.w_up)), self.w_down)
+
+
+class DifferentialAttention(nn.Module):
+    """Causal attention with two score maps over the same values,
+    combined as a1 - lam * a2, normed per head and gated by a projection
+    of the layer's input.
+
+    ``q_scale`` ([max_pos], set by the model) is the score factor of a
+    query at each position; ``softcap`` (None: off) bounds scores to
+    softcap * tanh(score / softcap)."""
+
+    def __init__(self, *, width, heads, kv_heads, dim, vdim, softcap, diff,
+                 eps, dtype, device):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        self.heads, self.kv_heads, self.dim, self.vdim = \
+            heads, kv_heads, dim, vdim
+        self.softcap, self.diff = softcap or 0.0, diff
+        self.eps, self.width = eps, width
+        self.dtype, self.device = dtype, device
+        self.out_width = heads * vdim
+        self.q_scale = None
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, H, G, D, V = (self.width, self.heads, self.kv_heads, self.dim,
+                         self.vdim)
+        return {"q": (H * 2 * D, W), "k": (G * 2 * D, W), "v": (G * V, W),
+                "lq1": (D,), "lk1": (D,), "lq2": (D,), "lk2": (D,),
+                "g": (H * V, W), "o": (W, H * V)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        stacked, offs = _stack_rows([w["q"], w["k"], w["v"], w["g"]])
+        self.w_in = _param(stacked.to(dtype=self.dtype, device=self.device))
+        _, self.k_off, self.v_off, self.g_off = offs
+        d1, d2 = ((w[f"lq{n}"].float() * w[f"lk{n}"].float()).sum().exp()
+                  for n in (1, 2))
+        self.lam = float(d1 - d2 + self.diff)
+
+    def cache_spec(self):
+        return PageSpec(self.kv_heads * (2 * self.dim + self.vdim))
+
+    def inner(self, x, b, cache, index: int, out) -> None:
+        proj = _linear(x, self.w_in)
+        pages = cache.pages[index]
+        hy.pair_append(proj, self.k_off, self.v_off, self.kv_heads,
+                       self.dim, self.vdim, b, pages)
+        hy.pair_attention(out, proj, self.g_off, self.heads, self.kv_heads,
+                          self.dim, self.vdim, pages, b, self.q_scale,
+                          self.softcap, self.lam, 1.0 - self.diff, self.eps)
+
+
+class GatedLinearAttention(nn.Module):
+    """S <- diag(alpha) S + k v^T, o = S^T q, with a decay per head and
+    key channel from a low-rank projection: alpha = sigmoid(z)^(1/tau).
+    Each head's output is normed and gated."""
+
+    def __init__(self, *, width, heads, dim, vdim, tau, decay_rank, eps,
+                 dtype, device):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.tau = heads, dim, vdim, tau
+        self.decay_rank, self.eps, self.width = decay_rank, eps, width
+        self.dtype, self.device = dtype, device
+        self.out_width = heads * vdim
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, n, v = self.width, self.heads * self.dim, self.heads * self.vdim
+        return {"q": (n, W), "k": (n, W), "v": (v, W), "g": (v, W),
+                "o": (W, v), "norm": (self.vdim,),
+                "a1": (self.decay_rank, W), "a2": (n, self.decay_rank),
+                "a2.b": (n,)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        to = dict(dtype=self.dtype, device=self.device)
+        stacked, offs = _stack_rows(
+            [w["q"], w["k"], w["v"], w["g"], w["a1"]])
+        self.w_in = _param(stacked.to(**to))
+        _, self.k_off, self.v_off, self.g_off, self.a_off = offs
+        self.w_a2 = _param(w["a2"].to(**to).contiguous())
+        self.b_a2, self.w_norm = (
+            _param(w[n].float().to(self.device).contiguous())
+            for n in ("a2.b", "norm"))
+
+    def cache_spec(self):
+        return StateSpec(self.heads, self.vdim, self.dim, 0, 0)
+
+    def inner(self, x, b, cache, index: int, out) -> None:
+        proj = _linear(x, self.w_in)
+        dec = _linear(proj[:, self.a_off:self.a_off + self.decay_rank],
+                      self.w_a2)
+        hy.gated_linear(out, proj, self.k_off, self.v_off, self.g_off, dec,
+                        self.b_a2, cache.state[index], b, self.w_norm,
+                        self.heads, self.dim, self.vdim, self.tau, self.eps)
+
+
+class StateSpaceDuality(nn.Module):
+    """Mamba-2: S <- exp(-exp(A) dt) S + dt B x^T, y = S^T C + D x, with
+    x, B and C from a short convolution and B, C shared by the heads of a
+    group; y is gated first and then normed in ``norm_groups`` parts."""
+
+    def __init__(self, *, width, heads, vdim, state, groups, taps,
+                 norm_groups, eps, dtype, device):
+        super().__init__()
+        if heads % groups or heads * vdim % norm_groups:
+            raise ValueError("groups must divide heads, and norm_groups "
+                             "heads * vdim")
+        self.heads, self.vdim, self.state, self.groups = \
+            heads, vdim, state, groups
+        self.taps, self.norm_groups = taps, norm_groups
+        self.eps, self.width = eps, width
+        self.dtype, self.device = dtype, device
+        self.out_width = heads * vdim
+        self.channels = heads * vdim + 2 * groups * state
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, inner, C, H = self.width, self.out_width, self.channels, self.heads
+        return {"in": (inner + C + H, W), "conv": (C, self.taps),
+                "conv.b": (C,), "dt_bias": (H,), "A_log": (H,), "D": (H,),
+                "norm": (inner,), "o": (W, inner)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        inner, C = self.out_width, self.channels
+        z, xbc, dt = torch.split(w["in"], [inner, C, self.heads])
+        # convolved channels first, as the kernels index them
+        stacked, (_, self.z_off, self.dt_off) = _stack_rows([xbc, z, dt])
+        self.w_in = _param(stacked.to(dtype=self.dtype, device=self.device))
+
+        def wide(t):
+            return _param(t.float().to(self.device).contiguous())
+
+        self.w_conv = wide(w["conv"].t())                  # [taps, C]
+        self.b_conv, self.w_norm = wide(w["conv.b"]), wide(w["norm"])
+        # per head: dt's bias, the rate exp(A_log), D
+        self.per_head = wide(torch.stack(
+            [w["dt_bias"].float(), w["A_log"].float().exp(),
+             w["D"].float()]))
+
+    def cache_spec(self):
+        return StateSpec(self.heads, self.vdim, self.state, self.channels,
+                         self.taps)
+
+    def inner(self, x, b, cache, index: int, out) -> None:
+        proj = _linear(x, self.w_in)
+        hy.state_space(out, proj, self.z_off, self.dt_off,
+                       cache.state[index], cache.ring[index], b, self.w_conv,
+                       self.b_conv, self.per_head, self.w_norm, self.groups,
+                       self.heads, self.state, self.vdim, self.taps,
+                       self.norm_groups, self.eps)
+
+
+class ClampedSwiGLU(nn.Module):
+    """g sigmoid(sharpness g) (u + 1) with g = min(gate x, limit) and
+    u = clamp(up x, -limit, limit)."""
+
+    def __init__(self, *, width, ff, limit, dtype, device, sharpness=1.702):
+        super().__init__()
+        self.width, self.ff, self.limit = width, ff, limit
+        self.sharpness = sharpness
+        self.dtype, self.device = dtype, device
+        self.out_width = ff
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        return {"gate": (self.ff, self.width), "up": (self.ff, self.width),
+                "down": (self.width, self.ff)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        stacked, (_, self.u_off) = _stack_rows([w["gate"], w["up"]])
+        self.w_in = _param(stacked.to(dtype=self.dtype, device=self.device))
+
+    def inner(self, x, out) -> None:
+        hy.clamped_swiglu(out, _linear(x, self.w_in), self.u_off, self.limit,
+                          self.sharpness)

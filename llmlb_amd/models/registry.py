@@ -11,15 +11,18 @@ from pathlib import Path
 
 from .dibelix import DibelixConfig, DibelixForCausalLM
 from .llama import LlamaConfig, LlamaForCausalLM
+from .taletar import TaletarConfig, TaletarForCausalLM
 
 MODELS = {
     LlamaConfig: LlamaForCausalLM,
     DibelixConfig: DibelixForCausalLM,
+    TaletarConfig: TaletarForCausalLM,
 }
 
 # architectures that can be read from a model folder
 FOLDERS = {
     DibelixConfig.architecture: DibelixConfig,
+    TaletarConfig.architecture: TaletarConfig,
 }
 
 PRESETS = {
@@ -32,6 +35,9 @@ PRESETS = {
     "dibelix-tiny": DibelixConfig.tiny,
     "dibelix-small": DibelixConfig.small,
     "dibelix-8b": DibelixConfig.base_8b,
+    "taletar-tiny": TaletarConfig.tiny,
+    "taletar-small": TaletarConfig.small,
+    "taletar-8b": TaletarConfig.base_8b,
 }
 
 

@@ -1,5 +1,6 @@
-"""Ops of the hybrid models: 32-bit residual stream with a norm on the
-sublayer's output, latent attention over pages, gated delta rule.
+"""Ops of the hybrid models: a 32-bit residual stream with norms before
+or after the sublayers, latent and differential attention over pages,
+gated delta rule and linear recurrences.
 
 The native library (csrc/hybrid) is loaded at first use.  GPU tensors
 always run the HIP kernels, in bfloat16 and in float32; CPU tensors run
@@ -55,16 +56,19 @@ def _dt(dtype: torch.dtype) -> ctypes.c_int:
 
 # -- rows ------------------------------------------------------------------
 
-def embed_rows(table, ids):
-    """(x float32 [T, W], the same in the storage type)."""
+def embed_rows(table, ids, copy: bool = True):
+    """(x float32 [T, W], the same in the storage type; None without
+    ``copy``)."""
     if not table.is_cuda:
-        return ref.embed_rows(table, ids)
+        return ref.embed_rows(table, ids, copy)
     T, W = ids.shape[0], table.shape[1]
     x = torch.empty(T, W, dtype=torch.float32, device=table.device)
-    xb = x if table.dtype == torch.float32 else torch.empty(
-        T, W, dtype=table.dtype, device=table.device)
+    xb = None
+    if copy:
+        xb = x if table.dtype == torch.float32 else torch.empty(
+            T, W, dtype=table.dtype, device=table.device)
     _check(native().hy_embed_rows(
-        _ptr(x), None if xb is x else _ptr(xb), _ptr(table), _ptr(ids),
+        _ptr(x), None if xb is x else _p(xb), _ptr(table), _ptr(ids),
         _i(T), _i(W), _i(table.shape[0]), _dt(table.dtype), _stream()),
         "hy_embed_rows")
     return x, xb
@@ -81,6 +85,23 @@ def post_norm_add(x, xb, y, w, eps, w_offset=0.0) -> None:
         _ptr(x), None if xb is x else _ptr(xb), _ptr(y), _ptr(w),
         _f(w_offset), _i(x.shape[0]), _i(x.shape[1]), _f(eps), _dt(y.dtype),
         _stream()), "hy_post_norm_add")
+
+
+def add_norms(x, y, w1, w2, eps, dtype):
+    """In place: x += y (None: nothing to add).  Returns rmsnorm(x) * w1
+    and rmsnorm(x) * w2 in ``dtype``, None for a weight that is None
+    (w2 alone may not be given)."""
+    if not x.is_cuda:
+        return ref.add_norms(x, y, w1, w2, eps, dtype)
+    assert y is None or (y.is_contiguous() and y.shape == x.shape
+                         and y.dtype == dtype)
+    h1, h2 = (None if w is None else
+              torch.empty(x.shape, dtype=dtype, device=x.device)
+              for w in (w1, w2))
+    _check(native().hy_add_norms(
+        _ptr(x), _p(y), _p(w1), _p(w2), _p(h1), _p(h2), _i(x.shape[0]),
+        _i(x.shape[1]), _f(eps), _dt(dtype), _stream()), "hy_add_norms")
+    return h1, h2
 
 
 def norm_rows(x, index, w, eps, dtype, w_offset=0.0):
@@ -105,6 +126,20 @@ def gelu_tanh_(y):
         _ptr(y), ctypes.c_longlong(y.numel()), _dt(y.dtype), _stream()),
         "hy_gelu_tanh")
     return y
+
+
+def clamped_swiglu(out, gu, u_off, limit, sharpness) -> None:
+    """out = g sigmoid(sharpness g) (u + 1), with g = min(gate, limit)
+    from the first columns of ``gu`` and u = clamp(up, -limit, limit)
+    from those at ``u_off``.  ``out`` may be columns of wider rows."""
+    if not gu.is_cuda:
+        ref.clamped_swiglu(out, gu, u_off, limit, sharpness)
+        return
+    assert gu.stride(1) == 1 and out.stride(1) == 1
+    _check(native().hy_clamped_swiglu(
+        _ptr(out), _i(out.stride(0)), _ptr(gu), _i(gu.stride(0)), _i(u_off),
+        _i(out.shape[0]), _i(out.shape[1]), _f(limit), _f(sharpness),
+        _dt(gu.dtype), _stream()), "hy_clamped_swiglu")
 
 
 def soft_cap(logits, cap):
@@ -267,3 +302,167 @@ def gated_delta(proj, b_off, dec, gate, state, ring, b, wconv, a_log,
         ld, _ptr(ring), _ptr(b.pos), _ptr(b.row), _ptr(b.tend), _i(T),
         *sizes, _i(taps), dt, st), "hy_delta_out")
     return out
+
+
+# -- differential attention ------------------------------------------------
+
+def pair_append(proj, k_off, v_off, kv_heads, dim, vdim, b, cache) -> None:
+    """Put every token's keys (both maps) and values into its page."""
+    if not proj.is_cuda:
+        ref.pair_append(proj, k_off, v_off, kv_heads, dim, vdim, b, cache)
+        return
+    assert proj.stride(1) == 1
+    _check(native().hy_pair_append(
+        _ptr(cache), _ptr(proj), _i(proj.stride(0)), _i(k_off), _i(v_off),
+        _i(kv_heads), _i(dim), _i(vdim), _ptr(b.pos), _ptr(b.row),
+        _ptr(b.block_tables), _i(b.block_tables.shape[1]), _i(b.n_tok),
+        _dt(proj.dtype), _stream()), "hy_pair_append")
+
+
+def can_pair_mfma(dtype, dim, vdim) -> bool:
+    """Sizes that the matrix-core kernels take."""
+    return (dtype == torch.bfloat16 and dim % 8 == 0 and vdim % 8 == 0
+            and dim <= 128 and vdim <= 256)
+
+
+def pair_parts(n: int, kv_heads: int, group: int, max_keys: int) -> int:
+    """How many workgroups share one query's keys: enough to fill the
+    chip, with at least two tiles of keys each."""
+    groups = n * kv_heads * ((group + 15) // 16)
+    return max(1, min(1024 // groups, max_keys // 128, 32))
+
+
+def pair_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
+                   q_scale, softcap, lam, gain, eps) -> None:
+    """Both maps' attention, their difference a1 - lam * a2, its norm per
+    head times ``gain`` and the sigmoid gate, into ``out`` [T, H * vdim]
+    (columns of wider rows).  ``proj`` starts with the queries."""
+    if not proj.is_cuda:
+        ref.pair_attention(out, proj, g_off, heads, kv_heads, dim, vdim,
+                           cache, b, q_scale, softcap, lam, gain, eps)
+        return
+    assert proj.stride(1) == 1 and out.stride(1) == 1
+    lib, bt, st = native(), b.block_tables, _stream()
+    H, G, D, V = heads, kv_heads, dim, vdim
+    dst = (_ptr(out), _i(out.stride(0)))
+    src = (_ptr(proj), _i(proj.stride(0)), _i(g_off), _ptr(cache))
+    sizes = (_i(H), _i(G), _i(D), _i(V))
+    consts = (_ptr(q_scale), _f(softcap), _f(lam), _f(gain), _f(eps))
+    where = (_ptr(bt), _i(bt.shape[1]))
+    # vector accesses need whole vectors in every row
+    if not (can_pair_mfma(proj.dtype, D, V) and proj.stride(0) % 8 == 0
+            and g_off % 8 == 0 and out.stride(0) % 8 == 0):
+        _check(lib.hy_pair_rows(
+            *dst, *src, _ptr(b.pos), _ptr(b.row), *where, *sizes, *consts,
+            _i(b.n_tok), _dt(proj.dtype), st), "hy_pair_rows")
+        return
+    n = b.n_short
+    if n:
+        parts = pair_parts(n, G, H // G, b.max_keys)
+        acc = torch.empty(n, H, 2, parts, V, dtype=torch.float32,
+                          device=proj.device)
+        ml = torch.empty(n, H, 2, parts, 2, dtype=torch.float32,
+                         device=proj.device)
+        _check(lib.hy_pair_decode(
+            *dst, _ptr(acc), _ptr(ml), *src, _ptr(b.pos), _ptr(b.row),
+            *where, *sizes, *consts, _i(n), _i(parts), st),
+            "hy_pair_decode")
+    if n < b.n_tok:
+        items, n_items = b.query_tiles(64)
+        _check(lib.hy_pair_flash(
+            *dst, *src, _ptr(items), _i(n_items), *where, *sizes, *consts,
+            st), "hy_pair_flash")
+
+
+# -- linear recurrences ----------------------------------------------------
+
+def _gated_norm(out, y, gate, g_off, w, groups, gate_first: bool,
+                eps) -> None:
+    """Rows of ``groups`` equal parts, each normed by its own rms and
+    times ``w`` (repeated along the row); silu(gate) before or after."""
+    T, W = y.shape
+    _check(native().hy_gated_norm(
+        _ptr(out), _i(out.stride(0)), _ptr(y), _ptr(gate),
+        _i(gate.stride(0)), _i(g_off), _ptr(w), _i(w.shape[0]), _i(T),
+        _i(groups), _i(W // groups), _i(gate_first), _f(eps),
+        _dt(out.dtype), _stream()), "hy_gated_norm")
+
+
+def gated_linear(out, proj, k_off, v_off, g_off, dec, dec_bias, state, b,
+                 w_norm, heads, dim, vdim, tau, eps) -> None:
+    """Gated linear attention of a packed batch into ``out``
+    [T, H * vdim] (columns of wider rows).  ``proj`` starts with the
+    queries; ``dec`` [T, H * dim] is the decays' projection.  Updates
+    ``state``."""
+    if not proj.is_cuda:
+        ref.gated_linear(out, proj, k_off, v_off, g_off, dec, dec_bias,
+                         state, b, w_norm, heads, dim, vdim, tau, eps)
+        return
+    assert proj.stride(1) == 1 and out.stride(1) == 1 \
+        and dec.is_contiguous()
+    lib, dt, st = native(), _dt(proj.dtype), _stream()
+    T, H, D, V = b.n_tok, heads, dim, vdim
+    ld, q_scale, rate = _i(proj.stride(0)), _f(D ** -0.5), _f(1.0 / tau)
+    if b.decode:
+        _check(lib.hy_gla_step(
+            _ptr(out), _i(out.stride(0)), _ptr(state), _ptr(proj), ld,
+            _i(k_off), _i(v_off), _i(g_off), _ptr(dec), _ptr(dec_bias),
+            _ptr(w_norm), _ptr(b.pos), _ptr(b.row), _i(T), _i(H), _i(D),
+            _i(V), q_scale, rate, _f(eps), dt, st), "hy_gla_step")
+        return
+    g = torch.empty(T, H * D, dtype=torch.float32, device=proj.device)
+    o = torch.empty(T, H * V, dtype=torch.float32, device=proj.device)
+    _check(lib.hy_gla_decay(
+        _ptr(g), _ptr(dec), _ptr(dec_bias), _i(T), _i(H * D), rate, dt, st),
+        "hy_gla_decay")
+    _check(lib.hy_linear_scan(
+        _ptr(o), _ptr(state), _ptr(proj), ld, _i(0), _i(k_off), _i(v_off),
+        _ptr(g), None, None, _ptr(b.e_start), _ptr(b.e_len), _ptr(b.e_pos),
+        _ptr(b.e_row), _i(len(b.entries)), _i(H), _i(H), _i(D), _i(V),
+        q_scale, dt, st), "hy_linear_scan")
+    _gated_norm(out, o, proj, g_off, w_norm, H, False, eps)
+
+
+def state_space(out, proj, z_off, dt_off, state, ring, b, wconv, bconv,
+                per_head, w_norm, groups, heads, dim, vdim, taps,
+                norm_groups, eps) -> None:
+    """Mamba-2 of a packed batch into ``out`` [T, H * vdim] (columns of
+    wider rows).  ``proj`` starts with the convolved x | B | C;
+    ``per_head`` rows are dt's bias, the decay rate and the skip factor.
+    Updates ``state`` and ``ring``."""
+    if not proj.is_cuda:
+        ref.state_space(out, proj, z_off, dt_off, state, ring, b, wconv,
+                        bconv, per_head, w_norm, groups, heads, dim, vdim,
+                        taps, norm_groups, eps)
+        return
+    assert proj.stride(1) == 1 and out.stride(1) == 1
+    lib, dt, st = native(), _dt(proj.dtype), _stream()
+    T, G, H, N, V = b.n_tok, groups, heads, dim, vdim
+    C = H * V + 2 * G * N
+    ld = _i(proj.stride(0))
+    o = torch.empty(T, H * V, dtype=torch.float32, device=proj.device)
+    conv = (_ptr(ring), _ptr(wconv), _ptr(bconv), _ptr(per_head))
+    if b.decode:
+        _check(lib.hy_ssm_step(
+            _ptr(o), _ptr(state), _ptr(proj), ld, _i(dt_off), *conv,
+            _ptr(b.pos), _ptr(b.row), _i(T), _i(G), _i(H), _i(N), _i(V),
+            _i(taps), dt, st), "hy_ssm_step")
+    else:
+        xbc = torch.empty(T, C, dtype=proj.dtype, device=proj.device)
+        steps = torch.empty(2, T, H, dtype=torch.float32,
+                            device=proj.device)
+        _check(lib.hy_ssm_prep(
+            _ptr(xbc), _ptr(steps), _ptr(proj), ld, _i(dt_off), *conv,
+            _ptr(b.pos), _ptr(b.row), _ptr(b.tstart), _i(T), _i(C), _i(H),
+            _i(taps), dt, st), "hy_ssm_prep")
+        _check(lib.hy_ring_store(
+            _ptr(ring), _ptr(proj), ld, _ptr(b.e_start), _ptr(b.e_len),
+            _ptr(b.e_pos), _ptr(b.e_row), _i(len(b.entries)), _i(C),
+            _i(taps), dt, st), "hy_ring_store")
+        _check(lib.hy_linear_scan(
+            _ptr(o), _ptr(state), _ptr(xbc), _i(C), _i(H * V + G * N),
+            _i(H * V), _i(0), _ptr(steps[0]), _ptr(steps[1]),
+            _ptr(per_head[2]), _ptr(b.e_start), _ptr(b.e_len),
+            _ptr(b.e_pos), _ptr(b.e_row), _i(len(b.entries)), _i(G), _i(H),
+            _i(N), _i(V), _f(1.0), dt, st), "hy_linear_scan")
+    _gated_norm(out, o, proj, z_off, w_norm, norm_groups, True, eps)

@@ -12,8 +12,10 @@ def _rms(x, eps):
     return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
 
 
-def embed_rows(table, ids):
+def embed_rows(table, ids, copy):
     x = table[ids.long()].float()
+    if not copy:
+        return x, None
     return x, x if table.dtype == torch.float32 else x.to(table.dtype)
 
 
@@ -23,6 +25,15 @@ def post_norm_add(x, xb, y, w, eps, w_offset):
         xb.copy_(x)
 
 
+def add_norms(x, y, w1, w2, eps, dtype):
+    if y is not None:
+        x += y.float()
+    if w1 is None:
+        return None, None
+    n = _rms(x, eps)
+    return (n * w1).to(dtype), None if w2 is None else (n * w2).to(dtype)
+
+
 def norm_rows(x, index, w, eps, dtype, w_offset):
     rows = x if index is None else x[index.long()]
     return (_rms(rows, eps) * (w_offset + w)).to(dtype)
@@ -30,6 +41,13 @@ def norm_rows(x, index, w, eps, dtype, w_offset):
 
 def gelu_tanh_(y):
     return y.copy_(F.gelu(y.float(), approximate="tanh"))
+
+
+def clamped_swiglu(out, gu, u_off, limit, sharpness):
+    n = out.shape[1]
+    g = gu[:, :n].float().clamp(max=limit)
+    u = gu[:, u_off:u_off + n].float().clamp(-limit, limit)
+    out.copy_(g * torch.sigmoid(sharpness * g) * (u + 1.0))
 
 
 def soft_cap(logits, cap):
@@ -115,3 +133,92 @@ def gated_delta(proj, b_off, dec, gate, state, ring, b, wconv, a_log,
             gate[start:start + n].float().view(n, H, V))
         outs.append(o.reshape(n, H * V))
     return torch.cat(outs).to(proj.dtype)
+
+
+def pair_append(proj, k_off, v_off, kv_heads, dim, vdim, b, cache):
+    T, G = b.n_tok, kv_heads
+    page = b.block_tables[b.row.long(), b.pos.long() // PAGE].long()
+    rows = cache.view(cache.shape[0], G, PAGE, 2 * dim + vdim)
+    k = proj[:, k_off:k_off + G * 2 * dim].reshape(T, G, 2 * dim)
+    v = proj[:, v_off:v_off + G * vdim].reshape(T, G, vdim)
+    rows[page, :, b.pos.long() % PAGE] = torch.cat([k, v], -1)
+
+
+def pair_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
+                   q_scale, softcap, lam, gain, eps):
+    H, G, D, V = heads, kv_heads, dim, vdim
+    rows = cache.view(cache.shape[0], G, PAGE, 2 * D + V)
+    head = torch.arange(H) // (H // G)
+    for t in range(b.n_tok):
+        p = int(b.pos[t])
+        js = torch.arange(p + 1)
+        page = b.block_tables[int(b.row[t]), js // PAGE].long()
+        kv = rows[page, :, js % PAGE].float()[:, head]         # [j, H, ..]
+        q = proj[t, :H * 2 * D].view(H, 2, D).float()
+        s = torch.einsum("hmd,jhmd->mhj", q,
+                         kv[..., :2 * D].unflatten(-1, (2, D))) * q_scale[p]
+        if softcap > 0:
+            s = softcap * torch.tanh(s / softcap)
+        a = torch.einsum("mhj,jhv->mhv", torch.softmax(s, -1),
+                         kv[..., 2 * D:])
+        o = _rms(a[0] - lam * a[1], eps) * gain
+        gate = torch.sigmoid(proj[t, g_off:g_off + H * V].float())
+        out[t] = (o.reshape(-1) * gate).to(out.dtype)
+
+
+def _scan(q, k, v, g, S, o):
+    """S [H, V, D] in place; q, k, g [n, H, D] (g may be [n, H, 1]),
+    v [n, H, V]; o [n, H, V] is filled."""
+    for t in range(q.shape[0]):
+        S *= g[t][:, None]
+        S += v[t][..., None] * k[t][:, None]
+        o[t] = torch.einsum("hvd,hd->hv", S, q[t])
+
+
+def gated_linear(out, proj, k_off, v_off, g_off, dec, dec_bias, state, b,
+                 w_norm, heads, dim, vdim, tau, eps):
+    H, D, V = heads, dim, vdim
+    for start, n, pos, row in b.entries:
+        x = proj[start:start + n].float()
+        z = dec[start:start + n].float() + dec_bias
+        g = torch.exp(F.logsigmoid(z) / tau).view(n, H, D)
+        S = state[row] if pos else state[row].zero_()
+        o = torch.empty(n, H, V)
+        _scan(x[:, :H * D].view(n, H, D) * D ** -0.5,
+              x[:, k_off:k_off + H * D].view(n, H, D),
+              x[:, v_off:v_off + H * V].view(n, H, V), g, S, o)
+        o = (_rms(o, eps) * w_norm).reshape(n, H * V)
+        out[start:start + n] = (
+            o * F.silu(x[:, g_off:g_off + H * V])).to(out.dtype)
+
+
+def state_space(out, proj, z_off, dt_off, state, ring, b, wconv, bconv,
+                per_head, w_norm, groups, heads, dim, vdim, taps,
+                norm_groups, eps):
+    G, H, N, V = groups, heads, dim, vdim
+    C = H * V + 2 * G * N
+    group = torch.arange(H) // (H // G)
+    for start, n, pos, row in b.entries:
+        x = proj[start:start + n, :C]
+        past = torch.zeros(taps - 1, C, dtype=x.dtype)
+        for back in range(1, taps):
+            if pos - back >= 0:
+                past[taps - 1 - back] = ring[row, (pos - back) % taps]
+        full = torch.cat([past, x]).float()
+        y = F.silu(bconv + sum(full[i:i + n] * wconv[i]
+                               for i in range(taps)))
+        xs = y[:, :H * V].view(n, H, V)
+        B = y[:, H * V:H * V + G * N].view(n, G, N)[:, group]
+        Cq = y[:, H * V + G * N:].view(n, G, N)[:, group]
+        dt = F.softplus(proj[start:start + n, dt_off:dt_off + H].float()
+                        + per_head[0], threshold=60.0)
+        g = torch.exp(-per_head[1] * dt)
+        S = state[row] if pos else state[row].zero_()
+        o = torch.empty(n, H, V)
+        _scan(Cq, B, dt[..., None] * xs, g[..., None], S, o)
+        for t in range(max(0, n - taps), n):
+            ring[row, (pos + t) % taps] = x[t]
+        o = (o + per_head[2][:, None] * xs).reshape(n, H * V)
+        o = o * F.silu(proj[start:start + n, z_off:z_off + H * V].float())
+        o = _rms(o.view(n, norm_groups, -1), eps).reshape(n, H * V) * w_norm
+        out[start:start + n] = o.to(out.dtype)
