@@ -23,27 +23,7 @@
 // multiplied with k AND q in one pass and
 //   o = S'^T q + (k . q) u,   S' = diag(g) S
 // leaves one cross-lane sum on the critical path of a token.
-#include "common.h"
-
-// silu(conv) of channel c at packed token t
-template <typename T>
-__device__ __forceinline__ float conv_silu(
-    const T* __restrict__ proj, int ld, const T* __restrict__ ring,
-    const float* __restrict__ wconv, int C, int taps, int c, int t, int pos,
-    int tstart, int slot) {
-  float acc = to_f(proj[(size_t)t * ld + c]) *
-              wconv[(size_t)(taps - 1) * C + c];
-  for (int back = 1; back < taps; ++back) {
-    const int p = pos - back;
-    if (p < 0) break;
-    const float in =
-        t - back >= tstart
-            ? to_f(proj[(size_t)(t - back) * ld + c])
-            : to_f(ring[((size_t)slot * taps + p % taps) * C + c]);
-    acc += in * wconv[(size_t)(taps - 1 - back) * C + c];
-  }
-  return silu_f(acc);
-}
+#include "recurrent.h"
 
 __device__ __forceinline__ float decay_of(float z, float a_log) {
   return expf(-expf(a_log) * softplus_f(z));
@@ -83,9 +63,9 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
       const int d = lane + j * WAVE;
       q[j] = k[j] = 0.f;
       if (d < D) {
-        q[j] = conv_silu(proj, ld, ring, wconv, C, taps, unit * D + d, t,
+        q[j] = conv_silu(proj, ld, ring, wconv, nullptr, C, taps, unit * D + d, t,
                          pos, ts, slot);
-        k[j] = conv_silu(proj, ld, ring, wconv, C, taps,
+        k[j] = conv_silu(proj, ld, ring, wconv, nullptr, C, taps,
                          (KH + unit) * D + d, t, pos, ts, slot);
       }
       qq += q[j] * q[j];
@@ -111,7 +91,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
     for (int j = lane; j < V; j += WAVE) {
       const int c = 2 * KH * D + h * V + j;
       w[at.v + h * V + j] =
-          conv_silu(proj, ld, ring, wconv, C, taps, c, t, pos, ts, slot);
+          conv_silu(proj, ld, ring, wconv, nullptr, C, taps, c, t, pos, ts, slot);
     }
     const float a = a_log[h];
     for (int d = lane; d < D; d += WAVE)
@@ -122,142 +102,6 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(
           sigmoid_f(to_f(proj[(size_t)t * ld + b_off + h]));
   }
 }
-
-// N consecutive elements, as wide as alignment allows; VEC: the address
-// is aligned to the whole run (or to 16 bytes).
-template <int N, bool VEC>
-__device__ __forceinline__ void load_run(const bf16_t* p, float* f) {
-  if (VEC && N % 8 == 0) {
-#pragma unroll
-    for (int i = 0; i < N; i += 8) load8(p + i, f + i);
-  } else if (VEC && N == 4) {
-    load4(p, f);
-  } else {
-#pragma unroll
-    for (int i = 0; i < N; ++i) f[i] = to_f(p[i]);
-  }
-}
-template <int N, bool VEC>
-__device__ __forceinline__ void load_run(const float* p, float* f) {
-  if (VEC && N % 4 == 0) {
-#pragma unroll
-    for (int i = 0; i < N; i += 4) load4(p + i, f + i);
-  } else {
-#pragma unroll
-    for (int i = 0; i < N; ++i) f[i] = p[i];
-  }
-}
-template <int N, bool VEC>
-__device__ __forceinline__ void store_run(float* p, const float* f) {
-  if (VEC && N % 4 == 0) {
-#pragma unroll
-    for (int i = 0; i < N; i += 4) store4(p + i, f + i);
-  } else {
-#pragma unroll
-    for (int i = 0; i < N; ++i) p[i] = f[i];
-  }
-}
-template <int N, bool VEC>
-__device__ __forceinline__ void store_run(bf16_t* p, const float* f) {
-  if (VEC && N % 8 == 0) {
-#pragma unroll
-    for (int i = 0; i < N; i += 8) store8(p + i, f + i);
-  } else if (VEC && N == 4) {
-    store4(p, f);
-  } else {
-#pragma unroll
-    for (int i = 0; i < N; ++i) p[i] = from_f<bf16_t>(f[i]);
-  }
-}
-// only the first ``valid`` of N elements exist
-template <int N, bool VEC, typename T>
-__device__ __forceinline__ void load_some(const T* p, int valid, float* f) {
-  if (VEC || valid >= N) {
-    load_run<N, VEC>(p, f);
-  } else {
-#pragma unroll
-    for (int i = 0; i < N; ++i) f[i] = i < valid ? to_f(p[i]) : 0.f;
-  }
-}
-template <int N, bool VEC, typename T>
-__device__ __forceinline__ void store_some(T* p, int valid, const float* f) {
-  if (VEC || valid >= N) {
-    store_run<N, VEC>(p, f);
-  } else {
-#pragma unroll
-    for (int i = 0; i < N; ++i)
-      if (i < valid) p[i] = from_f<T>(f[i]);
-  }
-}
-
-// 16-bit results take the hardware's exponential and logarithm
-template <typename T>
-__device__ __forceinline__ float sigmoid_t(float x) {
-  return sizeof(T) == 2 ? 1.f / (1.f + __expf(-x)) : sigmoid_f(x);
-}
-template <typename T>
-__device__ __forceinline__ float decay_t(float z, float rate) {
-  if (sizeof(T) == 2) {
-    const float e = __expf(-fabsf(z));
-    // log(1 + e) by its series where 1 + e would lose e
-    const float lp = e < 1e-3f ? e * (1.f - 0.5f * e) : __logf(1.f + e);
-    return __expf(-rate * (fmaxf(z, 0.f) + lp));
-  }
-  return expf(-rate * softplus_f(z));
-}
-
-// The convolution of N neighbouring channels over consecutive tokens,
-// each input read once: ``hist`` holds the last taps - 1 inputs.
-#define TAPS_MAX 4
-template <typename T, int N, bool VEC>
-struct ConvRun {
-  float w[TAPS_MAX][N], hist[TAPS_MAX - 1][N];
-  const T* proj;
-  const T* ring;
-  int ld, C, taps, c, valid;
-
-  __device__ __forceinline__ ConvRun(const T* proj_, int ld_, const T* ring_,
-                                     const float* wconv, int C_, int taps_,
-                                     int c_, int valid_)
-      : proj(proj_), ring(ring_), ld(ld_), C(C_), taps(taps_), c(c_),
-        valid(valid_) {
-#pragma unroll
-    for (int b = 0; b < TAPS_MAX; ++b)
-      if (b < taps)
-        load_some<N, VEC>(wconv + (size_t)(taps - 1 - b) * C + c, valid,
-                          w[b]);
-  }
-  // inputs before token t, from the batch or the sequence's ring
-  __device__ __forceinline__ void start(int t, int pos, int tstart,
-                                        int slot) {
-#pragma unroll
-    for (int b = 1; b < TAPS_MAX; ++b) {
-#pragma unroll
-      for (int i = 0; i < N; ++i) hist[b - 1][i] = 0.f;
-      if (b < taps && pos - b >= 0)
-        load_some<N, VEC>(
-            t - b >= tstart
-                ? proj + (size_t)(t - b) * ld + c
-                : ring + ((size_t)slot * taps + (pos - b) % taps) * C + c,
-            valid, hist[b - 1]);
-    }
-  }
-  __device__ __forceinline__ void step(int t, float* y) {
-    float x[N];
-    load_some<N, VEC>(proj + (size_t)t * ld + c, valid, x);
-#pragma unroll
-    for (int i = 0; i < N; ++i) {
-      float acc = x[i] * w[0][i];
-#pragma unroll
-      for (int b = 1; b < TAPS_MAX; ++b)
-        if (b < taps) acc += hist[b - 1][i] * w[b][i];
-#pragma unroll
-      for (int b = TAPS_MAX - 1; b > 1; --b) hist[b - 1][i] = hist[b - 2][i];
-      hist[0][i] = x[i];
-      y[i] = acc * sigmoid_t<T>(acc);
-    }
-  }
-};
 
 // delta_prep for at most TAPS_MAX taps and D <= 256: a workgroup walks
 // PREP_TOK tokens.  blockIdx.y ranges: q/k heads (16 lanes a head, 16
@@ -284,8 +128,10 @@ __global__ __launch_bounds__(256) void delta_prep_run_kernel(
     const int r0 = (threadIdx.x & 15) * RPL;
     const int valid = D - r0 < RPL ? (D - r0 > 0 ? D - r0 : 0) : RPL;
     const int cq = unit * D + (valid ? r0 : 0), ck = KH * D + cq;
-    ConvRun<T, RPL, VEC> q(proj, ld, ring, wconv, C, taps, cq, valid);
-    ConvRun<T, RPL, VEC> k(proj, ld, ring, wconv, C, taps, ck, valid);
+    ConvRun<T, RPL, VEC> q(proj, ld, ring, wconv, nullptr, C, taps, cq,
+                           valid);
+    ConvRun<T, RPL, VEC> k(proj, ld, ring, wconv, nullptr, C, taps, ck,
+                           valid);
     for (int t = t0; t < t1; ++t) {
       const int ts = tstart_[t];
       if (t == t0 || t == ts) {
@@ -322,8 +168,8 @@ __global__ __launch_bounds__(256) void delta_prep_run_kernel(
     const int j = (y * 256 + threadIdx.x) * 8;
     if (j >= H * V) return;
     const int valid = H * V - j < 8 ? H * V - j : 8;
-    ConvRun<T, 8, VEC> v(proj, ld, ring, wconv, C, taps, 2 * KH * D + j,
-                         valid);
+    ConvRun<T, 8, VEC> v(proj, ld, ring, wconv, nullptr, C, taps,
+                         2 * KH * D + j, valid);
     for (int t = t0; t < t1; ++t) {
       const int ts = tstart_[t];
       if (t == t0 || t == ts) v.start(t, pos_[t], ts, row_[t]);
@@ -354,38 +200,6 @@ __global__ __launch_bounds__(256) void delta_prep_run_kernel(
 #pragma unroll
     for (int i = 0; i < 8; ++i) f[i] = decay_t<T>(f[i] + bias[i], rate[i]);
     store_some<8, VEC>(ws + (size_t)t * at.size + at.g + j, valid, f);
-  }
-}
-
-template <int RPL, bool EXACT>
-__device__ __forceinline__ void load_rows(const float* __restrict__ p, int r0,
-                                          int D, float* f) {
-  if (EXACT && RPL % 4 == 0) {
-#pragma unroll
-    for (int i = 0; i < RPL / 4; ++i) {
-      const float4 v = reinterpret_cast<const float4*>(p + r0)[i];
-      f[i * 4] = v.x; f[i * 4 + 1] = v.y;
-      f[i * 4 + 2] = v.z; f[i * 4 + 3] = v.w;
-    }
-  } else {
-#pragma unroll
-    for (int i = 0; i < RPL; ++i)
-      f[i] = (EXACT || r0 + i < D) ? p[r0 + i] : 0.f;
-  }
-}
-
-template <int RPL, bool EXACT>
-__device__ __forceinline__ void store_rows(float* __restrict__ p, int r0,
-                                           int D, const float* f) {
-  if (EXACT && RPL % 4 == 0) {
-#pragma unroll
-    for (int i = 0; i < RPL / 4; ++i)
-      reinterpret_cast<float4*>(p + r0)[i] =
-          make_float4(f[i * 4], f[i * 4 + 1], f[i * 4 + 2], f[i * 4 + 3]);
-  } else {
-#pragma unroll
-    for (int i = 0; i < RPL; ++i)
-      if (EXACT || r0 + i < D) p[r0 + i] = f[i];
   }
 }
 
@@ -607,7 +421,7 @@ __global__ __launch_bounds__(256) void delta_step_kernel(
 
   T* keep = ring + ((size_t)slot * taps + pos % taps) * C;
   auto conv = [&](int c) {
-    const float y = conv_silu(proj, ld, ring, wconv, C, taps, c, s, pos, s,
+    const float y = conv_silu(proj, ld, ring, wconv, nullptr, C, taps, c, s, pos, s,
                               slot);
     keep[c] = proj[(size_t)s * ld + c];
     return y;
@@ -692,32 +506,11 @@ __global__ __launch_bounds__(256) void delta_step_kernel(
         from_f<T>(lo[j] * rn * w_norm[j] * sigmoid_f(to_f(gate[ob + j])));
 }
 
-static int rows_per_lane(int D) {
-  int r = 1;
-  while (r * 16 < D) r *= 2;
-  return r;
-}
-
 // every size the kernels of this file can take
 static bool delta_ok(int KH, int H, int D, int V, int taps) {
   return KH > 0 && H > 0 && H % KH == 0 && D > 0 && D <= 512 && V > 0 &&
          V <= 4096 && taps > 0;
 }
-
-#define HY_RPL(D, ...)                                                  \
-  do {                                                                  \
-    const int rpl__ = rows_per_lane(D);                                 \
-    const bool ex__ = rpl__ * 16 == (D);                                \
-    if (rpl__ == 1) { constexpr int RPL = 1; HY_EX(__VA_ARGS__); }      \
-    else if (rpl__ == 2) { constexpr int RPL = 2; HY_EX(__VA_ARGS__); } \
-    else if (rpl__ == 4) { constexpr int RPL = 4; HY_EX(__VA_ARGS__); } \
-    else if (rpl__ == 8) { constexpr int RPL = 8; HY_EX(__VA_ARGS__); } \
-    else if (rpl__ == 16) { constexpr int RPL = 16; HY_EX(__VA_ARGS__); } \
-    else { constexpr int RPL = 32; HY_EX(__VA_ARGS__); }                \
-  } while (0)
-#define HY_EX(...)                                        \
-  if (ex__) { constexpr bool EXACT = true; __VA_ARGS__; } \
-  else { constexpr bool EXACT = false; __VA_ARGS__; }
 
 extern "C" {
 

@@ -1,0 +1,589 @@
+// Linear recurrences with a matrix state per head:
+//   S <- diag(g) S + k v^T,   o = S^T q,   S [D key channels x V columns]
+//
+//  * gated linear attention: g per key channel, sigmoid(z)^(1/tau);
+//  * Mamba-2: g = exp(-rate dt) per head, v = dt x, and skip x is added to
+//    the output; q, k and x come from a short convolution, q and k serve
+//    all heads of a group.
+//
+// Tokens of several sequences lie packed one after another.  Per token:
+// pos (place in its sequence), row (its state slot), tstart (its
+// sequence's first packed token).  A sequence at position 0 starts from
+// zero whatever its slot holds.
+//
+// Everything that enters the state is float; q, k and v keep the storage
+// type they were projected or convolved in until they are used.
+#include "recurrent.h"
+
+// N consecutive elements as they lie in memory, widened on use, so that
+// elements in flight take half the registers and nothing waits for them.
+// VEC: the address is aligned to the whole run (or to 16 bytes).
+template <typename T, int N, bool VEC>
+struct Run;
+template <int N, bool VEC>
+struct Run<float, N, VEC> {
+  float f[N];
+  __device__ __forceinline__ void load(const float* p, int valid) {
+    load_some<N, VEC>(p, valid, f);
+  }
+  __device__ __forceinline__ float get(int i) const { return f[i]; }
+};
+template <int N>
+struct Run<bf16_t, N, false> {
+  unsigned short u[N];
+  __device__ __forceinline__ void load(const bf16_t* p, int valid) {
+#pragma unroll
+    for (int i = 0; i < N; ++i) u[i] = i < valid ? p[i].u : 0;
+  }
+  __device__ __forceinline__ float get(int i) const {
+    return __uint_as_float((unsigned)u[i] << 16);
+  }
+};
+template <>
+struct Run<bf16_t, 1, true> : Run<bf16_t, 1, false> {};
+template <int N>
+struct Run<bf16_t, N, true> {
+  unsigned w[N / 2];
+  __device__ __forceinline__ void load(const bf16_t* p, int) {
+    if (N % 8 == 0) {
+#pragma unroll
+      for (int i = 0; i < N / 8; ++i) {
+        const uint4 v = reinterpret_cast<const uint4*>(p)[i];
+        w[i * 4] = v.x; w[i * 4 + 1] = v.y;
+        w[i * 4 + 2] = v.z; w[i * 4 + 3] = v.w;
+      }
+    } else if (N == 4) {
+      const uint2 v = *reinterpret_cast<const uint2*>(p);
+      w[0] = v.x; w[N / 2 - 1] = v.y;
+    } else {
+      w[0] = *reinterpret_cast<const unsigned*>(p);
+    }
+  }
+  __device__ __forceinline__ float get(int i) const {
+    return __uint_as_float(i & 1 ? w[i / 2] & 0xffff0000u : w[i / 2] << 16);
+  }
+};
+
+// One wave = 4 CPL value columns of one head of one sequence: 16 lanes a
+// column, RPL key channels and CPL columns a lane.  The operands of the
+// next PF tokens are in flight while a token is worked on.  Nothing but
+// the state itself carries over from token to token; the sum over lanes
+// that makes an output is off that chain.
+//   q, k: columns q_off, k_off + group * D; v: v_off + head * V, of rows of
+//   ``in``;  g [T][H D] (CHANNEL) or [T][H];  dt [T][H], skip [H] or null
+template <typename T, int RPL, bool VEC, int CPL, bool CHANNEL>
+__global__ __launch_bounds__(64) void linear_scan_kernel(
+    float* __restrict__ o, float* __restrict__ state,
+    const T* __restrict__ in, int ld, int q_off, int k_off, int v_off,
+    const float* __restrict__ g_, const float* __restrict__ dt_,
+    const float* __restrict__ skip_, const int* __restrict__ e_start,
+    const int* __restrict__ e_len, const int* __restrict__ e_pos,
+    const int* __restrict__ e_row, int G, int H, int D, int V,
+    float q_scale) {
+  constexpr int PF = RPL <= 8 ? 4 : (RPL == 16 ? 2 : 1);
+  const int e = blockIdx.y;
+  const int nb = (V + 4 * CPL - 1) / (4 * CPL);
+  int head, cb;
+  if (H % 8 == 0) {  // all columns of a head on one XCD: its L2 serves them
+    const int x = blockIdx.x & 7, r = blockIdx.x >> 3;
+    head = x * (H / 8) + r / nb;
+    cb = r % nb;
+  } else {
+    head = blockIdx.x / nb;
+    cb = blockIdx.x % nb;
+  }
+  const int lane = threadIdx.x;
+  const int col = (cb * 4 + lane / 16) * CPL;  // the lane's first column
+  const int r0 = (lane & 15) * RPL;
+  const int valid = D - r0 < RPL ? (D - r0 > 0 ? D - r0 : 0) : RPL;
+  const int rr = valid ? r0 : 0;
+  const int group = head / (H / G);
+  const int len = e_len[e];
+  const size_t first = (size_t)e_start[e];
+  const T* qp = in + first * ld + q_off + group * D + rr;
+  const T* kp = in + first * ld + k_off + group * D + rr;
+  const T* vp = in + first * ld + v_off + head * V;
+  const float* gp = g_ + (CHANNEL ? first * H * D + (size_t)head * D + rr
+                                  : first * H + head);
+  const float* dp = dt_ ? dt_ + first * H + head : nullptr;
+  const float skip = skip_ ? skip_[head] : 0.f;
+  float* out = o + (first * H + head) * V;
+  float* sp = state + ((size_t)e_row[e] * H + head) * V * D;
+  int cc[CPL];
+#pragma unroll
+  for (int c = 0; c < CPL; ++c) cc[c] = col + c < V ? col + c : V - 1;
+
+  float S[CPL][RPL];
+  const bool resume = e_pos[e] > 0;
+#pragma unroll
+  for (int c = 0; c < CPL; ++c) {
+#pragma unroll
+    for (int i = 0; i < RPL; ++i) S[c][i] = 0.f;
+    if (resume) load_rows<RPL, VEC>(sp + (size_t)cc[c] * D, r0, D, S[c]);
+  }
+
+  constexpr int GN = CHANNEL ? RPL : 1;
+  Run<T, RPL, VEC> q[PF], k[PF];
+  float g[PF][GN], dt[PF];
+  T v[PF][CPL];
+  auto fetch = [&](int s, int t) {
+    t = t < len ? t : len - 1;
+    const size_t at = (size_t)t * ld;
+    q[s].load(qp + at, valid);
+    k[s].load(kp + at, valid);
+    if (CHANNEL) load_some<GN, VEC>(gp + (size_t)t * H * D, valid, g[s]);
+    else g[s][0] = gp[(size_t)t * H];
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) v[s][c] = vp[at + cc[c]];
+    dt[s] = dp ? dp[(size_t)t * H] : 1.f;
+  };
+#pragma unroll
+  for (int s = 0; s < PF; ++s) fetch(s, s);
+
+  // Every lane stores, the same value from several of them (and columns
+  // past the last one repeat it): no branch between the loads in flight
+  // and their use.
+  int oc = cc[0];
+#pragma unroll
+  for (int c = 1; c < CPL; ++c) oc = lane % CPL == c ? cc[c] : oc;
+  auto token = [&](int s, int t) {
+    float b[CPL], x[CPL];
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+      x[c] = to_f(v[s][c]);
+      const float u = x[c] * dt[s];
+      b[c] = 0.f;
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) {
+        S[c][i] = S[c][i] * g[s][CHANNEL ? i : 0] + k[s].get(i) * u;
+        b[c] += q[s].get(i) * S[c][i];
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) b[c] = row16_sum(b[c]);
+    float mine = b[0], xm = x[0];
+#pragma unroll
+    for (int c = 1; c < CPL; ++c) {
+      mine = lane % CPL == c ? b[c] : mine;
+      xm = lane % CPL == c ? x[c] : xm;
+    }
+    out[(size_t)t * H * V + oc] = mine * q_scale + skip * xm;
+  };
+  int t0 = 0;
+  for (; t0 + PF <= len; t0 += PF) {
+#pragma unroll
+    for (int s = 0; s < PF; ++s) {
+      token(s, t0 + s);
+      fetch(s, t0 + s + PF);
+    }
+  }
+#pragma unroll
+  for (int s = 0; s < PF; ++s)
+    if (t0 + s < len) token(s, t0 + s);
+#pragma unroll
+  for (int c = 0; c < CPL; ++c)
+    if (col + c < V)
+      store_rows<RPL, VEC>(sp + (size_t)(col + c) * D, r0, D, S[c]);
+}
+
+// g = sigmoid(dec + bias)^rate per channel
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void gla_decay_kernel(
+    float* __restrict__ g, const T* __restrict__ dec,
+    const float* __restrict__ bias, int n_tok, int C, float rate) {
+  constexpr int N = VEC ? 8 : 1;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * N;
+  if (c >= C) return;
+  float b[N];
+  load_run<N, VEC>(bias + c, b);
+  for (int t = blockIdx.x; t < n_tok; t += gridDim.x) {
+    float f[N];
+    load_run<N, VEC>(dec + (size_t)t * C + c, f);
+#pragma unroll
+    for (int i = 0; i < N; ++i) f[i] = decay_t<T>(-(f[i] + b[i]), rate);
+    store_run<N, VEC>(g + (size_t)t * C + c, f);
+  }
+}
+
+// dt = softplus(. + bias) and g = exp(-rate dt) of one head and token
+__device__ __forceinline__ void ssm_times(float raw, float bias, float rate,
+                                          float& dt, float& g) {
+  dt = softplus_f(raw + bias);
+  g = expf(-rate * dt);
+}
+
+// Convolved channels of a packed batch, one channel a thread (any taps).
+template <typename T>
+__global__ __launch_bounds__(256) void ssm_conv_kernel(
+    T* __restrict__ xbc, const T* __restrict__ proj, int ld,
+    const T* __restrict__ ring, const float* __restrict__ wconv,
+    const float* __restrict__ bias, const int* __restrict__ pos_,
+    const int* __restrict__ row_, const int* __restrict__ tstart_, int C,
+    int taps) {
+  const int t = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= C) return;
+  xbc[(size_t)t * C + c] =
+      from_f<T>(conv_silu(proj, ld, ring, wconv, bias, C, taps, c, t, pos_[t],
+                          tstart_[t], row_[t]));
+}
+
+// The same for at most TAPS_MAX taps: 8 channels a thread, each input of
+// PREP_TOK successive tokens read once.
+#define PREP_TOK 16
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void ssm_conv_run_kernel(
+    T* __restrict__ xbc, const T* __restrict__ proj, int ld,
+    const T* __restrict__ ring, const float* __restrict__ wconv,
+    const float* __restrict__ bias, const int* __restrict__ pos_,
+    const int* __restrict__ row_, const int* __restrict__ tstart_, int n_tok,
+    int C, int taps) {
+  const int t0 = blockIdx.x * PREP_TOK;
+  const int t1 = t0 + PREP_TOK < n_tok ? t0 + PREP_TOK : n_tok;
+  const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
+  if (c >= C) return;
+  const int valid = C - c < 8 ? C - c : 8;
+  ConvRun<T, 8, VEC> run(proj, ld, ring, wconv, bias, C, taps, c, valid);
+  for (int t = t0; t < t1; ++t) {
+    const int ts = tstart_[t];
+    if (t == t0 || t == ts) run.start(t, pos_[t], ts, row_[t]);
+    float f[8];
+    run.step(t, f);
+    store_some<8, VEC>(xbc + (size_t)t * C + c, valid, f);
+  }
+}
+
+// steps [2][T][H]: decay and dt.  per_head [3][H]: bias, rate, skip.
+template <typename T>
+__global__ __launch_bounds__(256) void ssm_times_kernel(
+    float* __restrict__ steps, const T* __restrict__ proj, int ld, int dt_off,
+    const float* __restrict__ per_head, int n_tok, int H) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i >= n_tok * H) return;
+  const int t = i / H, h = i - t * H;
+  float dt, g;
+  ssm_times(to_f(proj[(size_t)t * ld + dt_off + h]), per_head[h],
+            per_head[H + h], dt, g);
+  steps[i] = g;
+  steps[n_tok * H + i] = dt;
+}
+
+// The last inputs of every entry into its ring, once nothing reads the
+// ring any more.
+template <typename T>
+__global__ __launch_bounds__(256) void ring_store_kernel(
+    T* __restrict__ ring, const T* __restrict__ proj, int ld,
+    const int* __restrict__ e_start, const int* __restrict__ e_len,
+    const int* __restrict__ e_pos, const int* __restrict__ e_row, int C,
+    int taps) {
+  const int e = blockIdx.x, len = e_len[e];
+  const int n = len < taps ? len : taps;
+  for (int i = blockIdx.y; i < n; i += gridDim.y) {
+    const int j = len - n + i;
+    const T* src = proj + (size_t)(e_start[e] + j) * ld;
+    T* dst = ring + ((size_t)e_row[e] * taps + (e_pos[e] + j) % taps) * C;
+    for (int c = threadIdx.x; c < C; c += 256) dst[c] = src[c];
+  }
+}
+
+// Decode: one token of every sequence.  One workgroup per (head,
+// sequence); the state's loads are issued first so that everything the
+// token needs is computed behind them.
+//   CONV false: gated linear attention, out = silu(gate) norm(o)
+//   CONV true: Mamba-2, y = o + skip x (gate and norm span the heads)
+template <typename T, int RPL, bool EXACT, bool CONV>
+__global__ __launch_bounds__(256) void linear_step_kernel(
+    T* __restrict__ out, int ld_out, float* __restrict__ y,
+    float* __restrict__ state, const T* __restrict__ proj, int ld, int q_off,
+    int k_off, int v_off, int g_off, const T* __restrict__ dec,
+    const float* __restrict__ dec_bias, const float* __restrict__ w_norm,
+    T* __restrict__ ring, const float* __restrict__ wconv,
+    const float* __restrict__ conv_bias, const float* __restrict__ per_head,
+    const int* __restrict__ pos_, const int* __restrict__ row_, int G, int H,
+    int D, int V, int taps, float q_scale, float rate, float eps) {
+  constexpr int NU = 64 / RPL > 8 ? 8 : 64 / RPL;  // columns in flight
+  constexpr int DP = 16 * RPL;
+  extern __shared__ float lds[];
+  float* lq = lds;
+  float* lk = lq + DP;
+  float* lg = lk + DP;
+  float* lv = lg + DP;
+  float* lo = lv + V;
+  __shared__ float red[4];
+  const int h = blockIdx.x, s = blockIdx.y;
+  const int group = h / (H / G);
+  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
+  const int pos = pos_[s], slot = row_[s];
+  const int r0 = (lane & 15) * RPL;
+  const int col0 = wave * 4 + lane / 16;
+  float* sp = state + ((size_t)slot * H + h) * (size_t)V * D;
+
+  float S[NU][RPL];
+  auto fetch = [&](int base) {
+#pragma unroll
+    for (int n = 0; n < NU; ++n) {
+      const int col = base + n * 16 + col0;
+      if (pos > 0 && col < V) {
+        load_rows<RPL, EXACT>(sp + (size_t)col * D, r0, D, S[n]);
+      } else {
+#pragma unroll
+        for (int i = 0; i < RPL; ++i) S[n][i] = 0.f;
+      }
+    }
+  };
+  fetch(0);
+
+  const T* row = proj + (size_t)s * ld;
+  float gh = 0.f, dt = 1.f, skip = 0.f;
+  if constexpr (CONV) {
+    const int C = H * V + 2 * G * D;
+    T* keep = ring + ((size_t)slot * taps + pos % taps) * C;
+    auto conv = [&](int c) {
+      const float f = conv_silu(proj, ld, ring, wconv, conv_bias, C, taps, c,
+                                s, pos, s, slot);
+      keep[c] = row[c];
+      return f;
+    };
+    for (int d = tid; d < DP; d += 256) {
+      lq[d] = d < D ? conv(q_off + group * D + d) : 0.f;
+      lk[d] = d < D ? conv(k_off + group * D + d) : 0.f;
+    }
+    for (int j = tid; j < V; j += 256) lv[j] = conv(v_off + h * V + j);
+    ssm_times(to_f(row[g_off + h]), per_head[h], per_head[H + h], dt, gh);
+    skip = per_head[2 * H + h];
+  } else {
+    for (int d = tid; d < DP; d += 256) {
+      const bool ok = d < D;
+      lq[d] = ok ? to_f(row[q_off + h * D + d]) * q_scale : 0.f;
+      lk[d] = ok ? to_f(row[k_off + h * D + d]) : 0.f;
+      lg[d] = ok ? decay_t<T>(-(to_f(dec[((size_t)s * H + h) * D + d]) +
+                                dec_bias[h * D + d]),
+                              rate)
+                 : 0.f;
+    }
+    for (int j = tid; j < V; j += 256) lv[j] = to_f(row[v_off + h * V + j]);
+  }
+  __syncthreads();
+  float q[RPL], k[RPL], g[RPL];
+#pragma unroll
+  for (int i = 0; i < RPL; ++i) {
+    q[i] = lq[r0 + i];
+    k[i] = lk[r0 + i] * dt;
+    g[i] = CONV ? gh : lg[r0 + i];
+  }
+  float ssq = 0.f;
+  for (int base = 0; base < V; base += NU * 16) {
+    if (base) fetch(base);
+#pragma unroll
+    for (int n = 0; n < NU; ++n) {
+      const int col = base + n * 16 + col0;
+      const float v = lv[col < V ? col : 0];
+      float r = 0.f;
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) {
+        S[n][i] = S[n][i] * g[i] + k[i] * v;
+        r += q[i] * S[n][i];
+      }
+      r = row16_sum(r);
+      if (col < V) {
+        store_rows<RPL, EXACT>(sp + (size_t)col * D, r0, D, S[n]);
+        if ((lane & 15) == 0) {
+          lo[col] = r + skip * v;
+          ssq += r * r;
+        }
+      }
+    }
+  }
+  if constexpr (CONV) {
+    __syncthreads();
+    for (int j = tid; j < V; j += 256)
+      y[((size_t)s * H + h) * V + j] = lo[j];
+  } else {
+    ssq = block_sum_256(ssq, red);
+    const float rn = 1.f / sqrtf(ssq / V + eps);
+    for (int j = tid; j < V; j += 256)
+      out[(size_t)s * ld_out + h * V + j] =
+          from_f<T>(lo[j] * rn * w_norm[j] *
+                    silu_f(to_f(row[g_off + h * V + j])));
+  }
+}
+
+// every size the kernels of this file can take
+static bool scan_ok(int G, int H, int D, int V) {
+  return G > 0 && H > 0 && H % G == 0 && D > 0 && D <= 512 && V > 0 &&
+         V <= 4096;
+}
+
+template <bool CONV>
+static int launch_step(void* out, int ld_out, void* y, void* state,
+                       const void* proj, int ld, int q_off, int k_off,
+                       int v_off, int g_off, const void* dec,
+                       const void* dec_bias, const void* w_norm, void* ring,
+                       const void* wconv, const void* conv_bias,
+                       const void* per_head, const void* pos, const void* row,
+                       int n_seq, int G, int H, int D, int V, int taps,
+                       float q_scale, float rate, float eps, int dtype,
+                       void* stream) {
+  if (!scan_ok(G, H, D, V) || n_seq > 65535) return -2;
+  if (n_seq <= 0) return 0;
+  const size_t lds = (3 * 16 * rows_per_lane(D) + 2 * V) * sizeof(float);
+  const dim3 grid(H, n_seq), block(256);
+  HY_DTYPE(dtype, HY_RPL(D, hipLaunchKernelGGL(
+      (linear_step_kernel<T, RPL, EXACT, CONV>), grid, block, lds,
+      (hipStream_t)stream, (T*)out, ld_out, (float*)y, (float*)state,
+      (const T*)proj, ld, q_off, k_off, v_off, g_off, (const T*)dec,
+      (const float*)dec_bias, (const float*)w_norm, (T*)ring,
+      (const float*)wconv, (const float*)conv_bias, (const float*)per_head,
+      (const int*)pos, (const int*)row, G, H, D, V, taps, q_scale, rate,
+      eps)));
+  HY_CHECK();
+  return 0;
+}
+
+extern "C" {
+
+int hy_linear_scan(void* o, void* state, const void* in, int ld, int q_off,
+                   int k_off, int v_off, const void* g, const void* dt,
+                   const void* skip, const void* e_start, const void* e_len,
+                   const void* e_pos, const void* e_row, int n_entries, int G,
+                   int H, int D, int V, float q_scale, int dtype,
+                   void* stream) {
+  if (!scan_ok(G, H, D, V) || n_entries > 65535) return -2;
+  if (n_entries <= 0) return 0;
+  const bool channel = dt == nullptr;
+  if (channel && G != H) return -2;
+  // wide lanes where they still put waves enough on the 1024 SIMDs
+  const long long waves = (long long)n_entries * H * ((V + 3) / 4);
+  const bool vec = ld % 8 == 0 && q_off % 8 == 0 && k_off % 8 == 0 &&
+                   D % 8 == 0 && rows_per_lane(D) * 16 == D;
+#define RUN(CPL, CHANNEL, VEC)                                                \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                         \
+      (linear_scan_kernel<T, RPL, VEC, CPL, CHANNEL>),                        \
+      dim3(H * ((V + 4 * CPL - 1) / (4 * CPL)), n_entries), dim3(64), 0,      \
+      (hipStream_t)stream, (float*)o, (float*)state, (const T*)in, ld, q_off, \
+      k_off, v_off, (const float*)g, (const float*)dt, (const float*)skip,    \
+      (const int*)e_start, (const int*)e_len, (const int*)e_pos,              \
+      (const int*)e_row, G, H, D, V, q_scale))
+// (the wide forms are chosen for small D only)
+#define PICK(CPL)                               \
+  do {                                          \
+    if constexpr (RPL * CPL <= 32) {            \
+      if (channel && vec) RUN(CPL, true, true); \
+      else if (channel) RUN(CPL, true, false);  \
+      else if (vec) RUN(CPL, false, true);      \
+      else RUN(CPL, false, false);              \
+    }                                           \
+  } while (0)
+#define GO(CPL)                                                    \
+  do {                                                             \
+    switch (rows_per_lane(D)) {                                    \
+      case 1: { constexpr int RPL = 1; PICK(CPL); } break;         \
+      case 2: { constexpr int RPL = 2; PICK(CPL); } break;         \
+      case 4: { constexpr int RPL = 4; PICK(CPL); } break;         \
+      case 8: { constexpr int RPL = 8; PICK(CPL); } break;         \
+      case 16: { constexpr int RPL = 16; PICK(CPL); } break;       \
+      default: { constexpr int RPL = 32; PICK(CPL); } break;       \
+    }                                                              \
+  } while (0)
+  if (V >= 16 && D <= 128 && waves >= 8192) GO(4);
+  else if (V >= 8 && D <= 256 && waves >= 2048) GO(2);
+  else GO(1);
+#undef GO
+#undef PICK
+#undef RUN
+  HY_CHECK();
+  return 0;
+}
+
+int hy_gla_decay(void* g, const void* dec, const void* bias, int n_tok, int C,
+                 float rate, int dtype, void* stream) {
+  if (n_tok <= 0 || C <= 0) return 0;
+  const bool vec = C % 8 == 0;
+  const int cols = vec ? 2048 : 256;
+  const dim3 grid(n_tok < 2048 ? n_tok : 2048, (C + cols - 1) / cols);
+#define GO(VEC)                                                          \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                    \
+      (gla_decay_kernel<T, VEC>), grid, dim3(256), 0,                    \
+      (hipStream_t)stream, (float*)g, (const T*)dec, (const float*)bias, \
+      n_tok, C, rate))
+  if (vec) GO(true);
+  else GO(false);
+#undef GO
+  HY_CHECK();
+  return 0;
+}
+
+int hy_gla_step(void* out, int ld_out, void* state, const void* proj, int ld,
+                int k_off, int v_off, int g_off, const void* dec,
+                const void* dec_bias, const void* w_norm, const void* pos,
+                const void* row, int n_seq, int H, int D, int V,
+                float q_scale, float rate, float eps, int dtype,
+                void* stream) {
+  return launch_step<false>(out, ld_out, nullptr, state, proj, ld, 0, k_off,
+                            v_off, g_off, dec, dec_bias, w_norm, nullptr,
+                            nullptr, nullptr, nullptr, pos, row, n_seq, H, H,
+                            D, V, 1, q_scale, rate, eps, dtype, stream);
+}
+
+int hy_ssm_step(void* y, void* state, const void* proj, int ld, int dt_off,
+                void* ring, const void* wconv, const void* bias,
+                const void* per_head, const void* pos, const void* row,
+                int n_seq, int G, int H, int N, int V, int taps, int dtype,
+                void* stream) {
+  if (taps <= 0) return -2;
+  return launch_step<true>(nullptr, 0, y, state, proj, ld, H * V + G * N,
+                           H * V, 0, dt_off, nullptr, nullptr, nullptr, ring,
+                           wconv, bias, per_head, pos, row, n_seq, G, H, N, V,
+                           taps, 1.f, 0.f, 0.f, dtype, stream);
+}
+
+int hy_ssm_prep(void* xbc, void* steps, const void* proj, int ld, int dt_off,
+                const void* ring, const void* wconv, const void* bias,
+                const void* per_head, const void* pos, const void* row,
+                const void* tstart, int n_tok, int C, int H, int taps,
+                int dtype, void* stream) {
+  if (taps <= 0 || C <= 0 || H <= 0) return -2;
+  if (n_tok <= 0) return 0;
+  if ((long long)n_tok * H >= (1ll << 30)) return -2;
+  hipStream_t st = (hipStream_t)stream;
+  if (taps <= TAPS_MAX) {
+    const dim3 grid((n_tok + PREP_TOK - 1) / PREP_TOK, (C + 2047) / 2048);
+#define GO(VEC)                                                              \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (ssm_conv_run_kernel<T, VEC>), grid, dim3(256), 0, st, (T*)xbc,        \
+      (const T*)proj, ld, (const T*)ring, (const float*)wconv,               \
+      (const float*)bias, (const int*)pos, (const int*)row,                  \
+      (const int*)tstart, n_tok, C, taps))
+    if (C % 8 == 0 && ld % 8 == 0) GO(true);
+    else GO(false);
+#undef GO
+  } else {
+    HY_DTYPE(dtype, hipLaunchKernelGGL(
+        ssm_conv_kernel<T>, dim3(n_tok, (C + 255) / 256), dim3(256), 0, st,
+        (T*)xbc, (const T*)proj, ld, (const T*)ring, (const float*)wconv,
+        (const float*)bias, (const int*)pos, (const int*)row,
+        (const int*)tstart, C, taps));
+  }
+  HY_CHECK();
+  HY_DTYPE(dtype, hipLaunchKernelGGL(
+      ssm_times_kernel<T>, dim3((n_tok * H + 255) / 256), dim3(256), 0, st,
+      (float*)steps, (const T*)proj, ld, dt_off, (const float*)per_head,
+      n_tok, H));
+  HY_CHECK();
+  return 0;
+}
+
+int hy_ring_store(void* ring, const void* proj, int ld, const void* e_start,
+                  const void* e_len, const void* e_pos, const void* e_row,
+                  int n_entries, int C, int taps, int dtype, void* stream) {
+  if (taps <= 0 || C <= 0) return -2;
+  if (n_entries <= 0) return 0;
+  HY_DTYPE(dtype, hipLaunchKernelGGL(
+      ring_store_kernel<T>, dim3(n_entries, taps < 8 ? taps : 8), dim3(256),
+      0, (hipStream_t)stream, (T*)ring, (const T*)proj, ld,
+      (const int*)e_start, (const int*)e_len, (const int*)e_pos,
+      (const int*)e_row, C, taps));
+  HY_CHECK();
+  return 0;
+}
+
+}  // extern "C"

@@ -1,6 +1,6 @@
 // Row and elementwise kernels of the hybrid models: a residual stream
-// in 32-bit, an RMS norm applied to a sublayer's OUTPUT, the tanh form
-// of gelu and the soft cap of the logits.
+// in 32-bit, RMS norms of a sublayer's OUTPUT or of the stream itself,
+// gated norms of parts of a row, activations, the soft cap of logits.
 #include "common.h"
 
 // x[t] = table[ids[t]] in 32-bit, and a copy in the storage type for the
@@ -93,6 +93,166 @@ __global__ __launch_bounds__(256) void post_norm_add_kernel(
     }
 }
 
+// x += y; h1 = x / rms(x) * w1, h2 = x / rms(x) * w2 in the storage type.
+// y null: nothing is added; w2 (and h2) null: one norm; w1 null: the sum
+// alone.  One workgroup per row, kept in registers between the passes
+// where it fits.
+template <typename T>
+__global__ __launch_bounds__(256) void add_norms_kernel(
+    float* __restrict__ x, const T* __restrict__ y,
+    const float* __restrict__ w1, const float* __restrict__ w2,
+    T* __restrict__ h1, T* __restrict__ h2, int width, float eps) {
+  __shared__ float red[4];
+  const size_t base = (size_t)blockIdx.x * width;
+  const bool vec = (width & 7) == 0;
+  const int nvec = vec ? width >> 3 : 0;
+  float keep[NORM_KEEP][8];
+  float ssq = 0.f;
+  auto sum = [&](int i, float* f) {
+    load8(x + base + i * 8, f);
+    if (y) {
+      float d[8];
+      load8(y + base + i * 8, d);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] += d[j];
+      store8(x + base + i * 8, f);
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ssq += f[j] * f[j];
+  };
+#pragma unroll
+  for (int n = 0; n < NORM_KEEP; ++n) {
+    const int i = threadIdx.x + n * 256;
+    if (i < nvec) sum(i, keep[n]);
+  }
+  for (int i = threadIdx.x + NORM_KEEP * 256; i < nvec; i += 256) {
+    float f[8];
+    sum(i, f);
+  }
+  if (!vec)
+    for (int i = threadIdx.x; i < width; i += 256) {
+      float v = x[base + i];
+      if (y) {
+        v += to_f(y[base + i]);
+        x[base + i] = v;
+      }
+      ssq += v * v;
+    }
+  if (!w1) return;
+  const float r = 1.f / sqrtf(block_sum_256(ssq, red) / width + eps);
+
+  auto emit = [&](int i, const float* f) {
+    float w[8], o[8];
+    load8(w1 + i * 8, w);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = f[j] * r * w[j];
+    store8(h1 + base + i * 8, o);
+    if (!w2) return;
+    load8(w2 + i * 8, w);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = f[j] * r * w[j];
+    store8(h2 + base + i * 8, o);
+  };
+#pragma unroll
+  for (int n = 0; n < NORM_KEEP; ++n) {
+    const int i = threadIdx.x + n * 256;
+    if (i < nvec) emit(i, keep[n]);
+  }
+  // a thread reads back only what it wrote itself
+  for (int i = threadIdx.x + NORM_KEEP * 256; i < nvec; i += 256) {
+    float f[8];
+    load8(x + base + i * 8, f);
+    emit(i, f);
+  }
+  if (!vec)
+    for (int i = threadIdx.x; i < width; i += 256) {
+      const float v = x[base + i] * r;
+      h1[base + i] = from_f<T>(v * w1[i]);
+      if (w2) h2[base + i] = from_f<T>(v * w2[i]);
+    }
+}
+
+// Each of a row's ``groups`` parts of S columns divided by its rms, times
+// w (wl columns, repeated along the row), with silu(gate) applied before
+// the norm or after it.  L lanes a part: 16, a wave, or the workgroup.
+// Up to KEEP vectors a lane stay in registers between the passes.
+template <typename T, int L, bool GATE_FIRST, bool VEC>
+__global__ __launch_bounds__(256) void gated_norm_kernel(
+    T* __restrict__ out, int ld_out, const float* __restrict__ y,
+    const T* __restrict__ gate, int ld, int g_off,
+    const float* __restrict__ w, int wl, int parts, int groups, int S,
+    float eps) {
+  constexpr int N = VEC ? 8 : 1;
+  constexpr int KEEP = L == 256 ? 4 : (VEC ? 1 : 8);
+  __shared__ float red[4];
+  const int part = blockIdx.x * (256 / L) + threadIdx.x / L;
+  if (part >= parts) return;  // whole groups of L lanes
+  const int lane = threadIdx.x % L;
+  const int t = part / groups, g = part % groups;
+  const int c0 = g * S;  // the part's first column
+  const float* src = y + (size_t)t * groups * S + c0;
+  const T* gt = gate + (size_t)t * ld + g_off + c0;
+  auto fetch = [&](int i, float* f) {
+    if (VEC) load8(src + i, f);
+    else f[0] = src[i];
+    if (GATE_FIRST) {
+      float z[N];
+      if (VEC) load8(gt + i, z);
+      else z[0] = to_f(gt[i]);
+#pragma unroll
+      for (int j = 0; j < N; ++j) f[j] *= silu_f(z[j]);
+    }
+  };
+  float keep[KEEP][N], ssq = 0.f;
+#pragma unroll
+  for (int n = 0; n < KEEP; ++n) {
+    const int i = (lane + n * L) * N;
+    if (i < S) {
+      fetch(i, keep[n]);
+#pragma unroll
+      for (int j = 0; j < N; ++j) ssq += keep[n][j] * keep[n][j];
+    }
+  }
+  for (int i = (lane + KEEP * L) * N; i < S; i += L * N) {
+    float f[N];
+    fetch(i, f);
+#pragma unroll
+    for (int j = 0; j < N; ++j) ssq += f[j] * f[j];
+  }
+  ssq = L == 16 ? row16_sum(ssq)
+                : (L == 64 ? wave_sum(ssq) : block_sum_256(ssq, red));
+  const float r = 1.f / sqrtf(ssq / S + eps);
+  T* dst = out + (size_t)t * ld_out + c0;
+  auto emit = [&](int i, float* f) {
+    float wn[N];
+    const int wi = (c0 + i) % wl;
+    if (VEC) load8(w + wi, wn);
+    else wn[0] = w[wi];
+    float z[N];
+    if (!GATE_FIRST) {
+      if (VEC) load8(gt + i, z);
+      else z[0] = to_f(gt[i]);
+    }
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      f[j] *= r * wn[j];
+      if (!GATE_FIRST) f[j] *= silu_f(z[j]);
+    }
+    if (VEC) store8(dst + i, f);
+    else dst[i] = from_f<T>(f[0]);
+  };
+#pragma unroll
+  for (int n = 0; n < KEEP; ++n) {
+    const int i = (lane + n * L) * N;
+    if (i < S) emit(i, keep[n]);
+  }
+  for (int i = (lane + KEEP * L) * N; i < S; i += L * N) {
+    float f[N];
+    fetch(i, f);
+    emit(i, f);
+  }
+}
+
 // out[r] = norm(x[index[r]]) in the storage type (index null: row r).
 template <typename T>
 __global__ __launch_bounds__(256) void norm_rows_kernel(
@@ -157,6 +317,43 @@ __global__ __launch_bounds__(256) void gelu_tanh_kernel(T* __restrict__ y,
     y[i] = from_f<T>(gelu_tanh_f(to_f(y[i])));
 }
 
+// out = g sigmoid(sharpness g) (u + 1) with g = min(gate, limit) and
+// u = clamp(up, -limit, limit); gate and up lie u_off columns apart.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void clamped_swiglu_kernel(
+    T* __restrict__ out, int ld_out, const T* __restrict__ gu, int ld,
+    int u_off, int n_tok, int ff, float limit, float sharpness) {
+  constexpr int N = VEC ? 8 : 1;
+  const int per_row = ff / N;
+  const long long total = (long long)n_tok * per_row;
+  const long long step = (long long)gridDim.x * 256;
+  for (long long id = (long long)blockIdx.x * 256 + threadIdx.x; id < total;
+       id += step) {
+    const int t = (int)(id / per_row);
+    const int i = (int)(id - (long long)t * per_row) * N;
+    const T* src = gu + (size_t)t * ld + i;
+    float g[N], u[N];
+    if (VEC) {
+      load8(src, g);
+      load8(src + u_off, u);
+    } else {
+      g[0] = to_f(src[0]);
+      u[0] = to_f(src[u_off]);
+    }
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      g[j] = fminf(g[j], limit);
+      u[j] = fminf(fmaxf(u[j], -limit), limit);
+      const float e = sizeof(T) == 2 ? __expf(-sharpness * g[j])
+                                     : expf(-sharpness * g[j]);
+      g[j] = g[j] / (1.f + e) * (u[j] + 1.f);
+    }
+    T* dst = out + (size_t)t * ld_out + i;
+    if (VEC) store8(dst, g);
+    else dst[0] = from_f<T>(g[0]);
+  }
+}
+
 // out = cap * tanh(in / cap) in 32-bit (cap <= 0: a plain widening)
 template <typename T>
 __global__ __launch_bounds__(256) void soft_cap_kernel(
@@ -216,6 +413,51 @@ int hy_norm_rows(void* out, const void* x, const void* index, const void* w,
   return 0;
 }
 
+int hy_add_norms(void* x, const void* y, const void* w1, const void* w2,
+                 void* h1, void* h2, int n_tok, int width, float eps,
+                 int dtype, void* stream) {
+  if ((w1 && !h1) || (w2 && (!h2 || !w1))) return -2;
+  if (n_tok <= 0) return 0;
+  HY_DTYPE(dtype, hipLaunchKernelGGL(
+      add_norms_kernel<T>, dim3(n_tok), dim3(256), 0, (hipStream_t)stream,
+      (float*)x, (const T*)y, (const float*)w1, (const float*)w2, (T*)h1,
+      (T*)h2, width, eps));
+  HY_CHECK();
+  return 0;
+}
+
+int hy_gated_norm(void* out, int ld_out, const void* y, const void* gate,
+                  int ld, int g_off, const void* w, int wl, int n_tok,
+                  int groups, int S, int gate_first, float eps, int dtype,
+                  void* stream) {
+  if (groups <= 0 || S <= 0 || wl <= 0 || (groups * S) % wl) return -2;
+  if (n_tok <= 0) return 0;
+  if ((long long)n_tok * groups >= (1ll << 31)) return -2;
+  const int parts = n_tok * groups;
+  const bool vec = S % 8 == 0 && wl % 8 == 0 && ld % 8 == 0 &&
+                   ld_out % 8 == 0 && g_off % 8 == 0;
+#define GO(L, FIRST, VEC)                                                   \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                       \
+      (gated_norm_kernel<T, L, FIRST, VEC>),                                \
+      dim3((parts + 256 / L - 1) / (256 / L)), dim3(256), 0,                \
+      (hipStream_t)stream, (T*)out, ld_out, (const float*)y,                \
+      (const T*)gate, ld, g_off, (const float*)w, wl, parts, groups, S, eps))
+#define PICK(L)                                \
+  do {                                         \
+    if (gate_first && vec) GO(L, true, true);  \
+    else if (gate_first) GO(L, true, false);   \
+    else if (vec) GO(L, false, true);          \
+    else GO(L, false, false);                  \
+  } while (0)
+  if (S <= 128) PICK(16);
+  else if (S <= 512) PICK(64);
+  else PICK(256);
+#undef PICK
+#undef GO
+  HY_CHECK();
+  return 0;
+}
+
 static int grid_for(long long items) {
   long long g = (items + 255) / 256;
   return (int)(g < 1 ? 1 : (g > 8192 ? 8192 : g));
@@ -226,6 +468,26 @@ int hy_gelu_tanh(void* y, long long n, int dtype, void* stream) {
   HY_DTYPE(dtype, hipLaunchKernelGGL(
       gelu_tanh_kernel<T>, dim3(grid_for((n + 7) / 8)), dim3(256), 0,
       (hipStream_t)stream, (T*)y, n));
+  HY_CHECK();
+  return 0;
+}
+
+int hy_clamped_swiglu(void* out, int ld_out, const void* gu, int ld,
+                      int u_off, int n_tok, int ff, float limit,
+                      float sharpness, int dtype, void* stream) {
+  if (n_tok <= 0 || ff <= 0) return 0;
+  const bool vec =
+      ff % 8 == 0 && ld % 8 == 0 && ld_out % 8 == 0 && u_off % 8 == 0 &&
+      ((uintptr_t)out & (dtype == 0 ? 15 : 31)) == 0;
+  const int grid = grid_for((long long)n_tok * ff / (vec ? 8 : 1));
+#define GO(VEC)                                                            \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                      \
+      (clamped_swiglu_kernel<T, VEC>), dim3(grid), dim3(256), 0,           \
+      (hipStream_t)stream, (T*)out, ld_out, (const T*)gu, ld, u_off, n_tok, \
+      ff, limit, sharpness))
+  if (vec) GO(true);
+  else GO(false);
+#undef GO
   HY_CHECK();
   return 0;
 }

@@ -344,6 +344,7 @@ def pair_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
     assert proj.stride(1) == 1 and out.stride(1) == 1
     lib, bt, st = native(), b.block_tables, _stream()
     H, G, D, V = heads, kv_heads, dim, vdim
+    assert cache.shape[0] * G * 16 < 2 ** 31    # rows are 32-bit numbers
     dst = (_ptr(out), _i(out.stride(0)))
     src = (_ptr(proj), _i(proj.stride(0)), _i(g_off), _ptr(cache))
     sizes = (_i(H), _i(G), _i(D), _i(V))
