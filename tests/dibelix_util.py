@@ -1,20 +1,15 @@
-"""Small random Dibelix models and the runs that tests share.
+"""Small random Dibelix models and mixers for tests.
 
 Configurations are plain dictionaries in the layout of config.json, so
 that the oracle and the served model read the same thing.
 """
 from __future__ import annotations
 
-import json
-
 import torch
-from safetensors.torch import save_file
 
-from llmlb_amd.backend.engine import Engine, EngineConfig
-from llmlb_amd.backend.kv_cache import HybridCache
-from llmlb_amd.backend.ragged import RaggedBatch
-from llmlb_amd.models.dibelix import DibelixConfig
 from llmlb_amd.models.mixers import ChannelDelta, LatentAttention
+from packed_util import (MixerRun, engine, error, run_cuts,  # noqa: F401
+                         serve_at_random, tokens, write_model)
 
 
 def latent(heads, dim, rot, vdim, rank, window, base=1e4, scale=None,
@@ -112,48 +107,6 @@ def weights(cfg, seed=0, dtype=torch.bfloat16):
     return out
 
 
-def write_model(folder, cfg, w):
-    folder.mkdir(parents=True, exist_ok=True)
-    (folder / "config.json").write_text(json.dumps(cfg))
-    save_file(w, str(folder / "model.safetensors"))
-    return folder
-
-
-def engine(folder, device="cpu", dtype="float32", blocks=64, rows=6,
-           max_pos=1024, **kw):
-    cfg = DibelixConfig.from_dir(folder)
-    cfg.max_pos = max_pos
-    return Engine(EngineConfig(model=cfg, device=device, dtype=dtype,
-                               kv_cache_blocks=blocks, max_batch=rows,
-                               weights_path=str(folder), **kw))
-
-
-def tokens(n, vocab, seed):
-    g = torch.Generator().manual_seed(seed)
-    return torch.randint(0, vocab, (n,), generator=g).tolist()
-
-
-def run_cuts(eng, toks, cuts, close=True):
-    """All logits of one sequence fed in portions ending at ``cuts``."""
-    seq = eng.open_sequence()
-    out, at = [], 0
-    for c in list(cuts) + [len(toks)]:
-        if c > at:
-            out.append(eng.run_batch(
-                [(seq, toks[at:c], list(range(c - at)))]).cpu().double())
-            at = c
-    if close:
-        eng.close_sequence(seq)
-    return torch.cat(out)
-
-
-def error(got, want):
-    """Largest over positions of the rms logit error, relative to the
-    spread of the logits."""
-    d = got.cpu().double() - want
-    return (d.pow(2).mean(-1).sqrt().max() / want.std()).item()
-
-
 # -- one mixer alone -------------------------------------------------------
 
 def latent_mixer(m, w, eps, width, device="cpu", dtype=torch.float32,
@@ -178,47 +131,6 @@ def delta_mixer(m, w, eps, width, device="cpu", dtype=torch.float32):
         dtype=dtype, device=torch.device(device))
     mix.load({k: w[k] for k in mix.weight_shapes()})
     return mix
-
-
-class MixerRun:
-    """A mixer with a cache of its own; ``rows`` sequences, pages in a
-    shuffled order.  ``step([(row, inputs)])`` runs one packed batch."""
-
-    def __init__(self, mix, rows, max_tokens, seed=0):
-        nb = -(-max_tokens // 16)
-        g = torch.Generator().manual_seed(seed)
-        self.mix, self.dev = mix, mix.device
-        spec = mix.cache_spec()
-        self.cache = HybridCache([spec], 1 + rows * nb, rows, self.dev,
-                                 mix.dtype)
-        self.bt = (torch.randperm(rows * nb, generator=g) + 1).to(
-            torch.int32).view(rows, nb).to(self.dev)
-        self.at = [0] * rows
-
-    def step(self, work):
-        order = sorted(range(len(work)), key=lambda i: len(work[i][1]))
-        work = [work[i] for i in order]
-        runs = [(r, self.at[r], [0] * len(h)) for r, h in work]
-        b = RaggedBatch.build(runs, self.bt)
-        x = torch.cat([h for _, h in work]).to(self.mix.dtype).to(self.dev)
-        y = self.mix(x, b, self.cache, 0).double().cpu()
-        out = dict(zip((r for r, _ in work),
-                       torch.split(y, [len(h) for _, h in work])))
-        for r, h in work:
-            self.at[r] += len(h)
-        return out
-
-    def cuts(self, row, h, cuts):
-        """One sequence in portions ending at ``cuts``."""
-        out, at = [], 0
-        for c in list(cuts) + [len(h)]:
-            if c > at:
-                out.append(self.step([(row, h[at:c])])[row])
-                at = c
-        return torch.cat(out)
-
-    def restart(self, row):
-        self.at[row] = 0
 
 
 def planted_attention(m, width, T, pairs, seed=0, strength=9.0):

@@ -65,38 +65,14 @@ def test_unequal_batch_and_reuse(model):
     pages and slots of finished ones serve new ones."""
     cfg, w, folder = model
     eng = U.engine(folder, blocks=12, rows=3)
-    g = torch.Generator().manual_seed(7)
     reqs = [U.tokens(n, cfg["vocab"], 30 + n)
             for n in (1, 40, 2, 23, 50, 17, 33)]
     want = [O.forward(t, w, cfg) for t in reqs]
     free = eng.kv.free_blocks()
-    waiting, live = list(range(len(reqs))), {}
-    got = {i: [] for i in waiting}
-    while waiting or live:
-        while waiting and len(live) < 3:
-            i = waiting.pop(0)
-            live[i] = (eng.open_sequence(), 0)
-        work, who = [], []
-        for i, (seq, at) in live.items():
-            if torch.rand((), generator=g) < 0.25 and len(live) > 1:
-                continue
-            n = (1, 2, 5, 16, 19)[int(torch.randint(5, (), generator=g))]
-            part = reqs[i][at:at + n]
-            work.append((seq, part, list(range(len(part)))))
-            who.append((i, len(part)))
-        if not work:
-            continue
-        rows = eng.run_batch(work).split([n for _, n in who])
-        for (i, n), r in zip(who, rows):
-            got[i].append(r.double())
-            seq, at = live[i]
-            live[i] = (seq, at + n)
-            if at + n == len(reqs[i]):
-                eng.close_sequence(seq)
-                del live[i]
+    got = U.serve_at_random(eng, reqs, 3, (1, 2, 5, 16, 19))
     assert eng.kv.free_blocks() == free
     for i, rows in got.items():
-        assert U.error(torch.cat(rows), want[i]) < TOL, i
+        assert U.error(rows, want[i]) < TOL, i
 
 
 def greedy_oracle(w, cfg, prompt, n):

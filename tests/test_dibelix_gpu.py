@@ -59,39 +59,14 @@ def test_unequal_batches_alone_and_together(model, dtype):
     slots are those of the request alone."""
     cfg, w, folder = model
     eng = U.engine(folder, DEV, dtype, blocks=22, rows=4)
-    g = torch.Generator().manual_seed(7)
     reqs = [U.tokens(n, cfg["vocab"], 30 + n)
             for n in (1, 70, 2, 23, 80, 17, 66, 40)]
     want = [O.forward(t, w, cfg) for t in reqs]
     free = eng.kv.free_blocks()
-    waiting, live = list(range(len(reqs))), {}
-    got = {i: [] for i in waiting}
-    while waiting or live:
-        while waiting and len(live) < 4:
-            i = waiting.pop(0)
-            live[i] = (eng.open_sequence(), 0)
-        work, who = [], []
-        for i, (seq, at) in live.items():
-            if torch.rand((), generator=g) < 0.2:
-                continue
-            n = (1, 1, 2, 5, 16, 19, 33)[int(torch.randint(
-                7, (), generator=g))]
-            part = reqs[i][at:at + n]
-            work.append((seq, part, list(range(len(part)))))
-            who.append((i, len(part)))
-        if not work:
-            continue
-        rows = eng.run_batch(work).split([n for _, n in who])
-        for (i, n), r in zip(who, rows):
-            got[i].append(r.double().cpu())
-            seq, at = live[i]
-            live[i] = (seq, at + n)
-            if at + n == len(reqs[i]):
-                eng.close_sequence(seq)
-                del live[i]
+    got = U.serve_at_random(eng, reqs, 4, (1, 1, 2, 5, 16, 19, 33))
     assert eng.kv.free_blocks() == free
     for i, rows in got.items():
-        assert U.error(torch.cat(rows), want[i]) < LOGIT_TOL[dtype], i
+        assert U.error(rows, want[i]) < LOGIT_TOL[dtype], i
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])

@@ -1,0 +1,352 @@
+"""Taletar on the GPU: every kernel of its path, in bfloat16 and
+float32, against the plain implementation of taletar_oracle."""
+import pytest
+import torch
+
+import taletar_oracle as O
+import taletar_util as U
+from llmlb_amd.backend.sampler import SamplingParams
+from llmlb_amd.ops import hybrid as hy
+from test_taletar_cpu import greedy_oracle
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+F32, B16 = torch.float32, torch.bfloat16
+DTYPES = pytest.mark.parametrize("dtype", [B16, F32], ids=["bf16", "f32"])
+NAMES = pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+# rms logit error over the logits' spread
+LOGIT_TOL = {"float32": 1e-4, "bfloat16": 0.1}
+
+
+@pytest.fixture(scope="module", params=["ODD", "TILED", "PLAIN"])
+def model(request, tmp_path_factory):
+    cfg = getattr(U, request.param)
+    w = U.weights(cfg, seed=len(request.param))
+    return cfg, w, U.write_model(tmp_path_factory.mktemp(request.param),
+                                 cfg, w)
+
+
+@pytest.fixture(scope="module")
+def plain(tmp_path_factory):
+    cfg = U.PLAIN
+    w = U.weights(cfg, seed=3)
+    return cfg, w, U.write_model(tmp_path_factory.mktemp("plain"), cfg, w)
+
+
+def close(got, want, dtype, rel=None):
+    """Largest difference over the largest value."""
+    rel = rel or (2e-2 if dtype == B16 else 2e-5)
+    err = (got.double().cpu() - want).abs().max() / want.abs().max()
+    assert err < rel, float(err)
+
+
+# -- whole models ----------------------------------------------------------
+
+@NAMES
+def test_prompt_portions_and_decoding(model, dtype):
+    cfg, w, folder = model
+    toks = U.tokens(150, cfg["vocab"], 1)
+    want = O.forward(toks, w, cfg)
+    eng = U.engine(folder, DEV, dtype)
+    for cuts in ([], range(1, 150), range(2, 150, 2), range(9, 150, 9),
+                 range(64, 150, 17), [140] + list(range(141, 150))):
+        err = U.error(U.run_cuts(eng, toks, cuts), want)
+        assert err < LOGIT_TOL[dtype], (cuts, err)
+    assert eng._graphs and eng.use_graphs, "decode steps were not captured"
+
+
+@NAMES
+def test_unequal_batches_alone_and_together(model, dtype):
+    """Every request's logits in mixed batches with reused pages and
+    slots are those of the request alone."""
+    cfg, w, folder = model
+    eng = U.engine(folder, DEV, dtype, blocks=22, rows=4)
+    reqs = [U.tokens(n, cfg["vocab"], 30 + n)
+            for n in (1, 70, 2, 23, 80, 17, 66, 40)]
+    want = [O.forward(t, w, cfg) for t in reqs]
+    free = eng.kv.free_blocks()
+    got = U.serve_at_random(eng, reqs, 4, (1, 1, 2, 5, 16, 19, 33))
+    assert eng.kv.free_blocks() == free
+    for i, rows in got.items():
+        assert U.error(rows, want[i]) < LOGIT_TOL[dtype], i
+
+
+@NAMES
+def test_long_decoding(plain, dtype):
+    cfg, w, folder = plain
+    toks = U.tokens(400, cfg["vocab"], 8)
+    want = O.forward(toks, w, cfg)
+    eng = U.engine(folder, DEV, dtype)
+    got = U.run_cuts(eng, toks, range(3, 400))
+    assert U.error(got, want) < LOGIT_TOL[dtype]
+
+
+def test_captured_steps_match_eager_steps(model):
+    """Replays with other work and synchronizations between them; batch
+    sizes that pad their bucket."""
+    cfg, _, folder = model
+    engines = [U.engine(folder, DEV, "bfloat16", rows=6) for _ in range(2)]
+    engines[1].use_graphs = False
+    seqs = [[e.open_sequence() for _ in range(5)] for e in engines]
+    for e, ss in zip(engines, seqs):
+        for n, s in enumerate(ss):
+            e.run_batch([(s, U.tokens(7 * n + 3, cfg["vocab"], n), [])])
+    for step in range(8):
+        live = range(step % 2, 5 - step % 3)
+        res = []
+        for e, ss in zip(engines, seqs):
+            res.append(e.run_batch(
+                [(ss[i], U.tokens(1, cfg["vocab"], 50 * step + i), [0])
+                 for i in live]).clone())
+            e.run_batch([(ss[4], [step, step + 1], [])])
+            torch.cuda.synchronize()
+        d = (res[0] - res[1]).abs().max() / res[1].std()
+        assert d < 0.05, (step, float(d))
+    assert engines[0]._graphs and not engines[1]._graphs
+
+
+def test_greedy_generation(plain):
+    cfg, w, folder = plain
+    eng = U.engine(folder, DEV, "float32", blocks=40, rows=3,
+                   prefill_step_budget=24)
+    prompts = [U.tokens(n, cfg["vocab"], n) for n in (5, 60, 1, 31)]
+    want = [greedy_oracle(w, cfg, p, 6) for p in prompts]
+    queues = [eng.submit(p, SamplingParams(max_new_tokens=6))[1]
+              for p in prompts]
+    for _ in range(200):
+        if not eng.step():
+            break
+    for q, expect in zip(queues, want):
+        assert [q.get_nowait()[0] for _ in range(q.qsize())] == expect
+    assert eng.kv.free_blocks() == eng.kv.num_blocks - 1
+
+
+def test_preset_and_embeddings():
+    from llmlb_amd.backend.launcher import build_engine
+    eng = build_engine("taletar-tiny", DEV, kv_blocks=64, max_batch=4)
+    assert len(eng.generate_sync(list(range(40)), 5).token_ids) == 5
+    h = eng.model.forward_dense(torch.tensor([[1, 2, 3]] * 2, device=DEV))
+    assert torch.equal(h[0], h[1]) and h.isfinite().all()
+
+
+# -- differential attention alone ------------------------------------------
+
+# heads, kv_heads, dim, vdim, softcap: every tile shape with and without a
+# remainder and each way of capping; more than 16 heads to a key/value
+# head; sizes only the general kernel takes
+ATTENTION = [
+    (2, 1, 32, 64, 30.0), (3, 3, 24, 128, 60.0), (2, 2, 16, 256, 20.0),
+    (8, 2, 64, 64, None), (4, 1, 40, 96, 50.0), (2, 1, 64, 200, 61.0),
+    (2, 2, 128, 40, 15.0), (2, 1, 96, 128, None), (1, 1, 104, 256, 45.0),
+    (8, 8, 8, 8, 25.0), (17, 1, 16, 24, 30.0), (40, 2, 8, 40, 70.0),
+    (2, 1, 64, 256, 80.0), (3, 1, 120, 72, 100.0), (2, 1, 32, 136, None),
+    (6, 2, 7, 9, 12.0), (2, 1, 136, 16, None), (2, 2, 24, 300, 30.0),
+    (1, 1, 20, 600, 30.0), (4, 2, 12, 20, 40.0),
+]
+
+
+@pytest.mark.parametrize("sizes", ATTENTION, ids=str)
+@DTYPES
+def test_attention_planted(sizes, dtype):
+    """Scores that stand out at the first tokens, at page and tile
+    borders, just before and just after the query; whole, in portions,
+    and decoded."""
+    ly = U.attention(*sizes, q_temp=(0.3, 50))
+    T, width = 210, U.planted_width(ly["mixer"])
+    oracle, m, w = U.case(ly, width, sum(sizes[:4]))
+    h = U.plant(m, w, U.inputs(T, width, 3), U.far_triples(T))
+    want = oracle(h, w, "", m, 1e-5)
+    run = U.MixerRun(U.mixer("attention", m, w, 1e-5, width, DEV, dtype),
+                     2, T)
+    for cuts in ([], [130, 132, 135] + list(range(136, T)),
+                 list(range(9, T, 9)), [64, 128, 129, 192]):
+        run.restart(1)
+        close(run.cuts(1, h, cuts), want, dtype,
+              rel=5e-2 if dtype == B16 else 5e-5)
+
+
+@pytest.mark.parametrize("parts", [1, 2, 3, 8, 32])
+@pytest.mark.parametrize("heads", [(7, 1, 30.0), (42, 2, None)], ids=str)
+def test_decode_parts(parts, heads, monkeypatch):
+    monkeypatch.setattr(hy, "pair_parts", lambda *a: parts)
+    ly = U.attention(heads[0], heads[1], 16, 24, heads[2])
+    width = 96
+    lens = (1, 2, 16, 17, 64, 65, 128, 200)
+    oracle, m, w = U.case(ly, width, heads[0])
+    run = U.MixerRun(U.mixer("attention", m, w, 1e-5, width, DEV, B16),
+                     len(lens), 208)
+    hs = [U.inputs(n, width, n) for n in lens]
+    run.step([(i, h[:-1]) for i, h in enumerate(hs) if len(h) > 1])
+    got = run.step([(i, h[-1:]) for i, h in enumerate(hs)])
+    for i, h in enumerate(hs):
+        close(got[i][0], oracle(h, w, "", m, 1e-5)[-1], B16, 3e-2)
+
+
+def test_pages_of_others_do_not_matter():
+    """What earlier sequences left in a page's unused places, even
+    numbers that are none, changes nothing."""
+    for dtype in (B16, F32):
+        oracle, m, w = U.case(U.attention(4, 2, 16, 24), 64, 5)
+        run = U.MixerRun(U.mixer("attention", m, w, 1e-5, 64, DEV, dtype),
+                         1, 112)
+        for pages in run.cache.pages.values():
+            pages.fill_(float("nan"))
+        h = U.inputs(101, 64, 2)
+        for cuts in ([], [70, 71, 72], range(1, 101)):
+            run.restart(0)
+            close(run.cuts(0, h, cuts), oracle(h, w, "", m, 1e-5), dtype,
+                  3e-2 if dtype == B16 else 5e-5)
+
+
+# -- linear recurrences alone ----------------------------------------------
+
+# rows per lane 1..32 with and without a remainder; tau 1; every
+# convolution length, grouped heads, parts of every size for the norm
+RECURRENT = [U.gla(2, 16, 16), U.gla(4, 11, 7, tau=1.0, low=3),
+             U.gla(3, 32, 48), U.gla(8, 64, 96, tau=16.0, low=40),
+             U.gla(4, 50, 40), U.gla(2, 128, 128), U.gla(3, 100, 36),
+             U.gla(2, 256, 24), U.gla(2, 200, 50), U.gla(1, 512, 16),
+             U.gla(1, 300, 600),
+             U.mamba2(2, 16, 16), U.mamba2(6, 7, 11, 2, 3, 3),
+             U.mamba2(4, 48, 30, 4, 2, 2), U.mamba2(8, 64, 64, 2, 1, 4),
+             U.mamba2(8, 96, 50, 1, 6, 1), U.mamba2(4, 32, 128, 2, 4, 4),
+             U.mamba2(2, 36, 100, 1, 3, 1), U.mamba2(2, 24, 256, 1, 4, 1),
+             U.mamba2(3, 50, 200, 3, 2, 1), U.mamba2(1, 16, 512, 1, 5, 2)]
+
+
+@pytest.mark.parametrize("ly", RECURRENT, ids=str)
+@DTYPES
+def test_recurrent_mixer(ly, dtype):
+    width, T = 48, 75
+    oracle, m, w = U.case(ly, width, sum(map(ord, str(ly))) % 1000)
+    h = U.inputs(T, width, 2)
+    want = oracle(h, w, "", m, 1e-4)
+    run = U.MixerRun(U.mixer(ly["type"], m, w, 1e-4, width, DEV, dtype),
+                     2, T)
+    for cuts in ([], range(1, T), range(2, T, 2),
+                 [30, 33, 34, 35, 36, 60, 62]):
+        run.restart(1)
+        close(run.cuts(1, h, cuts), want, dtype,
+              rel=3e-2 if dtype == B16 else 5e-5)
+
+
+@pytest.mark.parametrize("rows", [3, 9, 33])
+@pytest.mark.parametrize("ly", [U.gla(8, 64, 128), U.gla(8, 128, 64),
+                                U.mamba2(8, 64, 128, 2),
+                                U.mamba2(16, 96, 40, 4)], ids=str)
+def test_recurrent_mixer_full_chip(ly, rows):
+    """Enough sequences for the scan's wide lanes; unequal lengths,
+    portions beside single tokens."""
+    width = 40
+    oracle, m, w = U.case(ly, width, rows)
+    hs = [U.inputs(5 + 2 * (i % 12), width, i) for i in range(rows)]
+    run = U.MixerRun(U.mixer(ly["type"], m, w, 1e-5, width, DEV, F32),
+                     rows, 48)
+    first = run.step([(i, h[:-3 - i % 2]) for i, h in enumerate(hs)])
+    second = run.step([(i, h[-3 - i % 2:-1] if i % 3 else
+                        h[-3 - i % 2:-2 - i % 2])
+                       for i, h in enumerate(hs)])
+    for i, h in enumerate(hs):
+        got = torch.cat([first[i], second[i]])
+        close(got, oracle(h, w, "", m, 1e-5)[:len(got)], F32)
+
+
+@pytest.mark.parametrize("ly", [U.gla(4, 32, 32), U.mamba2(4, 24, 32, 2)],
+                         ids=str)
+def test_slots_start_empty(ly):
+    """A slot's next sequence sees nothing of the last one, also when it
+    is shorter than the convolution."""
+    width = 40
+    oracle, m, w = U.case(ly, width, 1)
+    run = U.MixerRun(U.mixer(ly["type"], m, w, 1e-5, width, DEV, F32), 1, 64)
+    for n in (30, 2, 1, 3, 17):
+        h = U.inputs(n, width, n)
+        for cuts in ([], range(1, n)):
+            run.restart(0)
+            close(run.cuts(0, h, cuts), oracle(h, w, "", m, 1e-5), F32)
+
+
+# -- rows ------------------------------------------------------------------
+
+@pytest.mark.parametrize("width", [52, 256, 2048, 8200, 16384])
+@DTYPES
+def test_add_norms(width, dtype):
+    g = torch.Generator().manual_seed(width)
+    x = 3 * torch.randn(33, width, generator=g)
+    y = torch.randn(33, width, generator=g).to(dtype)
+    w1, w2 = (1 + 0.3 * torch.randn(width, generator=g) for _ in range(2))
+    tol = 1e-2 if dtype == B16 else 1e-6
+    for eps in (1e-5, 0.5):
+        for add, second in ((y, w2), (None, w2), (y, None)):
+            dev = x.to(DEV)
+            total = x.double() + (0 if add is None else add.double())
+            h1, h2 = hy.add_norms(
+                dev, None if add is None else add.to(DEV), w1.to(DEV),
+                None if second is None else second.to(DEV), eps, dtype)
+            close(dev, total, F32, 1e-6)
+            close(h1, O.rms(total, eps) * w1, dtype, tol)
+            if second is None:
+                assert h2 is None
+            else:
+                close(h2, O.rms(total, eps) * w2, dtype, tol)
+    dev = x.to(DEV)
+    assert hy.add_norms(dev, y.to(DEV), None, None, 1e-5, dtype) \
+        == (None, None)
+    close(dev, x.double() + y.double(), F32, 1e-6)
+
+
+# groups, columns of a group, repeated weight
+PARTS = [(5, 7, True), (3, 128, True), (16, 24, True), (4, 129, False),
+         (2, 512, True), (3, 333, False), (2, 520, False), (1, 8200, False),
+         (1, 12001, False), (2, 4096, True)]
+
+
+@pytest.mark.parametrize("parts", PARTS, ids=str)
+@DTYPES
+def test_gated_norm(parts, dtype):
+    groups, size, shared = parts
+    W = groups * size
+    g = torch.Generator().manual_seed(W)
+    y = torch.randn(9, W, generator=g)
+    gate = torch.randn(9, W + 16, generator=g).to(dtype)
+    w = 1 + 0.3 * torch.randn(size if shared else W, generator=g)
+    full = w.repeat(W // w.numel()).double()
+    z = O.silu(gate[:, 8:8 + W].double())
+    for first in (True, False):
+        n = (y.double() * z if first else y.double()).view(9, groups, size)
+        want = O.rms(n, 1e-2).reshape(9, W) * full
+        want = want if first else want * z
+        out = torch.full((9, W + 8), 7.0, dtype=dtype, device=DEV)
+        hy._gated_norm(out[:, :W], y.to(DEV), gate.to(DEV), 8, w.to(DEV),
+                       groups, first, 1e-2)
+        close(out[:, :W], want, dtype, 1e-2 if dtype == B16 else 1e-6)
+        assert (out[:, W:] == 7.0).all()
+
+
+@pytest.mark.parametrize("ff", [8, 70, 416, 5000])
+@DTYPES
+def test_clamped_swiglu(ff, dtype):
+    g = torch.Generator().manual_seed(ff)
+    off = ff + -ff % 8
+    gu = (3 * torch.randn(21, off + ff, generator=g)).to(dtype)
+    gu[0, :2] = 200.0
+    gu[0, 2:4] = -200.0
+    for limit, sharp in ((1.0, 1.702), (7.0, 1.0)):
+        a = gu[:, :ff].double().clamp(max=limit)
+        u = gu[:, off:].double().clamp(-limit, limit)
+        want = a * O.sigmoid(sharp * a) * (u + 1)
+        out = torch.full((21, ff + 5), 7.0, dtype=dtype, device=DEV)
+        hy.clamped_swiglu(out[:, 5:], gu.to(DEV), off, limit, sharp)
+        close(out[:, 5:], want, dtype, 1e-2 if dtype == B16 else 1e-6)
+        assert (out[:, :5] == 7.0).all()
+
+
+def test_sizes_out_of_bounds_are_refused():
+    """The host checks sizes before a kernel is launched."""
+    ly = U.gla(1, 513, 8)
+    _, m, w = U.case(ly, 24, 1)
+    run = U.MixerRun(U.mixer("gla", m, w, 1e-5, 24, DEV, F32), 1, 32)
+    with pytest.raises(RuntimeError):
+        run.step([(0, U.inputs(3, 24, 1))])
+    with pytest.raises(RuntimeError):
+        run.step([(0, U.inputs(1, 24, 1))])
