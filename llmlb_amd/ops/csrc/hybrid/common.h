@@ -6,6 +6,7 @@
 #include <hip/hip_runtime.h>
 #include <math.h>
 #include <stdint.h>
+#include <type_traits>
 
 #define WAVE 64
 #define PAGE 16  // tokens per cache page
@@ -105,6 +106,29 @@ __device__ __forceinline__ float row16_sum(float v) {
   v = dpp_add<0x141>(v);  // row_half_mirror
   v = dpp_add<0x140>(v);  // row_mirror
   return v;
+}
+
+__device__ __forceinline__ float row8_sum(float v) {  // of 8 lanes
+  v = dpp_add<0xB1>(v);
+  v = dpp_add<0x4E>(v);
+  return dpp_add<0x141>(v);
+}
+// Four sums over 16 lanes at once: lane l gets the one of v[l % 4].
+__device__ __forceinline__ float row16_sum4(const float* v) {
+  const bool odd = threadIdx.x & 1, high = threadIdx.x & 2;
+  float a = odd ? v[1] : v[0], b = odd ? v[3] : v[2];
+  const float a2 = odd ? v[0] : v[1], b2 = odd ? v[2] : v[3];
+  auto from = [](float x, auto ctrl) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(
+        0, __float_as_int(x), decltype(ctrl)::value, 0xf, 0xf, true));
+  };
+  a += from(a2, std::integral_constant<int, 0xB1>());  // lane ^ 1
+  b += from(b2, std::integral_constant<int, 0xB1>());
+  float c = high ? b : a;
+  const float c2 = high ? a : b;
+  c += from(c2, std::integral_constant<int, 0x4E>());  // lane ^ 2
+  c = dpp_add<0x124>(c);                               // row_ror:4
+  return dpp_add<0x128>(c);                            // row_ror:8
 }
 
 __device__ __forceinline__ float sigmoid_f(float x) {

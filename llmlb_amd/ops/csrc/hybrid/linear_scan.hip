@@ -26,6 +26,7 @@ struct Run<float, N, VEC> {
   __device__ __forceinline__ void load(const float* p, int valid) {
     load_some<N, VEC>(p, valid, f);
   }
+  __device__ __forceinline__ void set(int i, float x) { f[i] = x; }
   __device__ __forceinline__ float get(int i) const { return f[i]; }
 };
 template <int N>
@@ -35,6 +36,7 @@ struct Run<bf16_t, N, false> {
 #pragma unroll
     for (int i = 0; i < N; ++i) u[i] = i < valid ? p[i].u : 0;
   }
+  __device__ __forceinline__ void set(int i, bf16_t x) { u[i] = x.u; }
   __device__ __forceinline__ float get(int i) const {
     return __uint_as_float((unsigned)u[i] << 16);
   }
@@ -65,14 +67,16 @@ struct Run<bf16_t, N, true> {
 };
 
 // One wave = 4 CPL value columns of one head of one sequence: 16 lanes a
-// column, RPL key channels and CPL columns a lane.  The operands of the
+// column, RPL key channels and CPL columns a lane.  The waves of a
+// workgroup take neighbouring columns, so that a CU's cache serves them
+// the same rows and its SIMDs get the same number of waves.  The operands of the
 // next PF tokens are in flight while a token is worked on.  Nothing but
 // the state itself carries over from token to token; the sum over lanes
 // that makes an output is off that chain.
 //   q, k: columns q_off, k_off + group * D; v: v_off + head * V, of rows of
-//   ``in``;  g [T][H D] (CHANNEL) or [T][H];  dt [T][H], skip [H] or null
+//   ``in``;  g [T][H D] (CHANNEL) or [T][H];  dt [T][H] and skip [H] without CHANNEL
 template <typename T, int RPL, bool VEC, int CPL, bool CHANNEL>
-__global__ __launch_bounds__(64) void linear_scan_kernel(
+__global__ __launch_bounds__(256) void linear_scan_kernel(
     float* __restrict__ o, float* __restrict__ state,
     const T* __restrict__ in, int ld, int q_off, int k_off, int v_off,
     const float* __restrict__ g_, const float* __restrict__ dt_,
@@ -80,9 +84,11 @@ __global__ __launch_bounds__(64) void linear_scan_kernel(
     const int* __restrict__ e_len, const int* __restrict__ e_pos,
     const int* __restrict__ e_row, int G, int H, int D, int V,
     float q_scale) {
-  constexpr int PF = RPL <= 8 ? 4 : (RPL == 16 ? 2 : 1);
+  constexpr int PF = RPL <= 4 ? 32 / (CPL < 2 ? 2 : CPL)
+                              : (RPL == 8 ? 4 : (RPL == 16 ? 2 : 1));
   const int e = blockIdx.y;
-  const int nb = (V + 4 * CPL - 1) / (4 * CPL);
+  const int waves = blockDim.x / WAVE;
+  const int nb = (V + 4 * CPL - 1) / (4 * CPL) / waves;  // whole workgroups
   int head, cb;
   if (H % 8 == 0) {  // all columns of a head on one XCD: its L2 serves them
     const int x = blockIdx.x & 7, r = blockIdx.x >> 3;
@@ -92,7 +98,8 @@ __global__ __launch_bounds__(64) void linear_scan_kernel(
     head = blockIdx.x / nb;
     cb = blockIdx.x % nb;
   }
-  const int lane = threadIdx.x;
+  const int lane = threadIdx.x & (WAVE - 1);
+  cb = cb * waves + threadIdx.x / WAVE;
   const int col = (cb * 4 + lane / 16) * CPL;  // the lane's first column
   const int r0 = (lane & 15) * RPL;
   const int valid = D - r0 < RPL ? (D - r0 > 0 ? D - r0 : 0) : RPL;
@@ -100,18 +107,30 @@ __global__ __launch_bounds__(64) void linear_scan_kernel(
   const int group = head / (H / G);
   const int len = e_len[e];
   const size_t first = (size_t)e_start[e];
-  const T* qp = in + first * ld + q_off + group * D + rr;
-  const T* kp = in + first * ld + k_off + group * D + rr;
-  const T* vp = in + first * ld + v_off + head * V;
-  const float* gp = g_ + (CHANNEL ? first * H * D + (size_t)head * D + rr
-                                  : first * H + head);
-  const float* dp = dt_ ? dt_ + first * H + head : nullptr;
-  const float skip = skip_ ? skip_[head] : 0.f;
+  // a token's rows are the same for the wave, a lane's place in them is
+  // a 32-bit offset
+  const T* rows = in + first * ld;
+  const float* g_rows = g_ + first * H * (CHANNEL ? D : 1);
+  const float* dt_rows = CHANNEL ? nullptr : dt_ + first * H;
+  const unsigned q_at = (q_off + group * D + rr) * sizeof(T);
+  const unsigned k_at = (k_off + group * D + rr) * sizeof(T);
+  const unsigned v_at = (v_off + head * V) * sizeof(T);
+  const unsigned g_at = (head * D + rr) * sizeof(float);
+  // kept in a vector register: scalar loads return out of order, so that
+  // waiting for one token's would wait for the next ones' as well
+  unsigned head_at = head * sizeof(float);
+  asm("" : "+v"(head_at));
+  auto place = [](const auto* p, unsigned bytes) {
+    return reinterpret_cast<decltype(p)>(
+        reinterpret_cast<const char*>(p) + bytes);
+  };
+  const float skip = CHANNEL ? 0.f : skip_[head];
   float* out = o + (first * H + head) * V;
   float* sp = state + ((size_t)e_row[e] * H + head) * V * D;
   int cc[CPL];
 #pragma unroll
-  for (int c = 0; c < CPL; ++c) cc[c] = col + c < V ? col + c : V - 1;
+  for (int c = 0; c < CPL; ++c)
+    cc[c] = VEC || col + c < V ? col + c : V - 1;
 
   float S[CPL][RPL];
   const bool resume = e_pos[e] > 0;
@@ -124,18 +143,27 @@ __global__ __launch_bounds__(64) void linear_scan_kernel(
 
   constexpr int GN = CHANNEL ? RPL : 1;
   Run<T, RPL, VEC> q[PF], k[PF];
+  Run<T, CPL, VEC> v[PF];
   float g[PF][GN], dt[PF];
-  T v[PF][CPL];
   auto fetch = [&](int s, int t) {
     t = t < len ? t : len - 1;
-    const size_t at = (size_t)t * ld;
-    q[s].load(qp + at, valid);
-    k[s].load(kp + at, valid);
-    if (CHANNEL) load_some<GN, VEC>(gp + (size_t)t * H * D, valid, g[s]);
-    else g[s][0] = gp[(size_t)t * H];
+    const T* row = rows + (size_t)t * ld;
+    q[s].load(place(row, q_at), valid);
+    k[s].load(place(row, k_at), valid);
+    if (CHANNEL) {
+      load_some<GN, VEC>(place(g_rows + (size_t)t * H * D, g_at), valid, g[s]);
+      dt[s] = 1.f;
+    } else {
+      g[s][0] = *place(g_rows + (size_t)t * H, head_at);
+      dt[s] = *place(dt_rows + (size_t)t * H, head_at);
+    }
+    if constexpr (VEC) {
+      v[s].load(place(row, v_at + col * (unsigned)sizeof(T)), CPL);
+    } else {
 #pragma unroll
-    for (int c = 0; c < CPL; ++c) v[s][c] = vp[at + cc[c]];
-    dt[s] = dp ? dp[(size_t)t * H] : 1.f;
+      for (int c = 0; c < CPL; ++c)
+        v[s].set(c, *place(row, v_at + cc[c] * (unsigned)sizeof(T)));
+    }
   };
 #pragma unroll
   for (int s = 0; s < PF; ++s) fetch(s, s);
@@ -150,7 +178,7 @@ __global__ __launch_bounds__(64) void linear_scan_kernel(
     float b[CPL], x[CPL];
 #pragma unroll
     for (int c = 0; c < CPL; ++c) {
-      x[c] = to_f(v[s][c]);
+      x[c] = v[s].get(c);
       const float u = x[c] * dt[s];
       b[c] = 0.f;
 #pragma unroll
@@ -159,15 +187,25 @@ __global__ __launch_bounds__(64) void linear_scan_kernel(
         b[c] += q[s].get(i) * S[c][i];
       }
     }
+    float mine;
+    if constexpr (CPL == 4) {
+      mine = row16_sum4(b);
+    } else {
 #pragma unroll
-    for (int c = 0; c < CPL; ++c) b[c] = row16_sum(b[c]);
-    float mine = b[0], xm = x[0];
+      for (int c = 0; c < CPL; ++c) b[c] = row16_sum(b[c]);
+      mine = b[0];
 #pragma unroll
-    for (int c = 1; c < CPL; ++c) {
-      mine = lane % CPL == c ? b[c] : mine;
-      xm = lane % CPL == c ? x[c] : xm;
+      for (int c = 1; c < CPL; ++c) mine = lane % CPL == c ? b[c] : mine;
     }
-    out[(size_t)t * H * V + oc] = mine * q_scale + skip * xm;
+    if (!CHANNEL) {
+      float xm = x[0];
+#pragma unroll
+      for (int c = 1; c < CPL; ++c) xm = lane % CPL == c ? x[c] : xm;
+      mine += skip * xm;
+    } else {
+      mine *= q_scale;
+    }
+    out[(size_t)t * H * V + oc] = mine;
   };
   int t0 = 0;
   for (; t0 + PF <= len; t0 += PF) {
@@ -450,15 +488,23 @@ int hy_linear_scan(void* o, void* state, const void* in, int ld, int q_off,
   if (!scan_ok(G, H, D, V) || n_entries > 65535) return -2;
   if (n_entries <= 0) return 0;
   const bool channel = dt == nullptr;
-  if (channel && G != H) return -2;
+  if (channel ? G != H : !skip) return -2;
   // wide lanes where they still put waves enough on the 1024 SIMDs
+  // (measured; a decay per channel gains more from sharing its loads)
   const long long waves = (long long)n_entries * H * ((V + 3) / 4);
   const bool vec = ld % 8 == 0 && q_off % 8 == 0 && k_off % 8 == 0 &&
-                   D % 8 == 0 && rows_per_lane(D) * 16 == D;
+                   v_off % 8 == 0 && D % 8 == 0 && V % 16 == 0 &&
+                   rows_per_lane(D) * 16 == D;
+  // waves of a workgroup: all of a head's column blocks in whole groups
+  auto group = [&](int cpl) {
+    const int nb = (V + 4 * cpl - 1) / (4 * cpl);
+    return nb % 4 == 0 ? 4 : (nb % 2 == 0 ? 2 : 1);
+  };
 #define RUN(CPL, CHANNEL, VEC)                                                \
   HY_DTYPE(dtype, hipLaunchKernelGGL(                                         \
       (linear_scan_kernel<T, RPL, VEC, CPL, CHANNEL>),                        \
-      dim3(H * ((V + 4 * CPL - 1) / (4 * CPL)), n_entries), dim3(64), 0,      \
+      dim3(H * ((V + 4 * CPL - 1) / (4 * CPL)) / group(CPL), n_entries),      \
+      dim3(64 * group(CPL)), 0,                                               \
       (hipStream_t)stream, (float*)o, (float*)state, (const T*)in, ld, q_off, \
       k_off, v_off, (const float*)g, (const float*)dt, (const float*)skip,    \
       (const int*)e_start, (const int*)e_len, (const int*)e_pos,              \
@@ -484,7 +530,7 @@ int hy_linear_scan(void* o, void* state, const void* in, int ld, int q_off,
       default: { constexpr int RPL = 32; PICK(CPL); } break;       \
     }                                                              \
   } while (0)
-  if (V >= 16 && D <= 128 && waves >= 8192) GO(4);
+  if (V % 16 == 0 && D <= 128 && waves >= (channel ? 4096 : 8192)) GO(4);
   else if (V >= 8 && D <= 256 && waves >= 2048) GO(2);
   else GO(1);
 #undef GO

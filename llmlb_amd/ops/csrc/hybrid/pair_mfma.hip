@@ -465,41 +465,53 @@ void pair_decode_kernel(
   }
 }
 
-// Join the parts of both maps, subtract, norm, gate.  One wave a head.
+// Join the parts of both maps, subtract, norm, gate.  One wave a head;
+// lane a 32 + p first holds the weight of map a's part p.
+#define PARTS_MAX 32
 __global__ __launch_bounds__(256) void pair_merge_kernel(
     bf16_t* __restrict__ out, int ld_out, const float* __restrict__ ws_acc,
     const float* __restrict__ ws_ml, const bf16_t* __restrict__ proj, int ld,
     int g_off, int H, int V, int parts, float lam, float gain, float eps) {
   const int q = blockIdx.x, h = blockIdx.y * 4 + threadIdx.x / WAVE;
   if (h >= H) return;
-  const int c = (threadIdx.x & 63) * 4;  // V <= 256 columns
-  float o[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int a = 0; a < 2; ++a) {
-    const size_t at = (((size_t)q * H + h) * 2 + a) * parts;
-    float mx = -1e30f, sum = 0.f, x[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int p = 0; p < parts; ++p) mx = fmaxf(mx, ws_ml[(at + p) * 2]);
-    for (int p = 0; p < parts; ++p) {
-      const float w = __builtin_amdgcn_exp2f(ws_ml[(at + p) * 2] - mx);
-      sum += ws_ml[(at + p) * 2 + 1] * w;
-      if (c < V) {
-        float f[4];
-        load4(ws_acc + (at + p) * V + c, f);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) x[i] += f[i] * w;
-      }
-    }
-    const float inv = (a == 0 ? 1.f : -lam) / sum;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) o[i] += x[i] * inv;
+  const int lane = threadIdx.x & 63;
+  const size_t at = ((size_t)q * H + h) * 2 * parts;
+  const int c = lane * 4;  // V <= 256 columns
+  float z[4] = {0.f, 0.f, 0.f, 0.f};
+  if (c < V) load4(proj + (size_t)q * ld + g_off + (size_t)h * V + c, z);
+  float m = -1e30f, w = 0.f;
+  const int a = lane >> 5, p = lane & 31;
+  if (p < parts) {
+    const float2 ml =
+        *reinterpret_cast<const float2*>(ws_ml + (at + a * parts + p) * 2);
+    m = ml.x;
+    w = ml.y;
   }
-  float ssq = o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
+  float mx = m;
+#pragma unroll
+  for (int o = 16; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, WAVE));
+  const float f = __builtin_amdgcn_exp2f(m - mx);
+  float sum = w * f;
+#pragma unroll
+  for (int o = 16; o > 0; o >>= 1) sum += __shfl_xor(sum, o, WAVE);
+  w = f * (a == 0 ? 1.f : -lam) / sum;
+
+  float o[4] = {0.f, 0.f, 0.f, 0.f};
+  const float* src = ws_acc + at * V + (c < V ? c : 0);
+#pragma unroll 8
+  for (int i = 0; i < 2 * parts; ++i) {
+    const float wi = __shfl(w, i < parts ? i : 32 + i - parts, WAVE);
+    float x[4];
+    load4(src + (size_t)i * V, x);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] += x[j] * wi;
+  }
+  const float ssq =
+      c < V ? o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3] : 0.f;
   const float rn = gain / sqrtf(wave_sum(ssq) / V + eps);
   if (c >= V) return;
-  float z[4];
-  load4(proj + (size_t)q * ld + g_off + (size_t)h * V + c, z);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) o[i] *= rn / (1.f + __expf(-z[i]));
+  for (int j = 0; j < 4; ++j) o[j] *= rn / (1.f + __expf(-z[j]));
   store4(out + (size_t)q * ld_out + (size_t)h * V + c, o);
 }
 
@@ -560,7 +572,7 @@ int hy_pair_decode(void* out, int ld_out, void* acc, void* ml,
                    const void* q_scale, float cap, float lam, float gain,
                    float eps, int n_rows, int parts, void* stream) {
   if (!pair_ok(ld, ld_out, g_off, H, G, D, V) || parts < 1 ||
-      parts > 65535)
+      parts > PARTS_MAX)
     return -2;
   if (n_rows <= 0) return 0;
   const float to_z = cap > 0.f ? 2.f * LOG2E / cap : LOG2E;
