@@ -218,7 +218,7 @@ def main() -> None:
                          "llama-tiny on CPU)")
     ap.add_argument("--hybrid", action="store_true",
                     help="instead: prefill and decode throughput of the "
-                         "hybrid family beside Llama at equal size "
+                         "hybrid models beside Llama at equal size "
                          "(benchmarks/hybrid_bench.py)")
     args, rest = ap.parse_known_args()
     if args.hybrid:

@@ -113,6 +113,10 @@ __device__ __forceinline__ float row8_sum(float v) {  // of 8 lanes
   v = dpp_add<0x4E>(v);
   return dpp_add<0x141>(v);
 }
+__device__ __forceinline__ float half_wave_sum(float v) {  // of 32 lanes
+  v = row16_sum(v);
+  return v + __shfl_xor(v, 16, WAVE);
+}
 // Four sums over 16 lanes at once: lane l gets the one of v[l % 4].
 __device__ __forceinline__ float row16_sum4(const float* v) {
   const bool odd = threadIdx.x & 1, high = threadIdx.x & 2;

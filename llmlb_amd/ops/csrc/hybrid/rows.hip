@@ -174,7 +174,7 @@ __global__ __launch_bounds__(256) void add_norms_kernel(
 
 // Each of a row's ``groups`` parts of S columns divided by its rms, times
 // w (wl columns, repeated along the row), with silu(gate) applied before
-// the norm or after it.  L lanes a part: 8, 16, a wave, or the workgroup.
+// the norm or after it.  L lanes a part: 8 to 64, or the workgroup.
 // Up to KEEP vectors a lane stay in registers between the passes.
 template <typename T, int L, bool GATE_FIRST, bool VEC>
 __global__ __launch_bounds__(256) void gated_norm_kernel(
@@ -221,6 +221,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
   }
   ssq = L == 8    ? row8_sum(ssq)
         : L == 16 ? row16_sum(ssq)
+        : L == 32 ? half_wave_sum(ssq)
         : L == 64 ? wave_sum(ssq)
                   : block_sum_256(ssq, red);
   const float r = 1.f / sqrtf(ssq / S + eps);
@@ -453,6 +454,7 @@ int hy_gated_norm(void* out, int ld_out, const void* y, const void* gate,
   } while (0)
   if (S <= 64) PICK(8);
   else if (S <= 128) PICK(16);
+  else if (S <= 256) PICK(32);
   else if (S <= 512) PICK(64);
   else PICK(256);
 #undef PICK

@@ -297,6 +297,7 @@ def test_add_norms(width, dtype):
 
 # groups, columns of a group, repeated weight
 PARTS = [(5, 7, True), (3, 128, True), (16, 24, True), (4, 129, False),
+         (3, 200, False), (2, 256, True), (7, 64, False),
          (2, 512, True), (3, 333, False), (2, 520, False), (1, 8200, False),
          (1, 12001, False), (2, 4096, True)]
 
