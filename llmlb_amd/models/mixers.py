@@ -8,8 +8,13 @@ one matrix product.
 parallel layers have ``inner`` instead: it writes what the output
 projection reads (``out_width`` columns of a wider row), so that the
 layer applies the projections of mixer and feed-forward as one product.
+Where both also read the same norm, ``inputs`` names the weights of a
+module's input projections, and the layer stacks them into one product,
+whose sections start at the columns given to ``place``.
 """
 from __future__ import annotations
+
+import math
 
 import torch
 import torch.nn as nn
@@ -383,3 +388,120 @@ class ClampedSwiGLU(nn.Module):
     def inner(self, x, out) -> None:
         hy.clamped_swiglu(out, _linear(x, self.w_in), self.u_off, self.limit,
                           self.sharpness)
+
+
+class WindowedAttention(nn.Module):
+    """Causal attention over the last ``window`` tokens (None: all).
+    Queries and keys are normed over the whole projection and rotated on
+    the first ``rot`` numbers of each head; every head has a score
+    temperature and an output gate from a projection of the layer's
+    input.  ``cos_sin`` ([max_pos, rot]) is set by the model."""
+
+    inputs = ("q", "k", "v", "g")
+
+    def __init__(self, *, width, heads, kv_heads, dim, vdim, rot, scale,
+                 window, eps, dtype, device):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if rot % 2 or not 0 <= rot <= dim:
+            raise ValueError("rotated dimensions must be even and at most "
+                             "the head size")
+        if window is not None and window < 1:
+            raise ValueError("a window holds at least one token")
+        self.heads, self.kv_heads, self.dim, self.vdim = \
+            heads, kv_heads, dim, vdim
+        self.rot, self.scale = rot, scale
+        self.window = min(window or FULL_CONTEXT, FULL_CONTEXT)
+        self.eps, self.width = eps, width
+        self.dtype, self.device = dtype, device
+        self.out_width = heads * vdim
+        self.cos_sin = None
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, H, G, D, V = (self.width, self.heads, self.kv_heads, self.dim,
+                         self.vdim)
+        return {"q": (H * D, W), "k": (G * D, W), "v": (G * V, W),
+                "q.norm": (H * D,), "k.norm": (G * D,), "temp": (H,),
+                "g": (H, W), "o": (W, H * V)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        def wide(t):
+            return _param(t.to(self.device).contiguous())
+
+        # the kernels' softmax is of powers of two
+        factor = w["temp"].float() * (self.scale * math.log2(math.e))
+        self.w_q = wide(w["q.norm"].float()
+                        * factor.repeat_interleave(self.dim))
+        self.w_k = wide(w["k.norm"].float())
+
+    def place(self, offsets) -> None:
+        q, self.k_off, self.v_off, self.g_off = offsets
+        assert q == 0, "queries are the first section"
+
+    def cache_spec(self):
+        return PageSpec(self.kv_heads * (self.dim + self.vdim))
+
+    def inner(self, proj, b, cache, index: int, out) -> None:
+        pages = cache.pages[index]
+        sizes = (self.heads, self.kv_heads, self.dim, self.vdim)
+        hy.window_prep(proj, *sizes, self.rot, self.k_off, self.v_off,
+                       self.w_q, self.w_k, self.eps, self.cos_sin, b, pages)
+        hy.window_attention(out, proj, self.g_off, *sizes, pages, b,
+                            self.window)
+
+
+class RoutedExperts(nn.Module):
+    """Feed-forward experts down(relu(up x)^2), of which every token uses
+    the ``top`` that a router scores highest, besides one that all tokens
+    use (``shared``: its width, None: there is none).  Experts form
+    ``groups`` runs of neighbours; only those of the ``keep`` groups with
+    the largest best score can be chosen."""
+
+    def __init__(self, *, width, ff, experts, top, groups, keep, scale,
+                 shared, dtype, device):
+        super().__init__()
+        if groups < 1 or experts % groups or not 1 <= keep <= groups:
+            raise ValueError("expert groups must be equal, and some kept")
+        if not 1 <= top <= keep * (experts // groups):
+            raise ValueError("more experts a token than can be chosen")
+        self.width, self.ff, self.experts, self.top = width, ff, experts, top
+        self.groups, self.keep, self.scale = groups, keep, scale
+        self.dtype, self.device = dtype, device
+        self.out_width = shared or 0
+        self.inputs = ("shared.up",) if shared else ()
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W = self.width
+        out = {"router": (self.experts, W)}
+        for e in range(self.experts):
+            out[f"e{e}.up"] = (self.ff, W)
+            out[f"e{e}.down"] = (W, self.ff)
+        if self.out_width:
+            out["shared.up"] = (self.out_width, W)
+            out["shared.down"] = (W, self.out_width)
+        return out
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        to = dict(dtype=self.dtype, device=self.device)
+        self.w_router = _param(w["router"].to(**to).contiguous())
+        self.w_up, self.w_down = (
+            _param(torch.stack([w[f"e{e}.{n}"] for e in range(self.experts)])
+                   .to(**to)) for n in ("up", "down"))
+
+    def place(self, offsets) -> None:
+        self.u_off = offsets[0] if offsets else None
+
+    def inner(self, x, proj, out):
+        """Writes the shared expert's activations to ``out``; returns
+        what the routed experts add: (outputs [T, top, width], weights
+        [T, top])."""
+        if self.out_width:
+            hy.squared_relu(out, proj[:, self.u_off:
+                                      self.u_off + self.out_width])
+        few = x.shape[0] * self.top <= hy.FEW_PAIRS \
+            and hy.can_expert_mfma(x.dtype, self.width, self.ff)
+        index, weight, lists = hy.route(
+            x, self.w_router, self.top, self.groups, self.keep, self.scale,
+            lists=not few)
+        return hy.experts(x, index, lists, self.w_up, self.w_down), weight

@@ -5,7 +5,9 @@ A model's subclass builds ``layers_`` (modules with a mixer ``mix`` and a
 feed-forward ``ff``, which may be None), loads their weights and
 implements ``forward``.  Tensor names: ``embed``, ``head``,
 ``final.norm``, and per layer ``l<i>.norm1``, ``l<i>.mix.*``,
-``l<i>.norm2``, ``l<i>.mlp.*``.
+``l<i>.norm2`` (where mixer and feed-forward have norms of their own),
+``l<i>.mlp.*``.  ``runs`` lists the layer index of every layer run of a
+forward pass; each run has its own part of the cache.
 """
 from __future__ import annotations
 
@@ -40,6 +42,7 @@ class PackedCausalLM(nn.Module):
 
     ragged = True
     norm_offset = 0.0          # what a stored norm weight is added to
+    shared_norm = False        # one norm for mixer and feed-forward
 
     def __init__(self, cfg, tp: TPContext | None, dtype: torch.dtype,
                  device):
@@ -53,13 +56,19 @@ class PackedCausalLM(nn.Module):
 
     # -- weights ----------------------------------------------------------
 
+    @property
+    def norm_shape(self) -> tuple:
+        """Shape of a norm's weight on the residual stream."""
+        return (self.cfg.width,)
+
     def layer_shapes(self, i: int) -> dict[str, tuple]:
         """Names (without ``l<i>.``) and shapes of layer i's tensors."""
-        ly, W = self.layers_[i], self.cfg.width
-        out = {"norm1": (W,)}
+        ly = self.layers_[i]
+        out = {"norm1": self.norm_shape}
         out.update({f"mix.{k}": s for k, s in ly.mix.weight_shapes().items()})
         if ly.ff is not None:
-            out["norm2"] = (W,)
+            if not self.shared_norm:
+                out["norm2"] = self.norm_shape
             out.update({f"mlp.{k}": s
                         for k, s in ly.ff.weight_shapes().items()})
         return out
@@ -75,7 +84,7 @@ class PackedCausalLM(nn.Module):
 
     def weight_shapes(self) -> dict[str, tuple]:
         W = self.cfg.width
-        out = {"embed": (self.cfg.vocab, W), "final.norm": (W,),
+        out = {"embed": (self.cfg.vocab, W), "final.norm": self.norm_shape,
                "head": (self.cfg.vocab, W)}
         for i in range(len(self.layers_)):
             for k, s in self.layer_shapes(i).items():
@@ -131,8 +140,12 @@ class PackedCausalLM(nn.Module):
     # -- forward ----------------------------------------------------------
 
     @property
+    def runs(self) -> list[int]:
+        return list(range(len(self.layers_)))
+
+    @property
     def specs(self):
-        return [ly.mix.cache_spec() for ly in self.layers_]
+        return [self.layers_[i].mix.cache_spec() for i in self.runs]
 
     def make_cache(self, num_blocks: int, slots: int) -> HybridCache:
         return HybridCache(self.specs, num_blocks, slots, self.device,

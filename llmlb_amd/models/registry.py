@@ -10,6 +10,7 @@ import json
 from pathlib import Path
 
 from .dibelix import DibelixConfig, DibelixForCausalLM
+from .fidepel import FidepelConfig, FidepelForCausalLM
 from .llama import LlamaConfig, LlamaForCausalLM
 from .taletar import TaletarConfig, TaletarForCausalLM
 
@@ -17,12 +18,14 @@ MODELS = {
     LlamaConfig: LlamaForCausalLM,
     DibelixConfig: DibelixForCausalLM,
     TaletarConfig: TaletarForCausalLM,
+    FidepelConfig: FidepelForCausalLM,
 }
 
 # architectures that can be read from a model folder
 FOLDERS = {
     DibelixConfig.architecture: DibelixConfig,
     TaletarConfig.architecture: TaletarConfig,
+    FidepelConfig.architecture: FidepelConfig,
 }
 
 PRESETS = {
@@ -38,6 +41,9 @@ PRESETS = {
     "taletar-tiny": TaletarConfig.tiny,
     "taletar-small": TaletarConfig.small,
     "taletar-8b": TaletarConfig.base_8b,
+    "fidepel-tiny": FidepelConfig.tiny,
+    "fidepel-small": FidepelConfig.small,
+    "fidepel-8b": FidepelConfig.base_8b,
 }
 
 

@@ -26,4 +26,12 @@ __device__ __forceinline__ u32x4 load_columns(const unsigned short* p,
   return u32x4{a.x, a.y, b.x, b.y};
 }
 
+typedef __attribute__((ext_vector_type(2))) float f32x2;
+typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
+// two floats to bf16, nearest even
+__device__ __forceinline__ unsigned to_bf16x2(float lo, float hi) {
+  const f32x2 v = {lo, hi};
+  return __builtin_bit_cast(unsigned, __builtin_convertvector(v, bf16x2));
+}
+
 #define LOG2E 1.4426950408889634f

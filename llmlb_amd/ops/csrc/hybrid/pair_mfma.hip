@@ -14,7 +14,7 @@
 // Scores capped to |s| <= cap need no running maximum as long as
 // exp(cap) times any sum of values stays in float's range: weights are then
 // exp(s) itself (FIXED), for caps up to FIXED_CAP.
-#include "mfma.h"
+#include "paged_tiles.h"
 
 #define FIXED_CAP 60.f
 
@@ -30,92 +30,6 @@ __device__ __forceinline__ float cap_log2_of(float z, float cap_log2) {
   return cap_log2 - 2.f * cap_log2 * __builtin_amdgcn_rcpf(1.f + e);
 }
 
-typedef __attribute__((ext_vector_type(2))) float f32x2;
-typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
-// two floats to bf16, nearest even
-__device__ __forceinline__ unsigned to_bf16x2(float lo, float hi) {
-  const f32x2 v = {lo, hi};
-  return __builtin_bit_cast(unsigned, __builtin_convertvector(v, bf16x2));
-}
-
-// Stages tiles of 64 cached rows of one key/value head: K of both maps
-// into lk [64][2 DQ + 8], V into lv [64][DV + 8].  A thread's pieces of 16
-// bytes lie in pages that are the same for its whole wave.
-template <int DQ, int DV>
-struct Stage {
-  static constexpr int KP = 2 * DQ + 8, VP = DV + 8;
-  static constexpr int KR = 2 * DQ / 8, VR = DV / 8;  // pieces of a row
-  static constexpr int KL = 64 * KR / 256, VL = 64 * VR / 256;
-  const bf16_t* cache;
-  const int* pages;
-  size_t page_size;
-  int width, D, V, head_off, last_key, last_page;
-
-  __device__ __forceinline__ Stage(const bf16_t* cache_, const int* pages_,
-                                   int G, int g, int D_, int V_,
-                                   int last_key_)
-      : cache(cache_), pages(pages_), width(2 * D_ + V_), D(D_), V(V_),
-        last_key(last_key_), last_page(last_key_ / PAGE) {
-    page_size = (size_t)G * PAGE * width;
-    head_off = g * PAGE * width;
-  }
-  // page numbers of the 64 keys from j0 on
-  __device__ __forceinline__ void fetch_pages(int j0,
-                                              int (&pg)[4]) const {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int p = j0 / PAGE + i;
-      pg[i] = pages[p < last_page ? p : last_page];
-    }
-  }
-  // row r of the fetched tile; r / 16 is the same for the whole wave
-  __device__ __forceinline__ const bf16_t* row(int r,
-                                               const int (&pg)[4]) const {
-    const int s = __builtin_amdgcn_readfirstlane(r / PAGE);
-    const int p = s == 0 ? pg[0] : (s == 1 ? pg[1] : (s == 2 ? pg[2]
-                                                             : pg[3]));
-    return cache + (size_t)__builtin_amdgcn_readfirstlane(p) * page_size +
-           head_off + (r % PAGE) * width;
-  }
-  __device__ __forceinline__ void fetch(int j0, const int (&pg)[4],
-                                        u32x4 (&pk)[KL],
-                                        u32x4 (&pv)[VL]) const {
-#pragma unroll
-    for (int i = 0; i < KL; ++i) {
-      const int p = threadIdx.x + i * 256;
-      const int c = p % KR, d = c % (DQ / 8) * 8;
-      pk[i] = u32x4{0, 0, 0, 0};
-      if (d < D)
-        pk[i] = *reinterpret_cast<const u32x4*>(row(p / KR, pg) +
-                                                c / (DQ / 8) * D + d);
-    }
-#pragma unroll
-    for (int i = 0; i < VL; ++i) {
-      const int p = threadIdx.x + i * 256;
-      const int r = p / VR, d = p % VR * 8;
-      // rows past the last key meet zero weights and must be finite
-      pv[i] = u32x4{0, 0, 0, 0};
-      if (d < V && j0 + r <= last_key)
-        pv[i] = *reinterpret_cast<const u32x4*>(row(r, pg) + 2 * D + d);
-    }
-  }
-  static __device__ __forceinline__ void store(unsigned short* lk,
-                                               unsigned short* lv,
-                                               const u32x4 (&pk)[KL],
-                                               const u32x4 (&pv)[VL]) {
-#pragma unroll
-    for (int i = 0; i < KL; ++i) {
-      const int p = threadIdx.x + i * 256;
-      *reinterpret_cast<u32x4*>(&lk[p / KR * KP + p % KR * 8]) = pk[i];
-    }
-#pragma unroll
-    for (int i = 0; i < VL; ++i) {
-      const int p = threadIdx.x + i * 256;
-      *reinterpret_cast<u32x4*>(&lv[p / VR * VP + p % VR * 8]) = pv[i];
-    }
-  }
-};
-
 // ---------------------------------------------------------------------------
 // Prompt portions.  One workgroup: up to 64 queries of one head (16 a
 // wave), tiles of 64 keys through LDS, the next tile in registers.
@@ -129,7 +43,7 @@ void pair_flash_kernel(
     int H, int G, int D, int V, const float* __restrict__ q_scale,
     float to_z, float cap_log2, float lam, float gain, float eps) {
   constexpr int KD = DQ / 32, VT = DV / 16;
-  using St = Stage<DQ, DV>;
+  using St = Stage<2, DQ, DV>;
   __shared__ unsigned short lk[64 * St::KP];
   __shared__ unsigned short lv[64 * St::VP];
   const int* it = items + (blockIdx.x / H) * 4;
@@ -307,7 +221,7 @@ void pair_decode_kernel(
     const float* __restrict__ q_scale, float to_z, float cap_log2,
     int parts) {
   constexpr int KD = DQ / 32, NV = DV / 64, PP = 64 + 8;
-  using St = Stage<DQ, DV>;
+  using St = Stage<2, DQ, DV>;
   __shared__ unsigned short lk[64 * St::KP];
   __shared__ unsigned short lv[64 * St::VP];
   __shared__ unsigned short lp[2][16 * PP];

@@ -93,17 +93,23 @@ __global__ __launch_bounds__(256) void post_norm_add_kernel(
     }
 }
 
-// x += y; h1 = x / rms(x) * w1, h2 = x / rms(x) * w2 in the storage type.
-// y null: nothing is added; w2 (and h2) null: one norm; w1 null: the sum
-// alone.  One workgroup per row, kept in registers between the passes
-// where it fits.
-template <typename T>
+// x += mult y; h1 = x / rms(x) * w1, h2 = x / rms(x) * w2 in the storage
+// type.  y null: nothing is added; w2 (and h2) null: one norm; w1 null: the
+// sum alone.  ROUTED: x += mult (y + sum over k of zw[k] z[k]) with ``top``
+// more rows z of the token.  ONE: w1 and w2 are single numbers.  One
+// workgroup per row, kept in registers between the passes where it fits.
+template <typename T, bool ROUTED, bool ONE>
 __global__ __launch_bounds__(256) void add_norms_kernel(
     float* __restrict__ x, const T* __restrict__ y,
-    const float* __restrict__ w1, const float* __restrict__ w2,
+    const T* __restrict__ z, const float* __restrict__ zw, int top,
+    float mult, const float* __restrict__ w1, const float* __restrict__ w2,
     T* __restrict__ h1, T* __restrict__ h2, int width, float eps) {
   __shared__ float red[4];
   const size_t base = (size_t)blockIdx.x * width;
+  if (ROUTED) {
+    z += base * top;
+    zw += (size_t)blockIdx.x * top;
+  }
   const bool vec = (width & 7) == 0;
   const int nvec = vec ? width >> 3 : 0;
   float keep[NORM_KEEP][8];
@@ -113,8 +119,18 @@ __global__ __launch_bounds__(256) void add_norms_kernel(
     if (y) {
       float d[8];
       load8(y + base + i * 8, d);
+      if (ROUTED) {
+#pragma unroll 4
+        for (int k = 0; k < top; ++k) {
+          const float g = zw[k];
+          float e[8];
+          load8(z + (size_t)k * width + i * 8, e);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) f[j] += d[j];
+          for (int j = 0; j < 8; ++j) d[j] += g * e[j];
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) f[j] += mult * d[j];
       store8(x + base + i * 8, f);
     }
 #pragma unroll
@@ -133,7 +149,11 @@ __global__ __launch_bounds__(256) void add_norms_kernel(
     for (int i = threadIdx.x; i < width; i += 256) {
       float v = x[base + i];
       if (y) {
-        v += to_f(y[base + i]);
+        float d = to_f(y[base + i]);
+        if (ROUTED)
+          for (int k = 0; k < top; ++k)
+            d += zw[k] * to_f(z[(size_t)k * width + i]);
+        v += mult * d;
         x[base + i] = v;
       }
       ssq += v * v;
@@ -143,14 +163,14 @@ __global__ __launch_bounds__(256) void add_norms_kernel(
 
   auto emit = [&](int i, const float* f) {
     float w[8], o[8];
-    load8(w1 + i * 8, w);
+    if (!ONE) load8(w1 + i * 8, w);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) o[j] = f[j] * r * w[j];
+    for (int j = 0; j < 8; ++j) o[j] = f[j] * r * (ONE ? w1[0] : w[j]);
     store8(h1 + base + i * 8, o);
     if (!w2) return;
-    load8(w2 + i * 8, w);
+    if (!ONE) load8(w2 + i * 8, w);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) o[j] = f[j] * r * w[j];
+    for (int j = 0; j < 8; ++j) o[j] = f[j] * r * (ONE ? w2[0] : w[j]);
     store8(h2 + base + i * 8, o);
   };
 #pragma unroll
@@ -167,8 +187,8 @@ __global__ __launch_bounds__(256) void add_norms_kernel(
   if (!vec)
     for (int i = threadIdx.x; i < width; i += 256) {
       const float v = x[base + i] * r;
-      h1[base + i] = from_f<T>(v * w1[i]);
-      if (w2) h2[base + i] = from_f<T>(v * w2[i]);
+      h1[base + i] = from_f<T>(v * w1[ONE ? 0 : i]);
+      if (w2) h2[base + i] = from_f<T>(v * w2[ONE ? 0 : i]);
     }
 }
 
@@ -257,7 +277,8 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
 }
 
 // out[r] = norm(x[index[r]]) in the storage type (index null: row r).
-template <typename T>
+// ONE: w is a single number.
+template <typename T, bool ONE>
 __global__ __launch_bounds__(256) void norm_rows_kernel(
     T* __restrict__ out, const float* __restrict__ x,
     const int* __restrict__ index, const float* __restrict__ w,
@@ -277,9 +298,10 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(
     for (int i = threadIdx.x * 8; i < width; i += 2048) {
       float f[8], wr[8];
       load8(x + src + i, f);
-      load8(w + i, wr);
+      if (!ONE) load8(w + i, wr);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) f[j] *= r * (w_offset + wr[j]);
+      for (int j = 0; j < 8; ++j)
+        f[j] *= r * (w_offset + (ONE ? w[0] : wr[j]));
       store8(out + dst + i, f);
     }
     return;
@@ -288,7 +310,7 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(
     ssq += x[src + i] * x[src + i];
   const float r = 1.f / sqrtf(block_sum_256(ssq, red) / width + eps);
   for (int i = threadIdx.x; i < width; i += 256)
-    out[dst + i] = from_f<T>(x[src + i] * r * (w_offset + w[i]));
+    out[dst + i] = from_f<T>(x[src + i] * r * (w_offset + w[ONE ? 0 : i]));
 }
 
 __device__ __forceinline__ float gelu_tanh_f(float z) {
@@ -357,6 +379,34 @@ __global__ __launch_bounds__(256) void clamped_swiglu_kernel(
   }
 }
 
+// out = max(u, 0)^2
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void squared_relu_kernel(
+    T* __restrict__ out, int ld_out, const T* __restrict__ u, int ld,
+    int n_tok, int ff) {
+  constexpr int N = VEC ? 8 : 1;
+  const int per_row = ff / N;
+  const long long total = (long long)n_tok * per_row;
+  const long long step = (long long)gridDim.x * 256;
+  for (long long id = (long long)blockIdx.x * 256 + threadIdx.x; id < total;
+       id += step) {
+    const int t = (int)(id / per_row);
+    const int i = (int)(id - (long long)t * per_row) * N;
+    const T* src = u + (size_t)t * ld + i;
+    float f[N];
+    if (VEC) load8(src, f);
+    else f[0] = to_f(src[0]);
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      f[j] = fmaxf(f[j], 0.f);
+      f[j] *= f[j];
+    }
+    T* dst = out + (size_t)t * ld_out + i;
+    if (VEC) store8(dst, f);
+    else dst[0] = from_f<T>(f[0]);
+  }
+}
+
 // out = cap * tanh(in / cap) in 32-bit (cap <= 0: a plain widening)
 template <typename T>
 __global__ __launch_bounds__(256) void soft_cap_kernel(
@@ -405,26 +455,39 @@ int hy_post_norm_add(void* x, void* xb, const void* y, const void* w,
 }
 
 int hy_norm_rows(void* out, const void* x, const void* index, const void* w,
-                 float w_offset, int n_rows, int width, float eps, int dtype,
-                 void* stream) {
+                 int one, float w_offset, int n_rows, int width, float eps,
+                 int dtype, void* stream) {
   if (n_rows <= 0) return 0;
-  HY_DTYPE(dtype, hipLaunchKernelGGL(
-      norm_rows_kernel<T>, dim3(n_rows), dim3(256), 0, (hipStream_t)stream,
-      (T*)out, (const float*)x, (const int*)index, (const float*)w, w_offset,
-      width, eps));
+#define GO(ONE)                                                              \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (norm_rows_kernel<T, ONE>), dim3(n_rows), dim3(256), 0,                \
+      (hipStream_t)stream, (T*)out, (const float*)x, (const int*)index,      \
+      (const float*)w, w_offset, width, eps))
+  if (one) GO(true);
+  else GO(false);
+#undef GO
   HY_CHECK();
   return 0;
 }
 
-int hy_add_norms(void* x, const void* y, const void* w1, const void* w2,
-                 void* h1, void* h2, int n_tok, int width, float eps,
+int hy_add_norms(void* x, const void* y, const void* z, const void* zw,
+                 int top, float mult, const void* w1, const void* w2,
+                 int one, void* h1, void* h2, int n_tok, int width, float eps,
                  int dtype, void* stream) {
   if ((w1 && !h1) || (w2 && (!h2 || !w1))) return -2;
+  if (z && (!y || !zw || top < 1)) return -2;
   if (n_tok <= 0) return 0;
-  HY_DTYPE(dtype, hipLaunchKernelGGL(
-      add_norms_kernel<T>, dim3(n_tok), dim3(256), 0, (hipStream_t)stream,
-      (float*)x, (const T*)y, (const float*)w1, (const float*)w2, (T*)h1,
-      (T*)h2, width, eps));
+#define GO(ROUTED, ONE)                                                      \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (add_norms_kernel<T, ROUTED, ONE>), dim3(n_tok), dim3(256), 0,         \
+      (hipStream_t)stream, (float*)x, (const T*)y, (const T*)z,              \
+      (const float*)zw, top, mult, (const float*)w1, (const float*)w2,       \
+      (T*)h1, (T*)h2, width, eps))
+  if (z && one) GO(true, true);
+  else if (z) GO(true, false);
+  else if (one) GO(false, true);
+  else GO(false, false);
+#undef GO
   HY_CHECK();
   return 0;
 }
@@ -490,6 +553,24 @@ int hy_clamped_swiglu(void* out, int ld_out, const void* gu, int ld,
       (clamped_swiglu_kernel<T, VEC>), dim3(grid), dim3(256), 0,           \
       (hipStream_t)stream, (T*)out, ld_out, (const T*)gu, ld, u_off, n_tok, \
       ff, limit, sharpness))
+  if (vec) GO(true);
+  else GO(false);
+#undef GO
+  HY_CHECK();
+  return 0;
+}
+
+int hy_squared_relu(void* out, int ld_out, const void* u, int ld, int n_tok,
+                    int ff, int dtype, void* stream) {
+  if (n_tok <= 0 || ff <= 0) return 0;
+  const uintptr_t mask = dtype == 0 ? 15 : 31;
+  const bool vec = ff % 8 == 0 && ld % 8 == 0 && ld_out % 8 == 0 &&
+                   (((uintptr_t)out | (uintptr_t)u) & mask) == 0;
+  const int grid = grid_for((long long)n_tok * ff / (vec ? 8 : 1));
+#define GO(VEC)                                                              \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (squared_relu_kernel<T, VEC>), dim3(grid), dim3(256), 0,               \
+      (hipStream_t)stream, (T*)out, ld_out, (const T*)u, ld, n_tok, ff))
   if (vec) GO(true);
   else GO(false);
 #undef GO

@@ -1,0 +1,322 @@
+// Grouped-query attention over a sliding window of cached tokens, each
+// head's output times the sigmoid of a number of its own.
+//
+// Queries and keys are normed over the whole projection (all heads at
+// once) and rotated on the first ``rot`` numbers of each head.  A cached
+// token keeps, for each of G key/value heads, one row [key (D) | value
+// (V)]; a page is [G][16 tokens][D + V].  Query head h reads key/value
+// head h / (H / G).  The query's weights carry the scale of the scores
+// and log2(e): the softmax is over powers of two.
+#include "common.h"
+
+// One workgroup a token.  VEC: pieces of 8, each kept in registers
+// beside the piece it is rotated with (rows of up to 8192 numbers).
+#define PREP_KEEP 4
+
+struct PrepSection {  // the queries or the keys of a token
+  int off, heads;
+  const float* w;
+};
+
+template <typename T>
+__device__ __forceinline__ void rotate8(float* f, const float* other,
+                                        const float* cs, int d, int half) {
+  const bool low = d < half;
+  const int i = low ? d : d - half;
+  float c[8], s[8];
+  load8(cs + i, c);
+  load8(cs + half + i, s);
+#pragma unroll
+  for (int j = 0; j < 8; ++j)
+    f[j] = low ? f[j] * c[j] - other[j] * s[j] : f[j] * c[j] + other[j] * s[j];
+}
+
+template <typename T, int KEEP>
+__global__ __launch_bounds__(256) void window_prep_vec_kernel(
+    T* __restrict__ proj, int ld, T* __restrict__ cache, PrepSection q,
+    PrepSection k, int v_off, int D, int V, int rot,
+    const float* __restrict__ cos_sin, float eps,
+    const int* __restrict__ pos_, const int* __restrict__ row_,
+    const int* __restrict__ bt, int max_blocks) {
+  __shared__ float red[2][4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int pos = pos_[t], G = k.heads;
+  T* src = proj + (size_t)t * ld;
+  const int page = bt[(size_t)row_[t] * max_blocks + pos / PAGE];
+  T* rows = cache + ((size_t)page * G * PAGE + pos % PAGE) * (D + V);
+  const size_t head_step = (size_t)PAGE * (D + V);
+  const int half = rot / 2, per_head = D / 8;
+
+  float own[KEEP][8], other[KEEP][8], kown[8], kother[8];
+  float ssq = 0.f, kssq = 0.f;
+  auto fetch = [&](int off, int i, float* a, float* b) {
+    const int d = i % per_head * 8;
+    load8(src + off + i * 8, a);
+    if (d < rot) load8(src + off + i * 8 + (d < half ? half : -half), b);
+  };
+  const int nq = q.heads * per_head, nk = G * per_head;
+#pragma unroll
+  for (int n = 0; n < KEEP; ++n) {
+    const int i = tid + n * 256;
+    if (i < nq) {
+      fetch(q.off, i, own[n], other[n]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ssq += own[n][j] * own[n][j];
+    }
+  }
+  // keys are not changed in place: their first piece is kept, the rest
+  // is read again
+  if (tid < nk) fetch(k.off, tid, kown, kother);
+  for (int i = tid; i < nk; i += 256) {
+    float f[8];
+    if (i != tid) load8(src + k.off + i * 8, f);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float x = i == tid ? kown[j] : f[j];
+      kssq += x * x;
+    }
+  }
+  for (int i = tid; i < G * (V / 8); i += 256) {
+    const int g = i / (V / 8), d = i % (V / 8) * 8;
+    float f[8];
+    load8(src + v_off + i * 8, f);
+    store8(rows + g * head_step + D + d, f);
+  }
+  ssq = wave_sum(ssq);
+  kssq = wave_sum(kssq);
+  if ((tid & 63) == 0) {
+    red[0][tid / WAVE] = ssq;
+    red[1][tid / WAVE] = kssq;
+  }
+  __syncthreads();
+  const float rq = 1.f / sqrtf((red[0][0] + red[0][1] + red[0][2] +
+                                red[0][3]) / (q.heads * D) + eps);
+  const float rk = 1.f / sqrtf((red[1][0] + red[1][1] + red[1][2] +
+                                red[1][3]) / (G * D) + eps);
+  const float* cs = cos_sin + (size_t)pos * rot;
+  auto finish = [&](const float* w, float r, int i, float* a, float* b) {
+    const int d = i % per_head * 8;
+    float f[8];
+    load8(w + i * 8, f);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) a[j] *= r * f[j];
+    if (d >= rot) return;
+    load8(w + i * 8 + (d < half ? half : -half), f);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) b[j] *= r * f[j];
+    rotate8<T>(a, b, cs, d, half);
+  };
+#pragma unroll
+  for (int n = 0; n < KEEP; ++n) {
+    const int i = tid + n * 256;
+    if (i < nq) {
+      finish(q.w, rq, i, own[n], other[n]);
+      store8(src + q.off + i * 8, own[n]);
+    }
+  }
+  for (int i = tid; i < nk; i += 256) {
+    if (i != tid) fetch(k.off, i, kown, kother);
+    finish(k.w, rk, i, kown, kother);
+    store8(rows + i / per_head * head_step + i % per_head * 8, kown);
+  }
+}
+
+// Any sizes: the section's normed numbers go through LDS.
+template <typename T>
+__global__ __launch_bounds__(256) void window_prep_kernel(
+    T* __restrict__ proj, int ld, T* __restrict__ cache, PrepSection q,
+    PrepSection k, int v_off, int D, int V, int rot,
+    const float* __restrict__ cos_sin, float eps,
+    const int* __restrict__ pos_, const int* __restrict__ row_,
+    const int* __restrict__ bt, int max_blocks) {
+  extern __shared__ float lds[];
+  __shared__ float red[2][4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int pos = pos_[t], G = k.heads;
+  T* src = proj + (size_t)t * ld;
+  const int page = bt[(size_t)row_[t] * max_blocks + pos / PAGE];
+  T* rows = cache + ((size_t)page * G * PAGE + pos % PAGE) * (D + V);
+  const size_t head_step = (size_t)PAGE * (D + V);
+  const int half = rot / 2;
+  const float* cs = cos_sin + (size_t)pos * rot;
+  for (int i = tid; i < G * V; i += 256)
+    rows[i / V * head_step + D + i % V] = src[v_off + i];
+#pragma unroll
+  for (int s = 0; s < 2; ++s) {
+    const PrepSection sec = s == 0 ? q : k;
+    const int n = sec.heads * D;
+    float ssq = 0.f;
+    for (int i = tid; i < n; i += 256) {
+      const float x = to_f(src[sec.off + i]);
+      ssq += x * x;
+    }
+    const float r = 1.f / sqrtf(block_sum_256(ssq, red[s]) / n + eps);
+    for (int i = tid; i < n; i += 256)
+      lds[i] = to_f(src[sec.off + i]) * r * sec.w[i];
+    __syncthreads();
+    for (int i = tid; i < n; i += 256) {
+      const int d = i % D;
+      float x = lds[i];
+      if (d < half) x = x * cs[d] - lds[i + half] * cs[half + d];
+      else if (d < rot) x = x * cs[d - half] + lds[i - half] * cs[d];
+      T* dst = s == 0 ? src + sec.off + i : rows + i / D * head_step + d;
+      *dst = from_f<T>(x);
+    }
+    __syncthreads();
+  }
+}
+
+// Any sizes, 32-bit arithmetic: one workgroup per (query, head).  256 keys
+// at a time, a thread scores one of them; then CW threads take the value
+// columns of every (256 / CW)th key each.
+template <typename T, int NC>
+__global__ __launch_bounds__(256) void window_rows_kernel(
+    T* __restrict__ out, int ld_out, const T* __restrict__ proj, int ld,
+    int g_off, const T* __restrict__ cache, const int* __restrict__ pos_,
+    const int* __restrict__ row_, const int* __restrict__ bt, int max_blocks,
+    int H, int G, int D, int V, int CW, int window, bool vec) {
+  extern __shared__ float lds[];
+  float* lq = lds;                     // D query numbers
+  float* lp = lq + D;                  // weights of 256 keys
+  int* lrow = (int*)(lp + 256);        // rows of the keys
+  float* lacc = (float*)(lrow + 256);  // 256 x NC
+  __shared__ float red[4], red2[4];
+  const int t = blockIdx.x, h = blockIdx.y, g = h / (H / G);
+  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
+  const int pos = pos_[t];
+  const int* pages = bt + (size_t)row_[t] * max_blocks;
+  const int width = D + V;
+  const T* q = proj + (size_t)t * ld + (size_t)h * D;
+  for (int i = tid; i < D; i += 256) lq[i] = to_f(q[i]);
+  const int grp = tid / CW, ngrp = 256 / CW, c0 = tid % CW;
+  float m = -INFINITY, l = 0.f, acc[NC];
+#pragma unroll
+  for (int i = 0; i < NC; ++i) acc[i] = 0.f;
+  __syncthreads();
+  for (int j0 = pos - window + 1 > 0 ? pos - window + 1 : 0; j0 <= pos;
+       j0 += 256) {
+    const int j = j0 + tid;
+    float s = -INFINITY;
+    if (j <= pos) {
+      const int row = (pages[j / PAGE] * G + g) * PAGE + j % PAGE;
+      lrow[tid] = row;
+      const T* k = cache + (size_t)row * width;
+      float a = 0.f;
+      if (vec) {
+        for (int d = 0; d < D; d += 4) {
+          float f[4];
+          load4(k + d, f);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) a += f[i] * lq[d + i];
+        }
+      } else {
+        for (int d = 0; d < D; ++d) a += to_f(k[d]) * lq[d];
+      }
+      s = a;
+    }
+    float x = s;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) x = fmaxf(x, __shfl_xor(x, o, WAVE));
+    if (lane == 0) red[wave] = x;
+    __syncthreads();
+    x = fmaxf(fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])), m);
+    const float keep = exp2f(m - x);
+    m = x;
+    const float p = exp2f(s - x);
+    l = l * keep + p;
+    lp[tid] = p;
+    __syncthreads();
+    const int n_keys = pos - j0 + 1 < 256 ? pos - j0 + 1 : 256;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) acc[i] *= keep;
+    for (int k = grp; k < n_keys; k += ngrp) {
+      const T* v = cache + (size_t)lrow[k] * width + D;
+#pragma unroll
+      for (int i = 0; i < NC; ++i) {
+        const int c = c0 + i * CW;
+        acc[i] += lp[k] * (c < V ? to_f(v[c]) : 0.f);
+      }
+    }
+    __syncthreads();
+  }
+  l = wave_sum(l);
+  if (lane == 0) red2[wave] = l;
+#pragma unroll
+  for (int i = 0; i < NC; ++i) lacc[i * 256 + tid] = acc[i];
+  __syncthreads();
+  if (grp != 0) return;
+  const float f = sigmoid_f(to_f(proj[(size_t)t * ld + g_off + h])) /
+                  (red2[0] + red2[1] + red2[2] + red2[3]);
+  T* dst = out + (size_t)t * ld_out + (size_t)h * V;
+#pragma unroll
+  for (int i = 0; i < NC; ++i) {
+    const int c = c0 + i * CW;
+    float a = 0.f;
+    for (int k = 0; k < ngrp; ++k) a += lacc[i * 256 + k * CW + c0];
+    if (c < V) dst[c] = from_f<T>(a * f);
+  }
+}
+
+extern "C" {
+
+int hy_window_prep(void* proj, int ld, void* cache, int k_off, int v_off,
+                   int H, int G, int D, int V, int rot, const void* wq,
+                   const void* wk, const void* cos_sin, float eps,
+                   const void* pos, const void* row, const void* bt,
+                   int max_blocks, int n_tok, int dtype, void* stream) {
+  if (H <= 0 || G <= 0 || D <= 0 || V <= 0 || rot < 0 || rot > D || rot % 2 ||
+      (rot > 0 && !cos_sin) || H * D > 16384 || G * D > 16384)
+    return -2;
+  if (n_tok <= 0) return 0;
+  const PrepSection q{0, H, (const float*)wq}, k{k_off, G, (const float*)wk};
+  const bool vec = D % 8 == 0 && V % 8 == 0 && rot % 16 == 0 && ld % 8 == 0 &&
+                   k_off % 8 == 0 && v_off % 8 == 0 &&
+                   H * D <= 2048 * PREP_KEEP;
+#define ARGS                                                                 \
+  (hipStream_t)stream, (T*)proj, ld, (T*)cache, q, k, v_off, D, V, rot,      \
+      (const float*)cos_sin, eps, (const int*)pos, (const int*)row,          \
+      (const int*)bt, max_blocks
+#define GO(KEEP)                                                             \
+  HY_DTYPE(dtype, hipLaunchKernelGGL((window_prep_vec_kernel<T, KEEP>),      \
+                                     dim3(n_tok), dim3(256), 0, ARGS))
+  if (vec && H * D <= 2048) GO(1);
+  else if (vec && H * D <= 4096) GO(2);
+  else if (vec) GO(PREP_KEEP);
+  else
+    HY_DTYPE(dtype, hipLaunchKernelGGL(
+        window_prep_kernel<T>, dim3(n_tok), dim3(256),
+        (H > G ? H : G) * D * sizeof(float), ARGS));
+#undef GO
+#undef ARGS
+  HY_CHECK();
+  return 0;
+}
+
+int hy_window_rows(void* out, int ld_out, const void* proj, int ld, int g_off,
+                   const void* cache, const void* pos, const void* row,
+                   const void* bt, int max_blocks, int H, int G, int D, int V,
+                   int window, int n_rows, int dtype, void* stream) {
+  if (G <= 0 || H <= 0 || H % G || H > 65535 || D <= 0 || D > 1024 ||
+      V <= 0 || V > 1024 || window < 1)
+    return -2;
+  if (n_rows <= 0) return 0;
+  int cw = 1;
+  while (cw < V && cw < 256) cw *= 2;
+  const bool vec = D % 4 == 0 && V % 4 == 0;
+  const dim3 grid(n_rows, H), block(256);
+#define GO(NC)                                                              \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                       \
+      (window_rows_kernel<T, NC>), grid, block,                             \
+      (D + 512 + 256 * NC) * sizeof(float), (hipStream_t)stream, (T*)out,   \
+      ld_out, (const T*)proj, ld, g_off, (const T*)cache, (const int*)pos,  \
+      (const int*)row, (const int*)bt, max_blocks, H, G, D, V, cw, window,  \
+      vec))
+  if (V <= 256) GO(1);
+  else if (V <= 512) GO(2);
+  else GO(4);
+#undef GO
+  HY_CHECK();
+  return 0;
+}
+
+}  // extern "C"

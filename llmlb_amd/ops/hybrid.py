@@ -1,6 +1,6 @@
 """Ops of the hybrid models: a 32-bit residual stream with norms before
-or after the sublayers, latent and differential attention over pages,
-gated delta rule and linear recurrences.
+or after the sublayers, latent, differential and windowed attention over
+pages, gated delta rule, linear recurrences and mixtures of experts.
 
 The native library (csrc/hybrid) is loaded at first use.  GPU tensors
 always run the HIP kernels, in bfloat16 and in float32; CPU tensors run
@@ -87,32 +87,47 @@ def post_norm_add(x, xb, y, w, eps, w_offset=0.0) -> None:
         _stream()), "hy_post_norm_add")
 
 
-def add_norms(x, y, w1, w2, eps, dtype):
-    """In place: x += y (None: nothing to add).  Returns rmsnorm(x) * w1
-    and rmsnorm(x) * w2 in ``dtype``, None for a weight that is None
-    (w2 alone may not be given)."""
+def add_norms(x, y, w1, w2, eps, dtype, mult=1.0, routed=None):
+    """In place: x += mult * y (None: nothing to add).  Returns
+    rmsnorm(x) * w1 and rmsnorm(x) * w2 in ``dtype``, None for a weight
+    that is None (w2 alone may not be given); weights are rows or single
+    numbers.  ``routed``: (z [T, n, W], g [T, n]) whose weighted sum
+    over n is added to y first."""
     if not x.is_cuda:
-        return ref.add_norms(x, y, w1, w2, eps, dtype)
+        return ref.add_norms(x, y, w1, w2, eps, dtype, mult, routed)
     assert y is None or (y.is_contiguous() and y.shape == x.shape
                          and y.dtype == dtype)
+    z, g = routed or (None, None)
+    n = 0
+    if z is not None:
+        n = z.shape[1]
+        assert z.is_contiguous() and g.is_contiguous() and z.dtype == dtype \
+            and z.shape == (x.shape[0], n, x.shape[1]) \
+            and g.shape == (x.shape[0], n)
+    one = w1 is not None and w1.numel() == 1 and x.shape[1] > 1
+    for w in (w1, w2):
+        assert w is None or w.numel() == (1 if one else x.shape[1])
     h1, h2 = (None if w is None else
               torch.empty(x.shape, dtype=dtype, device=x.device)
               for w in (w1, w2))
     _check(native().hy_add_norms(
-        _ptr(x), _p(y), _p(w1), _p(w2), _p(h1), _p(h2), _i(x.shape[0]),
-        _i(x.shape[1]), _f(eps), _dt(dtype), _stream()), "hy_add_norms")
+        _ptr(x), _p(y), _p(z), _p(g), _i(n), _f(mult), _p(w1), _p(w2),
+        _i(one), _p(h1), _p(h2), _i(x.shape[0]), _i(x.shape[1]), _f(eps),
+        _dt(dtype), _stream()), "hy_add_norms")
     return h1, h2
 
 
 def norm_rows(x, index, w, eps, dtype, w_offset=0.0):
     """rmsnorm(x[index]) * (w_offset + w) in ``dtype``; index may be
-    None (every row)."""
+    None (every row), w a row or a single number."""
     if not x.is_cuda:
         return ref.norm_rows(x, index, w, eps, dtype, w_offset)
     n = x.shape[0] if index is None else index.shape[0]
+    one = w.numel() == 1 and x.shape[1] > 1
+    assert w.numel() == (1 if one else x.shape[1])
     out = torch.empty(n, x.shape[1], dtype=dtype, device=x.device)
     _check(native().hy_norm_rows(
-        _ptr(out), _ptr(x), _p(index), _ptr(w), _f(w_offset), _i(n),
+        _ptr(out), _ptr(x), _p(index), _ptr(w), _i(one), _f(w_offset), _i(n),
         _i(x.shape[1]), _f(eps), _dt(dtype), _stream()), "hy_norm_rows")
     return out
 
@@ -140,6 +155,18 @@ def clamped_swiglu(out, gu, u_off, limit, sharpness) -> None:
         _ptr(out), _i(out.stride(0)), _ptr(gu), _i(gu.stride(0)), _i(u_off),
         _i(out.shape[0]), _i(out.shape[1]), _f(limit), _f(sharpness),
         _dt(gu.dtype), _stream()), "hy_clamped_swiglu")
+
+
+def squared_relu(out, u) -> None:
+    """out = max(u, 0)^2; both may be columns of wider rows."""
+    if not u.is_cuda:
+        ref.squared_relu(out, u)
+        return
+    assert u.stride(1) == 1 and out.stride(1) == 1 and u.shape == out.shape
+    _check(native().hy_squared_relu(
+        _ptr(out), _i(out.stride(0)), _ptr(u), _i(u.stride(0)),
+        _i(out.shape[0]), _i(out.shape[1]), _dt(u.dtype), _stream()),
+        "hy_squared_relu")
 
 
 def soft_cap(logits, cap):
@@ -467,3 +494,151 @@ def state_space(out, proj, z_off, dt_off, state, ring, b, wconv, bconv,
             _ptr(b.e_pos), _ptr(b.e_row), _i(len(b.entries)), _i(G), _i(H),
             _i(N), _i(V), _f(1.0), dt, st), "hy_linear_scan")
     _gated_norm(out, o, proj, z_off, w_norm, norm_groups, True, eps)
+
+
+# -- windowed attention ----------------------------------------------------
+
+def window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk,
+                eps, cos_sin, b, cache) -> None:
+    """Norm queries (the first columns of ``proj``) and keys over all
+    heads, rotate the first ``rot`` numbers of each head, the queries in
+    place; put keys and values into the pages.  ``wq`` carries the
+    scores' scale and log2(e)."""
+    if not proj.is_cuda:
+        ref.window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off,
+                        wq, wk, eps, cos_sin, b, cache)
+        return
+    assert proj.stride(1) == 1 and wq.numel() == heads * dim \
+        and wk.numel() == kv_heads * dim
+    bt = b.block_tables
+    _check(native().hy_window_prep(
+        _ptr(proj), _i(proj.stride(0)), _ptr(cache), _i(k_off), _i(v_off),
+        _i(heads), _i(kv_heads), _i(dim), _i(vdim), _i(rot), _ptr(wq),
+        _ptr(wk), _p(cos_sin), _f(eps), _ptr(b.pos), _ptr(b.row), _ptr(bt),
+        _i(bt.shape[1]), _i(b.n_tok), _dt(proj.dtype), _stream()),
+        "hy_window_prep")
+
+
+def can_window_mfma(dtype, group, dim, vdim) -> bool:
+    """Sizes that the matrix-core kernels take."""
+    return (dtype == torch.bfloat16 and dim % 8 == 0 and vdim % 8 == 0
+            and dim <= 256 and vdim <= 256 and group <= 128)
+
+
+def window_parts(n: int, kv_heads: int, group: int, keys: int) -> int:
+    """How many workgroups share one query's keys: enough to fill the
+    chip, with at least two tiles of keys each."""
+    groups = n * kv_heads * ((group + 15) // 16)
+    return max(1, min(1024 // groups, keys // 128, 64))
+
+
+def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
+                     window) -> None:
+    """Attention of the prepared queries over the last ``window`` tokens,
+    times the sigmoid of the heads' numbers at column ``g_off``, into
+    ``out`` [T, H * vdim] (columns of wider rows)."""
+    if not proj.is_cuda:
+        ref.window_attention(out, proj, g_off, heads, kv_heads, dim, vdim,
+                             cache, b, window)
+        return
+    assert proj.stride(1) == 1 and out.stride(1) == 1
+    lib, bt, st = native(), b.block_tables, _stream()
+    H, G, D, V = heads, kv_heads, dim, vdim
+    assert cache.shape[0] * G * 16 < 2 ** 31    # rows are 32-bit numbers
+    dst = (_ptr(out), _i(out.stride(0)))
+    src = (_ptr(proj), _i(proj.stride(0)), _i(g_off), _ptr(cache))
+    where = (_ptr(bt), _i(bt.shape[1]))
+    sizes = (_i(H), _i(G), _i(D), _i(V), _i(window))
+    # vector accesses need whole vectors in every row
+    if not (can_window_mfma(proj.dtype, H // G, D, V)
+            and proj.stride(0) % 8 == 0 and out.stride(0) % 8 == 0):
+        _check(lib.hy_window_rows(
+            *dst, *src, _ptr(b.pos), _ptr(b.row), *where, *sizes,
+            _i(b.n_tok), _dt(proj.dtype), st), "hy_window_rows")
+        return
+    n = b.n_short
+    if n:
+        parts = window_parts(n, G, H // G, min(window, b.max_keys))
+        acc = ml = None
+        if parts > 1:
+            acc = torch.empty(n, H, parts, V, dtype=torch.float32,
+                              device=proj.device)
+            ml = torch.empty(n, H, parts, 2, dtype=torch.float32,
+                             device=proj.device)
+        _check(lib.hy_window_decode(
+            *dst, _p(acc), _p(ml), *src, _ptr(b.pos), _ptr(b.row), *where,
+            *sizes, _i(n), _i(parts), st), "hy_window_decode")
+    if n < b.n_tok:
+        items, n_items = b.query_tiles(128 // (H // G))
+        _check(lib.hy_window_flash(
+            *dst, *src, _ptr(items), _i(n_items), *where, *sizes, st),
+            "hy_window_flash")
+
+
+# -- mixture of experts ----------------------------------------------------
+
+FEW_PAIRS = 1024     # (token, choice) pairs that need no lists of experts
+
+
+def can_expert_mfma(dtype, width, ff) -> bool:
+    """Sizes that the matrix-core kernels take."""
+    return dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0
+
+
+def route(h, w, top, groups, keep, scale, lists: bool = True):
+    """The experts of every token: (index [T, top] int32, weight [T, top]
+    float32, lists).  Logits w h in 32-bit, softmax over all experts, the
+    ``top`` best among the ``keep`` groups of neighbours with the largest
+    best score, weights over their sum times ``scale``.  ``lists``: also
+    every expert's (token, choice) pairs, as (counts, pairs)."""
+    if not h.is_cuda:
+        return *ref.route(h, w, top, groups, keep, scale), None
+    T, W = h.shape
+    E = w.shape[0]
+    assert h.is_contiguous() and w.is_contiguous() and w.shape[1] == W
+    index = torch.empty(T, top, dtype=torch.int32, device=h.device)
+    weight = torch.empty(T, top, dtype=torch.float32, device=h.device)
+    counts = pairs = None
+    if lists:
+        counts = torch.zeros(E, dtype=torch.int32, device=h.device)
+        pairs = torch.empty(E, T, dtype=torch.int32, device=h.device)
+    _check(native().hy_route(
+        _ptr(index), _ptr(weight), _p(counts), _p(pairs), _ptr(h), _ptr(w),
+        _i(W), _i(E), _i(top), _i(groups), _i(keep), _f(scale), _i(T),
+        _dt(h.dtype), _stream()), "hy_route")
+    return index, weight, (counts, pairs) if lists else None
+
+
+def experts(h, index, lists, w_up, w_down):
+    """down(relu(up h)^2) of every token's experts -> [T, top, W].
+    w_up [E, ff, W], w_down [E, W, ff]; ``lists``: of ``route``, may be
+    None for few pairs on the matrix cores."""
+    if not h.is_cuda:
+        return ref.experts(h, index, w_up, w_down)
+    T, top = index.shape
+    E, F, W = w_up.shape
+    assert h.is_contiguous() and w_up.is_contiguous() \
+        and w_down.is_contiguous() and w_down.shape == (E, W, F) \
+        and h.shape == (T, W)
+    lib, st = native(), _stream()
+    u = torch.empty(T * top, F, dtype=h.dtype, device=h.device)
+    z = torch.empty(T, top, W, dtype=h.dtype, device=h.device)
+    up = (_ptr(u), _ptr(h), _ptr(w_up))
+    down = (_ptr(z), _ptr(u), _ptr(w_down))
+    up_size = (_i(E), _i(F), _i(W), _i(top), _i(1))
+    down_size = (_i(E), _i(W), _i(F), _i(1), _i(0))
+    if lists is None:
+        for data, size in ((up, up_size), (down, down_size)):
+            _check(lib.hy_expert_few(*data, _ptr(index), *size, _i(T * top),
+                                     st), "hy_expert_few")
+        return z
+    where = (_ptr(lists[0]), _ptr(lists[1]))
+    tiles = can_expert_mfma(h.dtype, W, F)
+    for data, size in ((up, up_size), (down, down_size)):
+        args = (*data, *where, *size, _i(T), _i(T * top))
+        if tiles:
+            _check(lib.hy_expert_tiles(*args, st), "hy_expert_tiles")
+        else:
+            _check(lib.hy_expert_rows(*args, _dt(h.dtype), st),
+                   "hy_expert_rows")
+    return z

@@ -50,12 +50,13 @@ def rope_apply(q: torch.Tensor, k: torch.Tensor, cos_sin: torch.Tensor,
 
 
 def build_cos_sin_table(max_pos: int, head_dim: int, rope_theta: float,
-                        device="cpu") -> torch.Tensor:
-    """[max_pos, head_dim] fp32: cos(f_i * p) | sin(f_i * p)."""
+                        device="cpu", factor: float = 1.0) -> torch.Tensor:
+    """[max_pos, head_dim] fp32: cos(f_i * p) | sin(f_i * p), with all
+    frequencies divided by ``factor`` (linear scaling)."""
     half = head_dim // 2
     inv_freq = 1.0 / (
         rope_theta ** (torch.arange(0, half, dtype=torch.float64) / half)
-    )
+    ) / factor
     pos = torch.arange(max_pos, dtype=torch.float64)
     angles = torch.outer(pos, inv_freq)  # [max_pos, half]
     table = torch.cat([angles.cos(), angles.sin()], dim=-1).float()

@@ -6,6 +6,7 @@ import torch
 import torch.nn.functional as F
 
 PAGE = 16
+LN2 = 0.6931471805599453
 
 
 def _rms(x, eps):
@@ -25,9 +26,12 @@ def post_norm_add(x, xb, y, w, eps, w_offset):
         xb.copy_(x)
 
 
-def add_norms(x, y, w1, w2, eps, dtype):
+def add_norms(x, y, w1, w2, eps, dtype, mult=1.0, routed=None):
     if y is not None:
-        x += y.float()
+        x += mult * y.float()
+    if routed is not None:
+        z, g = routed
+        x += mult * torch.einsum("tkw,tk->tw", z.float(), g)
     if w1 is None:
         return None, None
     n = _rms(x, eps)
@@ -48,6 +52,10 @@ def clamped_swiglu(out, gu, u_off, limit, sharpness):
     g = gu[:, :n].float().clamp(max=limit)
     u = gu[:, u_off:u_off + n].float().clamp(-limit, limit)
     out.copy_(g * torch.sigmoid(sharpness * g) * (u + 1.0))
+
+
+def squared_relu(out, u):
+    out.copy_(u.float().clamp(min=0).square())
 
 
 def soft_cap(logits, cap):
@@ -222,3 +230,66 @@ def state_space(out, proj, z_off, dt_off, state, ring, b, wconv, bconv,
         o = o * F.silu(proj[start:start + n, z_off:z_off + H * V].float())
         o = _rms(o.view(n, norm_groups, -1), eps).reshape(n, H * V) * w_norm
         out[start:start + n] = o.to(out.dtype)
+
+
+# -- windowed attention ----------------------------------------------------
+
+def window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk,
+                eps, cos_sin, b, cache):
+    T, H, G, D, V = b.n_tok, heads, kv_heads, dim, vdim
+    pos = b.pos.long()
+
+    def normed(at, n, w):
+        x = proj[:, at:at + n * D]
+        y = (_rms(x.float(), eps) * w).view(T, n, D)
+        if rot:
+            y = torch.cat([_turn(y[..., :rot], cos_sin[pos]), y[..., rot:]],
+                          -1)
+        return y.to(proj.dtype)
+
+    proj[:, :H * D] = normed(0, H, wq).reshape(T, -1)
+    page = b.block_tables[b.row.long(), pos // PAGE].long()
+    rows = cache.view(cache.shape[0], G, PAGE, D + V)
+    v = proj[:, v_off:v_off + G * V].reshape(T, G, V)
+    rows[page, :, pos % PAGE] = torch.cat([normed(k_off, G, wk), v], -1)
+
+
+def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
+                     window):
+    H, G, D, V = heads, kv_heads, dim, vdim
+    rows = cache.view(cache.shape[0], G, PAGE, D + V)
+    head = torch.arange(H) // (H // G)
+    for t in range(b.n_tok):
+        p = int(b.pos[t])
+        js = torch.arange(max(0, p - window + 1), p + 1)
+        page = b.block_tables[int(b.row[t]), js // PAGE].long()
+        kv = rows[page, :, js % PAGE].float()[:, head]         # [j, H, ..]
+        s = torch.einsum("hd,jhd->hj", proj[t, :H * D].view(H, D).float(),
+                         kv[..., :D])
+        a = torch.softmax(s * LN2, -1)
+        o = torch.einsum("hj,jhv->hv", a, kv[..., D:])
+        gate = torch.sigmoid(proj[t, g_off:g_off + H].float())
+        out[t] = (o * gate[:, None]).reshape(-1).to(out.dtype)
+
+
+# -- mixture of experts ----------------------------------------------------
+
+def route(h, w, top, groups, keep, scale):
+    s = torch.softmax(h.float() @ w.float().T, -1)
+    T, E = s.shape
+    best = s.view(T, groups, -1).amax(-1).topk(keep, -1).indices
+    allowed = torch.zeros(T, groups, dtype=torch.bool).scatter_(
+        1, best, True).repeat_interleave(E // groups, 1)
+    g, index = s.masked_fill(~allowed, -1.0).topk(top, -1)
+    return index.int(), g / (g.sum(-1, keepdim=True) + 1e-20) * scale
+
+
+def experts(h, index, w_up, w_down):
+    T, top = index.shape
+    z = torch.empty(T, top, h.shape[1], dtype=h.dtype)
+    for e in index.unique().tolist():
+        t, k = (index == e).nonzero(as_tuple=True)
+        u = (h[t].float() @ w_up[e].float().T).to(h.dtype)
+        u = u.float().clamp(min=0).square().to(h.dtype)
+        z[t, k] = (u.float() @ w_down[e].float().T).to(h.dtype)
+    return z
