@@ -1,6 +1,6 @@
 #!/usr/bin/env python3
-"""Prefill and decode throughput of the hybrid models (Dibelix, Taletar)
-beside the Llama family at equal width, depth and parameter count
+"""Prefill and decode throughput of the hybrid models (Dibelix, Taletar,
+Fidepel) beside the Llama family at equal width, depth and parameter count
 (random weights, one GPU).
 
   python bench.py --hybrid [--steps K --warmup W]      all sizes, one JSON
@@ -85,8 +85,25 @@ def taletar_config(size: str):
     return build(fit_ff(TaletarForCausalLM, build, size, 3))
 
 
+def fidepel_config(size: str):
+    """The same width, depth and heads, with a window; 16 experts and a
+    shared one take up the Llama model's feed-forward, 4 of 16 (and the
+    shared one) compute a token."""
+    from llmlb_amd.models.fidepel import FidepelConfig, FidepelForCausalLM
+    w, n, h, d, kv, inter = SIZES[size]
+
+    def build(ff):
+        return FidepelConfig.build(
+            n, vocab=VOCAB, width=w, heads=h, kv_heads=kv, dim=d, vdim=d,
+            window=WINDOW, ff=ff, experts=16, top=4, groups=4, keep=2,
+            shared_ff=ff, residual_mult=0.4, max_pos=8192,
+            name=f"fidepel-{size}")
+
+    return build(fit_ff(FidepelForCausalLM, build, size, 2 * 17))
+
+
 CONFIGS = {"llama": llama_config, "dibelix": dibelix_config,
-           "taletar": taletar_config}
+           "taletar": taletar_config, "fidepel": fidepel_config}
 
 
 def make_engine(cfg, args):
@@ -169,7 +186,7 @@ def measure(kind: str, size: str, args) -> dict:
 
 def add_arguments(ap) -> None:
     ap.add_argument("--size", default="s,m,l", help="of s, m, l")
-    ap.add_argument("--only", default="llama,dibelix,taletar")
+    ap.add_argument("--only", default="llama,dibelix,taletar,fidepel")
     ap.add_argument("--phase", default="all",
                     choices=("all", "prefill", "decode"))
     ap.add_argument("--prompts", type=int, default=8)
@@ -198,7 +215,9 @@ def run(args) -> dict:
                                       "layers, shared latents; repeated",
                            "taletar": "differential attention, gated "
                                       "linear attention, Mamba-2, gated "
-                                      "linear attention; repeated"}},
+                                      "linear attention; repeated",
+                           "fidepel": "windowed attention and 4 of 16 "
+                                      "experts beside a shared one"}},
             "steps": args.steps, "warmup": args.warmup, "sizes": sizes}
 
 

@@ -160,10 +160,15 @@ class FidepelLayer(nn.Module):
         proj = _linear(h, self.w_in)
         mid = torch.empty(h.shape[0], self.w_out.shape[1], dtype=h.dtype,
                           device=h.device)
-        self.mix.inner(proj, b, cache, run, mid[:, :n])
-        routed = None if self.ff is None \
-            else self.ff.inner(h, proj, mid[:, n:])
-        return _linear(mid, self.w_out), routed
+        if self.ff is None:
+            self.mix.inner(proj, b, cache, run, mid[:, :n])
+            return _linear(mid, self.w_out), None
+        index, weight, lists = hy.window_front(
+            self.mix.prep(proj, b, cache, run), self.ff.routing(h),
+            self.ff.act(proj, mid[:, n:]))
+        self.mix.attend(proj, b, cache, run, mid[:, :n])
+        z = self.ff.routed(h, index, lists)
+        return _linear(mid, self.w_out), (z, weight)
 
 
 class FidepelForCausalLM(PackedCausalLM):

@@ -442,13 +442,20 @@ class WindowedAttention(nn.Module):
     def cache_spec(self):
         return PageSpec(self.kv_heads * (self.dim + self.vdim))
 
-    def inner(self, proj, b, cache, index: int, out) -> None:
-        pages = cache.pages[index]
-        sizes = (self.heads, self.kv_heads, self.dim, self.vdim)
-        hy.window_prep(proj, *sizes, self.rot, self.k_off, self.v_off,
-                       self.w_q, self.w_k, self.eps, self.cos_sin, b, pages)
-        hy.window_attention(out, proj, self.g_off, *sizes, pages, b,
+    def prep(self, proj, b, cache, index: int) -> tuple:
+        """Arguments of ``hybrid.window_prep``."""
+        return (proj, self.heads, self.kv_heads, self.dim, self.vdim,
+                self.rot, self.k_off, self.v_off, self.w_q, self.w_k,
+                self.eps, self.cos_sin, b, cache.pages[index])
+
+    def attend(self, proj, b, cache, index: int, out) -> None:
+        hy.window_attention(out, proj, self.g_off, self.heads, self.kv_heads,
+                            self.dim, self.vdim, cache.pages[index], b,
                             self.window)
+
+    def inner(self, proj, b, cache, index: int, out) -> None:
+        hy.window_prep(*self.prep(proj, b, cache, index))
+        self.attend(proj, b, cache, index, out)
 
 
 class RoutedExperts(nn.Module):
@@ -492,16 +499,19 @@ class RoutedExperts(nn.Module):
     def place(self, offsets) -> None:
         self.u_off = offsets[0] if offsets else None
 
-    def inner(self, x, proj, out):
-        """Writes the shared expert's activations to ``out``; returns
-        what the routed experts add: (outputs [T, top, width], weights
-        [T, top])."""
-        if self.out_width:
-            hy.squared_relu(out, proj[:, self.u_off:
-                                      self.u_off + self.out_width])
+    def routing(self, x) -> tuple:
+        """Arguments of ``hybrid.route``."""
         few = x.shape[0] * self.top <= hy.FEW_PAIRS \
             and hy.can_expert_mfma(x.dtype, self.width, self.ff)
-        index, weight, lists = hy.route(
-            x, self.w_router, self.top, self.groups, self.keep, self.scale,
-            lists=not few)
-        return hy.experts(x, index, lists, self.w_up, self.w_down), weight
+        return (x, self.w_router, self.top, self.groups, self.keep,
+                self.scale, not few)
+
+    def act(self, proj, out) -> tuple | None:
+        """Arguments of ``hybrid.squared_relu``: the shared expert's
+        activation (None: there is none)."""
+        n = self.out_width
+        return (out, proj[:, self.u_off:self.u_off + n]) if n else None
+
+    def routed(self, x, index, lists):
+        """The chosen experts' outputs [T, top, width]."""
+        return hy.experts(x, index, lists, self.w_up, self.w_down)

@@ -6,37 +6,62 @@
 #pragma once
 #include "common.h"
 
-// The expert and the tile of BM pairs of its list that workgroup number
-// ``tile`` computes, experts one after another; false past the last one.
-// Called by whole waves.
+// A tile is BM pairs of one expert's list, or what remains of it.  All whole
+// tiles are numbered first, expert after expert, then the remainders: they
+// are the quick ones, and come last.
 struct ExpertTile {
   int expert, first, n;  // n pairs from ``first`` on
 };
+#define EXPERTS_MAX 1024
+
 template <int BM>
-__device__ __forceinline__ bool find_tile(const int* counts, int E, int tile,
-                                          ExpertTile& out) {
-  const int lane = threadIdx.x & (WAVE - 1);
-  for (int e0 = 0; e0 < E; e0 += WAVE) {
-    const int n = e0 + lane < E ? counts[e0 + lane] : 0;
-    const int tiles = (n + BM - 1) / BM;
-    int sum = tiles;  // of this lane's and all earlier experts
+struct ExpertTiles {
+  // tiles of the experts up to and with each: whole ones, remainders
+  int whole[EXPERTS_MAX], rest[EXPERTS_MAX];
+
+  // one wave
+  __device__ __forceinline__ void count(const int* counts, int E) {
+    const int lane = threadIdx.x & (WAVE - 1);
+    int w0 = 0, r0 = 0;
+    for (int e0 = 0; e0 < E; e0 += WAVE) {
+      const int n = e0 + lane < E ? counts[e0 + lane] : 0;
+      int w = n / BM, r = n % BM != 0;
 #pragma unroll
-    for (int o = 1; o < WAVE; o *= 2) {
-      const int x = __shfl_up(sum, o, WAVE);
-      if (lane >= o) sum += x;
+      for (int o = 1; o < WAVE; o *= 2) {
+        const int x = __shfl_up(w, o, WAVE), y = __shfl_up(r, o, WAVE);
+        if (lane >= o) {
+          w += x;
+          r += y;
+        }
+      }
+      if (e0 + lane < E) {
+        whole[e0 + lane] = w0 + w;
+        rest[e0 + lane] = r0 + r;
+      }
+      w0 += __shfl(w, WAVE - 1, WAVE);
+      r0 += __shfl(r, WAVE - 1, WAVE);
     }
-    const int all = __shfl(sum, WAVE - 1, WAVE);
-    if (tile < all) {
-      const unsigned long long past = __ballot(sum > tile);
-      const int l = __ffsll((long long)past) - 1;
-      const int before = __shfl(sum - tiles, l, WAVE);
-      out.expert = e0 + l;
-      out.first = (tile - before) * BM;
-      out.n = __shfl(n, l, WAVE) - out.first;
-      out.n = out.n < BM ? out.n : BM;
-      return true;
-    }
-    tile -= all;
   }
-  return false;
-}
+  // first expert with ends[e] > i, by whole waves
+  static __device__ __forceinline__ int find(const int* ends, int E, int i) {
+    const int lane = threadIdx.x & (WAVE - 1);
+    for (int e0 = 0; e0 < E; e0 += WAVE) {
+      const unsigned long long past =
+          __ballot(e0 + lane < E && ends[e0 + lane] > i);
+      if (past)
+        return __builtin_amdgcn_readfirstlane(
+            e0 + __ffsll((long long)past) - 1);
+    }
+    return E - 1;
+  }
+  // whole waves: tile i of the whole ones, or of the remainders
+  __device__ __forceinline__ ExpertTile get(const int* counts, int E, int i,
+                                            bool is_rest) const {
+    ExpertTile t;
+    t.expert = find(is_rest ? rest : whole, E, i);
+    const int before = t.expert ? whole[t.expert - 1] : 0;
+    t.first = (is_rest ? whole[t.expert] - before : i - before) * BM;
+    t.n = is_rest ? counts[t.expert] - t.first : BM;
+    return t;
+  }
+};

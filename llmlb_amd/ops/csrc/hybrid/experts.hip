@@ -14,8 +14,13 @@ __global__ __launch_bounds__(256) void expert_rows_kernel(
     const int* __restrict__ counts, const int* __restrict__ pairs, int E,
     int N, int K, int div, int act, int n_tok) {
   __shared__ float la[BM][BK + 1], lb[BN][BK + 1];
-  ExpertTile t;
-  if (!find_tile<BM>(counts, E, blockIdx.x, t)) return;
+  __shared__ ExpertTiles<BM> tiles;
+  if (threadIdx.x < WAVE) tiles.count(counts, E);
+  __syncthreads();
+  const int i = blockIdx.x, whole = tiles.whole[E - 1];
+  if (i >= whole + tiles.rest[E - 1]) return;
+  const ExpertTile t =
+      tiles.get(counts, E, i < whole ? i : i - whole, i >= whole);
   const int* list = pairs + (size_t)t.expert * n_tok + t.first;
   const T* we = w + (size_t)t.expert * N * K;
   const int n0 = blockIdx.y * BN;
@@ -62,7 +67,7 @@ extern "C" int hy_expert_rows(void* out, const void* in, const void* w,
                               const void* counts, const void* pairs, int E,
                               int N, int K, int div, int act, int n_tok,
                               int n_pairs, int dtype, void* stream) {
-  if (E <= 0 || N <= 0 || K <= 0 || div <= 0 || N > 65535 * BN) return -2;
+  if (E <= 0 || E > EXPERTS_MAX || N <= 0 || K <= 0 || div <= 0 || N > 65535 * BN) return -2;
   if (n_tok <= 0 || n_pairs <= 0) return 0;
   const int tiles = n_pairs / BM + (E < n_pairs ? E : n_pairs);
   HY_DTYPE(dtype, hipLaunchKernelGGL(

@@ -7,159 +7,51 @@
 // (V)]; a page is [G][16 tokens][D + V].  Query head h reads key/value
 // head h / (H / G).  The query's weights carry the scale of the scores
 // and log2(e): the softmax is over powers of two.
-#include "common.h"
+#include "window_prep.h"
 
-// One workgroup a token.  VEC: pieces of 8, each kept in registers
-// beside the piece it is rotated with (rows of up to 8192 numbers).
-#define PREP_KEEP 4
-
-struct PrepSection {  // the queries or the keys of a token
-  int off, heads;
-  const float* w;
-};
-
-template <typename T>
-__device__ __forceinline__ void rotate8(float* f, const float* other,
-                                        const float* cs, int d, int half) {
-  const bool low = d < half;
-  const int i = low ? d : d - half;
-  float c[8], s[8];
-  load8(cs + i, c);
-  load8(cs + half + i, s);
-#pragma unroll
-  for (int j = 0; j < 8; ++j)
-    f[j] = low ? f[j] * c[j] - other[j] * s[j] : f[j] * c[j] + other[j] * s[j];
+// Four tokens a workgroup, a wave each.
+template <int KQ, int KK>
+__global__ __launch_bounds__(256) void window_prep_wave_kernel(WindowPrep a) {
+  const int t =
+      blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE);
+  if (t < a.n_tok) window_prep_wave<bf16_t, KQ, KK>(a, t);
 }
 
-template <typename T, int KEEP>
-__global__ __launch_bounds__(256) void window_prep_vec_kernel(
-    T* __restrict__ proj, int ld, T* __restrict__ cache, PrepSection q,
-    PrepSection k, int v_off, int D, int V, int rot,
-    const float* __restrict__ cos_sin, float eps,
-    const int* __restrict__ pos_, const int* __restrict__ row_,
-    const int* __restrict__ bt, int max_blocks) {
-  __shared__ float red[2][4];
-  const int t = blockIdx.x, tid = threadIdx.x;
-  const int pos = pos_[t], G = k.heads;
-  T* src = proj + (size_t)t * ld;
-  const int page = bt[(size_t)row_[t] * max_blocks + pos / PAGE];
-  T* rows = cache + ((size_t)page * G * PAGE + pos % PAGE) * (D + V);
-  const size_t head_step = (size_t)PAGE * (D + V);
-  const int half = rot / 2, per_head = D / 8;
-
-  float own[KEEP][8], other[KEEP][8], kown[8], kother[8];
-  float ssq = 0.f, kssq = 0.f;
-  auto fetch = [&](int off, int i, float* a, float* b) {
-    const int d = i % per_head * 8;
-    load8(src + off + i * 8, a);
-    if (d < rot) load8(src + off + i * 8 + (d < half ? half : -half), b);
-  };
-  const int nq = q.heads * per_head, nk = G * per_head;
-#pragma unroll
-  for (int n = 0; n < KEEP; ++n) {
-    const int i = tid + n * 256;
-    if (i < nq) {
-      fetch(q.off, i, own[n], other[n]);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) ssq += own[n][j] * own[n][j];
-    }
-  }
-  // keys are not changed in place: their first piece is kept, the rest
-  // is read again
-  if (tid < nk) fetch(k.off, tid, kown, kother);
-  for (int i = tid; i < nk; i += 256) {
-    float f[8];
-    if (i != tid) load8(src + k.off + i * 8, f);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const float x = i == tid ? kown[j] : f[j];
-      kssq += x * x;
-    }
-  }
-  for (int i = tid; i < G * (V / 8); i += 256) {
-    const int g = i / (V / 8), d = i % (V / 8) * 8;
-    float f[8];
-    load8(src + v_off + i * 8, f);
-    store8(rows + g * head_step + D + d, f);
-  }
-  ssq = wave_sum(ssq);
-  kssq = wave_sum(kssq);
-  if ((tid & 63) == 0) {
-    red[0][tid / WAVE] = ssq;
-    red[1][tid / WAVE] = kssq;
-  }
-  __syncthreads();
-  const float rq = 1.f / sqrtf((red[0][0] + red[0][1] + red[0][2] +
-                                red[0][3]) / (q.heads * D) + eps);
-  const float rk = 1.f / sqrtf((red[1][0] + red[1][1] + red[1][2] +
-                                red[1][3]) / (G * D) + eps);
-  const float* cs = cos_sin + (size_t)pos * rot;
-  auto finish = [&](const float* w, float r, int i, float* a, float* b) {
-    const int d = i % per_head * 8;
-    float f[8];
-    load8(w + i * 8, f);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) a[j] *= r * f[j];
-    if (d >= rot) return;
-    load8(w + i * 8 + (d < half ? half : -half), f);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) b[j] *= r * f[j];
-    rotate8<T>(a, b, cs, d, half);
-  };
-#pragma unroll
-  for (int n = 0; n < KEEP; ++n) {
-    const int i = tid + n * 256;
-    if (i < nq) {
-      finish(q.w, rq, i, own[n], other[n]);
-      store8(src + q.off + i * 8, own[n]);
-    }
-  }
-  for (int i = tid; i < nk; i += 256) {
-    if (i != tid) fetch(k.off, i, kown, kother);
-    finish(k.w, rk, i, kown, kother);
-    store8(rows + i / per_head * head_step + i % per_head * 8, kown);
-  }
-}
-
-// Any sizes: the section's normed numbers go through LDS.
+// Any sizes, a workgroup a token: the section's normed numbers go through LDS.
 template <typename T>
-__global__ __launch_bounds__(256) void window_prep_kernel(
-    T* __restrict__ proj, int ld, T* __restrict__ cache, PrepSection q,
-    PrepSection k, int v_off, int D, int V, int rot,
-    const float* __restrict__ cos_sin, float eps,
-    const int* __restrict__ pos_, const int* __restrict__ row_,
-    const int* __restrict__ bt, int max_blocks) {
+__global__ __launch_bounds__(256) void window_prep_kernel(WindowPrep a) {
   extern __shared__ float lds[];
   __shared__ float red[2][4];
   const int t = blockIdx.x, tid = threadIdx.x;
-  const int pos = pos_[t], G = k.heads;
-  T* src = proj + (size_t)t * ld;
-  const int page = bt[(size_t)row_[t] * max_blocks + pos / PAGE];
-  T* rows = cache + ((size_t)page * G * PAGE + pos % PAGE) * (D + V);
+  const int pos = a.pos[t], G = a.G, D = a.D, V = a.V, rot = a.rot;
+  T* src = (T*)a.proj + (size_t)t * a.ld;
+  const int page = a.bt[(size_t)a.row[t] * a.max_blocks + pos / PAGE];
+  T* rows = (T*)a.cache + ((size_t)page * G * PAGE + pos % PAGE) * (D + V);
   const size_t head_step = (size_t)PAGE * (D + V);
   const int half = rot / 2;
-  const float* cs = cos_sin + (size_t)pos * rot;
+  const float* cs = a.cos_sin + (size_t)pos * rot;
   for (int i = tid; i < G * V; i += 256)
-    rows[i / V * head_step + D + i % V] = src[v_off + i];
+    rows[i / V * head_step + D + i % V] = src[a.v_off + i];
 #pragma unroll
   for (int s = 0; s < 2; ++s) {
-    const PrepSection sec = s == 0 ? q : k;
-    const int n = sec.heads * D;
+    const int off = s == 0 ? 0 : a.k_off;
+    const float* w = s == 0 ? a.wq : a.wk;
+    const int n = (s == 0 ? a.H : G) * D;
     float ssq = 0.f;
     for (int i = tid; i < n; i += 256) {
-      const float x = to_f(src[sec.off + i]);
+      const float x = to_f(src[off + i]);
       ssq += x * x;
     }
-    const float r = 1.f / sqrtf(block_sum_256(ssq, red[s]) / n + eps);
+    const float r = 1.f / sqrtf(block_sum_256(ssq, red[s]) / n + a.eps);
     for (int i = tid; i < n; i += 256)
-      lds[i] = to_f(src[sec.off + i]) * r * sec.w[i];
+      lds[i] = to_f(src[off + i]) * r * w[i];
     __syncthreads();
     for (int i = tid; i < n; i += 256) {
       const int d = i % D;
       float x = lds[i];
       if (d < half) x = x * cs[d] - lds[i + half] * cs[half + d];
       else if (d < rot) x = x * cs[d - half] + lds[i - half] * cs[d];
-      T* dst = s == 0 ? src + sec.off + i : rows + i / D * head_step + d;
+      T* dst = s == 0 ? src + off + i : rows + i / D * head_step + d;
       *dst = from_f<T>(x);
     }
     __syncthreads();
@@ -264,30 +156,30 @@ int hy_window_prep(void* proj, int ld, void* cache, int k_off, int v_off,
                    const void* wk, const void* cos_sin, float eps,
                    const void* pos, const void* row, const void* bt,
                    int max_blocks, int n_tok, int dtype, void* stream) {
-  if (H <= 0 || G <= 0 || D <= 0 || V <= 0 || rot < 0 || rot > D || rot % 2 ||
-      (rot > 0 && !cos_sin) || H * D > 16384 || G * D > 16384)
-    return -2;
+  const WindowPrep a{proj,
+                     cache,
+                     (const float*)wq,
+                     (const float*)wk,
+                     (const float*)cos_sin,
+                     (const int*)pos,
+                     (const int*)row,
+                     (const int*)bt,
+                     ld, k_off, v_off, H, G, D, V, rot, max_blocks, n_tok,
+                     eps};
+  if (!window_prep_ok(a)) return -2;
   if (n_tok <= 0) return 0;
-  const PrepSection q{0, H, (const float*)wq}, k{k_off, G, (const float*)wk};
-  const bool vec = D % 8 == 0 && V % 8 == 0 && rot % 16 == 0 && ld % 8 == 0 &&
-                   k_off % 8 == 0 && v_off % 8 == 0 &&
-                   H * D <= 2048 * PREP_KEEP;
-#define ARGS                                                                 \
-  (hipStream_t)stream, (T*)proj, ld, (T*)cache, q, k, v_off, D, V, rot,      \
-      (const float*)cos_sin, eps, (const int*)pos, (const int*)row,          \
-      (const int*)bt, max_blocks
-#define GO(KEEP)                                                             \
-  HY_DTYPE(dtype, hipLaunchKernelGGL((window_prep_vec_kernel<T, KEEP>),      \
-                                     dim3(n_tok), dim3(256), 0, ARGS))
-  if (vec && H * D <= 2048) GO(1);
-  else if (vec && H * D <= 4096) GO(2);
-  else if (vec) GO(PREP_KEEP);
-  else
+  if (dtype == 0 && window_prep_wave_ok(a)) {
+#define GO(KQ, KK)                                                        \
+  hipLaunchKernelGGL((window_prep_wave_kernel<KQ, KK>),                   \
+                     dim3((n_tok + 3) / 4), dim3(256), 0,                 \
+                     (hipStream_t)stream, a)
+    WINDOW_PREP_UNITS(H * D, G * D);
+#undef GO
+  } else {
     HY_DTYPE(dtype, hipLaunchKernelGGL(
         window_prep_kernel<T>, dim3(n_tok), dim3(256),
-        (H > G ? H : G) * D * sizeof(float), ARGS));
-#undef GO
-#undef ARGS
+        (H > G ? H : G) * D * sizeof(float), (hipStream_t)stream, a));
+  }
   HY_CHECK();
   return 0;
 }

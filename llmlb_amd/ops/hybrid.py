@@ -519,6 +519,44 @@ def window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk,
         "hy_window_prep")
 
 
+def window_front(prep, routing, act=None):
+    """``window_prep(*prep)``, ``route(*routing)`` and, with ``act``,
+    ``squared_relu(*act)`` of columns of the same ``proj``: what a
+    parallel layer does between its input projections and its attention,
+    in one launch.  Returns what ``route`` does."""
+    proj = prep[0]
+    if proj.is_cuda:
+        (proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk, eps,
+         cos_sin, b, cache) = prep
+        h, w, top, groups, keep, scale, lists = routing
+        out, u = act or (None, None)
+        u_off = ff = ld_act = 0
+        if act:
+            assert out.stride(1) == 1 and out.shape == u.shape \
+                and u.stride() == proj.stride() and u.dtype == proj.dtype
+            u_off = (u.data_ptr() - proj.data_ptr()) // proj.element_size()
+            ff, ld_act = u.shape[1], out.stride(0)
+        assert proj.stride(1) == 1 and wq.numel() == heads * dim \
+            and wk.numel() == kv_heads * dim and h.shape[0] == b.n_tok
+        index, weight, counts, pairs = _routing_buffers(h, w, top, lists)
+        bt = b.block_tables
+        done = native().hy_window_front(
+            _ptr(index), _ptr(weight), _p(counts), _p(pairs), _ptr(h),
+            _ptr(w), _i(h.shape[1]), _i(w.shape[0]), _i(top), _i(groups),
+            _i(keep), _f(scale), _ptr(proj), _i(proj.stride(0)), _ptr(cache),
+            _i(k_off), _i(v_off), _i(heads), _i(kv_heads), _i(dim), _i(vdim),
+            _i(rot), _ptr(wq), _ptr(wk), _p(cos_sin), _f(eps), _ptr(b.pos),
+            _ptr(b.row), _ptr(bt), _i(bt.shape[1]), _p(out), _i(ld_act),
+            _i(u_off), _i(ff), _i(b.n_tok), _dt(proj.dtype), _stream())
+        if done == 1:
+            return index, weight, (counts, pairs) if lists else None
+        _check(done, "hy_window_front")
+    window_prep(*prep)
+    if act:
+        squared_relu(*act)
+    return route(*routing)
+
+
 def can_window_mfma(dtype, group, dim, vdim) -> bool:
     """Sizes that the matrix-core kernels take."""
     return (dtype == torch.bfloat16 and dim % 8 == 0 and vdim % 8 == 0
@@ -529,7 +567,7 @@ def window_parts(n: int, kv_heads: int, group: int, keys: int) -> int:
     """How many workgroups share one query's keys: enough to fill the
     chip, with at least two tiles of keys each."""
     groups = n * kv_heads * ((group + 15) // 16)
-    return max(1, min(1024 // groups, keys // 128, 64))
+    return max(1, min(256 // groups, keys // 128, 64))
 
 
 def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
@@ -577,12 +615,25 @@ def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
 
 # -- mixture of experts ----------------------------------------------------
 
-FEW_PAIRS = 1024     # (token, choice) pairs that need no lists of experts
+FEW_PAIRS = 512      # (token, choice) pairs that need no lists of experts
 
 
 def can_expert_mfma(dtype, width, ff) -> bool:
     """Sizes that the matrix-core kernels take."""
     return dtype == torch.bfloat16 and width % 8 == 0 and ff % 8 == 0
+
+
+def _routing_buffers(h, w, top, lists: bool):
+    T, E = h.shape[0], w.shape[0]
+    assert h.is_contiguous() and w.is_contiguous() \
+        and w.shape[1] == h.shape[1] and w.dtype == h.dtype
+    index = torch.empty(T, top, dtype=torch.int32, device=h.device)
+    weight = torch.empty(T, top, dtype=torch.float32, device=h.device)
+    if not lists:
+        return index, weight, None, None
+    return (index, weight,
+            torch.zeros(E, dtype=torch.int32, device=h.device),
+            torch.empty(E, T, dtype=torch.int32, device=h.device))
 
 
 def route(h, w, top, groups, keep, scale, lists: bool = True):
@@ -595,18 +646,22 @@ def route(h, w, top, groups, keep, scale, lists: bool = True):
         return *ref.route(h, w, top, groups, keep, scale), None
     T, W = h.shape
     E = w.shape[0]
-    assert h.is_contiguous() and w.is_contiguous() and w.shape[1] == W
-    index = torch.empty(T, top, dtype=torch.int32, device=h.device)
-    weight = torch.empty(T, top, dtype=torch.float32, device=h.device)
-    counts = pairs = None
-    if lists:
-        counts = torch.zeros(E, dtype=torch.int32, device=h.device)
-        pairs = torch.empty(E, T, dtype=torch.int32, device=h.device)
+    index, weight, counts, pairs = _routing_buffers(h, w, top, lists)
     _check(native().hy_route(
         _ptr(index), _ptr(weight), _p(counts), _p(pairs), _ptr(h), _ptr(w),
         _i(W), _i(E), _i(top), _i(groups), _i(keep), _f(scale), _i(T),
         _dt(h.dtype), _stream()), "hy_route")
     return index, weight, (counts, pairs) if lists else None
+
+
+def expert_tile(pairs: int, experts: int, n: int, k: int) -> int:
+    """Tile of ``hy_expert_tiles`` for products of depth k with n
+    outputs: 128 x 128 where experts have few pairs or outputs, 256 x 256
+    for deep products, 128 x 256 (two a compute unit, so that one stores
+    while the other multiplies) for shallow ones."""
+    if pairs < 192 * experts or n <= 256:
+        return 0
+    return 1 if k > 1024 else 2
 
 
 def experts(h, index, lists, w_up, w_down):
@@ -634,10 +689,12 @@ def experts(h, index, lists, w_up, w_down):
         return z
     where = (_ptr(lists[0]), _ptr(lists[1]))
     tiles = can_expert_mfma(h.dtype, W, F)
-    for data, size in ((up, up_size), (down, down_size)):
+    for data, size, n, k in ((up, up_size, F, W), (down, down_size, W, F)):
         args = (*data, *where, *size, _i(T), _i(T * top))
         if tiles:
-            _check(lib.hy_expert_tiles(*args, st), "hy_expert_tiles")
+            _check(lib.hy_expert_tiles(
+                *args, _i(expert_tile(T * top, E, n, k)), st),
+                "hy_expert_tiles")
         else:
             _check(lib.hy_expert_rows(*args, _dt(h.dtype), st),
                    "hy_expert_rows")

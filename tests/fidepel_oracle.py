@@ -102,6 +102,28 @@ def routing(h, w_router, router):
     return out
 
 
+def margins(h, w_router, router):
+    """By how much each token's choice of experts is clear, as the ratio
+    of scores (logarithm): between the last expert taken and the first
+    one left, and between the last group kept and the next."""
+    out = []
+    count = (router.get("groups") or {}).get("count", 1)
+    keep = (router.get("groups") or {}).get("keep", 1)
+    for z in h @ w_router.T:
+        chosen = choose(torch.softmax(z, -1), router["top"],
+                        router.get("groups"))
+        best = z.view(count, -1).amax(-1).sort(descending=True).values
+        gaps = [best[keep - 1] - best[keep]] if keep < count else []
+        size = z.numel() // count
+        open_ = z.view(count, -1).amax(-1) >= best[keep - 1]
+        rest = [z[e] for e in range(z.numel())
+                if open_[e // size] and e not in chosen]
+        if rest:
+            gaps.append(z[chosen[-1]] - max(rest))
+        out.append(float(min(gaps)) if gaps else float("inf"))
+    return torch.tensor(out)
+
+
 def mixture(h, w, p, mlp):
     y = torch.zeros_like(h)
     picks = routing(h, w[p + "router"], mlp["router"])
@@ -127,18 +149,25 @@ def layer_runs(cfg):
             + list(range(loop["stop"], n)))
 
 
-def forward(tokens, w, cfg, layers_out=None):
-    """Logits [T, vocab] in double precision."""
+def forward(tokens, w, cfg, layers_out=None, clear=None):
+    """Logits [T, vocab] in double precision.  ``clear`` (a list) gets
+    every position's smallest margin over all layer runs."""
     w = {k: t.to(F64) for k, t in w.items()}
     eps, mult = cfg["norm"]["eps"], cfg["residual_mult"]
     x = w["embed"][torch.tensor(tokens, dtype=torch.long)]
+    least = torch.full((len(tokens),), float("inf"))
     for i in layer_runs(cfg):
         layer = cfg["layers"][i]
         h = rms(x, eps) * w[f"l{i}.norm1"]
         y = attention(h, w, f"l{i}.mix.", layer["mixer"], eps)
         if layer.get("mlp") is not None:
             y = y + mixture(h, w, f"l{i}.mlp.", layer["mlp"])
+            if clear is not None:
+                least = torch.minimum(least, margins(
+                    h, w[f"l{i}.mlp.router"], layer["mlp"]["router"]))
         x = x + mult * y
         if layers_out is not None:
             layers_out.append(x)
+    if clear is not None:
+        clear.extend(least.tolist())
     return (rms(x, eps) * w["final.norm"]) @ w["head"].T
