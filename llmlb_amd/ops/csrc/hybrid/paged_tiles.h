@@ -61,9 +61,9 @@ struct Stage {
       const int r = p / VR, d = p % VR * 8;
       pv[i] = *reinterpret_cast<const u32x4*>(row(r, pg) + MAPS * D +
                                               (d < V ? d : 0));
-      // columns past V are dropped; rows past the last key meet zero
-      // weights and must be finite
-      if (j0 + r > last_key) pv[i] = u32x4{0, 0, 0, 0};
+      // columns past V are zeros; rows past the last key meet zero weights
+      // and must be finite
+      if (j0 + r > last_key || d >= V) pv[i] = u32x4{0, 0, 0, 0};
     }
   }
   static __device__ __forceinline__ void store(unsigned short* lk,
