@@ -245,7 +245,7 @@ def test_pages_of_others_do_not_matter():
 
 # experts, choices a token, (groups, kept), width, tokens: up to 16, 32, 64
 # and 256 experts in the matrix-core kernel, more in the general one
-ROUTES = [(3, 1, (1, 1), 24, 5), (12, 4, (3, 2), 200, 70),
+ROUTES = [(3, 1, (1, 1), 24, 5), (15, 4, (5, 3), 200, 70),
           (16, 16, (1, 1), 1000, 33), (20, 6, (5, 3), 264, 129),
           (32, 2, (8, 2), 64, 16), (64, 8, (8, 4), 520, 50),
           (63, 5, (9, 9), 128, 17), (70, 3, (7, 3), 96, 40),
@@ -301,7 +301,7 @@ def test_route_survives_numbers_that_are_none():
 
 # experts, choices, width, ff, tokens: depths and heights with and without
 # remainders, experts with no pair, one pair and many
-EXPERTS = [(4, 2, 64, 32, 1), (12, 4, 256, 96, 60), (5, 1, 72, 40, 130),
+EXPERTS = [(4, 2, 64, 32, 1), (14, 5, 264, 88, 60), (5, 1, 72, 40, 130),
            (3, 3, 200, 264, 90), (16, 4, 128, 136, 700), (8, 2, 320, 520, 64),
            (40, 3, 48, 8, 33), (2, 1, 1032, 24, 300)]
 
