@@ -122,16 +122,18 @@ class PageSpec:
 @dataclass(frozen=True)
 class StateSpec:
     """A recurrent layer: per sequence a float state of
-    heads x vdim x dim and the last ``taps`` inputs of ``channels``
-    convolved channels (both 0: no convolution)."""
+    heads x vdim x dim, the last ``taps`` inputs of ``channels``
+    convolved channels (both 0: no convolution), and ``extra`` more
+    floats a head."""
     heads: int
     vdim: int
     dim: int
     channels: int
     taps: int
+    extra: int = 0
 
     def slot_bytes(self, esize: int) -> int:
-        return (4 * self.heads * self.vdim * self.dim
+        return (4 * self.heads * (self.vdim * self.dim + self.extra)
                 + esize * self.taps * self.channels)
 
 
@@ -151,7 +153,7 @@ class HybridCache(PagePool):
     def __init__(self, specs, num_blocks: int, slots: int, device, dtype):
         super().__init__(num_blocks)
         self.slots = slots
-        self.pages, self.state, self.ring = {}, {}, {}
+        self.pages, self.state, self.ring, self.extra = {}, {}, {}, {}
         for i, s in enumerate(specs):
             if isinstance(s, PageSpec):
                 self.pages[i] = torch.zeros(num_blocks, BLOCK_SIZE, s.width,
@@ -162,6 +164,9 @@ class HybridCache(PagePool):
                     dtype=torch.float32, device=device)
                 self.ring[i] = torch.zeros(slots + 1, s.taps, s.channels,
                                            dtype=dtype, device=device)
+                self.extra[i] = torch.zeros(
+                    slots + 1, s.heads, s.extra, dtype=torch.float32,
+                    device=device)
 
     @staticmethod
     def block_bytes(specs, dtype) -> int:

@@ -51,15 +51,31 @@ def _stack_rows(parts, align: int = 8):
     return torch.cat(rows).contiguous(), offs
 
 
+def _halves(dim: int, rot: int) -> torch.Tensor:
+    """Order of a head's ``dim`` numbers that takes neighbours (2i, 2i+1)
+    of the first ``rot`` to places i and i + rot/2, where the kernels
+    rotate pairs.  Scores do not change when queries and keys share an
+    order."""
+    order = torch.arange(dim)
+    order[:rot] = torch.cat([torch.arange(0, rot, 2),
+                             torch.arange(1, rot, 2)])
+    return order
+
+
 class LatentAttention(nn.Module):
     """Multi-head attention whose keys and values are linear maps of one
     cached latent per token, plus a rotated key part shared by the
     heads.  ``kv_from`` names the layer whose latents this one reads
-    (None: its own)."""
+    (None: its own).  ``interleaved``: neighbouring numbers turn
+    together.  ``sink``: the softmax has a learned score per head without
+    a key.  ``gate``: the heads' outputs are multiplied with the sigmoid
+    of a projection of the layer's input."""
 
     def __init__(self, *, width, heads, dim, rot_dim, vdim, kv_rank, scale,
-                 window, kv_from, eps, dtype, device):
+                 window, kv_from, eps, dtype, device, interleaved=False,
+                 sink=False, gate=False):
         super().__init__()
+        self.interleaved, self.sink, self.gate = interleaved, sink, gate
         self.heads, self.dim, self.rot, self.vdim = heads, dim, rot_dim, vdim
         self.rank, self.scale, self.kv_from = kv_rank, scale, kv_from
         self.window = min(window or FULL_CONTEXT, FULL_CONTEXT)
@@ -77,15 +93,35 @@ class LatentAttention(nn.Module):
         if self.kv_from is None:
             out["dkv"] = (R + self.rot, self.width)
             out["dkv.norm"] = (R,)
+        if self.sink:
+            out["sink"] = (H,)
+        if self.gate:
+            out["g"] = (H * self.vdim, self.width)
         return out
 
     def load(self, w: dict[str, torch.Tensor]) -> None:
         to = dict(dtype=self.dtype, device=self.device)
         own = self.kv_from is None
-        stacked, offs = _stack_rows(
-            [w["q"], w["dkv"]] if own else [w["q"]])
+        parts = {"q": w["q"]}
+        if own:
+            parts["dkv"] = w["dkv"]
+        if self.interleaved:
+            turn = self.dim + _halves(self.rot, self.rot)
+            order = torch.cat([torch.arange(self.dim), turn])
+            parts["q"] = w["q"].view(self.heads, -1, self.width)[
+                :, order].reshape(w["q"].shape)
+            if own:
+                parts["dkv"] = w["dkv"][torch.cat(
+                    [torch.arange(self.rank), turn - self.dim + self.rank])]
+        if self.gate:
+            parts["g"] = w["g"]
+        stacked, offs = _stack_rows(list(parts.values()))
+        offs = dict(zip(parts, offs))
         self.w_in = _param(stacked.to(**to))
-        self.c_off = offs[1] if own else 0
+        self.c_off = offs.get("dkv", 0)
+        self.g_off = offs.get("g")
+        self.w_sink = _param(w["sink"].float().to(self.device).contiguous()) \
+            if self.sink else None
         self.w_uk = _param(w["uk"].reshape(
             self.heads, self.dim, self.rank).to(**to).contiguous())
         uv = w["uv"].reshape(self.heads, self.vdim, self.rank).to(**to)
@@ -114,13 +150,13 @@ class LatentAttention(nn.Module):
             o = torch.empty(T, self.heads * self.vdim, dtype=x.dtype,
                             device=x.device)
             if n:
-                o[:n] = self._absorbed(proj, b, pages, n)
+                self._absorbed(proj, b, pages, n, o[:n])
             hy.latent_flash(o, proj, self.heads, self.dim, self.rot,
                             self.w_uk, self.w_uv, pages, b, self.window,
-                            self.scale)
+                            self.scale, self.w_sink, self.g_off)
         return _linear(o, self.w_o)
 
-    def _absorbed(self, proj, b, pages, n):
+    def _absorbed(self, proj, b, pages, n, out=None):
         """The first n tokens of the batch -> [n, heads * vdim]."""
         H, D = self.heads, self.dim
         q = proj[:n, :H * (D + self.rot)].unflatten(
@@ -129,9 +165,16 @@ class LatentAttention(nn.Module):
         attend = hy.latent_decode if self.tiled and proj.is_cuda \
             else hy.latent_rows
         lat = attend(qa, proj, D, self.rot, pages, b, self.window,
-                     self.scale)
+                     self.scale, self.w_sink)
         o = torch.bmm(lat, self.w_uv_t)                 # [H, n, vdim]
-        return o.transpose(0, 1).reshape(n, H * self.vdim)
+        if self.gate:
+            if out is None:
+                out = torch.empty(n, H * self.vdim, dtype=o.dtype,
+                                  device=o.device)
+            hy.join_heads(out, o, proj, self.g_off)
+            return out
+        o = o.transpose(0, 1).reshape(n, H * self.vdim)
+        return o if out is None else out.copy_(o)
 
 
 class ChannelDelta(nn.Module):
@@ -199,12 +242,16 @@ class ChannelDelta(nn.Module):
 
 
 class DenseFF(nn.Module):
-    """down(gelu(up x)), the tanh form of gelu."""
+    """down(act(up x)); ``act``: "gelu" (its tanh form) or "relu2", the
+    square of relu."""
 
-    def __init__(self, *, width, ff, dtype, device):
+    def __init__(self, *, width, ff, dtype, device, act="gelu"):
         super().__init__()
+        if act not in ("gelu", "relu2"):
+            raise ValueError(f"unknown activation '{act}'")
         self.width, self.ff, self.dtype, self.device = \
             width, ff, dtype, device
+        self.act = act
 
     def weight_shapes(self) -> dict[str, tuple]:
         return {"up": (self.ff, self.width), "down": (self.width, self.ff)}
@@ -215,7 +262,12 @@ class DenseFF(nn.Module):
         self.w_down = _param(w["down"].to(**to))
 
     def forward(self, x):
-        return _linear(hy.gelu_tanh_(_linear(x, self.w_up)), self.w_down)
+        u = _linear(x, self.w_up)
+        if self.act == "gelu":
+            hy.gelu_tanh_(u)
+        else:
+            hy.squared_relu(u, u)
+        return _linear(u, self.w_down)
 
 
 class DifferentialAttention(nn.Module):
@@ -456,6 +508,147 @@ class WindowedAttention(nn.Module):
     def inner(self, proj, b, cache, index: int, out) -> None:
         hy.window_prep(*self.prep(proj, b, cache, index))
         self.attend(proj, b, cache, index, out)
+
+
+class GroupedAttention(nn.Module):
+    """Causal attention with grouped key/value heads, over the last
+    ``window`` tokens or (``chunk``) those of the query's own run of
+    ``window`` positions (None: all).  Queries and keys are normed per
+    head and rotated on the first ``rot`` numbers of each; with
+    ``interleaved`` neighbouring numbers turn together.  ``bias``: their
+    projections have biases.  ``tied``: the values are the keys as
+    projected, before norm and rotation.  ``cos_sin`` ([max_pos, rot]) is
+    set by the model."""
+
+    def __init__(self, *, width, heads, kv_heads, dim, vdim, rot, scale,
+                 window, chunk, bias, tied, interleaved, eps, dtype, device):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if rot % 2 or not 0 <= rot <= dim:
+            raise ValueError("rotated dimensions must be even and at most "
+                             "the head size")
+        if window is not None and window < 1:
+            raise ValueError("a window or chunk holds at least one token")
+        if tied and vdim != dim:
+            raise ValueError("values that are the keys have their size")
+        self.heads, self.kv_heads, self.dim, self.vdim = \
+            heads, kv_heads, dim, vdim
+        self.rot, self.scale = rot, scale
+        self.window = min(window or FULL_CONTEXT, FULL_CONTEXT)
+        self.chunk = chunk and window is not None
+        self.bias, self.tied, self.interleaved = bias, tied, interleaved
+        self.eps, self.width = eps, width
+        self.dtype, self.device = dtype, device
+        self.cos_sin = None
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, H, G, D, V = (self.width, self.heads, self.kv_heads, self.dim,
+                         self.vdim)
+        out = {"q": (H * D, W), "k": (G * D, W), "q.norm": (D,),
+               "k.norm": (D,), "o": (W, H * V)}
+        if self.bias:
+            out.update({"q.b": (H * D,), "k.b": (G * D,)})
+        if not self.tied:
+            out["v"] = (G * V, W)
+        return out
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        D = self.dim
+        order = _halves(D, self.rot) if self.interleaved \
+            else torch.arange(D)
+
+        def heads_in(t):
+            """Rows of every head in the kernels' order."""
+            return t.reshape(-1, D, *t.shape[1:])[:, order].reshape(t.shape)
+
+        def wide(t):
+            return _param(t.float().to(self.device).contiguous())
+
+        to = dict(dtype=self.dtype, device=self.device)
+        parts = [heads_in(w["q"]), heads_in(w["k"])]
+        if not self.tied:
+            parts.append(w["v"])
+        stacked, offs = _stack_rows(parts)
+        self.w_in = _param(stacked.to(**to))
+        self.k_off = offs[1]
+        self.v_off = None if self.tied else offs[2]
+        self.b_q = wide(heads_in(w["q.b"])) if self.bias else None
+        self.b_k = wide(heads_in(w["k.b"])) if self.bias else None
+        # the kernels' softmax is of powers of two
+        self.w_q = wide(w["q.norm"].float()[order]
+                        * (self.scale * math.log2(math.e)))
+        self.w_k = wide(w["k.norm"][order])
+        w_o = w["o"]
+        if self.tied:      # the heads' outputs are in the keys' order
+            w_o = w_o.view(self.width, -1, D)[:, :, order].reshape(w_o.shape)
+        self.w_o = _param(w_o.to(**to).contiguous())
+
+    def cache_spec(self):
+        return PageSpec(self.kv_heads * (self.dim + self.vdim))
+
+    def forward(self, x, b, cache, index: int):
+        H, G, D, V = self.heads, self.kv_heads, self.dim, self.vdim
+        proj, pages = _linear(x, self.w_in), cache.pages[index]
+        hy.head_prep(proj, H, G, D, V, self.rot, self.k_off, self.v_off,
+                     self.b_q, self.b_k, self.w_q, self.w_k, self.eps,
+                     self.cos_sin, b, pages)
+        o = torch.empty(x.shape[0], H * V, dtype=x.dtype, device=x.device)
+        hy.window_attention(o, proj, None, H, G, D, V, pages, b, self.window,
+                            self.chunk)
+        return _linear(o, self.w_o)
+
+
+class MatrixMemory(nn.Module):
+    """mLSTM: S <- exp(f) S + exp(i) k v^T with a normaliser n of the same
+    gates, o = S^T q / max(|n . q|, 1), kept in range by a running
+    maximum of the gates' logarithms; i = cap tanh(. / cap) and
+    f = log sigmoid(cap tanh(. / cap)).  Each head's output is normed,
+    weighted and gated."""
+
+    def __init__(self, *, width, heads, dim, vdim, gate_cap, eps, dtype,
+                 device):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.cap = \
+            heads, dim, vdim, gate_cap
+        self.eps, self.width = eps, width
+        self.dtype, self.device = dtype, device
+
+    def weight_shapes(self) -> dict[str, tuple]:
+        W, H = self.width, self.heads
+        n, v = H * self.dim, H * self.vdim
+        return {"q": (n, W), "k": (n, W), "v": (v, W), "g": (v, W),
+                "i": (H, W), "f": (H, W), "i.b": (H,), "f.b": (H,),
+                "norm": (v,), "o": (W, v)}
+
+    def load(self, w: dict[str, torch.Tensor]) -> None:
+        to = dict(dtype=self.dtype, device=self.device)
+        stacked, offs = _stack_rows(
+            [w["q"], w["k"], w["v"], w["g"], torch.cat([w["i"], w["f"]])])
+        self.w_in = _param(stacked.to(**to))
+        _, self.k_off, self.v_off, self.g_off, self.i_off = offs
+
+        def wide(t):
+            return _param(t.float().to(self.device).contiguous())
+
+        self.b_gate = wide(torch.stack([w["i.b"], w["f.b"]]))
+        self.w_norm = wide(w["norm"])
+        self.w_o = _param(w["o"].to(**to))
+
+    def cache_spec(self):
+        return StateSpec(self.heads, self.vdim, self.dim, 0, 0,
+                         hy.memory_extra(self.dim))
+
+    def forward(self, x, b, cache, index: int):
+        proj = _linear(x, self.w_in)
+        o = torch.empty(x.shape[0], self.heads * self.vdim, dtype=x.dtype,
+                        device=x.device)
+        hy.matrix_memory(o, proj, self.k_off, self.v_off, self.g_off,
+                         self.i_off, self.b_gate, self.cap,
+                         cache.state[index], cache.extra[index], b,
+                         self.w_norm, self.heads, self.dim, self.vdim,
+                         self.eps)
+        return _linear(o, self.w_o)
 
 
 class RoutedExperts(nn.Module):

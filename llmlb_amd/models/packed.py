@@ -6,8 +6,10 @@ feed-forward ``ff``, which may be None), loads their weights and
 implements ``forward``.  Tensor names: ``embed``, ``head``,
 ``final.norm``, and per layer ``l<i>.norm1``, ``l<i>.mix.*``,
 ``l<i>.norm2`` (where mixer and feed-forward have norms of their own),
+``l<i>.norm1b`` and ``l<i>.norm2b`` (where their outputs are normed too),
 ``l<i>.mlp.*``.  ``runs`` lists the layer index of every layer run of a
-forward pass; each run has its own part of the cache.
+forward pass; each run has its own part of the cache.  ``owners`` lists
+the layers that have tensors.
 """
 from __future__ import annotations
 
@@ -43,6 +45,8 @@ class PackedCausalLM(nn.Module):
     ragged = True
     norm_offset = 0.0          # what a stored norm weight is added to
     shared_norm = False        # one norm for mixer and feed-forward
+    output_norms = False       # sublayers' outputs are normed as well
+    centred_norms = False      # layer norms instead of RMS norms
 
     def __init__(self, cfg, tp: TPContext | None, dtype: torch.dtype,
                  device):
@@ -65,10 +69,14 @@ class PackedCausalLM(nn.Module):
         """Names (without ``l<i>.``) and shapes of layer i's tensors."""
         ly = self.layers_[i]
         out = {"norm1": self.norm_shape}
+        if self.output_norms:
+            out["norm1b"] = self.norm_shape
         out.update({f"mix.{k}": s for k, s in ly.mix.weight_shapes().items()})
         if ly.ff is not None:
             if not self.shared_norm:
                 out["norm2"] = self.norm_shape
+            if self.output_norms:
+                out["norm2b"] = self.norm_shape
             out.update({f"mlp.{k}": s
                         for k, s in ly.ff.weight_shapes().items()})
         return out
@@ -86,7 +94,7 @@ class PackedCausalLM(nn.Module):
         W = self.cfg.width
         out = {"embed": (self.cfg.vocab, W), "final.norm": self.norm_shape,
                "head": (self.cfg.vocab, W)}
-        for i in range(len(self.layers_)):
+        for i in self.owners:
             for k, s in self.layer_shapes(i).items():
                 out[f"l{i}.{k}"] = s
         return out
@@ -103,7 +111,7 @@ class PackedCausalLM(nn.Module):
 
         self.embed, self.head = mat("embed"), mat("head")
         self.final_norm = vec("final.norm")
-        for i in range(len(self.layers_)):
+        for i in self.owners:
             self.load_layer(i, lambda k: take(f"l{i}.{k}"),
                             lambda k: vec(f"l{i}.{k}"))
 
@@ -140,6 +148,10 @@ class PackedCausalLM(nn.Module):
     # -- forward ----------------------------------------------------------
 
     @property
+    def owners(self) -> list[int]:
+        return list(range(len(self.layers_)))
+
+    @property
     def runs(self) -> list[int]:
         return list(range(len(self.layers_)))
 
@@ -155,7 +167,8 @@ class PackedCausalLM(nn.Module):
         """Final-norm hidden states of the rows ``index`` (int32; None:
         all) of the residual stream."""
         return hy.norm_rows(x, index, self.final_norm, self.cfg.eps,
-                            self.dtype, self.norm_offset)
+                            self.dtype, self.norm_offset,
+                            self.centred_norms)
 
     def logits(self, x: torch.Tensor, index=None) -> torch.Tensor:
         """float32 logits of the rows ``index`` (int32; None: all)."""

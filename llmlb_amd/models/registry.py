@@ -12,6 +12,7 @@ from pathlib import Path
 from .dibelix import DibelixConfig, DibelixForCausalLM
 from .fidepel import FidepelConfig, FidepelForCausalLM
 from .llama import LlamaConfig, LlamaForCausalLM
+from .rasodra import RasodraConfig, RasodraForCausalLM
 from .taletar import TaletarConfig, TaletarForCausalLM
 
 MODELS = {
@@ -19,6 +20,7 @@ MODELS = {
     DibelixConfig: DibelixForCausalLM,
     TaletarConfig: TaletarForCausalLM,
     FidepelConfig: FidepelForCausalLM,
+    RasodraConfig: RasodraForCausalLM,
 }
 
 # architectures that can be read from a model folder
@@ -26,6 +28,7 @@ FOLDERS = {
     DibelixConfig.architecture: DibelixConfig,
     TaletarConfig.architecture: TaletarConfig,
     FidepelConfig.architecture: FidepelConfig,
+    RasodraConfig.architecture: RasodraConfig,
 }
 
 PRESETS = {
@@ -44,6 +47,9 @@ PRESETS = {
     "fidepel-tiny": FidepelConfig.tiny,
     "fidepel-small": FidepelConfig.small,
     "fidepel-8b": FidepelConfig.base_8b,
+    "rasodra-tiny": RasodraConfig.tiny,
+    "rasodra-small": RasodraConfig.small,
+    "rasodra-8b": RasodraConfig.base_8b,
 }
 
 

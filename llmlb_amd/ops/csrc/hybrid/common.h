@@ -150,6 +150,21 @@ __device__ __forceinline__ size_t page_slot(const int* bt, int max_blocks,
          pos % PAGE;
 }
 
+// Which keys the query at position i sees: the last ``size`` ones, or those
+// of its own chunk of ``size`` positions.
+struct Mask {
+  int size;
+  bool chunk;
+  // how far back the first of them lies (it may be before position 0)
+  __device__ __forceinline__ int span(int i) const {
+    return chunk ? i % size : size - 1;
+  }
+  __device__ __forceinline__ int first(int i) const {
+    const int j = i - span(i);
+    return j > 0 ? j : 0;
+  }
+};
+
 #define HY_CHECK()                                  \
   do {                                              \
     if (hipGetLastError() != hipSuccess) return -1; \

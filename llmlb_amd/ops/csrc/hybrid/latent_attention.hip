@@ -5,7 +5,8 @@
 // and its value W_uv c, so with qa = W_uk^T q (the "absorbed" query)
 //   score = (qa . c + qr . kr) * scale,   out = W_uv (sum_j p_j c_j):
 // the cache is read as it is, once for all heads.  A query at position i
-// sees the keys j with 0 <= i - j < window.
+// sees the keys j with 0 <= i - j < window.  With ``sink`` (a number per
+// head) the softmax's sum also contains exp(sink), which has no value.
 //
 // Cache layout: [pages][16 tokens][rank + R].
 #include "common.h"
@@ -121,7 +122,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(
     int ld, int D, int R, int rank, const T* __restrict__ cache,
     const int* __restrict__ pos_, const int* __restrict__ row_,
     const int* __restrict__ bt, int max_blocks, int window, float scale,
-    int N) {
+    const float* __restrict__ sink, int N) {
   extern __shared__ float lds[];
   float* lq = lds;               // rank + R query numbers
   float* lacc = lds + rank + R;  // 4 waves x rank
@@ -138,6 +139,10 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(
   __syncthreads();
 
   float m = -INFINITY, l = 0.f, acc[NR];
+  if (sink && wave == 0) {
+    m = sink[h];
+    l = 1.f;
+  }
 #pragma unroll
   for (int i = 0; i < NR; ++i) acc[i] = 0.f;
   for (int j = first + wave; j <= pos; j += 4) {
@@ -183,7 +188,58 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(
   }
 }
 
+// out[t][h V ..] = o[h][t][..] sigmoid(gate[t][h V ..]), the absorbed
+// form's values side by side.  N columns a thread.
+template <typename T, int N>
+__global__ __launch_bounds__(256) void join_heads_kernel(
+    T* __restrict__ out, const T* __restrict__ o, const T* __restrict__ gate,
+    int ld, int n_tok, int H, int V) {
+  const int per = V / N;
+  const long long id = (long long)blockIdx.x * 256 + threadIdx.x;
+  if (id >= (long long)n_tok * H * per) return;
+  const int c = (int)(id % per) * N;
+  const long long th = id / per;
+  const int t = (int)(th / H), h = (int)(th - (long long)t * H);
+  const T* src = o + ((size_t)h * n_tok + t) * V + c;
+  const T* g = gate + (size_t)t * ld + (size_t)h * V + c;
+  T* dst = out + ((size_t)t * H + h) * V + c;
+  float f[N], z[N];
+  if constexpr (N == 8) {
+    load8(src, f);
+    load8(g, z);
+  } else {
+    f[0] = to_f(src[0]);
+    z[0] = to_f(g[0]);
+  }
+#pragma unroll
+  for (int i = 0; i < N; ++i) f[i] *= sigmoid_f(z[i]);
+  if constexpr (N == 8) store8(dst, f);
+  else dst[0] = from_f<T>(f[0]);
+}
+
 extern "C" {
+
+int hy_join_heads(void* out, const void* o, const void* gate, int ld,
+                  int n_tok, int H, int V, int dtype, void* stream) {
+  if (H <= 0 || V <= 0) return -2;
+  if (n_tok <= 0) return 0;
+  const uintptr_t mask = dtype == 0 ? 15 : 31;
+  const bool vec = V % 8 == 0 && ld % 8 == 0 &&
+                   (((uintptr_t)out | (uintptr_t)o | (uintptr_t)gate) &
+                    mask) == 0;
+  const long long n = (long long)n_tok * H * (V / (vec ? 8 : 1));
+  if (n >= (1ll << 38)) return -2;
+  const dim3 grid((unsigned)((n + 255) / 256)), block(256);
+#define GO(N)                                                              \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                      \
+      (join_heads_kernel<T, N>), grid, block, 0, (hipStream_t)stream,      \
+      (T*)out, (const T*)o, (const T*)gate, ld, n_tok, H, V))
+  if (vec) GO(8);
+  else GO(1);
+#undef GO
+  HY_CHECK();
+  return 0;
+}
 
 int hy_latent_prep(void* proj, int ld, int H, int D, int R, int c_off,
                    int rank, const void* w_norm, float eps,
@@ -214,8 +270,8 @@ int hy_latent_prep(void* proj, int ld, int H, int D, int R, int c_off,
 int hy_latent_rows(void* out, const void* qa, const void* proj, int ld, int H,
                    int D, int R, int rank, const void* cache, const void* pos,
                    const void* row, const void* bt, int max_blocks,
-                   int window, float scale, int n_rows, int dtype,
-                   void* stream) {
+                   int window, float scale, const void* sink, int n_rows,
+                   int dtype, void* stream) {
   if (rank <= 0 || rank > 2048 || R > 2048 || window <= 0 || H > 65535)
     return -2;
   if (n_rows <= 0) return 0;
@@ -226,7 +282,7 @@ int hy_latent_rows(void* out, const void* qa, const void* proj, int ld, int H,
       (latent_rows_kernel<T, NR>), grid, block, lds, (hipStream_t)stream,    \
       (T*)out, (const T*)qa, (const T*)proj, ld, D, R, rank,                 \
       (const T*)cache, (const int*)pos, (const int*)row, (const int*)bt,     \
-      max_blocks, window, scale, n_rows))
+      max_blocks, window, scale, (const float*)sink, n_rows))
   if (rank <= 128) GO(2);
   else if (rank <= 256) GO(4);
   else if (rank <= 512) GO(8);

@@ -47,13 +47,16 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(
 //           position of that row); key rows of an item are consecutive
 //   q   = proj + h * (D + R), kx [keys][H D], kr [keys][R],
 //   vt [H V][key_ld]  (values transposed), out [tokens][H V]
+//   sink (null: none): a number per head whose power joins the sum
+//   g_off >= 0: out times the sigmoid of proj's columns from there on
 template <int DQ, int DV>
 __global__ __launch_bounds__(256, DQ * 2 + DV <= 512 ? 2 : 1)
 void latent_flash_kernel(
     bf16_t* __restrict__ out, const bf16_t* __restrict__ proj, int ld,
     const bf16_t* __restrict__ kx, const bf16_t* __restrict__ kr,
     const bf16_t* __restrict__ vt, int key_ld, const int* __restrict__ items,
-    int H, int D, int R, int V, int window, float scale_log2) {
+    int H, int D, int R, int V, int window, float scale_log2,
+    const float* __restrict__ sink, int g_off) {
   constexpr int KD = DQ / 32, VT = DV / 16;
   constexpr int KP = DQ + 8, VP = 64 + 8;  // LDS pitches
   constexpr int KL = 64 * DQ / 8 / 256, VL = DV * 64 / 8 / 256;
@@ -125,8 +128,8 @@ void latent_flash_kernel(
   float m[2], l[2];
 #pragma unroll
   for (int a = 0; a < 2; ++a) {
-    m[a] = -1e30f;
-    l[a] = 0.f;
+    m[a] = sink ? sink[h] * LOG2E : -1e30f;
+    l[a] = sink && g == 0 ? 1.f : 0.f;
 #pragma unroll
     for (int v = 0; v < VT; ++v) o[a][v] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
@@ -230,6 +233,24 @@ void latent_flash_kernel(
     const int r = wave * 32 + a * 16 + n;
     if (r >= n_q) continue;
     bf16_t* dst = out + ((size_t)(q_row + r) * H + h) * V;
+    if (g_off >= 0) {
+      const bf16_t* gate =
+          proj + (size_t)(q_row + r) * ld + g_off + (size_t)h * V;
+#pragma unroll
+      for (int v = 0; v < VT; ++v) {
+        const int d = v * 16 + g * 4;
+        float z[4] = {0.f, 0.f, 0.f, 0.f};
+        if ((V & 3) == 0 && (g_off & 3) == 0) {
+          if (d < V) load4(gate + d, z);
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (d + i < V) z[i] = to_f(gate[d + i]);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[a][v][i] /= 1.f + __expf(-z[i]);
+      }
+    }
 #pragma unroll
     for (int v = 0; v < VT; ++v) {
       const int d = v * 16 + g * 4;
@@ -262,7 +283,8 @@ void latent_decode_kernel(
     const bf16_t* __restrict__ proj, int ld, int D, int R, int rank, int H,
     const bf16_t* __restrict__ cache, const int* __restrict__ pos_,
     const int* __restrict__ row_, const int* __restrict__ bt, int max_blocks,
-    int window, float scale_log2, int N, int parts) {
+    int window, float scale_log2, const float* __restrict__ sink, int N,
+    int parts) {
   constexpr int KD = NT * 2 + 2;         // 32-wide steps over rank + R
   constexpr int KEYS = 64 / HT, KT = KEYS / 16;
   constexpr int PITCH = KD * 32 + 8;
@@ -347,9 +369,13 @@ void latent_decode_kernel(
 
   f32x4 o[HT][NT];
   float m[HT], l = 0.f;  // m of head n per tile; l of this wave's keys
+  // the sink counts once: in the first part, with the first keys
+  const bool sunk = sink && part == 0;
+  if (sunk && kt == 0 && g == 0) l = 1.f;
 #pragma unroll
   for (int a = 0; a < HT; ++a) {
-    m[a] = -1e30f;
+    const int h = h0 + a * 16 + n;
+    m[a] = sunk ? sink[h < H ? h : 0] * LOG2E : -1e30f;
 #pragma unroll
     for (int t = 0; t < NT; ++t) o[a][t] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
@@ -497,8 +523,8 @@ static int launch_decode(void* out, void* acc, void* ml, const void* qa,
                          const void* proj, int ld, int D, int R, int rank,
                          int H, const void* cache, const void* pos,
                          const void* row, const void* bt, int max_blocks,
-                         int window, float scale, int N, int parts,
-                         hipStream_t s) {
+                         int window, float scale, const void* sink, int N,
+                         int parts, hipStream_t s) {
   constexpr int lds = (64 / HT) * ((NT * 2 + 2) * 32 + 8) * 2;
   static const hipError_t ready = hipFuncSetAttribute(
       reinterpret_cast<const void*>(latent_decode_kernel<NT, HT>),
@@ -510,7 +536,7 @@ static int launch_decode(void* out, void* acc, void* ml, const void* qa,
                      (const bf16_t*)qa, (const bf16_t*)proj, ld, D, R, rank,
                      H, (const bf16_t*)cache, (const int*)pos,
                      (const int*)row, (const int*)bt, max_blocks, window,
-                     scale * LOG2E, N, parts);
+                     scale * LOG2E, (const float*)sink, N, parts);
   HY_CHECK();
   if (parts > 1) {
     hipLaunchKernelGGL(latent_merge_kernel, dim3(N, H), block, 0, s,
@@ -539,7 +565,8 @@ int hy_latent_gather(void* c, void* kr, const void* cache, const void* blocks,
 int hy_latent_flash(void* out, const void* proj, int ld, const void* kx,
                     const void* kr, const void* vt, int key_ld,
                     const void* items, int n_items, int H, int D, int R,
-                    int V, int window, float scale, void* stream) {
+                    int V, int window, float scale, const void* sink,
+                    int g_off, void* stream) {
   if (D % 8 || R % 8 || ld % 8 || key_ld % 64 || D + R > 256 || V > 256)
     return -2;
   if (n_items <= 0) return 0;
@@ -549,7 +576,8 @@ int hy_latent_flash(void* out, const void* proj, int ld, const void* kx,
                      (hipStream_t)stream, (bf16_t*)out,                     \
                      (const bf16_t*)proj, ld, (const bf16_t*)kx,            \
                      (const bf16_t*)kr, (const bf16_t*)vt, key_ld,          \
-                     (const int*)items, H, D, R, V, window, scale * LOG2E)
+                     (const int*)items, H, D, R, V, window, scale * LOG2E,  \
+                     (const float*)sink, g_off)
   const int dq = D + R;
   if (V <= 64) {
     if (dq <= 64) GO(64, 64);
@@ -574,7 +602,7 @@ int hy_latent_decode(void* out, void* acc, void* ml, const void* qa,
                      const void* proj, int ld, int H, int D, int R, int rank,
                      const void* cache, const void* pos, const void* row,
                      const void* bt, int max_blocks, int window, float scale,
-                     int N, int parts, void* stream) {
+                     const void* sink, int N, int parts, void* stream) {
   if (rank % 8 || R % 8 || D % 8 || ld % 8 || R > 64 || rank > 512 ||
       window <= 0 || parts < 1 || parts > 65535)
     return -2;
@@ -583,11 +611,11 @@ int hy_latent_decode(void* out, void* acc, void* ml, const void* qa,
   return H <= 16                                                             \
              ? launch_decode<NT, 1>(out, acc, ml, qa, proj, ld, D, R, rank,  \
                                     H, cache, pos, row, bt, max_blocks,      \
-                                    window, scale, N, parts,                 \
+                                    window, scale, sink, N, parts,           \
                                     (hipStream_t)stream)                     \
              : launch_decode<NT, 2>(out, acc, ml, qa, proj, ld, D, R, rank,  \
                                     H, cache, pos, row, bt, max_blocks,      \
-                                    window, scale, N, parts,                 \
+                                    window, scale, sink, N, parts,           \
                                     (hipStream_t)stream)
   if (rank <= 64) GO(1);
   if (rank <= 128) GO(2);

@@ -4,7 +4,12 @@
 //  * gated linear attention: g per key channel, sigmoid(z)^(1/tau);
 //  * Mamba-2: g = exp(-rate dt) per head, v = dt x, and skip x is added to
 //    the output; q, k and x come from a short convolution, q and k serve
-//    all heads of a group.
+//    all heads of a group;
+//  * matrix memory (mLSTM): g and the weight of v from exponential gates
+//    per head, kept in range by a running maximum m; beside S a normaliser
+//    n [D], the same recurrence with v = 1, and o is divided by
+//    max(|n . q|, exp(-m)) + 1e-6.  n and m are the state's ``extra``:
+//    [slots][H][extra_row(D)], n first, m at extra_row(D) - 4.
 //
 // Tokens of several sequences lie packed one after another.  Per token:
 // pos (place in its sequence), row (its state slot), tstart (its
@@ -14,6 +19,21 @@
 // Everything that enters the state is float; q, k and v keep the storage
 // type they were projected or convolved in until they are used.
 #include "recurrent.h"
+
+enum Kind { CHANNEL, HEAD, MEMORY };  // gated linear, Mamba-2, mLSTM
+
+__host__ __device__ __forceinline__ int extra_row(int D) {
+  return (D + 3) / 4 * 4 + 4;
+}
+
+// Log input and forget gates of one head and token, cap tanh(z / cap) and
+// the logarithm of its sigmoid.
+__device__ __forceinline__ void memory_gates(float zi, float zf, float cap,
+                                             float& li, float& lf) {
+  li = cap * tanhf(zi / cap);
+  lf = -softplus_f(-cap * tanhf(zf / cap));
+}
+#define MEMORY_EPS 1e-6f
 
 // N consecutive elements as they lie in memory, widened on use, so that
 // elements in flight take half the registers and nothing waits for them.
@@ -74,8 +94,11 @@ struct Run<bf16_t, N, true> {
 // the state itself carries over from token to token; the sum over lanes
 // that makes an output is off that chain.
 //   q, k: columns q_off, k_off + group * D; v: v_off + head * V, of rows of
-//   ``in``;  g [T][H D] (CHANNEL) or [T][H];  dt [T][H] and skip [H] without CHANNEL
-template <typename T, int RPL, bool VEC, int CPL, bool CHANNEL>
+//   ``in``;  g [T][H D] (CHANNEL) or [T][H];  dt [T][H] without CHANNEL
+//   skip: [H] (HEAD), exp(-m) [T][H] (MEMORY)
+// MEMORY: every wave carries the normaliser as well, from n0 [entries][H][D];
+// one of a head's waves leaves the last one in ``extra``.
+template <typename T, int RPL, bool VEC, int CPL, Kind KIND>
 __global__ __launch_bounds__(256) void linear_scan_kernel(
     float* __restrict__ o, float* __restrict__ state,
     const T* __restrict__ in, int ld, int q_off, int k_off, int v_off,
@@ -83,7 +106,9 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
     const float* __restrict__ skip_, const int* __restrict__ e_start,
     const int* __restrict__ e_len, const int* __restrict__ e_pos,
     const int* __restrict__ e_row, int G, int H, int D, int V,
-    float q_scale) {
+    float q_scale, const float* __restrict__ n0, float* __restrict__ extra) {
+  constexpr bool CHANNEL = KIND == Kind::CHANNEL;
+  constexpr bool MEMORY = KIND == Kind::MEMORY;
   constexpr int PF = RPL <= 4 ? 32 / (CPL < 2 ? 2 : CPL)
                               : (RPL == 8 ? 4 : (RPL == 16 ? 2 : 1));
   const int e = blockIdx.y;
@@ -124,7 +149,8 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
     return reinterpret_cast<decltype(p)>(
         reinterpret_cast<const char*>(p) + bytes);
   };
-  const float skip = CHANNEL ? 0.f : skip_[head];
+  const float skip = KIND == HEAD ? skip_[head] : 0.f;
+  const float* e_rows = MEMORY ? skip_ + first * H : nullptr;
   float* out = o + (first * H + head) * V;
   float* sp = state + ((size_t)e_row[e] * H + head) * V * D;
   int cc[CPL];
@@ -132,7 +158,9 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
   for (int c = 0; c < CPL; ++c)
     cc[c] = VEC || col + c < V ? col + c : V - 1;
 
-  float S[CPL][RPL];
+  float S[CPL][RPL], N[RPL];
+  if (MEMORY)
+    load_rows<RPL, VEC>(n0 + ((size_t)e * H + head) * D, r0, D, N);
   const bool resume = e_pos[e] > 0;
 #pragma unroll
   for (int c = 0; c < CPL; ++c) {
@@ -144,7 +172,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
   constexpr int GN = CHANNEL ? RPL : 1;
   Run<T, RPL, VEC> q[PF], k[PF];
   Run<T, CPL, VEC> v[PF];
-  float g[PF][GN], dt[PF];
+  float g[PF][GN], dt[PF], floor_[MEMORY ? PF : 1];
   auto fetch = [&](int s, int t) {
     t = t < len ? t : len - 1;
     const T* row = rows + (size_t)t * ld;
@@ -156,6 +184,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
     } else {
       g[s][0] = *place(g_rows + (size_t)t * H, head_at);
       dt[s] = *place(dt_rows + (size_t)t * H, head_at);
+      if (MEMORY) floor_[s] = *place(e_rows + (size_t)t * H, head_at);
     }
     if constexpr (VEC) {
       v[s].load(place(row, v_at + col * (unsigned)sizeof(T)), CPL);
@@ -197,7 +226,16 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
 #pragma unroll
       for (int c = 1; c < CPL; ++c) mine = lane % CPL == c ? b[c] : mine;
     }
-    if (!CHANNEL) {
+    if (MEMORY) {
+      float a = 0.f;
+#pragma unroll
+      for (int i = 0; i < RPL; ++i) {
+        N[i] = N[i] * g[s][0] + k[s].get(i) * dt[s];
+        a += q[s].get(i) * N[i];
+      }
+      a = fabsf(row16_sum(a) * q_scale);
+      mine *= q_scale / (fmaxf(a, floor_[MEMORY ? s : 0]) + MEMORY_EPS);
+    } else if (!CHANNEL) {
       float xm = x[0];
 #pragma unroll
       for (int c = 1; c < CPL; ++c) xm = lane % CPL == c ? x[c] : xm;
@@ -222,6 +260,68 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
   for (int c = 0; c < CPL; ++c)
     if (col + c < V)
       store_rows<RPL, VEC>(sp + (size_t)(col + c) * D, r0, D, S[c]);
+  if (MEMORY && col == 0)
+    store_rows<RPL, VEC>(
+        extra + ((size_t)e_row[e] * H + head) * extra_row(D), r0, D, N);
+}
+
+// What matrix memory's scan needs of every token and head, one wave per
+// (head, entry): the running maximum m as a scan of max(a + ., b), 64
+// tokens at a time, then steps [3][T][H] = exp(f + m' - m), exp(i - m),
+// exp(-m).  bias [2][H]: input gates', forget gates'.  Also copies the
+// normaliser out of the state (several workgroups of the scan read it and
+// one replaces it) and leaves the last m there.
+template <typename T>
+__global__ __launch_bounds__(64) void memory_gates_kernel(
+    float* __restrict__ steps, float* __restrict__ n0,
+    float* __restrict__ extra, const T* __restrict__ proj, int ld, int i_off,
+    int f_off, const float* __restrict__ bias, const int* __restrict__ e_start,
+    const int* __restrict__ e_len, const int* __restrict__ e_pos,
+    const int* __restrict__ e_row, int n_tok, int H, int D, float cap) {
+  const int h = blockIdx.x, e = blockIdx.y, lane = threadIdx.x;
+  const int len = e_len[e], first = e_start[e];
+  const bool resume = e_pos[e] > 0;
+  float* ex = extra + ((size_t)e_row[e] * H + h) * extra_row(D);
+  for (int d = lane; d < D; d += WAVE)
+    n0[((size_t)e * H + h) * D + d] = resume ? ex[d] : 0.f;
+  float m = resume ? ex[extra_row(D) - 4] : 0.f;
+  const float bi = bias[h], bf = bias[H + h];
+  const size_t plane = (size_t)n_tok * H;
+  auto fetch = [&](int t, float& zi, float& zf) {
+    t = t < len ? t : len - 1;
+    const T* row = proj + (size_t)(first + t) * ld + h;
+    zi = to_f(row[i_off]);
+    zf = to_f(row[f_off]);
+  };
+  float zi, zf;
+  fetch(lane, zi, zf);
+  for (int t0 = 0; t0 < len; t0 += WAVE) {
+    const int t = t0 + lane;
+    float li, lf;
+    memory_gates(zi + bi, zf + bf, cap, li, lf);
+    if (t0 + WAVE < len) fetch(t + WAVE, zi, zf);
+    float a = lf, b = li;
+#pragma unroll
+    for (int o = 1; o < WAVE; o <<= 1) {
+      const float a1 = __shfl_up(a, o, WAVE), b1 = __shfl_up(b, o, WAVE);
+      if (lane >= o) {
+        b = fmaxf(b1 + a, b);
+        a += a1;
+      }
+    }
+    const float now = fmaxf(a + m, b);
+    float before = __shfl_up(now, 1, WAVE);
+    if (lane == 0) before = m;
+    if (t < len) {
+      const size_t at = (size_t)(first + t) * H + h;
+      steps[at] = expf(lf + before - now);
+      steps[plane + at] = expf(li - now);
+      steps[2 * plane + at] = expf(-now);
+    }
+    const int last = len - t0 < WAVE ? len - t0 - 1 : WAVE - 1;
+    m = __shfl(now, last, WAVE);
+  }
+  if (lane == 0) ex[extra_row(D) - 4] = m;
 }
 
 // g = sigmoid(dec + bias)^rate per channel
@@ -326,9 +426,12 @@ __global__ __launch_bounds__(256) void ring_store_kernel(
 // Decode: one token of every sequence.  One workgroup per (head,
 // sequence); the state's loads are issued first so that everything the
 // token needs is computed behind them.
-//   CONV false: gated linear attention, out = silu(gate) norm(o)
-//   CONV true: Mamba-2, y = o + skip x (gate and norm span the heads)
-template <typename T, int RPL, bool EXACT, bool CONV>
+//   CHANNEL: gated linear attention, out = silu(gate) norm(o)
+//   HEAD: Mamba-2, y = o + skip x (gate and norm span the heads)
+//   MEMORY: mLSTM, out = sigmoid(gate) norm(o); ``dec`` points to the
+//     input gates' projections (the forget gates' follow), per_head [2][H]
+//     are their biases and ``rate`` the cap
+template <typename T, int RPL, bool EXACT, Kind KIND>
 __global__ __launch_bounds__(256) void linear_step_kernel(
     T* __restrict__ out, int ld_out, float* __restrict__ y,
     float* __restrict__ state, const T* __restrict__ proj, int ld, int q_off,
@@ -336,8 +439,10 @@ __global__ __launch_bounds__(256) void linear_step_kernel(
     const float* __restrict__ dec_bias, const float* __restrict__ w_norm,
     T* __restrict__ ring, const float* __restrict__ wconv,
     const float* __restrict__ conv_bias, const float* __restrict__ per_head,
-    const int* __restrict__ pos_, const int* __restrict__ row_, int G, int H,
-    int D, int V, int taps, float q_scale, float rate, float eps) {
+    float* __restrict__ extra, const int* __restrict__ pos_,
+    const int* __restrict__ row_, int G, int H, int D, int V, int taps,
+    float q_scale, float rate, float eps) {
+  constexpr bool CONV = KIND == HEAD;
   constexpr int NU = 64 / RPL > 8 ? 8 : 64 / RPL;  // columns in flight
   constexpr int DP = 16 * RPL;
   extern __shared__ float lds[];
@@ -372,6 +477,8 @@ __global__ __launch_bounds__(256) void linear_step_kernel(
 
   const T* row = proj + (size_t)s * ld;
   float gh = 0.f, dt = 1.f, skip = 0.f;
+  float N[RPL], m = 0.f, inv = 1.f;
+  float* ex = nullptr;
   if constexpr (CONV) {
     const int C = H * V + 2 * G * D;
     T* keep = ring + ((size_t)slot * taps + pos % taps) * C;
@@ -388,6 +495,25 @@ __global__ __launch_bounds__(256) void linear_step_kernel(
     for (int j = tid; j < V; j += 256) lv[j] = conv(v_off + h * V + j);
     ssm_times(to_f(row[g_off + h]), per_head[h], per_head[H + h], dt, gh);
     skip = per_head[2 * H + h];
+  } else if constexpr (KIND == MEMORY) {
+    for (int d = tid; d < DP; d += 256) {
+      const bool ok = d < D;
+      lq[d] = ok ? to_f(row[q_off + h * D + d]) * q_scale : 0.f;
+      lk[d] = ok ? to_f(row[k_off + h * D + d]) : 0.f;
+    }
+    for (int j = tid; j < V; j += 256) lv[j] = to_f(row[v_off + h * V + j]);
+    const T* z = dec + (size_t)s * ld + h;
+    float li, lf;
+    memory_gates(to_f(z[0]) + per_head[h], to_f(z[H]) + per_head[H + h], rate,
+                 li, lf);
+    ex = extra + ((size_t)slot * H + h) * extra_row(D);
+    const float before = pos > 0 ? ex[extra_row(D) - 4] : 0.f;
+    m = fmaxf(lf + before, li);
+    gh = expf(lf + before - m);
+    dt = expf(li - m);
+#pragma unroll
+    for (int i = 0; i < RPL; ++i) N[i] = 0.f;
+    if (pos > 0) load_rows<RPL, EXACT>(ex, r0, D, N);
   } else {
     for (int d = tid; d < DP; d += 256) {
       const bool ok = d < D;
@@ -406,7 +532,19 @@ __global__ __launch_bounds__(256) void linear_step_kernel(
   for (int i = 0; i < RPL; ++i) {
     q[i] = lq[r0 + i];
     k[i] = lk[r0 + i] * dt;
-    g[i] = CONV ? gh : lg[r0 + i];
+    g[i] = KIND == CHANNEL ? lg[r0 + i] : gh;
+  }
+  if constexpr (KIND == MEMORY) {
+    // every 16 lanes make the normaliser; what it was has been read
+    float a = 0.f;
+#pragma unroll
+    for (int i = 0; i < RPL; ++i) {
+      N[i] = N[i] * gh + k[i];
+      a += q[i] * N[i];
+    }
+    inv = 1.f / (fmaxf(fabsf(row16_sum(a)), expf(-m)) + MEMORY_EPS);
+    if (tid < 16) store_rows<RPL, EXACT>(ex, r0, D, N);
+    if (tid == 0) ex[extra_row(D) - 4] = m;
   }
   float ssq = 0.f;
   for (int base = 0; base < V; base += NU * 16) {
@@ -422,6 +560,7 @@ __global__ __launch_bounds__(256) void linear_step_kernel(
         r += q[i] * S[n][i];
       }
       r = row16_sum(r);
+      if (KIND == MEMORY) r *= inv;
       if (col < V) {
         store_rows<RPL, EXACT>(sp + (size_t)col * D, r0, D, S[n]);
         if ((lane & 15) == 0) {
@@ -438,10 +577,12 @@ __global__ __launch_bounds__(256) void linear_step_kernel(
   } else {
     ssq = block_sum_256(ssq, red);
     const float rn = 1.f / sqrtf(ssq / V + eps);
-    for (int j = tid; j < V; j += 256)
-      out[(size_t)s * ld_out + h * V + j] =
-          from_f<T>(lo[j] * rn * w_norm[j] *
-                    silu_f(to_f(row[g_off + h * V + j])));
+    for (int j = tid; j < V; j += 256) {
+      const float z = to_f(row[g_off + h * V + j]);
+      const float f = KIND == MEMORY ? w_norm[h * V + j] * sigmoid_f(z)
+                                     : w_norm[j] * silu_f(z);
+      out[(size_t)s * ld_out + h * V + j] = from_f<T>(lo[j] * rn * f);
+    }
   }
 }
 
@@ -451,14 +592,14 @@ static bool scan_ok(int G, int H, int D, int V) {
          V <= 4096;
 }
 
-template <bool CONV>
+template <Kind KIND>
 static int launch_step(void* out, int ld_out, void* y, void* state,
                        const void* proj, int ld, int q_off, int k_off,
                        int v_off, int g_off, const void* dec,
                        const void* dec_bias, const void* w_norm, void* ring,
                        const void* wconv, const void* conv_bias,
-                       const void* per_head, const void* pos, const void* row,
-                       int n_seq, int G, int H, int D, int V, int taps,
+                       const void* per_head, void* extra, const void* pos,
+                       const void* row, int n_seq, int G, int H, int D, int V, int taps,
                        float q_scale, float rate, float eps, int dtype,
                        void* stream) {
   if (!scan_ok(G, H, D, V) || n_seq > 65535) return -2;
@@ -466,13 +607,13 @@ static int launch_step(void* out, int ld_out, void* y, void* state,
   const size_t lds = (3 * 16 * rows_per_lane(D) + 2 * V) * sizeof(float);
   const dim3 grid(H, n_seq), block(256);
   HY_DTYPE(dtype, HY_RPL(D, hipLaunchKernelGGL(
-      (linear_step_kernel<T, RPL, EXACT, CONV>), grid, block, lds,
+      (linear_step_kernel<T, RPL, EXACT, KIND>), grid, block, lds,
       (hipStream_t)stream, (T*)out, ld_out, (float*)y, (float*)state,
       (const T*)proj, ld, q_off, k_off, v_off, g_off, (const T*)dec,
       (const float*)dec_bias, (const float*)w_norm, (T*)ring,
       (const float*)wconv, (const float*)conv_bias, (const float*)per_head,
-      (const int*)pos, (const int*)row, G, H, D, V, taps, q_scale, rate,
-      eps)));
+      (float*)extra, (const int*)pos, (const int*)row, G, H, D, V, taps,
+      q_scale, rate, eps)));
   HY_CHECK();
   return 0;
 }
@@ -483,12 +624,13 @@ int hy_linear_scan(void* o, void* state, const void* in, int ld, int q_off,
                    int k_off, int v_off, const void* g, const void* dt,
                    const void* skip, const void* e_start, const void* e_len,
                    const void* e_pos, const void* e_row, int n_entries, int G,
-                   int H, int D, int V, float q_scale, int dtype,
-                   void* stream) {
+                   int H, int D, int V, float q_scale, const void* n0,
+                   void* extra, int dtype, void* stream) {
   if (!scan_ok(G, H, D, V) || n_entries > 65535) return -2;
   if (n_entries <= 0) return 0;
-  const bool channel = dt == nullptr;
+  const bool channel = dt == nullptr, memory = n0 != nullptr;
   if (channel ? G != H : !skip) return -2;
+  if (memory && (channel || !extra)) return -2;
   // wide lanes where they still put waves enough on the 1024 SIMDs
   // (measured; a decay per channel gains more from sharing its loads)
   const long long waves = (long long)n_entries * H * ((V + 3) / 4);
@@ -500,23 +642,26 @@ int hy_linear_scan(void* o, void* state, const void* in, int ld, int q_off,
     const int nb = (V + 4 * cpl - 1) / (4 * cpl);
     return nb % 4 == 0 ? 4 : (nb % 2 == 0 ? 2 : 1);
   };
-#define RUN(CPL, CHANNEL, VEC)                                                \
+#define RUN(CPL, KIND, VEC)                                                   \
   HY_DTYPE(dtype, hipLaunchKernelGGL(                                         \
-      (linear_scan_kernel<T, RPL, VEC, CPL, CHANNEL>),                        \
+      (linear_scan_kernel<T, RPL, VEC, CPL, KIND>),                           \
       dim3(H * ((V + 4 * CPL - 1) / (4 * CPL)) / group(CPL), n_entries),      \
       dim3(64 * group(CPL)), 0,                                               \
       (hipStream_t)stream, (float*)o, (float*)state, (const T*)in, ld, q_off, \
       k_off, v_off, (const float*)g, (const float*)dt, (const float*)skip,    \
       (const int*)e_start, (const int*)e_len, (const int*)e_pos,              \
-      (const int*)e_row, G, H, D, V, q_scale))
+      (const int*)e_row, G, H, D, V, q_scale, (const float*)n0,               \
+      (float*)extra))
 // (the wide forms are chosen for small D only)
 #define PICK(CPL)                               \
   do {                                          \
     if constexpr (RPL * CPL <= 32) {            \
-      if (channel && vec) RUN(CPL, true, true); \
-      else if (channel) RUN(CPL, true, false);  \
-      else if (vec) RUN(CPL, false, true);      \
-      else RUN(CPL, false, false);              \
+      if (channel && vec) RUN(CPL, CHANNEL, true); \
+      else if (channel) RUN(CPL, CHANNEL, false);  \
+      else if (memory && vec) RUN(CPL, MEMORY, true); \
+      else if (memory) RUN(CPL, MEMORY, false);    \
+      else if (vec) RUN(CPL, HEAD, true);          \
+      else RUN(CPL, HEAD, false);                  \
     }                                           \
   } while (0)
 #define GO(CPL)                                                    \
@@ -564,10 +709,42 @@ int hy_gla_step(void* out, int ld_out, void* state, const void* proj, int ld,
                 const void* row, int n_seq, int H, int D, int V,
                 float q_scale, float rate, float eps, int dtype,
                 void* stream) {
-  return launch_step<false>(out, ld_out, nullptr, state, proj, ld, 0, k_off,
-                            v_off, g_off, dec, dec_bias, w_norm, nullptr,
-                            nullptr, nullptr, nullptr, pos, row, n_seq, H, H,
-                            D, V, 1, q_scale, rate, eps, dtype, stream);
+  return launch_step<CHANNEL>(out, ld_out, nullptr, state, proj, ld, 0,
+                              k_off, v_off, g_off, dec, dec_bias, w_norm,
+                              nullptr, nullptr, nullptr, nullptr, nullptr,
+                              pos, row, n_seq, H, H, D, V, 1, q_scale, rate,
+                              eps, dtype, stream);
+}
+
+int hy_memory_step(void* out, int ld_out, void* state, void* extra,
+                   const void* proj, int ld, int k_off, int v_off, int g_off,
+                   int i_off, const void* bias, const void* w_norm,
+                   const void* pos, const void* row, int n_seq, int H, int D,
+                   int V, float q_scale, float cap, float eps, int dtype,
+                   void* stream) {
+  const size_t esize = dtype == 0 ? 2 : 4;
+  return launch_step<MEMORY>(out, ld_out, nullptr, state, proj, ld, 0, k_off,
+                             v_off, g_off, (const char*)proj + i_off * esize,
+                             nullptr, w_norm, nullptr, nullptr, nullptr, bias,
+                             extra, pos, row, n_seq, H, H, D, V, 1, q_scale,
+                             cap, eps, dtype, stream);
+}
+
+int hy_memory_gates(void* steps, void* n0, void* extra, const void* proj,
+                    int ld, int i_off, const void* bias, const void* e_start,
+                    const void* e_len, const void* e_pos, const void* e_row,
+                    int n_entries, int n_tok, int H, int D, float cap,
+                    int dtype, void* stream) {
+  if (!scan_ok(H, H, D, 1) || n_entries > 65535 || !(cap > 0.f)) return -2;
+  if (n_entries <= 0 || n_tok <= 0) return 0;
+  HY_DTYPE(dtype, hipLaunchKernelGGL(
+      memory_gates_kernel<T>, dim3(H, n_entries), dim3(WAVE), 0,
+      (hipStream_t)stream, (float*)steps, (float*)n0, (float*)extra,
+      (const T*)proj, ld, i_off, i_off + H, (const float*)bias,
+      (const int*)e_start, (const int*)e_len, (const int*)e_pos,
+      (const int*)e_row, n_tok, H, D, cap));
+  HY_CHECK();
+  return 0;
 }
 
 int hy_ssm_step(void* y, void* state, const void* proj, int ld, int dt_off,
@@ -576,10 +753,10 @@ int hy_ssm_step(void* y, void* state, const void* proj, int ld, int dt_off,
                 int n_seq, int G, int H, int N, int V, int taps, int dtype,
                 void* stream) {
   if (taps <= 0) return -2;
-  return launch_step<true>(nullptr, 0, y, state, proj, ld, H * V + G * N,
+  return launch_step<HEAD>(nullptr, 0, y, state, proj, ld, H * V + G * N,
                            H * V, 0, dt_off, nullptr, nullptr, nullptr, ring,
-                           wconv, bias, per_head, pos, row, n_seq, G, H, N, V,
-                           taps, 1.f, 0.f, 0.f, dtype, stream);
+                           wconv, bias, per_head, nullptr, pos, row, n_seq, G,
+                           H, N, V, taps, 1.f, 0.f, 0.f, dtype, stream);
 }
 
 int hy_ssm_prep(void* xbc, void* steps, const void* proj, int ld, int dt_off,

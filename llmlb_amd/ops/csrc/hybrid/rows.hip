@@ -1,6 +1,7 @@
 // Row and elementwise kernels of the hybrid models: a residual stream
-// in 32-bit, RMS norms of a sublayer's OUTPUT or of the stream itself,
-// gated norms of parts of a row, activations, the soft cap of logits.
+// in 32-bit, RMS and layer norms of a sublayer's OUTPUT or of the stream
+// itself, gated norms of parts of a row, activations, the soft cap of
+// logits.
 #include "common.h"
 
 // x[t] = table[ids[t]] in 32-bit, and a copy in the storage type for the
@@ -194,14 +195,14 @@ __global__ __launch_bounds__(256) void add_norms_kernel(
 
 // Each of a row's ``groups`` parts of S columns divided by its rms, times
 // w (wl columns, repeated along the row), with silu(gate) applied before
-// the norm or after it.  L lanes a part: 8 to 64, or the workgroup.
+// the norm or after it, or sigmoid(gate) after it (``sigm``).  L lanes a part: 8 to 64, or the workgroup.
 // Up to KEEP vectors a lane stay in registers between the passes.
 template <typename T, int L, bool GATE_FIRST, bool VEC>
 __global__ __launch_bounds__(256) void gated_norm_kernel(
     T* __restrict__ out, int ld_out, const float* __restrict__ y,
     const T* __restrict__ gate, int ld, int g_off,
     const float* __restrict__ w, int wl, int parts, int groups, int S,
-    float eps) {
+    bool sigm, float eps) {
   constexpr int N = VEC ? 8 : 1;
   constexpr int KEEP = L == 256 ? 4 : (VEC ? 1 : 8);
   __shared__ float red[4];
@@ -259,7 +260,7 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
 #pragma unroll
     for (int j = 0; j < N; ++j) {
       f[j] *= r * wn[j];
-      if (!GATE_FIRST) f[j] *= silu_f(z[j]);
+      if (!GATE_FIRST) f[j] *= (sigm ? 1.f : z[j]) * sigmoid_f(z[j]);
     }
     if (VEC) store8(dst + i, f);
     else dst[i] = from_f<T>(f[0]);
@@ -277,22 +278,27 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(
 }
 
 // out[r] = norm(x[index[r]]) in the storage type (index null: row r).
-// ONE: w is a single number.
-template <typename T, bool ONE>
+// ONE: w is a single number.  CENTRED: the row's mean is taken off first.
+template <typename T, bool ONE, bool CENTRED>
 __global__ __launch_bounds__(256) void norm_rows_kernel(
     T* __restrict__ out, const float* __restrict__ x,
     const int* __restrict__ index, const float* __restrict__ w,
     float w_offset, int width, float eps) {
-  __shared__ float red[4];
+  __shared__ float red[4], red2[4];
   const size_t src = (size_t)(index ? index[blockIdx.x] : blockIdx.x) * width;
   const size_t dst = (size_t)blockIdx.x * width;
-  float ssq = 0.f;
+  float ssq = 0.f, mean = 0.f;
+  if (CENTRED) {
+    float sum = 0.f;
+    for (int i = threadIdx.x; i < width; i += 256) sum += x[src + i];
+    mean = block_sum_256(sum, red2) / width;
+  }
   if ((width & 7) == 0) {
     for (int i = threadIdx.x * 8; i < width; i += 2048) {
       float f[8];
       load8(x + src + i, f);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) ssq += f[j] * f[j];
+      for (int j = 0; j < 8; ++j) ssq += (f[j] - mean) * (f[j] - mean);
     }
     const float r = 1.f / sqrtf(block_sum_256(ssq, red) / width + eps);
     for (int i = threadIdx.x * 8; i < width; i += 2048) {
@@ -301,16 +307,134 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(
       if (!ONE) load8(w + i, wr);
 #pragma unroll
       for (int j = 0; j < 8; ++j)
-        f[j] *= r * (w_offset + (ONE ? w[0] : wr[j]));
+        f[j] = (f[j] - mean) * r * (w_offset + (ONE ? w[0] : wr[j]));
       store8(out + dst + i, f);
     }
     return;
   }
   for (int i = threadIdx.x; i < width; i += 256)
-    ssq += x[src + i] * x[src + i];
+    ssq += (x[src + i] - mean) * (x[src + i] - mean);
   const float r = 1.f / sqrtf(block_sum_256(ssq, red) / width + eps);
   for (int i = threadIdx.x; i < width; i += 256)
-    out[dst + i] = from_f<T>(x[src + i] * r * (w_offset + w[ONE ? 0 : i]));
+    out[dst + i] = from_f<T>((x[src + i] - mean) * r *
+                             (w_offset + w[ONE ? 0 : i]));
+}
+
+// x += norm(y) w_post, h = norm(x) w_pre in the storage type: what lies
+// between two sublayers whose outputs are normed as well as their inputs.
+// y null: nothing is added; w_pre (and h) null: the sum alone.  CENTRED:
+// layer norms, else RMS norms.  One workgroup per row; KEEP runs of N
+// neighbours a thread stay in registers between the passes, the rest is
+// read again.
+template <typename T, int N, int KEEP, bool CENTRED>
+__global__ __launch_bounds__(256) void post_pre_norm_kernel(
+    float* __restrict__ x, const T* __restrict__ y,
+    const float* __restrict__ w_post, const float* __restrict__ w_pre,
+    T* __restrict__ h, int width, float eps) {
+  __shared__ float red[4][4];
+  const int runs = width / N, tid = threadIdx.x;
+  const float inv = 1.f / width;
+  float* xr = x + (size_t)blockIdx.x * width;
+  const T* yr = y ? y + (size_t)blockIdx.x * width : nullptr;
+  auto load = [](const auto* p, float* f) {
+    if constexpr (N == 8) load8(p, f);
+    else f[0] = to_f(p[0]);
+  };
+  auto store = [](auto* p, const float* f) {
+    using S = std::remove_reference_t<decltype(*p)>;
+    if constexpr (N == 8) store8(p, f);
+    else p[0] = from_f<S>(f[0]);
+  };
+  float keep[KEEP][N], mean = 0.f;
+  // sums over the row of ``src``, of which the first runs are kept
+  auto total = [&](const auto* src, float* red) {
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if (tid + k * 256 < runs)
+#pragma unroll
+        for (int j = 0; j < N; ++j) s += keep[k][j];
+    for (int i = tid + KEEP * 256; i < runs; i += 256) {
+      float f[N];
+      load(src + (size_t)i * N, f);
+#pragma unroll
+      for (int j = 0; j < N; ++j) s += f[j];
+    }
+    return block_sum_256(s, red);
+  };
+  auto squares = [&](const auto* src, float* red) {
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if (tid + k * 256 < runs)
+#pragma unroll
+        for (int j = 0; j < N; ++j)
+          s += (keep[k][j] - mean) * (keep[k][j] - mean);
+    for (int i = tid + KEEP * 256; i < runs; i += 256) {
+      float f[N];
+      load(src + (size_t)i * N, f);
+#pragma unroll
+      for (int j = 0; j < N; ++j) s += (f[j] - mean) * (f[j] - mean);
+    }
+    return block_sum_256(s, red);
+  };
+  if (y) {
+    // the stream's loads fly behind the norm of y
+    float xk[KEEP][N];
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if (tid + k * 256 < runs) load(yr + (size_t)(tid + k * 256) * N, keep[k]);
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if (tid + k * 256 < runs) load(xr + (size_t)(tid + k * 256) * N, xk[k]);
+    if (CENTRED) mean = total(yr, red[0]) * inv;
+    const float r = 1.f / sqrtf(squares(yr, red[1]) * inv + eps);
+    auto add = [&](int i, const float* f, float* out) {
+      float w[N];
+      load(w_post + (size_t)i * N, w);
+#pragma unroll
+      for (int j = 0; j < N; ++j) out[j] += (f[j] - mean) * r * w[j];
+      store(xr + (size_t)i * N, out);
+    };
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if (tid + k * 256 < runs) {
+        add(tid + k * 256, keep[k], xk[k]);
+#pragma unroll
+        for (int j = 0; j < N; ++j) keep[k][j] = xk[k][j];
+      }
+    for (int i = tid + KEEP * 256; i < runs; i += 256) {
+      float f[N], v[N];
+      load(yr + (size_t)i * N, f);
+      load(xr + (size_t)i * N, v);
+      add(i, f, v);
+    }
+  } else {
+#pragma unroll
+    for (int k = 0; k < KEEP; ++k)
+      if (tid + k * 256 < runs) load(xr + (size_t)(tid + k * 256) * N, keep[k]);
+  }
+  if (!w_pre) return;
+  // beyond the kept runs a thread reads back only what it wrote itself
+  mean = 0.f;
+  if (CENTRED) mean = total(xr, red[2]) * inv;
+  const float r = 1.f / sqrtf(squares(xr, red[3]) * inv + eps);
+  T* hr = h + (size_t)blockIdx.x * width;
+  auto emit = [&](int i, float* f) {
+    float w[N];
+    load(w_pre + (size_t)i * N, w);
+#pragma unroll
+    for (int j = 0; j < N; ++j) f[j] = (f[j] - mean) * r * w[j];
+    store(hr + (size_t)i * N, f);
+  };
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k)
+    if (tid + k * 256 < runs) emit(tid + k * 256, keep[k]);
+  for (int i = tid + KEEP * 256; i < runs; i += 256) {
+    float f[N];
+    load(xr + (size_t)i * N, f);
+    emit(i, f);
+  }
 }
 
 __device__ __forceinline__ float gelu_tanh_f(float z) {
@@ -455,16 +579,43 @@ int hy_post_norm_add(void* x, void* xb, const void* y, const void* w,
 }
 
 int hy_norm_rows(void* out, const void* x, const void* index, const void* w,
-                 int one, float w_offset, int n_rows, int width, float eps,
-                 int dtype, void* stream) {
+                 int one, float w_offset, int centred, int n_rows, int width,
+                 float eps, int dtype, void* stream) {
   if (n_rows <= 0) return 0;
-#define GO(ONE)                                                              \
+#define GO(ONE, CENTRED)                                                     \
   HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
-      (norm_rows_kernel<T, ONE>), dim3(n_rows), dim3(256), 0,                \
+      (norm_rows_kernel<T, ONE, CENTRED>), dim3(n_rows), dim3(256), 0,       \
       (hipStream_t)stream, (T*)out, (const float*)x, (const int*)index,      \
       (const float*)w, w_offset, width, eps))
-  if (one) GO(true);
-  else GO(false);
+  if (one && centred) GO(true, true);
+  else if (one) GO(true, false);
+  else if (centred) GO(false, true);
+  else GO(false, false);
+#undef GO
+  HY_CHECK();
+  return 0;
+}
+
+int hy_post_pre_norm(void* x, const void* y, const void* w_post,
+                     const void* w_pre, void* h, int centred, int n_tok,
+                     int width, float eps, int dtype, void* stream) {
+  if ((y && !w_post) || (w_pre && !h) || width <= 0) return -2;
+  if (n_tok <= 0) return 0;
+#define GO(N, KEEP, CENTRED)                                                 \
+  HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
+      (post_pre_norm_kernel<T, N, KEEP, CENTRED>), dim3(n_tok), dim3(256),   \
+      0, (hipStream_t)stream, (float*)x, (const T*)y, (const float*)w_post,  \
+      (const float*)w_pre, (T*)h, width, eps))
+#define PICK(N, KEEP)                 \
+  do {                                \
+    if (centred) GO(N, KEEP, true);   \
+    else GO(N, KEEP, false);          \
+  } while (0)
+  if (width % 8) PICK(1, 4);
+  else if (width <= 2048) PICK(8, 1);
+  else if (width <= 4096) PICK(8, 2);
+  else PICK(8, 4);
+#undef PICK
 #undef GO
   HY_CHECK();
   return 0;
@@ -494,8 +645,9 @@ int hy_add_norms(void* x, const void* y, const void* z, const void* zw,
 
 int hy_gated_norm(void* out, int ld_out, const void* y, const void* gate,
                   int ld, int g_off, const void* w, int wl, int n_tok,
-                  int groups, int S, int gate_first, float eps, int dtype,
-                  void* stream) {
+                  int groups, int S, int gate_first, int sigm, float eps,
+                  int dtype, void* stream) {
+  if (sigm && gate_first) return -2;
   if (groups <= 0 || S <= 0 || wl <= 0 || (groups * S) % wl) return -2;
   if (n_tok <= 0) return 0;
   if ((long long)n_tok * groups >= (1ll << 31)) return -2;
@@ -507,7 +659,8 @@ int hy_gated_norm(void* out, int ld_out, const void* y, const void* gate,
       (gated_norm_kernel<T, L, FIRST, VEC>),                                \
       dim3((parts + 256 / L - 1) / (256 / L)), dim3(256), 0,                \
       (hipStream_t)stream, (T*)out, ld_out, (const float*)y,                \
-      (const T*)gate, ld, g_off, (const float*)w, wl, parts, groups, S, eps))
+      (const T*)gate, ld, g_off, (const float*)w, wl, parts, groups, S,     \
+      sigm != 0, eps))
 #define PICK(L)                                \
   do {                                         \
     if (gate_first && vec) GO(L, true, true);  \

@@ -1,8 +1,11 @@
-// Grouped-query attention over a sliding window of cached tokens, each
-// head's output times the sigmoid of a number of its own.
+// Grouped-query attention over a sliding window of cached tokens, or over
+// the tokens of the query's own chunk (chunks are counted from position
+// 0), each head's output times the sigmoid of a number of its own (column
+// g_off of its token's row; g_off < 0: no gate).
 //
-// Queries and keys are normed over the whole projection (all heads at
-// once) and rotated on the first ``rot`` numbers of each head.  A cached
+// Queries and keys are prepared by window_prep (normed over the whole
+// projection, all heads at once) or by head_prep (each head by itself),
+// and rotated on the first ``rot`` numbers of each head.  A cached
 // token keeps, for each of G key/value heads, one row [key (D) | value
 // (V)]; a page is [G][16 tokens][D + V].  Query head h reads key/value
 // head h / (H / G).  The query's weights carry the scale of the scores
@@ -66,7 +69,7 @@ __global__ __launch_bounds__(256) void window_rows_kernel(
     T* __restrict__ out, int ld_out, const T* __restrict__ proj, int ld,
     int g_off, const T* __restrict__ cache, const int* __restrict__ pos_,
     const int* __restrict__ row_, const int* __restrict__ bt, int max_blocks,
-    int H, int G, int D, int V, int CW, int window, bool vec) {
+    int H, int G, int D, int V, int CW, Mask mask, bool vec) {
   extern __shared__ float lds[];
   float* lq = lds;                     // D query numbers
   float* lp = lq + D;                  // weights of 256 keys
@@ -85,8 +88,7 @@ __global__ __launch_bounds__(256) void window_rows_kernel(
 #pragma unroll
   for (int i = 0; i < NC; ++i) acc[i] = 0.f;
   __syncthreads();
-  for (int j0 = pos - window + 1 > 0 ? pos - window + 1 : 0; j0 <= pos;
-       j0 += 256) {
+  for (int j0 = mask.first(pos); j0 <= pos; j0 += 256) {
     const int j = j0 + tid;
     float s = -INFINITY;
     if (j <= pos) {
@@ -137,8 +139,9 @@ __global__ __launch_bounds__(256) void window_rows_kernel(
   for (int i = 0; i < NC; ++i) lacc[i * 256 + tid] = acc[i];
   __syncthreads();
   if (grp != 0) return;
-  const float f = sigmoid_f(to_f(proj[(size_t)t * ld + g_off + h])) /
-                  (red2[0] + red2[1] + red2[2] + red2[3]);
+  const float gate =
+      g_off < 0 ? 1.f : sigmoid_f(to_f(proj[(size_t)t * ld + g_off + h]));
+  const float f = gate / (red2[0] + red2[1] + red2[2] + red2[3]);
   T* dst = out + (size_t)t * ld_out + (size_t)h * V;
 #pragma unroll
   for (int i = 0; i < NC; ++i) {
@@ -187,7 +190,8 @@ int hy_window_prep(void* proj, int ld, void* cache, int k_off, int v_off,
 int hy_window_rows(void* out, int ld_out, const void* proj, int ld, int g_off,
                    const void* cache, const void* pos, const void* row,
                    const void* bt, int max_blocks, int H, int G, int D, int V,
-                   int window, int n_rows, int dtype, void* stream) {
+                   int window, int chunk, int n_rows, int dtype,
+                   void* stream) {
   if (G <= 0 || H <= 0 || H % G || H > 65535 || D <= 0 || D > 1024 ||
       V <= 0 || V > 1024 || window < 1)
     return -2;
@@ -195,13 +199,14 @@ int hy_window_rows(void* out, int ld_out, const void* proj, int ld, int g_off,
   int cw = 1;
   while (cw < V && cw < 256) cw *= 2;
   const bool vec = D % 4 == 0 && V % 4 == 0;
+  const Mask mask{window, chunk != 0};
   const dim3 grid(n_rows, H), block(256);
 #define GO(NC)                                                              \
   HY_DTYPE(dtype, hipLaunchKernelGGL(                                       \
       (window_rows_kernel<T, NC>), grid, block,                             \
       (D + 512 + 256 * NC) * sizeof(float), (hipStream_t)stream, (T*)out,   \
       ld_out, (const T*)proj, ld, g_off, (const T*)cache, (const int*)pos,  \
-      (const int*)row, (const int*)bt, max_blocks, H, G, D, V, cw, window,  \
+      (const int*)row, (const int*)bt, max_blocks, H, G, D, V, cw, mask,    \
       vec))
   if (V <= 256) GO(1);
   else if (V <= 512) GO(2);

@@ -1,5 +1,5 @@
-// Matrix-core forms of windowed grouped-query attention (see
-// window_attention.hip for the cache layout), bf16 storage, float softmax.
+// Matrix-core forms of windowed and chunked grouped-query attention (see
+// window_attention.hip for the masks, the gate and the cache layout), bf16 storage, float softmax.
 //
 //  * window_flash_kernel   prompts: 128 rows a workgroup, a row being one
 //    head of one query; all heads of a key/value head are rows side by
@@ -23,7 +23,7 @@ void window_flash_kernel(
     bf16_t* __restrict__ out, int ld_out, const bf16_t* __restrict__ proj,
     int ld, int g_off, const bf16_t* __restrict__ cache,
     const int* __restrict__ items, const int* __restrict__ bt, int max_blocks,
-    int H, int G, int D, int V, int window) {
+    int H, int G, int D, int V, Mask mask) {
   constexpr int KD = DQ / 32, VT = DV / 16;
   using St = Stage<1, DQ, DV>;
   __shared__ unsigned short lk[64 * St::KP];
@@ -35,7 +35,7 @@ void window_flash_kernel(
   const int n = lane & 15, g = lane >> 4;
   const int last = q_pos + it[2] - 1;
 
-  int qi[2], at[2];  // this lane's queries and heads
+  int qi[2], at[2], span[2];  // this lane's queries, heads, keys before
   u32x4 qf[2][KD];
 #pragma unroll
   for (int a = 0; a < 2; ++a) {
@@ -43,6 +43,7 @@ void window_flash_kernel(
     r = r < n_rows ? r : n_rows - 1;
     qi[a] = r / R;
     at[a] = kv * R + r - qi[a] * R;
+    span[a] = mask.span(q_pos + qi[a]);
     const bf16_t* q =
         proj + (size_t)(q_row + qi[a]) * ld + (size_t)at[a] * D;
 #pragma unroll
@@ -55,8 +56,10 @@ void window_flash_kernel(
   // positions of the wave's first and last query
   const int w_lo = q_pos + wave * 32 / R;
   const int w_hi = q_pos + (wave * 32 + 31) / R;
-  const int first = q_pos - window + 1;
-  const int lo = first > 0 ? first & ~(PAGE - 1) : 0;
+  // and the first keys they see
+  const int w_lo_key = w_lo - mask.span(w_lo);
+  const int w_hi_key = w_hi - mask.span(w_hi);
+  const int lo = mask.first(q_pos) & ~(PAGE - 1);
 
   St st(cache, bt + (size_t)it[3] * max_blocks, G, kv, D, V, last);
   u32x4 pk[St::KL], pv[St::VL];
@@ -82,7 +85,7 @@ void window_flash_kernel(
       if (j0 + 128 <= last) st.fetch_pages(j0 + 128, pg);
     }
     // a tile none of the wave's queries sees is skipped
-    if (j0 <= w_hi && j0 + 63 > w_lo - window) {
+    if (j0 <= w_hi && j0 + 63 >= w_lo_key) {
       f32x4 s[2][4];
 #pragma unroll
       for (int t = 0; t < 4; ++t) {
@@ -95,7 +98,7 @@ void window_flash_kernel(
           s[1][t] = mfma(kf, qf[1][k], s[1][t]);
         }
       }
-      const bool whole = j0 + 63 <= w_lo && j0 > w_hi - window;
+      const bool whole = j0 + 63 <= w_lo && j0 >= w_hi_key;
       u32x4 pf[2][2];
 #pragma unroll
       for (int a = 0; a < 2; ++a) {
@@ -105,9 +108,10 @@ void window_flash_kernel(
           for (int t = 0; t < 4; ++t)
 #pragma unroll
             for (int i = 0; i < 4; ++i)
-              s[a][t][i] = (unsigned)(age - t * 16 - i) < (unsigned)window
-                               ? s[a][t][i]
-                               : -INFINITY;
+              s[a][t][i] =
+                  (unsigned)(age - t * 16 - i) <= (unsigned)span[a]
+                      ? s[a][t][i]
+                      : -INFINITY;
         }
         float mx = m[a];
 #pragma unroll
@@ -158,8 +162,9 @@ void window_flash_kernel(
     sum += __shfl_xor(sum, 32, WAVE);
     if (wave * 32 + a * 16 + n >= n_rows) continue;
     const size_t tok = q_row + qi[a];
-    const float f =
-        1.f / (sum * (1.f + __expf(-to_f(proj[tok * ld + g_off + at[a]]))));
+    float f = 1.f / sum;
+    if (g_off >= 0)
+      f = 1.f / (sum * (1.f + __expf(-to_f(proj[tok * ld + g_off + at[a]]))));
     bf16_t* dst = out + tok * ld_out + (size_t)at[a] * V;
 #pragma unroll
     for (int v = 0; v < VT; ++v) {
@@ -187,7 +192,7 @@ void window_decode_kernel(
     int g_off, const bf16_t* __restrict__ cache,
     const int* __restrict__ pos_, const int* __restrict__ row_,
     const int* __restrict__ bt, int max_blocks, int H, int G, int D, int V,
-    int window, int parts) {
+    Mask mask, int parts) {
   constexpr int KD = DQ / 32, NV = DV / 64, PP = 64 + 8;
   using St = Stage<1, DQ, DV>;
   __shared__ unsigned short lk[64 * St::KP];
@@ -203,8 +208,8 @@ void window_decode_kernel(
   const int h = kv * R + h0 + n;  // this lane's head
   const bool real = h0 + n < R;
 
-  const int first = pos - window + 1;
-  const int lo = first > 0 ? first & ~(PAGE - 1) : 0;
+  const int span = mask.span(pos);
+  const int lo = mask.first(pos) & ~(PAGE - 1);
   const int tiles = (pos - lo) / 64 + 1;
   const int per = (tiles + parts - 1) / parts;
   const int t_lo = part * per;
@@ -227,7 +232,10 @@ void window_decode_kernel(
       qf[k] = *reinterpret_cast<const u32x4*>(proj + (size_t)q * ld +
                                               (size_t)h * D + d);
   }
-  float z = real ? to_f(proj[(size_t)q * ld + g_off + h]) : 0.f;
+  // what the sum is multiplied with to gate
+  float z = 1.f;
+  if (real && g_off >= 0)
+    z += __expf(-to_f(proj[(size_t)q * ld + g_off + h]));
 
   f32x4 o[NV];
   float m = -1e30f, l = 0.f;
@@ -249,7 +257,7 @@ void window_decode_kernel(
                qf[k], s);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      s[i] = (unsigned)(pos - j - i) < (unsigned)window ? s[i] : -INFINITY;
+      s[i] = (unsigned)(pos - j - i) <= (unsigned)span ? s[i] : -INFINITY;
     float mx = fmaxf(fmaxf(s[0], s[1]), fmaxf(s[2], s[3]));
     mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
     mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
@@ -291,7 +299,7 @@ void window_decode_kernel(
   if (!real) return;
   l = lsum[n][0] + lsum[n][1] + lsum[n][2] + lsum[n][3];
   if (parts == 1) {
-    const float f = 1.f / (l * (1.f + __expf(-z)));
+    const float f = 1.f / (l * z);
     bf16_t* dst = out + (size_t)q * ld_out + (size_t)h * V;
 #pragma unroll
     for (int v = 0; v < NV; ++v) {
@@ -329,7 +337,7 @@ __global__ __launch_bounds__(256) void window_merge_kernel(
   const int lane = threadIdx.x & 63;
   const size_t at = ((size_t)q * H + h) * parts;
   const int c = lane * 4;  // V <= 256 columns
-  const float z = to_f(proj[(size_t)q * ld + g_off + h]);
+  const float z = g_off < 0 ? 0.f : to_f(proj[(size_t)q * ld + g_off + h]);
   float m = -1e30f, w = 0.f;
   if (lane < parts) {
     const float2 ml =
@@ -341,7 +349,8 @@ __global__ __launch_bounds__(256) void window_merge_kernel(
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) mx = fmaxf(mx, __shfl_xor(mx, o, WAVE));
   const float f = __builtin_amdgcn_exp2f(m - mx);
-  w = f / (wave_sum(w * f) * (1.f + __expf(-z)));
+  const float gate = g_off < 0 ? 1.f : 1.f + __expf(-z);
+  w = f / (wave_sum(w * f) * gate);
 
   float o[4] = {0.f, 0.f, 0.f, 0.f};
   const float* src = ws_acc + at * V + (c < V ? c : 0);
@@ -384,16 +393,17 @@ extern "C" {
 int hy_window_flash(void* out, int ld_out, const void* proj, int ld,
                     int g_off, const void* cache, const void* items,
                     int n_items, const void* bt, int max_blocks, int H, int G,
-                    int D, int V, int window, void* stream) {
+                    int D, int V, int window, int chunk, void* stream) {
   if (!window_ok(ld, ld_out, H, G, D, V, window) || H / G > 128) return -2;
   if (n_items <= 0) return 0;
+  const Mask mask{window, chunk != 0};
 #define GO(DQ, DV)                                                           \
   hipLaunchKernelGGL((window_flash_kernel<DQ, DV>),                          \
                      dim3((unsigned)n_items * G), dim3(256), 0,              \
                      (hipStream_t)stream, (bf16_t*)out, ld_out,              \
                      (const bf16_t*)proj, ld, g_off, (const bf16_t*)cache,   \
                      (const int*)items, (const int*)bt, max_blocks, H, G, D, \
-                     V, window)
+                     V, mask)
   WINDOW_SIZES(D, V);
 #undef GO
   HY_CHECK();
@@ -404,20 +414,21 @@ int hy_window_decode(void* out, int ld_out, void* acc, void* ml,
                      const void* proj, int ld, int g_off, const void* cache,
                      const void* pos, const void* row, const void* bt,
                      int max_blocks, int H, int G, int D, int V, int window,
-                     int n_rows, int parts, void* stream) {
+                     int chunk, int n_rows, int parts, void* stream) {
   if (!window_ok(ld, ld_out, H, G, D, V, window) || parts < 1 ||
       parts > PARTS_MAX || (parts > 1 && (!acc || !ml)))
     return -2;
   if (n_rows <= 0) return 0;
   const int tiles = (H / G + 15) / 16;
   if (G * tiles > 65535) return -2;
+  const Mask mask{window, chunk != 0};
 #define GO(DQ, DV)                                                           \
   hipLaunchKernelGGL((window_decode_kernel<DQ, DV>),                         \
                      dim3(n_rows, G * tiles, parts), dim3(256), 0,           \
                      (hipStream_t)stream, (bf16_t*)out, ld_out, (float*)acc, \
                      (float*)ml, (const bf16_t*)proj, ld, g_off,             \
                      (const bf16_t*)cache, (const int*)pos, (const int*)row, \
-                     (const int*)bt, max_blocks, H, G, D, V, window, parts)
+                     (const int*)bt, max_blocks, H, G, D, V, mask, parts)
   WINDOW_SIZES(D, V);
 #undef GO
   HY_CHECK();

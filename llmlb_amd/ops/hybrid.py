@@ -1,6 +1,7 @@
 """Ops of the hybrid models: a 32-bit residual stream with norms before
-or after the sublayers, latent, differential and windowed attention over
-pages, gated delta rule, linear recurrences and mixtures of experts.
+or after the sublayers or both, latent, differential, windowed and chunked
+attention over pages, gated delta rule, linear recurrences and mixtures of
+experts.
 
 The native library (csrc/hybrid) is loaded at first use.  GPU tensors
 always run the HIP kernels, in bfloat16 and in float32; CPU tensors run
@@ -117,18 +118,40 @@ def add_norms(x, y, w1, w2, eps, dtype, mult=1.0, routed=None):
     return h1, h2
 
 
-def norm_rows(x, index, w, eps, dtype, w_offset=0.0):
-    """rmsnorm(x[index]) * (w_offset + w) in ``dtype``; index may be
-    None (every row), w a row or a single number."""
+def post_pre_norm(x, y, w_post, w_pre, eps, dtype, centred: bool):
+    """In place: x += norm(y) * w_post (y None: nothing to add).  Returns
+    norm(x) * w_pre in ``dtype`` (w_pre None: nothing).  ``centred``:
+    layer norms, else RMS norms."""
     if not x.is_cuda:
-        return ref.norm_rows(x, index, w, eps, dtype, w_offset)
+        return ref.post_pre_norm(x, y, w_post, w_pre, eps, dtype, centred)
+    assert x.is_contiguous()
+    assert y is None or (y.is_contiguous() and y.shape == x.shape
+                         and y.dtype == dtype
+                         and w_post.numel() == x.shape[1])
+    assert w_pre is None or w_pre.numel() == x.shape[1]
+    h = None if w_pre is None else torch.empty(x.shape, dtype=dtype,
+                                               device=x.device)
+    _check(native().hy_post_pre_norm(
+        _ptr(x), _p(y), None if y is None else _ptr(w_post), _p(w_pre),
+        _p(h), _i(centred), _i(x.shape[0]), _i(x.shape[1]), _f(eps),
+        _dt(dtype), _stream()), "hy_post_pre_norm")
+    return h
+
+
+def norm_rows(x, index, w, eps, dtype, w_offset=0.0, centred=False):
+    """norm(x[index]) * (w_offset + w) in ``dtype``; index may be None
+    (every row), w a row or a single number.  ``centred``: a layer norm,
+    else an RMS norm."""
+    if not x.is_cuda:
+        return ref.norm_rows(x, index, w, eps, dtype, w_offset, centred)
     n = x.shape[0] if index is None else index.shape[0]
     one = w.numel() == 1 and x.shape[1] > 1
     assert w.numel() == (1 if one else x.shape[1])
     out = torch.empty(n, x.shape[1], dtype=dtype, device=x.device)
     _check(native().hy_norm_rows(
-        _ptr(out), _ptr(x), _p(index), _ptr(w), _i(one), _f(w_offset), _i(n),
-        _i(x.shape[1]), _f(eps), _dt(dtype), _stream()), "hy_norm_rows")
+        _ptr(out), _ptr(x), _p(index), _ptr(w), _i(one), _f(w_offset),
+        _i(centred), _i(n), _i(x.shape[1]), _f(eps), _dt(dtype), _stream()),
+        "hy_norm_rows")
     return out
 
 
@@ -203,11 +226,13 @@ def latent_prep(proj, heads, dim, rot, rank, c_off, w_norm, eps, cos_sin, b,
         _i(b.n_tok), _dt(proj.dtype), _stream()), "hy_latent_prep")
 
 
-def latent_rows(qa, proj, dim, rot, cache, b, window, scale):
+def latent_rows(qa, proj, dim, rot, cache, b, window, scale, sink=None):
     """Absorbed attention: qa [H, N, rank] (the batch's first N tokens)
-    -> weighted latents [H, N, rank]."""
+    -> weighted latents [H, N, rank].  ``sink`` [H] float32 (None: none):
+    a score of every head that has no key and no value."""
     if not qa.is_cuda:
-        return ref.latent_rows(qa, proj, dim, rot, cache, b, window, scale)
+        return ref.latent_rows(qa, proj, dim, rot, cache, b, window, scale,
+                               sink)
     H, N, rank = qa.shape
     assert qa.is_contiguous()
     out = torch.empty_like(qa)
@@ -215,7 +240,8 @@ def latent_rows(qa, proj, dim, rot, cache, b, window, scale):
         _ptr(out), _ptr(qa), _ptr(proj), _i(proj.stride(0)), _i(H), _i(dim),
         _i(rot), _i(rank), _ptr(cache), _ptr(b.pos), _ptr(b.row),
         _ptr(b.block_tables), _i(b.block_tables.shape[1]), _i(window),
-        _f(scale), _i(N), _dt(qa.dtype), _stream()), "hy_latent_rows")
+        _f(scale), _p(sink), _i(N), _dt(qa.dtype), _stream()),
+        "hy_latent_rows")
     return out
 
 
@@ -233,7 +259,7 @@ def decode_parts(n: int, heads: int, window: int, max_keys: int) -> int:
     return max(1, min(256 // groups, keys // 64, 16))
 
 
-def latent_decode(qa, proj, dim, rot, cache, b, window, scale):
+def latent_decode(qa, proj, dim, rot, cache, b, window, scale, sink=None):
     """``latent_rows`` on the matrix cores (bf16, GPU)."""
     H, N, rank = qa.shape
     assert qa.is_contiguous()
@@ -250,8 +276,24 @@ def latent_decode(qa, proj, dim, rot, cache, b, window, scale):
         _ptr(out), _p(acc), _p(ml), _ptr(qa), _ptr(proj),
         _i(proj.stride(0)), _i(H), _i(dim), _i(rot), _i(rank), _ptr(cache),
         _ptr(b.pos), _ptr(b.row), _ptr(bt), _i(bt.shape[1]), _i(window),
-        _f(scale), _i(N), _i(parts), _stream()), "hy_latent_decode")
+        _f(scale), _p(sink), _i(N), _i(parts), _stream()),
+        "hy_latent_decode")
     return out
+
+
+def join_heads(out, o, proj, g_off) -> None:
+    """out [N, H * V] = the heads of o [H, N, V] side by side, times the
+    sigmoid of the columns of ``proj`` from ``g_off`` on."""
+    if not o.is_cuda:
+        ref.join_heads(out, o, proj, g_off)
+        return
+    H, N, V = o.shape
+    gate = proj[:N, g_off:g_off + H * V]
+    assert o.is_contiguous() and out.is_contiguous() \
+        and out.shape == gate.shape == (N, H * V) and gate.stride(1) == 1
+    _check(native().hy_join_heads(
+        _ptr(out), _ptr(o), _ptr(gate), _i(proj.stride(0)), _i(N), _i(H),
+        _i(V), _dt(o.dtype), _stream()), "hy_join_heads")
 
 
 def can_flash(dtype, dim, rot, rank, vdim) -> bool:
@@ -261,11 +303,12 @@ def can_flash(dtype, dim, rot, rank, vdim) -> bool:
 
 
 def latent_flash(out, proj, heads, dim, rot, w_uk, w_uv, cache, b, window,
-                 scale) -> None:
+                 scale, sink=None, g_off=None) -> None:
     """Attention of the batch's long entries into ``out`` [T, H * vdim]:
     their visible latents are copied out of the pages and expanded to
     keys and (transposed) values.  w_uk [H, dim, rank], w_uv
-    [H, vdim, rank]."""
+    [H, vdim, rank].  With ``g_off`` times the sigmoid of the columns of
+    ``proj`` from there on."""
     H, V, rank = w_uv.shape
     blocks, items, n_blocks, n_items = b.long_plan(window)
     n = 64 * n_blocks
@@ -280,7 +323,8 @@ def latent_flash(out, proj, heads, dim, rot, w_uk, w_uv, cache, b, window,
     _check(lib.hy_latent_flash(
         _ptr(out), _ptr(proj), _i(proj.stride(0)), _ptr(kx), _ptr(kr),
         _ptr(vt), _i(n), _ptr(items), _i(n_items), _i(H), _i(dim), _i(rot),
-        _i(V), _i(window), _f(scale), st), "hy_latent_flash")
+        _i(V), _i(window), _f(scale), _p(sink),
+        _i(-1 if g_off is None else g_off), st), "hy_latent_flash")
 
 
 # -- gated delta rule ------------------------------------------------------
@@ -404,15 +448,16 @@ def pair_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
 
 # -- linear recurrences ----------------------------------------------------
 
-def _gated_norm(out, y, gate, g_off, w, groups, gate_first: bool,
-                eps) -> None:
+def _gated_norm(out, y, gate, g_off, w, groups, gate_first: bool, eps,
+                sigm: bool = False) -> None:
     """Rows of ``groups`` equal parts, each normed by its own rms and
-    times ``w`` (repeated along the row); silu(gate) before or after."""
+    times ``w`` (repeated along the row); silu(gate) before or after, or
+    sigmoid(gate) after (``sigm``)."""
     T, W = y.shape
     _check(native().hy_gated_norm(
         _ptr(out), _i(out.stride(0)), _ptr(y), _ptr(gate),
         _i(gate.stride(0)), _i(g_off), _ptr(w), _i(w.shape[0]), _i(T),
-        _i(groups), _i(W // groups), _i(gate_first), _f(eps),
+        _i(groups), _i(W // groups), _i(gate_first), _i(sigm), _f(eps),
         _dt(out.dtype), _stream()), "hy_gated_norm")
 
 
@@ -447,7 +492,7 @@ def gated_linear(out, proj, k_off, v_off, g_off, dec, dec_bias, state, b,
         _ptr(o), _ptr(state), _ptr(proj), ld, _i(0), _i(k_off), _i(v_off),
         _ptr(g), None, None, _ptr(b.e_start), _ptr(b.e_len), _ptr(b.e_pos),
         _ptr(b.e_row), _i(len(b.entries)), _i(H), _i(H), _i(D), _i(V),
-        q_scale, dt, st), "hy_linear_scan")
+        q_scale, None, None, dt, st), "hy_linear_scan")
     _gated_norm(out, o, proj, g_off, w_norm, H, False, eps)
 
 
@@ -492,11 +537,89 @@ def state_space(out, proj, z_off, dt_off, state, ring, b, wconv, bconv,
             _i(H * V), _i(0), _ptr(steps[0]), _ptr(steps[1]),
             _ptr(per_head[2]), _ptr(b.e_start), _ptr(b.e_len),
             _ptr(b.e_pos), _ptr(b.e_row), _i(len(b.entries)), _i(G), _i(H),
-            _i(N), _i(V), _f(1.0), dt, st), "hy_linear_scan")
+            _i(N), _i(V), _f(1.0), None, None, dt, st), "hy_linear_scan")
     _gated_norm(out, o, proj, z_off, w_norm, norm_groups, True, eps)
 
 
+def memory_extra(dim: int) -> int:
+    """Floats per head that matrix memory keeps beside its matrix: the
+    normaliser, padded to whole vectors, and a vector whose first number
+    is the running maximum."""
+    return -(-dim // 4) * 4 + 4
+
+
+def matrix_memory(out, proj, k_off, v_off, g_off, i_off, gate_bias, cap,
+                  state, extra, b, w_norm, heads, dim, vdim, eps) -> None:
+    """mLSTM of a packed batch into ``out`` [T, H * vdim] (columns of
+    wider rows): recurrence, head norms and output gate.  ``proj`` starts
+    with the queries; the input gates are H columns from ``i_off`` on,
+    the forget gates the next H; ``gate_bias`` [2, H].  ``w_norm``
+    [H * vdim].  Updates ``state`` [slots, H, vdim, dim] and ``extra``
+    [slots, H, memory_extra(dim)]."""
+    if not proj.is_cuda:
+        ref.matrix_memory(out, proj, k_off, v_off, g_off, i_off, gate_bias,
+                          cap, state, extra, b, w_norm, heads, dim, vdim,
+                          eps)
+        return
+    T, H, D, V = b.n_tok, heads, dim, vdim
+    assert proj.stride(1) == 1 and out.stride(1) == 1 \
+        and extra.shape[1:] == (H, memory_extra(D)) \
+        and w_norm.numel() == H * V and gate_bias.numel() == 2 * H
+    lib, dt, st = native(), _dt(proj.dtype), _stream()
+    ld, q_scale = _i(proj.stride(0)), _f(D ** -0.5)
+    if b.decode:
+        _check(lib.hy_memory_step(
+            _ptr(out), _i(out.stride(0)), _ptr(state), _ptr(extra),
+            _ptr(proj), ld, _i(k_off), _i(v_off), _i(g_off), _i(i_off),
+            _ptr(gate_bias), _ptr(w_norm), _ptr(b.pos), _ptr(b.row), _i(T),
+            _i(H), _i(D), _i(V), q_scale, _f(cap), _f(eps), dt, st),
+            "hy_memory_step")
+        return
+    E = len(b.entries)
+    f32 = dict(dtype=torch.float32, device=proj.device)
+    steps = torch.empty(3, T, H, **f32)
+    n0 = torch.empty(E, H, D, **f32)
+    o = torch.empty(T, H * V, **f32)
+    runs = (_ptr(b.e_start), _ptr(b.e_len), _ptr(b.e_pos), _ptr(b.e_row),
+            _i(E))
+    _check(lib.hy_memory_gates(
+        _ptr(steps), _ptr(n0), _ptr(extra), _ptr(proj), ld, _i(i_off),
+        _ptr(gate_bias), *runs, _i(T), _i(H), _i(D), _f(cap), dt, st),
+        "hy_memory_gates")
+    _check(lib.hy_linear_scan(
+        _ptr(o), _ptr(state), _ptr(proj), ld, _i(0), _i(k_off), _i(v_off),
+        _ptr(steps[0]), _ptr(steps[1]), _ptr(steps[2]), *runs, _i(H), _i(H),
+        _i(D), _i(V), q_scale, _ptr(n0), _ptr(extra), dt, st),
+        "hy_linear_scan")
+    _gated_norm(out, o, proj, g_off, w_norm, H, False, eps, True)
+
+
 # -- windowed attention ----------------------------------------------------
+
+def head_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, bq, bk,
+              wq, wk, eps, cos_sin, b, cache) -> None:
+    """Add biases (``bq``, ``bk`` float32, None: none) to queries (the
+    first columns of ``proj``) and keys, norm each head by itself with
+    the weights ``wq`` and ``wk`` [dim], rotate its first ``rot`` numbers
+    (pairs half of them apart), the queries in place; put keys and values
+    into the pages.  ``v_off`` None: the values are the keys with their
+    biases, before norm and rotation.  ``wq`` carries the scores' scale
+    and log2(e)."""
+    if not proj.is_cuda:
+        ref.head_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off,
+                      bq, bk, wq, wk, eps, cos_sin, b, cache)
+        return
+    assert proj.stride(1) == 1 and wq.numel() == dim == wk.numel() \
+        and (bq is None or bq.numel() == heads * dim) \
+        and (bk is None or bk.numel() == kv_heads * dim)
+    bt = b.block_tables
+    _check(native().hy_head_prep(
+        _ptr(proj), _i(proj.stride(0)), _ptr(cache), _i(k_off),
+        _i(-1 if v_off is None else v_off), _i(heads), _i(kv_heads), _i(dim),
+        _i(vdim), _i(rot), _p(bq), _p(bk), _ptr(wq), _ptr(wk), _p(cos_sin),
+        _f(eps), _ptr(b.pos), _ptr(b.row), _ptr(bt), _i(bt.shape[1]),
+        _i(b.n_tok), _dt(proj.dtype), _stream()), "hy_head_prep")
+
 
 def window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk,
                 eps, cos_sin, b, cache) -> None:
@@ -571,14 +694,17 @@ def window_parts(n: int, kv_heads: int, group: int, keys: int) -> int:
 
 
 def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
-                     window) -> None:
+                     window, chunk: bool = False) -> None:
     """Attention of the prepared queries over the last ``window`` tokens,
-    times the sigmoid of the heads' numbers at column ``g_off``, into
-    ``out`` [T, H * vdim] (columns of wider rows)."""
+    or (``chunk``) over those of the query's own run of ``window``
+    positions, times the sigmoid of the heads' numbers at column
+    ``g_off`` (None: no gate), into ``out`` [T, H * vdim] (columns of
+    wider rows)."""
     if not proj.is_cuda:
         ref.window_attention(out, proj, g_off, heads, kv_heads, dim, vdim,
-                             cache, b, window)
+                             cache, b, window, chunk)
         return
+    g_off = -1 if g_off is None else g_off
     assert proj.stride(1) == 1 and out.stride(1) == 1
     lib, bt, st = native(), b.block_tables, _stream()
     H, G, D, V = heads, kv_heads, dim, vdim
@@ -586,7 +712,7 @@ def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
     dst = (_ptr(out), _i(out.stride(0)))
     src = (_ptr(proj), _i(proj.stride(0)), _i(g_off), _ptr(cache))
     where = (_ptr(bt), _i(bt.shape[1]))
-    sizes = (_i(H), _i(G), _i(D), _i(V), _i(window))
+    sizes = (_i(H), _i(G), _i(D), _i(V), _i(window), _i(chunk))
     # vector accesses need whole vectors in every row
     if not (can_window_mfma(proj.dtype, H // G, D, V)
             and proj.stride(0) % 8 == 0 and out.stride(0) % 8 == 0):

@@ -38,9 +38,20 @@ def add_norms(x, y, w1, w2, eps, dtype, mult=1.0, routed=None):
     return (n * w1).to(dtype), None if w2 is None else (n * w2).to(dtype)
 
 
-def norm_rows(x, index, w, eps, dtype, w_offset):
+def _norm(x, eps, centred):
+    return _rms(x - x.mean(-1, keepdim=True) if centred else x, eps)
+
+
+def post_pre_norm(x, y, w_post, w_pre, eps, dtype, centred):
+    if y is not None:
+        x += _norm(y.float(), eps, centred) * w_post
+    return None if w_pre is None else (_norm(x, eps, centred)
+                                       * w_pre).to(dtype)
+
+
+def norm_rows(x, index, w, eps, dtype, w_offset, centred):
     rows = x if index is None else x[index.long()]
-    return (_rms(rows, eps) * (w_offset + w)).to(dtype)
+    return (_norm(rows, eps, centred) * (w_offset + w)).to(dtype)
 
 
 def gelu_tanh_(y):
@@ -88,7 +99,7 @@ def latent_prep(proj, heads, dim, rot, rank, c_off, w_norm, eps, cos_sin, b,
         proj[:, c_off + rank:c_off + rank + rot], cs)
 
 
-def latent_rows(qa, proj, dim, rot, cache, b, window, scale):
+def latent_rows(qa, proj, dim, rot, cache, b, window, scale, sink):
     H, N, rank = qa.shape
     out = torch.empty_like(qa)
     q = proj[:N, :H * (dim + rot)].reshape(N, H, dim + rot)
@@ -98,9 +109,18 @@ def latent_rows(qa, proj, dim, rot, cache, b, window, scale):
         page = b.block_tables[int(b.row[n]), js // PAGE].long()
         key = cache[page, js % PAGE].float()
         full = torch.cat([qa[:, n], q[n, :, dim:]], -1).float()
-        a = torch.softmax(full @ key.T * scale, -1)
+        s = full @ key.T * scale
+        if sink is not None:
+            s = torch.cat([s, sink[:, None]], -1)
+        a = torch.softmax(s, -1)[:, :len(js)]
         out[:, n] = (a @ key[:, :rank]).to(out.dtype)
     return out
+
+
+def join_heads(out, o, proj, g_off):
+    H, N, V = o.shape
+    gate = torch.sigmoid(proj[:N, g_off:g_off + H * V].float())
+    out.copy_(o.transpose(0, 1).reshape(N, H * V) * gate)
 
 
 def gated_delta(proj, b_off, dec, gate, state, ring, b, wconv, a_log,
@@ -232,7 +252,64 @@ def state_space(out, proj, z_off, dt_off, state, ring, b, wconv, bconv,
         out[start:start + n] = o.to(out.dtype)
 
 
+def matrix_memory(out, proj, k_off, v_off, g_off, i_off, gate_bias, cap,
+                  state, extra, b, w_norm, heads, dim, vdim, eps):
+    H, D, V = heads, dim, vdim
+    for start, n, pos, row in b.entries:
+        x = proj[start:start + n].float()
+        q = x[:, :H * D].view(n, H, D) * D ** -0.5
+        k = x[:, k_off:k_off + H * D].view(n, H, D)
+        v = x[:, v_off:v_off + H * V].view(n, H, V)
+        z = x[:, i_off:i_off + 2 * H].view(n, 2, H) + gate_bias.view(2, H)
+        z = cap * torch.tanh(z / cap)
+        li, lf = z[:, 0], F.logsigmoid(z[:, 1])
+        S, N, m = state[row], extra[row, :, :D], extra[row, :, -4]
+        if not pos:
+            for t in (S, N, m):
+                t.zero_()
+        o = torch.empty(n, H, V)
+        for t in range(n):
+            now = torch.maximum(lf[t] + m, li[t])
+            keep = torch.exp(lf[t] + m - now)[:, None]
+            put = torch.exp(li[t] - now)[:, None] * k[t]
+            S *= keep[..., None]
+            S += v[t][..., None] * put[:, None]
+            N.mul_(keep).add_(put)
+            m.copy_(now)
+            den = torch.maximum((N * q[t]).sum(-1).abs(), torch.exp(-m))
+            o[t] = torch.einsum("hvd,hd->hv", S, q[t]) \
+                / (den + 1e-6)[:, None]
+        o = _rms(o, eps).reshape(n, H * V) * w_norm
+        gate = torch.sigmoid(x[:, g_off:g_off + H * V])
+        out[start:start + n] = (o * gate).to(out.dtype)
+
+
 # -- windowed attention ----------------------------------------------------
+
+def head_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, bq, bk,
+              wq, wk, eps, cos_sin, b, cache):
+    T, H, G, D, V = b.n_tok, heads, kv_heads, dim, vdim
+    pos = b.pos.long()
+
+    def section(at, n, bias):
+        x = proj[:, at:at + n * D].float()
+        return (x if bias is None else x + bias).view(T, n, D)
+
+    def normed(x, w):
+        y = _rms(x, eps) * w
+        if rot:
+            y = torch.cat([_turn(y[..., :rot], cos_sin[pos]), y[..., rot:]],
+                          -1)
+        return y.to(proj.dtype)
+
+    q, k = section(0, H, bq), section(k_off, G, bk)
+    v = k if v_off is None else proj[:, v_off:v_off + G * V].reshape(T, G, V)
+    proj[:, :H * D] = normed(q, wq).reshape(T, -1)
+    page = b.block_tables[b.row.long(), pos // PAGE].long()
+    rows = cache.view(cache.shape[0], G, PAGE, D + V)
+    rows[page, :, pos % PAGE] = torch.cat(
+        [normed(k, wk), v.to(proj.dtype)], -1)
+
 
 def window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk,
                 eps, cos_sin, b, cache):
@@ -255,21 +332,23 @@ def window_prep(proj, heads, kv_heads, dim, vdim, rot, k_off, v_off, wq, wk,
 
 
 def window_attention(out, proj, g_off, heads, kv_heads, dim, vdim, cache, b,
-                     window):
+                     window, chunk):
     H, G, D, V = heads, kv_heads, dim, vdim
     rows = cache.view(cache.shape[0], G, PAGE, D + V)
     head = torch.arange(H) // (H // G)
     for t in range(b.n_tok):
         p = int(b.pos[t])
-        js = torch.arange(max(0, p - window + 1), p + 1)
+        first = p - p % window if chunk else max(0, p - window + 1)
+        js = torch.arange(first, p + 1)
         page = b.block_tables[int(b.row[t]), js // PAGE].long()
         kv = rows[page, :, js % PAGE].float()[:, head]         # [j, H, ..]
         s = torch.einsum("hd,jhd->hj", proj[t, :H * D].view(H, D).float(),
                          kv[..., :D])
         a = torch.softmax(s * LN2, -1)
         o = torch.einsum("hj,jhv->hv", a, kv[..., D:])
-        gate = torch.sigmoid(proj[t, g_off:g_off + H].float())
-        out[t] = (o * gate[:, None]).reshape(-1).to(out.dtype)
+        if g_off is not None:
+            o = o * torch.sigmoid(proj[t, g_off:g_off + H].float())[:, None]
+        out[t] = o.reshape(-1).to(out.dtype)
 
 
 # -- mixture of experts ----------------------------------------------------
