@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Prefill and decode throughput of the hybrid models (Dibelix, Taletar,
-Fidepel) beside the Llama family at equal width, depth and parameter count
-(random weights, one GPU).
+Fidepel, Rasodra) beside the Llama family at equal width, depth and
+parameter count (random weights, one GPU).
 
   python bench.py --hybrid [--steps K --warmup W]      all sizes, one JSON
   python benchmarks/hybrid_bench.py --size m --only dibelix --phase decode
@@ -31,7 +31,7 @@ SIZES = {
     "m": (2048, 8, 16, 128, 4, 5632),
     "l": (4096, 8, 32, 128, 8, 14336),
 }
-VOCAB, WINDOW = 32000, 1024
+VOCAB, WINDOW, CHUNK = 32000, 1024, 2048
 
 
 def llama_config(size: str):
@@ -102,8 +102,26 @@ def fidepel_config(size: str):
     return build(fit_ff(FidepelForCausalLM, build, size, 2 * 17))
 
 
+def rasodra_config(size: str):
+    """The same width, depth and heads in every mixer; chunks hold a whole
+    prompt, so that attention sees what the Llama model's does."""
+    from llmlb_amd.models.rasodra import RasodraConfig, RasodraForCausalLM
+    w, n, h, d, kv, inter = SIZES[size]
+
+    def build(ff):
+        return RasodraConfig.build(
+            "AMLM" * (n // 4), vocab=VOCAB, width=w, ff=ff, heads=h,
+            kv_heads=kv, dim=d, chunk=CHUNK, latent_heads=h, latent_dim=d,
+            rot_dim=d // 2, latent_vdim=d, kv_rank=4 * d, memory_heads=h,
+            memory_dim=d, memory_vdim=d, max_pos=8192,
+            name=f"rasodra-{size}")
+
+    return build(fit_ff(RasodraForCausalLM, build, size, 2))
+
+
 CONFIGS = {"llama": llama_config, "dibelix": dibelix_config,
-           "taletar": taletar_config, "fidepel": fidepel_config}
+           "taletar": taletar_config, "fidepel": fidepel_config,
+           "rasodra": rasodra_config}
 
 
 def make_engine(cfg, args):
@@ -186,7 +204,7 @@ def measure(kind: str, size: str, args) -> dict:
 
 def add_arguments(ap) -> None:
     ap.add_argument("--size", default="s,m,l", help="of s, m, l")
-    ap.add_argument("--only", default="llama,dibelix,taletar,fidepel")
+    ap.add_argument("--only", default="llama,dibelix,taletar,fidepel,rasodra")
     ap.add_argument("--phase", default="all",
                     choices=("all", "prefill", "decode"))
     ap.add_argument("--prompts", type=int, default=8)
@@ -210,6 +228,7 @@ def run(args) -> dict:
             "config": {"prompts": args.prompts,
                        "prompt_len": args.prompt_len, "batch": args.batch,
                        "context": args.context, "window": WINDOW,
+                       "chunk": CHUNK,
                        "layers": {
                            "dibelix": "latent attention, two gated delta "
                                       "layers, shared latents; repeated",
@@ -217,7 +236,9 @@ def run(args) -> dict:
                                       "linear attention, Mamba-2, gated "
                                       "linear attention; repeated",
                            "fidepel": "windowed attention and 4 of 16 "
-                                      "experts beside a shared one"}},
+                                      "experts beside a shared one",
+                           "rasodra": "chunked attention, mLSTM, latent "
+                                      "attention, mLSTM; repeated"}},
             "steps": args.steps, "warmup": args.warmup, "sizes": sizes}
 
 

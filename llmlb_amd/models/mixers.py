@@ -57,9 +57,8 @@ def _halves(dim: int, rot: int) -> torch.Tensor:
     rotate pairs.  Scores do not change when queries and keys share an
     order."""
     order = torch.arange(dim)
-    order[:rot] = torch.cat([torch.arange(0, rot, 2),
-                             torch.arange(1, rot, 2)])
-    return order
+    turned = order[:rot]
+    return torch.cat([turned[0::2], turned[1::2], order[rot:]])
 
 
 class LatentAttention(nn.Module):
@@ -258,8 +257,11 @@ class DenseFF(nn.Module):
 
     def load(self, w: dict[str, torch.Tensor]) -> None:
         to = dict(dtype=self.dtype, device=self.device)
-        self.w_up = _param(w["up"].to(**to))
-        self.w_down = _param(w["down"].to(**to))
+        # an uneven depth would keep the staged decode GEMM from the
+        # product down; what is added is zero in both matrices
+        gap = -self.ff % 256 if self.ff >= 4096 else 0
+        self.w_up = _param(F.pad(w["up"], (0, 0, 0, gap)).to(**to))
+        self.w_down = _param(F.pad(w["down"], (0, gap)).to(**to))
 
     def forward(self, x):
         u = _linear(x, self.w_up)

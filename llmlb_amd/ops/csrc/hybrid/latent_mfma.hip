@@ -313,13 +313,14 @@ void latent_decode_kernel(
 
   // the thread's pieces of a page, as offsets into it and into LDS
   // (threads past the last piece repeat it)
-  int p_from[PL], p_to[PL];
+  int p_from[PL], p_to[PL], p_row[PL];
 #pragma unroll
   for (int i = 0; i < PL; ++i) {
     int p = tid + i * 256;
     p = p < PAGE * pieces ? p : PAGE * pieces - 1;
     p_from[i] = p * 8;
-    p_to[i] = p / pieces * PITCH + p % pieces * 8;
+    p_row[i] = p / pieces;
+    p_to[i] = p_row[i] * PITCH + p % pieces * 8;
   }
   // page numbers are wave-uniform and fetched a tile ahead of the rows
   int pg[PAGES];
@@ -380,6 +381,15 @@ void latent_decode_kernel(
     for (int t = 0; t < NT; ++t) o[a][t] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   for (int t = t_lo; t < t_hi; ++t) {
+    // rows past the last key meet zero weights and must be finite
+    const int left = pos - base - t * KEYS;
+    if (left < KEYS - 1) {
+#pragma unroll
+      for (int k = 0; k < PAGES; ++k)
+#pragma unroll
+        for (int i = 0; i < PL; ++i)
+          if (k * PAGE + p_row[i] > left) pk[k][i] = u32x4{0, 0, 0, 0};
+    }
 #pragma unroll
     for (int k = 0; k < PAGES; ++k)
 #pragma unroll

@@ -18,22 +18,10 @@
 //
 // Everything that enters the state is float; q, k and v keep the storage
 // type they were projected or convolved in until they are used.
+#include "memory.h"
 #include "recurrent.h"
 
 enum Kind { CHANNEL, HEAD, MEMORY };  // gated linear, Mamba-2, mLSTM
-
-__host__ __device__ __forceinline__ int extra_row(int D) {
-  return (D + 3) / 4 * 4 + 4;
-}
-
-// Log input and forget gates of one head and token, cap tanh(z / cap) and
-// the logarithm of its sigmoid.
-__device__ __forceinline__ void memory_gates(float zi, float zf, float cap,
-                                             float& li, float& lf) {
-  li = cap * tanhf(zi / cap);
-  lf = -softplus_f(-cap * tanhf(zf / cap));
-}
-#define MEMORY_EPS 1e-6f
 
 // N consecutive elements as they lie in memory, widened on use, so that
 // elements in flight take half the registers and nothing waits for them.

@@ -548,6 +548,12 @@ def memory_extra(dim: int) -> int:
     return -(-dim // 4) * 4 + 4
 
 
+def can_memory_mfma(dtype, dim, vdim) -> bool:
+    """Sizes that the matrix-core kernel takes."""
+    return (dtype == torch.bfloat16 and dim % 8 == 0 and vdim % 8 == 0
+            and dim <= 256)
+
+
 def matrix_memory(out, proj, k_off, v_off, g_off, i_off, gate_bias, cap,
                   state, extra, b, w_norm, heads, dim, vdim, eps) -> None:
     """mLSTM of a packed batch into ``out`` [T, H * vdim] (columns of
@@ -578,10 +584,21 @@ def matrix_memory(out, proj, k_off, v_off, g_off, i_off, gate_bias, cap,
     E = len(b.entries)
     f32 = dict(dtype=torch.float32, device=proj.device)
     steps = torch.empty(3, T, H, **f32)
-    n0 = torch.empty(E, H, D, **f32)
     o = torch.empty(T, H * V, **f32)
     runs = (_ptr(b.e_start), _ptr(b.e_len), _ptr(b.e_pos), _ptr(b.e_row),
             _i(E))
+    if can_memory_mfma(proj.dtype, D, V) and proj.stride(0) % 8 == 0 \
+            and k_off % 8 == 0 and v_off % 8 == 0:
+        carry = torch.empty(E, H, memory_extra(D), **f32)
+        _check(lib.hy_memory_chunk(
+            _ptr(o), _ptr(steps), _ptr(carry), _ptr(state), _ptr(extra),
+            _ptr(proj), ld, _i(k_off), _i(v_off), _i(i_off),
+            _ptr(gate_bias), *runs, _i(max(n for _, n, _, _ in b.entries)),
+            _i(T), _i(H), _i(D), _i(V), q_scale, _f(cap), st),
+            "hy_memory_chunk")
+        _gated_norm(out, o, proj, g_off, w_norm, H, False, eps, True)
+        return
+    n0 = torch.empty(E, H, D, **f32)
     _check(lib.hy_memory_gates(
         _ptr(steps), _ptr(n0), _ptr(extra), _ptr(proj), ld, _i(i_off),
         _ptr(gate_bias), *runs, _i(T), _i(H), _i(D), _f(cap), dt, st),

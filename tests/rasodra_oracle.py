@@ -7,8 +7,6 @@ llmlb_amd, keeps no cache, and always runs a sequence from its start.
 """
 from __future__ import annotations
 
-import math
-
 import torch
 
 F64 = torch.float64
@@ -35,13 +33,12 @@ def rotate(x, base, n):
     """x [T, heads, D]: neighbours (2i, 2i + 1) among the first n numbers
     of every head turn by position times base^(-2i/n)."""
     out = x.clone()
-    for p in range(x.shape[0]):
-        for i in range(n // 2):
-            a = p * base ** (-2.0 * i / n)
-            c, s = math.cos(a), math.sin(a)
-            u, v = x[p, :, 2 * i], x[p, :, 2 * i + 1]
-            out[p, :, 2 * i] = u * c - v * s
-            out[p, :, 2 * i + 1] = v * c + u * s
+    p = torch.arange(x.shape[0], dtype=F64)[:, None]
+    for i in range(n // 2):
+        a = p * base ** (-2.0 * i / n)
+        u, v = x[:, :, 2 * i], x[:, :, 2 * i + 1]
+        out[:, :, 2 * i] = u * a.cos() - v * a.sin()
+        out[:, :, 2 * i + 1] = v * a.cos() + u * a.sin()
     return out
 
 
