@@ -323,19 +323,24 @@ __global__ __launch_bounds__(256) void norm_rows_kernel(
 // x += norm(y) w_post, h = norm(x) w_pre in the storage type: what lies
 // between two sublayers whose outputs are normed as well as their inputs.
 // y null: nothing is added; w_pre (and h) null: the sum alone.  CENTRED:
-// layer norms, else RMS norms.  One workgroup per row; KEEP runs of N
-// neighbours a thread stay in registers between the passes, the rest is
-// read again.
-template <typename T, int N, int KEEP, bool CENTRED>
+// layer norms, else RMS norms.  L threads a row, a wave or the workgroup;
+// KEEP runs of N neighbours a thread stay in registers between the passes,
+// the rest is read again.
+template <typename T, int L, int N, int KEEP, bool CENTRED>
 __global__ __launch_bounds__(256) void post_pre_norm_kernel(
     float* __restrict__ x, const T* __restrict__ y,
     const float* __restrict__ w_post, const float* __restrict__ w_pre,
-    T* __restrict__ h, int width, float eps) {
+    T* __restrict__ h, int n_tok, int width, float eps) {
   __shared__ float red[4][4];
-  const int runs = width / N, tid = threadIdx.x;
+  const int runs = width / N, tid = threadIdx.x % L;
+  const int row = blockIdx.x * (256 / L) + threadIdx.x / L;
+  if (row >= n_tok) return;  // whole waves
   const float inv = 1.f / width;
-  float* xr = x + (size_t)blockIdx.x * width;
-  const T* yr = y ? y + (size_t)blockIdx.x * width : nullptr;
+  float* xr = x + (size_t)row * width;
+  const T* yr = y ? y + (size_t)row * width : nullptr;
+  auto over_row = [](float s, float* red) {
+    return L == WAVE ? wave_sum(s) : block_sum_256(s, red);
+  };
   auto load = [](const auto* p, float* f) {
     if constexpr (N == 8) load8(p, f);
     else f[0] = to_f(p[0]);
@@ -351,42 +356,42 @@ __global__ __launch_bounds__(256) void post_pre_norm_kernel(
     float s = 0.f;
 #pragma unroll
     for (int k = 0; k < KEEP; ++k)
-      if (tid + k * 256 < runs)
+      if (tid + k * L < runs)
 #pragma unroll
         for (int j = 0; j < N; ++j) s += keep[k][j];
-    for (int i = tid + KEEP * 256; i < runs; i += 256) {
+    for (int i = tid + KEEP * L; i < runs; i += L) {
       float f[N];
       load(src + (size_t)i * N, f);
 #pragma unroll
       for (int j = 0; j < N; ++j) s += f[j];
     }
-    return block_sum_256(s, red);
+    return over_row(s, red);
   };
   auto squares = [&](const auto* src, float* red) {
     float s = 0.f;
 #pragma unroll
     for (int k = 0; k < KEEP; ++k)
-      if (tid + k * 256 < runs)
+      if (tid + k * L < runs)
 #pragma unroll
         for (int j = 0; j < N; ++j)
           s += (keep[k][j] - mean) * (keep[k][j] - mean);
-    for (int i = tid + KEEP * 256; i < runs; i += 256) {
+    for (int i = tid + KEEP * L; i < runs; i += L) {
       float f[N];
       load(src + (size_t)i * N, f);
 #pragma unroll
       for (int j = 0; j < N; ++j) s += (f[j] - mean) * (f[j] - mean);
     }
-    return block_sum_256(s, red);
+    return over_row(s, red);
   };
   if (y) {
     // the stream's loads fly behind the norm of y
     float xk[KEEP][N];
 #pragma unroll
     for (int k = 0; k < KEEP; ++k)
-      if (tid + k * 256 < runs) load(yr + (size_t)(tid + k * 256) * N, keep[k]);
+      if (tid + k * L < runs) load(yr + (size_t)(tid + k * L) * N, keep[k]);
 #pragma unroll
     for (int k = 0; k < KEEP; ++k)
-      if (tid + k * 256 < runs) load(xr + (size_t)(tid + k * 256) * N, xk[k]);
+      if (tid + k * L < runs) load(xr + (size_t)(tid + k * L) * N, xk[k]);
     if (CENTRED) mean = total(yr, red[0]) * inv;
     const float r = 1.f / sqrtf(squares(yr, red[1]) * inv + eps);
     auto add = [&](int i, const float* f, float* out) {
@@ -398,12 +403,12 @@ __global__ __launch_bounds__(256) void post_pre_norm_kernel(
     };
 #pragma unroll
     for (int k = 0; k < KEEP; ++k)
-      if (tid + k * 256 < runs) {
-        add(tid + k * 256, keep[k], xk[k]);
+      if (tid + k * L < runs) {
+        add(tid + k * L, keep[k], xk[k]);
 #pragma unroll
         for (int j = 0; j < N; ++j) keep[k][j] = xk[k][j];
       }
-    for (int i = tid + KEEP * 256; i < runs; i += 256) {
+    for (int i = tid + KEEP * L; i < runs; i += L) {
       float f[N], v[N];
       load(yr + (size_t)i * N, f);
       load(xr + (size_t)i * N, v);
@@ -412,14 +417,14 @@ __global__ __launch_bounds__(256) void post_pre_norm_kernel(
   } else {
 #pragma unroll
     for (int k = 0; k < KEEP; ++k)
-      if (tid + k * 256 < runs) load(xr + (size_t)(tid + k * 256) * N, keep[k]);
+      if (tid + k * L < runs) load(xr + (size_t)(tid + k * L) * N, keep[k]);
   }
   if (!w_pre) return;
   // beyond the kept runs a thread reads back only what it wrote itself
   mean = 0.f;
   if (CENTRED) mean = total(xr, red[2]) * inv;
   const float r = 1.f / sqrtf(squares(xr, red[3]) * inv + eps);
-  T* hr = h + (size_t)blockIdx.x * width;
+  T* hr = h + (size_t)row * width;
   auto emit = [&](int i, float* f) {
     float w[N];
     load(w_pre + (size_t)i * N, w);
@@ -429,8 +434,8 @@ __global__ __launch_bounds__(256) void post_pre_norm_kernel(
   };
 #pragma unroll
   for (int k = 0; k < KEEP; ++k)
-    if (tid + k * 256 < runs) emit(tid + k * 256, keep[k]);
-  for (int i = tid + KEEP * 256; i < runs; i += 256) {
+    if (tid + k * L < runs) emit(tid + k * L, keep[k]);
+  for (int i = tid + KEEP * L; i < runs; i += L) {
     float f[N];
     load(xr + (size_t)i * N, f);
     emit(i, f);
@@ -601,20 +606,23 @@ int hy_post_pre_norm(void* x, const void* y, const void* w_post,
                      int width, float eps, int dtype, void* stream) {
   if ((y && !w_post) || (w_pre && !h) || width <= 0) return -2;
   if (n_tok <= 0) return 0;
-#define GO(N, KEEP, CENTRED)                                                 \
+#define GO(L, N, KEEP, CENTRED)                                              \
   HY_DTYPE(dtype, hipLaunchKernelGGL(                                        \
-      (post_pre_norm_kernel<T, N, KEEP, CENTRED>), dim3(n_tok), dim3(256),   \
-      0, (hipStream_t)stream, (float*)x, (const T*)y, (const float*)w_post,  \
-      (const float*)w_pre, (T*)h, width, eps))
-#define PICK(N, KEEP)                 \
-  do {                                \
-    if (centred) GO(N, KEEP, true);   \
-    else GO(N, KEEP, false);          \
+      (post_pre_norm_kernel<T, L, N, KEEP, CENTRED>),                        \
+      dim3((n_tok + 256 / L - 1) / (256 / L)), dim3(256), 0,                 \
+      (hipStream_t)stream, (float*)x, (const T*)y, (const float*)w_post,     \
+      (const float*)w_pre, (T*)h, n_tok, width, eps))
+#define PICK(L, N, KEEP)                 \
+  do {                                   \
+    if (centred) GO(L, N, KEEP, true);   \
+    else GO(L, N, KEEP, false);          \
   } while (0)
-  if (width % 8) PICK(1, 4);
-  else if (width <= 2048) PICK(8, 1);
-  else if (width <= 4096) PICK(8, 2);
-  else PICK(8, 4);
+  if (width % 8) PICK(256, 1, 4);
+  else if (width <= 512) PICK(64, 8, 1);
+  else if (width <= 1024) PICK(64, 8, 2);
+  else if (width <= 2048) PICK(256, 8, 1);
+  else if (width <= 4096) PICK(256, 8, 2);
+  else PICK(256, 8, 4);
 #undef PICK
 #undef GO
   HY_CHECK();

@@ -369,8 +369,8 @@ def test_memory_full_chip(ly, rows, dtype):
 
 # -- rows ------------------------------------------------------------------
 
-@pytest.mark.parametrize("width", [7, 52, 256, 2048, 4096, 8200, 16384,
-                                   9001])
+@pytest.mark.parametrize("width", [7, 52, 256, 520, 1024, 2048, 4096, 8200,
+                                   16384, 9001])
 @DTYPES
 def test_post_pre_norm(width, dtype):
     g = torch.Generator().manual_seed(width)
