@@ -4,8 +4,9 @@ Each library is built from its own sources, so a program that needs one
 model family compiles only that family's kernels:
 
   kernels   csrc/*.hip          Llama-family ops and decode GEMMs
-  hybrid    csrc/hybrid/*.hip   latent and differential attention,
-                                recurrences, the 32-bit residual stream
+  hybrid    csrc/hybrid/*.hip   latent, differential, windowed and
+                                chunked attention, recurrences, the
+                                32-bit residual stream
 
 Command line: ``python -m llmlb_amd.ops.build [name ...]`` (all without
 a name).

@@ -24,8 +24,8 @@
 // Per token and head F, c = i - F and b, as gates [3][H][n_tok]; also
 // copies normaliser and maximum out of the state to ``carry``
 // [entries][H][extra_row(D)] (several workgroups read them later, and one
-// replaces them).  A workgroup: a chunk and 16 heads.
-__global__ __launch_bounds__(256) void memory_chunk_gates_kernel(
+// replaces them).  A workgroup: a chunk and 16 heads, a wave each.
+__global__ __launch_bounds__(1024) void memory_chunk_gates_kernel(
     float* __restrict__ gates, float* __restrict__ carry,
     const float* __restrict__ extra, const bf16_t* __restrict__ proj, int ld,
     int i_off, const float* __restrict__ bias, const int* __restrict__ e_start,
@@ -43,10 +43,10 @@ __global__ __launch_bounds__(256) void memory_chunk_gates_kernel(
     const bool resume = e_pos[e] > 0;
     const float* src = extra + ((size_t)e_row[e] * H + h0) * row;
     float* dst = carry + ((size_t)e * H + h0) * row;
-    for (int i = tid; i < heads * row; i += 256)
+    for (int i = tid; i < heads * row; i += 1024)
       dst[i] = resume ? src[i] : 0.f;
   }
-  for (int i = tid; i < CHUNK * 32; i += 256) {
+  for (int i = tid; i < CHUNK * 32; i += 1024) {
     const int t = t0 + i / 32, c = i % 32, h = c % 16;
     if (h < heads)
       z[i / 32][c] =
@@ -54,7 +54,8 @@ __global__ __launch_bounds__(256) void memory_chunk_gates_kernel(
                     c / 16 * H + h0 + h]);
   }
   __syncthreads();
-  for (int h = wave; h < heads; h += 4) {
+  const int h = wave;
+  if (h < heads) {
     float li, lf;
     memory_gates(z[lane][h] + bias[h0 + h], z[lane][16 + h] + bias[H + h0 + h],
                  cap, li, lf);
@@ -408,7 +409,7 @@ int hy_memory_chunk(void* o, void* gates, void* carry, void* state,
   hipLaunchKernelGGL(
       memory_chunk_gates_kernel,
       dim3((max_len + CHUNK - 1) / CHUNK, n_entries, (H + 15) / 16),
-      dim3(256), 0, s, (float*)gates, (float*)carry, (const float*)extra,
+      dim3(1024), 0, s, (float*)gates, (float*)carry, (const float*)extra,
       (const bf16_t*)proj, ld, i_off, (const float*)bias,
       (const int*)e_start, (const int*)e_len, (const int*)e_pos,
       (const int*)e_row, n_tok, H, D, cap);

@@ -617,9 +617,11 @@ int hy_post_pre_norm(void* x, const void* y, const void* w_post,
     if (centred) GO(L, N, KEEP, true);   \
     else GO(L, N, KEEP, false);          \
   } while (0)
+  // a wave a row where there are rows enough for all of them
+  const bool many = n_tok >= 2048;
   if (width % 8) PICK(256, 1, 4);
-  else if (width <= 512) PICK(64, 8, 1);
-  else if (width <= 1024) PICK(64, 8, 2);
+  else if (many && width <= 512) PICK(64, 8, 1);
+  else if (many && width <= 1024) PICK(64, 8, 2);
   else if (width <= 2048) PICK(256, 8, 1);
   else if (width <= 4096) PICK(256, 8, 2);
   else PICK(256, 8, 4);
